@@ -5,7 +5,7 @@ set -e
 cd "$(dirname "$0")/../phi-3-vision-mlx_amd/csrc"
 NAME=$1; UNIT=$2; shift 2
 OBJ=../../build/obj; mkdir -p $OBJ
-FLAGS="--offload-arch=gfx950 -O3 -std=c++17 -fPIC -Wno-unused-result"
+FLAGS="--offload-arch=gfx950 -O3 -std=c++17 -fPIC -Wno-unused-result -Xclang -target-feature -Xclang -packed-fp32-ops"
 for f in *.hip; do
   [ "$f" = "$UNIT" ] && continue
   if [ ! -f $OBJ/${f%.hip}.o ] || [ $f -nt $OBJ/${f%.hip}.o ] || [ p3v_common.h -nt $OBJ/${f%.hip}.o ] || [ ../../include/p3v.h -nt $OBJ/${f%.hip}.o ]; then
