@@ -73,7 +73,8 @@ enum {
   P3V_EPI_RESID_BF16 = 5,  /* out bf16 = resid + bf16(acc)                    phi.py:460,483-485 */
   P3V_EPI_SILU_MUL = 6,    /* W = [gate;up] (2N rows): out bf16[M,N] = silu(g)*u  phi.py:469-471 */
   P3V_EPI_PATCH = 7,       /* out f32 row (m/P)*(P+1)+1+m%P = acc + pos[1+m%P]   phi.py:199-205 */
-  P3V_EPI_F32 = 8          /* out f32 = acc (+ bias if given)                               */
+  P3V_EPI_F32 = 8,         /* out f32 = acc (+ bias if given)                               */
+  P3V_EPI_SCALE_RESID_F32 = 9 /* out f32 = resid_f32 + col_scale[n] * acc (a residual branch with a per-channel scale) */
 };
 typedef struct {
   const uint16_t* A;   /* [M, lda] bf16 */
@@ -88,6 +89,7 @@ typedef struct {
   int patches_per_img; /* P3V_EPI_PATCH: P (=576) */
   void* ws;            /* caller-owned device workspace (16-byte aligned) or null */
   int64_t ws_bytes;    /* its size; see p3v_gemm_ws_bytes */
+  const uint16_t* col_scale; /* P3V_EPI_SCALE_RESID_F32: [N] bf16 */
 } p3v_gemm_args_t;
 /* Operands are addressed with 32-bit byte offsets: M * lda * 2 and rows(W) * ldw * 2 must stay below 4 GiB
  * (P3V_ERR_UNSUPPORTED otherwise).  Shapes with 17 <= M <= 1024 and fewer than 256 output tiles (short prompts) run split
@@ -428,6 +430,56 @@ int p3v_gemv_step(const p3v_gemv_args_t* args /* host */, const p3v_gemv_step_t*
 int p3v_gemv_fp8_step(const p3v_gemv_fp8_args_t* args /* host */, const p3v_gemv_step_t* step /* host */, void* stream);
 /* and on MLX 4-bit group-64 weights (`args` as for p3v_gemv_q4, one row, no epilogue) */
 int p3v_gemv_q4_step(const p3v_gemv_q4_args_t* args /* host */, const p3v_gemv_step_t* step /* host */, void* stream);
+
+/* ---- layered text decoders (config.py: LayerSpec).  Activations are bf16, or fp32 where a call says so (f32 / out_f32 / a_f32 != 0);
+ * the residual stream is fp32; weights are bf16. */
+/* x[n, hidden] fp32 = table[clamp(id)] * scale */
+int p3v_embed_scale(const int32_t* ids, const uint16_t* table, float* out, int n_tok, int hidden, int vocab, float scale, void* stream);
+
+/* dynamic tanh: h = tanh(alpha x) w + b per channel.  With mu, a token shift behind it: out_t = h_t + (h_{t-1} - h_t) mu, where h_{t-1}
+ * of a call's first token comes from `hist` [B, hist_rows, H] fp32 (row = cache column % hist_rows; the call stores its last
+ * hist_rows unshifted h there) and is zero for a sequence's first token (column pad_len[b], or 0). */
+typedef struct {
+  const float* x; const uint16_t* w; const uint16_t* b; const uint16_t* mu; float* hist; const int32_t* pad_len; const int32_t* d_past;
+  float alpha;
+  int past, hist_rows, B, L, H;
+} p3v_dyt_args_t;
+int p3v_dyt(const p3v_dyt_args_t* args /* host */, void* out, int out_f32, void* stream);
+
+/* p3v_gemm for every size and for fp32 A (a_f32: A is float*), plain fp32 arithmetic.  Epilogues NONE (out in A's type), F32, SILU_MUL,
+ * SCALE_RESID_F32. */
+int p3v_gemm_any(const p3v_gemm_args_t* args /* host */, int a_f32, void* stream);
+
+/* Attention with scores mixed across heads, a sink, value mixing and an output gate.  qkv rows [B*L, ld]: H*dim query, G*dim key,
+ * G*vdim value columns, then anything (the H gate logits: `gate` points at the first one, row stride ld as well).
+ *   q = rms(query row) q_norm,  k = rms(key row) k_norm   (one RMS over the whole projection, fp32)
+ *   v = value, or with v_first (row stride ld_first) (1 - vmix) value + vmix v_first
+ *   s_h = scale sum_g talk[h, g] (q_g . k_g);  p = softmax of s over the keys pad_len[b] .. own position with exp(sink_h) added to the
+ *   denominator;  out row = sigmoid(gate_h) sum p v.
+ * Caches: k [B, G, Tp, dimp], v [B, G, Tp/16, vdimp, 16] (dimp % 32 == 0, vdimp % 16 == 0, the padding zero), Tp % 32 == 0.
+ * p3v_qkv_heads writes q [B, H, L, dimp] and appends k, v; p3v_attn_mix attends from q over the cache (new tokens included);
+ * p3v_attn_mix_decode does both for L = 1 (P3V_ERR_UNSUPPORTED: run the two).  n_split from p3v_attn_mix_plan (0: the any-size kernel),
+ * ws of p3v_attn_mix_ws_bytes.  n_keys of the plan: the cache capacity for L = 1, past + L otherwise. */
+typedef struct {
+  const void* qkv; const uint16_t* q_norm; const uint16_t* k_norm; const void* v_first;
+  void* q; void* k; void* v;
+  const uint16_t* talk; const uint16_t* sink; const void* gate; void* out; float* ws;
+  const int32_t* pad_len; const int32_t* d_past;
+  float eps, vmix, scale;
+  int B, L, H, G, dim, vdim, dimp, vdimp, ld, ld_first, past, Tp, n_split, f32;
+} p3v_mix_args_t;
+int p3v_qkv_heads(const p3v_mix_args_t* args /* host */, void* stream);
+int p3v_attn_mix(const p3v_mix_args_t* args /* host */, void* stream);
+int p3v_attn_mix_decode(const p3v_mix_args_t* args /* host */, void* stream);
+int p3v_attn_mix_plan(int B, int L, int H, int G, int dim, int vdim, int n_keys, int f32);
+int64_t p3v_attn_mix_ws_bytes(int B, int L, int H, int vdim, int n_split);
+
+/* p3v_argmax / p3v_log_softmax / p3v_topk / p3v_step_end on fp32 logits */
+int p3v_argmax_f32(const float* logits, int32_t* out, int rows, int n, int64_t row_stride, void* stream);
+int p3v_log_softmax_f32(const float* x, float* y, int rows, int n, void* stream);
+int p3v_topk_f32(const float* x, int32_t* idx_out, int rows, int n, int k, int64_t row_stride, void* stream);
+int p3v_step_end_f32(const float* logits, int32_t* next_tok, int32_t* tok, int32_t* history, int32_t* d_step, int32_t* d_past, int32_t* ticket,
+                     int B, int n, int max_steps, void* stream);
 
 /* ---- hipGraph helpers: capture a sequence of the launches above and replay it */
 int p3v_graph_begin(void* stream);

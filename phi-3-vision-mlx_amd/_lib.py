@@ -4,14 +4,17 @@ The library is the product: there is NO fallback.  If it is missing or fails to
 load, every op raises -- a silent PyTorch path would void the parity claims.
 """
 import ctypes as C
+import hashlib
 import os
+import subprocess
+import sys
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.environ.get("P3V_LIB") or os.path.join(_HERE, "libp3v.so")     # P3V_LIB: debug builds only
 
 P3V_OK = 0
 (EPI_NONE, EPI_BIAS, EPI_BIAS_QGELU, EPI_BIAS_GELU, EPI_BIAS_RESID_F32, EPI_RESID_BF16, EPI_SILU_MUL, EPI_PATCH,
- EPI_F32) = range(9)
+ EPI_F32, EPI_SCALE_RESID_F32) = range(10)
 DECODE_MAX_L = 16
 
 vp, i32, i64, f32 = C.c_void_p, C.c_int, C.c_int64, C.c_float
@@ -25,7 +28,7 @@ class Props(C.Structure):
 class GemmArgs(C.Structure):
     _fields_ = [("A", vp), ("W", vp), ("out", vp), ("bias", vp), ("resid", vp), ("pos", vp),
                 ("M", i32), ("N", i32), ("K", i32), ("lda", i32), ("ldw", i32), ("ldo", i32),
-                ("epilogue", i32), ("patches_per_img", i32), ("ws", vp), ("ws_bytes", i64)]
+                ("epilogue", i32), ("patches_per_img", i32), ("ws", vp), ("ws_bytes", i64), ("col_scale", vp)]
 
 
 class QkvSplit(C.Structure):
@@ -89,6 +92,18 @@ class AttnDecQ8Args(C.Structure):
                 ("o_proj_w8", vp), ("o_proj_scale", vp), ("o_proj_x", vp), ("o_rearm", vp), ("o_n", i32)]   # optional fused o_proj (e4m3)
 
 
+class DytArgs(C.Structure):
+    _fields_ = [("x", vp), ("w", vp), ("b", vp), ("mu", vp), ("hist", vp), ("pad_len", vp), ("d_past", vp), ("alpha", f32),
+                ("past", i32), ("hist_rows", i32), ("B", i32), ("L", i32), ("H", i32)]
+
+
+class MixArgs(C.Structure):
+    _fields_ = [("qkv", vp), ("q_norm", vp), ("k_norm", vp), ("v_first", vp), ("q", vp), ("k", vp), ("v", vp), ("talk", vp), ("sink", vp),
+                ("gate", vp), ("out", vp), ("ws", vp), ("pad_len", vp), ("d_past", vp), ("eps", f32), ("vmix", f32), ("scale", f32),
+                ("B", i32), ("L", i32), ("H", i32), ("G", i32), ("dim", i32), ("vdim", i32), ("dimp", i32), ("vdimp", i32),
+                ("ld", i32), ("ld_first", i32), ("past", i32), ("Tp", i32), ("n_split", i32), ("f32", i32)]
+
+
 # name -> (restype, argtypes); must list every symbol include/p3v.h declares
 SIGNATURES = {
     "p3v_version": (i32, []),
@@ -141,6 +156,18 @@ SIGNATURES = {
     "p3v_lora_up": (i32, [vp, vp, vp, f32, i32, vp, vp, i32, i32, i32, vp]),
     "p3v_step_begin": (i32, [vp, vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, i32, i32, vp, i32, vp]),
     "p3v_step_end": (i32, [vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, vp]),
+    "p3v_embed_scale": (i32, [vp, vp, vp, i32, i32, i32, f32, vp]),
+    "p3v_dyt": (i32, [C.POINTER(DytArgs), vp, i32, vp]),
+    "p3v_gemm_any": (i32, [C.POINTER(GemmArgs), i32, vp]),
+    "p3v_qkv_heads": (i32, [C.POINTER(MixArgs), vp]),
+    "p3v_attn_mix": (i32, [C.POINTER(MixArgs), vp]),
+    "p3v_attn_mix_decode": (i32, [C.POINTER(MixArgs), vp]),
+    "p3v_attn_mix_plan": (i32, [i32, i32, i32, i32, i32, i32, i32, i32]),
+    "p3v_attn_mix_ws_bytes": (i64, [i32, i32, i32, i32, i32]),
+    "p3v_argmax_f32": (i32, [vp, vp, i32, i32, i64, vp]),
+    "p3v_log_softmax_f32": (i32, [vp, vp, i32, i32, vp]),
+    "p3v_topk_f32": (i32, [vp, vp, i32, i32, i32, i64, vp]),
+    "p3v_step_end_f32": (i32, [vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, vp]),
     "p3v_graph_begin": (i32, [vp]),
     "p3v_graph_end": (i32, [vp, C.POINTER(vp)]),
     "p3v_graph_launch": (i32, [vp, vp]),
@@ -154,6 +181,35 @@ SIGNATURES = {
 _lib = None
 
 
+class _Partial:
+    """A library built from some translation units only (build_units): an entry point it does not have raises when it is called."""
+
+    def __init__(self, l):
+        for name in SIGNATURES:
+            fn = getattr(l, name, None)
+            setattr(self, name, fn if fn is not None else self._absent(name))
+
+    @staticmethod
+    def _absent(name):
+        def absent(*_):
+            raise RuntimeError(f"{name} is not part of this partial library: build all of it (csrc/build.sh)")
+        return absent
+
+
+def build_units(units):
+    """For a program that runs one model family (registry.Family.units): use the full library if it is built, else build and use one of
+    these translation units alone."""
+    global LIB_PATH, _lib
+    if os.path.exists(LIB_PATH) or _lib is not None:
+        return
+    path = os.path.join(_HERE, "libp3v_part_" + hashlib.sha256(" ".join(units).encode()).hexdigest()[:8] + ".so")
+    src = [os.path.join(_HERE, "csrc", f) for f in os.listdir(os.path.join(_HERE, "csrc"))] + [os.path.join(_HERE, "..", "include", "p3v.h")]
+    if not os.path.exists(path) or os.path.getmtime(path) < max(os.path.getmtime(f) for f in src):
+        subprocess.run(["bash", os.path.join(_HERE, "csrc", "build.sh")], check=True, stdout=sys.stderr,
+                       env=dict(os.environ, P3V_UNITS=" ".join(units), P3V_OUT=path))
+    LIB_PATH = path
+
+
 def lib():
     """Load libp3v.so once; raise loudly when it is not there."""
     global _lib
@@ -164,10 +220,13 @@ def lib():
                 "`python -c 'import __graft_entry__ as g; g.build()'` (or csrc/build.sh). "
                 "There is no CPU/PyTorch fallback for the hot path.")
         l = C.CDLL(LIB_PATH)
+        partial = os.path.basename(LIB_PATH).startswith("libp3v_part_")
         for name, (res, args) in SIGNATURES.items():
+            if partial and not hasattr(l, name):
+                continue
             fn = getattr(l, name)          # AttributeError if the ABI and the header drift apart
             fn.restype, fn.argtypes = res, args
-        _lib = l
+        _lib = _Partial(l) if partial else l
     return _lib
 
 

@@ -29,8 +29,8 @@ import numpy as np
 import torch
 
 from . import ops as model_ops
-from .config import is_vision, load_config, make_config, phi3v_config_dict, tiny_config_dict
-from .processor import Phi3FProcessor, Phi3VProcessor
+from .config import load_config, make_config, phi3v_config_dict, tiny_config_dict
+from .registry import family
 from .weights import load_adapter, load_safetensors_dir, resolve_adapter, synth_weights
 
 PATH_ADAPTERS = "adapters"
@@ -121,7 +121,7 @@ class LogitStopper:
     def __call__(self, logits):
         if not self.early_stop:
             return False
-        if logits.shape[0] > 1:
+        if logits.shape[0] > 1 or logits.shape[-1] <= ID_EOS:     # (a vocabulary without the end token: nothing to stop at)
             self.early_stop = False
             return False
         log_prob = model_ops.log_softmax(logits[:, -1, :].contiguous())
@@ -209,18 +209,17 @@ def _get_cfg(json_path, **kwargs):
 
 
 def _make_processor(cfg, model_path, return_mx=True):
-    cls = Phi3VProcessor if is_vision(cfg) else Phi3FProcessor
-    return cls(model_path, return_mx=return_mx)
+    f = family(cfg)
+    return f.processor_cls(model_path, return_mx=return_mx, **({"vocab_size": cfg.vocab_size} if f.layered else {}))
 
 
 def _load(model_path=PATH_ORIGINAL_PHI3_VISION, adapter_path=None, return_mx=True, device=None, **kwargs):
     """reference phi_3_vision_mlx.py:257-274: config -> model class by `architectures[0]`,
     HF safetensors -> device weights."""
-    from .model import Phi3VModel
     cfg = _get_cfg(f"{model_path}/config.json", **kwargs)
     processor = _make_processor(cfg, model_path, return_mx)
     device = device or f"cuda:{torch.cuda.current_device()}"
-    model = Phi3VModel(cfg, load_safetensors_dir(model_path, cfg, device="cpu"), device=device)
+    model = family(cfg).model_cls(cfg, load_safetensors_dir(model_path, cfg, device="cpu"), device=device)
     if adapter_path:
         _attach_adapter(model, adapter_path, model_path)
     return model, processor
@@ -237,20 +236,21 @@ def _attach_adapter(model, adapter_path, model_path=None):
     lora_cfg, tensors = load_adapter(adapter_path)
     if model_path is not None and lora_cfg.get("model_path") != model_path:
         print(f"WARNING: LoRA trained for {lora_cfg.get('model_path')} is being used with {model_path}")
+    if not hasattr(model, "set_adapters"):
+        raise ValueError(f"LoRA adapters are not available for {model.cfg.architectures[0]}")
     model.set_adapters(resolve_adapter(model.cfg, lora_cfg, tensors))
 
 
 def load_synthetic(blind_model=False, tiny=False, seed=0, device=None, std_scale=1.0, adapter_path=None, lm_head_spread=0.0,
-                   lm_head_seed=0, outliers=None, residual_scale=None, **kwargs):
-    """Seeded random weights of the real (or tiny) architecture -- no checkpoint needed.
+                   lm_head_seed=0, outliers=None, residual_scale=None, config=None, **kwargs):
+    """Seeded random weights of the real (or tiny) architecture -- no checkpoint needed.  config: a config dict of any family instead.
     lm_head_spread / lm_head_seed: decisive-argmax head of the parity fixtures (weights.peaked_lm_head);
     outliers: heavy-tailed activations (weights.add_outliers); residual_scale: the well-conditioned checkpoint (weights.synth_weights)."""
-    from .model import Phi3VModel
-    d = tiny_config_dict(vision=not blind_model) if tiny else phi3v_config_dict(vision=not blind_model)
+    d = config if config is not None else tiny_config_dict(vision=not blind_model) if tiny else phi3v_config_dict(vision=not blind_model)
     cfg = make_config(d, **kwargs)
     device = device or f"cuda:{torch.cuda.current_device()}"
-    model = Phi3VModel(cfg, synth_weights(cfg, seed=seed, device=device, std_scale=std_scale, lm_head_spread=lm_head_spread,
-                                          lm_head_seed=lm_head_seed, outliers=outliers, residual_scale=residual_scale), device=device)
+    model = family(cfg).model_cls(cfg, synth_weights(cfg, seed=seed, device=device, std_scale=std_scale, lm_head_spread=lm_head_spread,
+                                                         lm_head_seed=lm_head_seed, outliers=outliers, residual_scale=residual_scale), device=device)
     if adapter_path:
         _attach_adapter(model, adapter_path)
     return model, _make_processor(cfg, None)
@@ -335,7 +335,7 @@ def greedy_loop(model, token, cache, n_steps, streamer, token_stopper, logit_sto
         if n_done == fail_at:                                       # (tests) what a poisoned step leaves: a negative token, NaN cache rows
             rows, fail_at = [-1] * len(rows), -1
             torch.cuda.synchronize()
-            if not st.quantized:
+            if not st.quantized and torch.is_tensor(st.v):
                 st.v[..., st.offset - (i - n_done):st.offset] = float("nan")
                 st.k[:, :, :, st.offset - (i - n_done):st.offset] = float("nan")
         if min(rows) < 0:

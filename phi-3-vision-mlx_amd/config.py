@@ -8,7 +8,9 @@ reference's own notebook (assets/su_rope_explained.ipynb, cell 9); a real
 """
 import json
 import math
+from dataclasses import dataclass
 from types import SimpleNamespace
+from typing import Optional
 
 SHORT_FACTOR = [
     1.05, 1.05, 1.05, 1.1, 1.1, 1.1, 1.2500000000000002, 1.2500000000000002,
@@ -84,11 +86,70 @@ def tiny_config_dict(vision=True):
 def make_config(d=None, **kwargs):
     """dict (+ kwargs overlay, as reference `_get_cfg`) -> SimpleNamespace."""
     d = dict(d if d is not None else phi3v_config_dict())
+    if "architecture" in d:
+        return layered_config(d, **kwargs)
+    if kwargs.get("dtype") not in (None, "bfloat16"):
+        raise ValueError(f"dtype {kwargs['dtype']!r}: this model runs in bfloat16")
     d.update(kwargs)
     cfg = SimpleNamespace(**d)
     if getattr(cfg, "img_processor", None) is not None and not hasattr(cfg, "clip"):
         cfg.clip = dict(CLIP_L_336)
     return cfg
+
+
+# ---------------------------------------------------------------- layered text decoders
+@dataclass(frozen=True)
+class Mixer:
+    """One attention mixer: H query heads over G key / value heads (query head h uses key / value head h // (H / G))."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    v_mix: bool
+
+
+@dataclass(frozen=True)
+class Mlp:
+    ff: int
+
+
+@dataclass(frozen=True)
+class LayerSpec:
+    mixer: Mixer
+    mlp: Optional[Mlp]
+
+
+def _layer_spec(i, d):
+    if d["type"] != "attention":
+        raise ValueError(f"layer {i}: unknown mixer type {d['type']!r}")
+    m = d["mixer"]
+    mixer = Mixer(int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"]), float(m["scale"]), bool(m["v_mix"]))
+    if mixer.heads % mixer.kv_heads:
+        raise ValueError(f"layer {i}: {mixer.heads} query heads over {mixer.kv_heads} key / value heads")
+    mlp = d.get("mlp")
+    if mlp is not None and mlp["kind"] != "dense":
+        raise ValueError(f"layer {i}: unknown feed-forward kind {mlp['kind']!r}")
+    return LayerSpec(mixer, None if mlp is None else Mlp(int(mlp["ff"])))
+
+
+def layered_config(d, dtype=None, shift_rows=128, **kwargs):
+    """config.json of a layered decoder -> SimpleNamespace.  dtype: "bfloat16" (default) or "float32" activations; shift_rows: columns of
+    token-shift history a state keeps (how far a cache can be rewound)."""
+    for k in ("use_quantized_cache", "quantized_fp8", "quantized_int4"):
+        if kwargs.pop(k, False):
+            raise ValueError(f"{k} is not available for {d['architecture']}")
+    if dtype not in (None, "bfloat16", "float32"):
+        raise ValueError(f"dtype must be 'bfloat16' or 'float32', got {dtype!r}")
+    layers = tuple(_layer_spec(i, x) for i, x in enumerate(d["layers"]))
+    mixing = {s.mixer.kv_heads * s.mixer.vdim for s in layers if s.mixer.v_mix}
+    if len(mixing) > 1:
+        raise ValueError(f"value-mixing layers of different value widths {sorted(mixing)}")
+    if not layers:
+        raise ValueError("a model without layers")
+    return SimpleNamespace(architectures=[d["architecture"]], layers=layers, num_hidden_layers=len(layers), hidden_size=int(d["width"]),
+                           vocab_size=int(d["vocab"]), norm_eps=float(d["norm"]["eps"]), embed_scale=float(d["embedding"]["scale"]),
+                           dtype=dtype or "bfloat16", shift_rows=int(shift_rows), **kwargs)
 
 
 def load_config(json_path, **kwargs):

@@ -8,7 +8,7 @@
 set -e
 cd "$(dirname "$0")"
 OUT=${P3V_OUT:-../libp3v.so}
-UNITS=${P3V_UNITS:-elementwise gemm gemm256 gemm_skinny gemm_rows gemm_fp8 gemv gemv_fp8 gemv_q4 attention lora preprocess runtime}
+UNITS=${P3V_UNITS:-elementwise gemm gemm256 gemm_skinny gemm_rows gemm_fp8 gemv gemv_fp8 gemv_q4 attention layered attn_mix lora preprocess runtime}
 # packed fp32 instructions stay off: hipcc forms them from ordinary float code and some of their forms have given wrong results on this chip
 FLAGS="--offload-arch=gfx950 -O3 -std=c++17 -fPIC -Wno-unused-result -Xclang -target-feature -Xclang -packed-fp32-ops"
 OBJ=$(mktemp -d "${TMPDIR:-/tmp}/p3v_build.XXXXXX")

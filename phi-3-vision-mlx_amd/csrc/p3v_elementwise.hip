@@ -673,7 +673,24 @@ __device__ __forceinline__ ValIdx row_argmax_partial(const bf16_t* __restrict__ 
   return m;
 }
 
-__global__ void __launch_bounds__(1024) k_argmax(const bf16_t* __restrict__ x, int32_t* __restrict__ out, int n,
+// the same on an fp32 row
+__device__ __forceinline__ ValIdx row_argmax_partial(const float* __restrict__ r, int n) {
+  ValIdx m = {-INFINITY, 0x7fffffff};
+  for (int i = threadIdx.x; i < n; i += blockDim.x) {
+    float v = r[i];
+    int k = i;
+    if (v != v) { v = INFINITY; k = -1; }
+    if (v > m.v || (v == m.v && k < m.i) || m.i == 0x7fffffff) { m.v = v; m.i = k; }
+  }
+  return m;
+}
+__device__ __forceinline__ float logit_f32(bf16_t v) { return bf16_to_f32(v); }
+__device__ __forceinline__ float logit_f32(float v) { return v; }
+__device__ __forceinline__ void logit_store(bf16_t* p, float v) { *p = f32_to_bf16(v); }
+__device__ __forceinline__ void logit_store(float* p, float v) { *p = v; }
+
+template <typename T>
+__global__ void __launch_bounds__(1024) k_argmax(const T* __restrict__ x, int32_t* __restrict__ out, int n,
                                                  int64_t stride) {
   __shared__ ValIdx red[16];
   ValIdx m = row_argmax_partial(x + (size_t)blockIdx.x * stride, n);
@@ -681,49 +698,63 @@ __global__ void __launch_bounds__(1024) k_argmax(const bf16_t* __restrict__ x, i
   if (threadIdx.x == 0) out[blockIdx.x] = m.i;
 }
 
-extern "C" int p3v_argmax(const uint16_t* logits, int32_t* out, int rows, int n, int64_t row_stride, void* stream) {
+template <typename T>
+static int launch_argmax(const T* logits, int32_t* out, int rows, int n, int64_t row_stride, void* stream) {
   if (!logits || !out || rows < 0 || n <= 0) return P3V_ERR_ARG;
   if (rows == 0) return P3V_OK;
-  hipLaunchKernelGGL(k_argmax, dim3(rows), dim3(1024), 0, (hipStream_t)stream, logits, out, n, row_stride);
+  hipLaunchKernelGGL(k_argmax<T>, dim3(rows), dim3(1024), 0, (hipStream_t)stream, logits, out, n, row_stride);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
 }
+extern "C" int p3v_argmax(const uint16_t* logits, int32_t* out, int rows, int n, int64_t row_stride, void* stream) {
+  return launch_argmax(logits, out, rows, n, row_stride, stream);
+}
+extern "C" int p3v_argmax_f32(const float* logits, int32_t* out, int rows, int n, int64_t row_stride, void* stream) {
+  return launch_argmax(logits, out, rows, n, row_stride, stream);
+}
 
-__global__ void __launch_bounds__(1024) k_log_softmax(const bf16_t* __restrict__ x, bf16_t* __restrict__ y, int n) {
+template <typename T>
+__global__ void __launch_bounds__(1024) k_log_softmax(const T* __restrict__ x, T* __restrict__ y, int n) {
   __shared__ float red[16];
-  const bf16_t* r = x + (size_t)blockIdx.x * n;
-  bf16_t* o = y + (size_t)blockIdx.x * n;
+  const T* r = x + (size_t)blockIdx.x * n;
+  T* o = y + (size_t)blockIdx.x * n;
   float m = -INFINITY;
-  for (int i = threadIdx.x; i < n; i += blockDim.x) m = fmaxf(m, bf16_to_f32(r[i]));
+  for (int i = threadIdx.x; i < n; i += blockDim.x) m = fmaxf(m, logit_f32(r[i]));
   m = block_max(m, red);
   float s = 0.f;
-  for (int i = threadIdx.x; i < n; i += blockDim.x) s += expf(bf16_to_f32(r[i]) - m);
+  for (int i = threadIdx.x; i < n; i += blockDim.x) s += expf(logit_f32(r[i]) - m);
   s = block_sum(s, red);
-  // nn.log_softmax(x) = x - mx.logsumexp(x): the normaliser is itself a bf16 array before the subtraction rounds again
-  const float lse = bf16_round(m + logf(s));
-  for (int i = threadIdx.x; i < n; i += blockDim.x) o[i] = f32_to_bf16(bf16_to_f32(r[i]) - lse);
+  // nn.log_softmax(x) = x - mx.logsumexp(x): the normaliser is itself an array of x's type before the subtraction rounds again
+  T lse_t;
+  logit_store(&lse_t, m + logf(s));
+  const float lse = logit_f32(lse_t);
+  for (int i = threadIdx.x; i < n; i += blockDim.x) logit_store(o + i, logit_f32(r[i]) - lse);
 }
 
-extern "C" int p3v_log_softmax(const uint16_t* x, uint16_t* y, int rows, int n, void* stream) {
+template <typename T>
+static int launch_log_softmax(const T* x, T* y, int rows, int n, void* stream) {
   if (!x || !y || rows < 0 || n <= 0) return P3V_ERR_ARG;
   if (rows == 0) return P3V_OK;
-  hipLaunchKernelGGL(k_log_softmax, dim3(rows), dim3(1024), 0, (hipStream_t)stream, x, y, n);
+  hipLaunchKernelGGL(k_log_softmax<T>, dim3(rows), dim3(1024), 0, (hipStream_t)stream, x, y, n);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
 }
+extern "C" int p3v_log_softmax(const uint16_t* x, uint16_t* y, int rows, int n, void* stream) { return launch_log_softmax(x, y, rows, n, stream); }
+extern "C" int p3v_log_softmax_f32(const float* x, float* y, int rows, int n, void* stream) { return launch_log_softmax(x, y, rows, n, stream); }
 
-__global__ void __launch_bounds__(1024) k_topk(const bf16_t* __restrict__ x, int32_t* __restrict__ out, int n, int k,
+template <typename T>
+__global__ void __launch_bounds__(1024) k_topk(const T* __restrict__ x, int32_t* __restrict__ out, int n, int k,
                                                int64_t stride) {
   __shared__ ValIdx red[16];
   __shared__ int picked[8];
-  const bf16_t* r = x + (size_t)blockIdx.x * stride;
+  const T* r = x + (size_t)blockIdx.x * stride;
   for (int round = 0; round < k; ++round) {
     ValIdx m = {-INFINITY, 0x7fffffff};
     for (int i = threadIdx.x; i < n; i += blockDim.x) {
       bool skip = false;
       for (int p = 0; p < round; ++p) skip |= (picked[p] == i);
       if (skip) continue;
-      const float v = bf16_to_f32(r[i]);
+      const float v = logit_f32(r[i]);
       if (v > m.v || (v == m.v && i < m.i) || m.i == 0x7fffffff) { m.v = v; m.i = i; }
     }
     m = block_argmax(m, red);
@@ -732,12 +763,19 @@ __global__ void __launch_bounds__(1024) k_topk(const bf16_t* __restrict__ x, int
   }
 }
 
-extern "C" int p3v_topk(const uint16_t* x, int32_t* idx_out, int rows, int n, int k, int64_t row_stride, void* stream) {
+template <typename T>
+static int launch_topk(const T* x, int32_t* idx_out, int rows, int n, int k, int64_t row_stride, void* stream) {
   if (!x || !idx_out || rows < 0 || n <= 0 || k <= 0 || k > 8 || k > n) return P3V_ERR_ARG;
   if (rows == 0) return P3V_OK;
-  hipLaunchKernelGGL(k_topk, dim3(rows), dim3(1024), 0, (hipStream_t)stream, x, idx_out, n, k, row_stride);
+  hipLaunchKernelGGL(k_topk<T>, dim3(rows), dim3(1024), 0, (hipStream_t)stream, x, idx_out, n, k, row_stride);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
+}
+extern "C" int p3v_topk(const uint16_t* x, int32_t* idx_out, int rows, int n, int k, int64_t row_stride, void* stream) {
+  return launch_topk(x, idx_out, rows, n, k, row_stride, stream);
+}
+extern "C" int p3v_topk_f32(const float* x, int32_t* idx_out, int rows, int n, int k, int64_t row_stride, void* stream) {
+  return launch_topk(x, idx_out, rows, n, k, row_stride, stream);
 }
 
 // ---------------------------------------------------------------- device-resident loop state
@@ -807,7 +845,8 @@ extern "C" int p3v_step_begin(const int32_t* tok, const uint16_t* table, uint16_
   return P3V_OK;
 }
 
-__global__ void __launch_bounds__(1024) k_step_end(const bf16_t* __restrict__ logits, int32_t* __restrict__ next_tok,
+template <typename T>
+__global__ void __launch_bounds__(1024) k_step_end(const T* __restrict__ logits, int32_t* __restrict__ next_tok,
                                                    int32_t* __restrict__ tok, int32_t* __restrict__ hist, int32_t* d_step,
                                                    int32_t* d_past, int32_t* ticket, int n, int max_steps) {
   __shared__ ValIdx red[16];
@@ -835,11 +874,20 @@ __global__ void __launch_bounds__(1024) k_step_end(const bf16_t* __restrict__ lo
   }
 }
 
-extern "C" int p3v_step_end(const uint16_t* logits, int32_t* next_tok, int32_t* tok, int32_t* history, int32_t* d_step,
-                            int32_t* d_past, int32_t* ticket, int B, int n, int max_steps, void* stream) {
+template <typename T>
+static int launch_step_end(const T* logits, int32_t* next_tok, int32_t* tok, int32_t* history, int32_t* d_step, int32_t* d_past, int32_t* ticket,
+                           int B, int n, int max_steps, void* stream) {
   if (!logits || !next_tok || !tok || !history || !d_step || !d_past || !ticket || B <= 0 || n <= 0) return P3V_ERR_ARG;
-  hipLaunchKernelGGL(k_step_end, dim3(B), dim3(1024), 0, (hipStream_t)stream, logits, next_tok, tok, history, d_step, d_past,
+  hipLaunchKernelGGL(k_step_end<T>, dim3(B), dim3(1024), 0, (hipStream_t)stream, logits, next_tok, tok, history, d_step, d_past,
                      ticket, n, max_steps);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
+}
+extern "C" int p3v_step_end(const uint16_t* logits, int32_t* next_tok, int32_t* tok, int32_t* history, int32_t* d_step,
+                            int32_t* d_past, int32_t* ticket, int B, int n, int max_steps, void* stream) {
+  return launch_step_end(logits, next_tok, tok, history, d_step, d_past, ticket, B, n, max_steps, stream);
+}
+extern "C" int p3v_step_end_f32(const float* logits, int32_t* next_tok, int32_t* tok, int32_t* history, int32_t* d_step,
+                                int32_t* d_past, int32_t* ticket, int B, int n, int max_steps, void* stream) {
+  return launch_step_end(logits, next_tok, tok, history, d_step, d_past, ticket, B, n, max_steps, stream);
 }

@@ -79,7 +79,8 @@ class Request:
 class ContinuousEngine:
     def __init__(self, model, processor, slots=8, window=ROPE_WINDOW, patience=64):
         self.model, self.processor, self.slots, self.window, self.patience = model, processor, slots, window, patience
-        self.long_rope = window > ROPE_WINDOW
+        self.regimes = getattr(model, "rope_regimes", True)     # False: positions pick no table, any window serves any length
+        self.long_rope = self.regimes and window > ROPE_WINDOW
         self.rows = [None] * slots                               # row -> active Request
         self.waiting = collections.deque()
         self.lock = threading.Lock()
@@ -100,7 +101,7 @@ class ContinuousEngine:
         """Does a request of this shape belong to this engine's RoPE regime and fit its window?"""
         if max_tokens < 1 or S < 1 or S + max_tokens > self.window:
             return False
-        return (S + max_tokens > ROPE_WINDOW) == self.long_rope
+        return not self.regimes or (S + max_tokens > ROPE_WINDOW) == self.long_rope
 
     def submit(self, inputs, max_tokens):
         """inputs: a B = 1 `processor(text[, images])` result.  Returns the Request; wait on `.done`, read `.tokens`."""

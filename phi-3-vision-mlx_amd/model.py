@@ -22,134 +22,29 @@ Dtype flow differs from the reference only where stated in DESIGN.md
 tolerance the parity tests state.
 """
 import math
-import copy
 import os
 
 import numpy as np
 import torch
 
 from . import ops
+from .cache import CacheState, LayerCache  # noqa: F401
 from .config import head_dim, is_vision, rope_scaling_factor
+from .decoder import DecoderModel, on_device
 from .weights import Q4Weight, mlx_quantize, q4_repack
 from .ops import (BF16, EPI_BIAS, EPI_BIAS_GELU, EPI_BIAS_QGELU, EPI_BIAS_RESID_F32, EPI_NONE, EPI_PATCH,
                   EPI_RESID_BF16, EPI_SILU_MUL, F32, I32)
-
-import functools
-import weakref
-
-
-def _on_device(fn):
-    """Run a model entry point with the model's GPU as the current device: ops.py launches on
-    `torch.cuda.current_stream()` of the CURRENT device, and a thread other than the one that loaded the model (the
-    server's engine thread) starts on device 0."""
-    @functools.wraps(fn)
-    def wrapped(self, *a, **kw):
-        with torch.cuda.device(self.device):
-            return fn(self, *a, **kw)
-    return wrapped
 
 
 V_PREFIX = "model.vision_embed_tokens.img_processor.vision_model."
 E_PREFIX = "model.vision_embed_tokens."
 
 
-class CacheState:
-    """All layers' KV cache + per-prompt RoPE tables / pad lengths.
+class Phi3VModel(DecoderModel):
+    rope_regimes = True
 
-    Mirrors reference KVCache (phi.py:509-548) semantics: `offset` auto-advances
-    by L, can be rewound (`advance_offset`), `max_tokens < 1` disables caching,
-    `n_beam > 1` reads the cache without writing it."""
-
-    def __init__(self, cfg, B, S, max_tokens, device):
-        self.B, self.S, self.max_tokens = B, S, max_tokens
-        self.T = S + max(max_tokens, 0)
-        self.quantized = bool(getattr(cfg, "use_quantized_cache", False))
-        # cache_format="mlx4" (opt-in): the reference's OWN quantised cache -- MLX 4-bit group-32 codes of the PROMPT's K / V, later
-        # tokens unquantised (phi.py:528-540).  The codes are kept in the reference's format (k4 / v4 + scale | bias), and the
-        # bf16 cache rows hold their dequantised values, which is what every later call of the reference attends on: the decode
-        # path is then the plain bf16 one.  (Default for quantize_cache=True: int8 for all tokens, BASELINE config 5.)
-        self.mlx4 = self.quantized and getattr(cfg, "cache_format", "int8") == "mlx4"
-        if self.quantized and getattr(cfg, "cache_format", "int8") not in ("int8", "mlx4"):
-            raise ValueError(f"cache_format must be 'int8' or 'mlx4', got {cfg.cache_format!r}")
-        if self.mlx4:
-            self.quantized = False
-        # row/column stride of the caches: whole 128-key tiles (the decode attention takes one 128-key tile per workgroup
-        # when the capacity allows it)
-        gran = 128
-        self.Tp = (self.T + gran - 1) // gran * gran
-        if (self.Tp // gran) % 2 == 0:
-            # V^T rows are Tp * 2 bytes apart: at multiples of 512 B the 96 rows of a tile crowd the same memory channels
-            # (measured decode step at B = 1: +3.5 % at Tp = 2560, +2 % at 3584, +1.4 % at 4096, +5.7 % at 33024 = 258 tiles
-            # against the neighbouring lengths) -- an ODD number of 128-key tiles keeps the stride off that grid
-            self.Tp += gran
-        nl, nkv, hd = cfg.num_hidden_layers, cfg.num_key_value_heads, head_dim(cfg)
-        if self.quantized:
-            # int8 KV (quantize_cache=True): offset-binary bytes + one fp32 scale per (layer, row, head, token);
-            # one bf16 K / V^T scratch layer holds the exact prompt keys while a layer's prefill attends (phi.py:531-533)
-            self.k8 = torch.full((nl, B, nkv, self.Tp, hd), 128, dtype=torch.uint8, device=device)
-            self.v8 = torch.full((nl, B, nkv, hd, self.Tp), 128, dtype=torch.uint8, device=device)
-            self.ks = torch.ones((nl, B, nkv, self.Tp), dtype=F32, device=device)
-            self.vs = torch.ones((nl, B, nkv, self.Tp), dtype=F32, device=device)
-            self.k_tmp = torch.empty((B, nkv, self.Tp, hd), dtype=BF16, device=device)
-            self.v_tmp = torch.zeros((B, nkv, hd, self.Tp), dtype=BF16, device=device)
-        else:
-            self.k = torch.empty((nl, B, nkv, self.Tp, hd), dtype=BF16, device=device)    # K   [.., t, hd]
-            self.v = torch.zeros((nl, B, nkv, hd, self.Tp), dtype=BF16, device=device)    # V^T [.., hd, t] (zero: tail keys stay finite)
-        if self.mlx4:
-            g = hd // 32
-            self.k4 = torch.zeros((nl, B, nkv, max(S, 1), g, 4), dtype=I32, device=device)
-            self.v4 = torch.zeros_like(self.k4)
-            self.k_sb = torch.zeros((nl, B, nkv, max(S, 1), g, 2), dtype=F32, device=device)
-            self.v_sb = torch.zeros_like(self.k_sb)
-            self.mlx4_tokens = 0                                # prompt tokens held as codes (set by the first call)
-        self.offset = 0
-        self.cos = self.sin = self.pad_len = None
-        self.graphs = {}
-        self.epoch = None                                       # model.epoch the graphs were captured under
-        self.shared = {"dirty": False}                          # shared by the per-request views of a captured-prefill entry (copy.copy)
-
-    def mark_dirty(self):
-        """An unrecovered failed step may have left NaN rows beyond the offset and half-armed buffers in the decode graph: a
-        captured-prefill entry built on these buffers must not be reused (model._prefill_captured drops it)."""
-        self.shared["dirty"] = True
-
-    def scrub(self, lo, hi):
-        """Forget cache positions [lo, hi) that a FAILED step wrote (api.greedy_loop's recovery): a poisoned step leaves NaN there,
-        and the decode attention multiplies every V^T column of a tile -- live or not -- by its (zero) probability."""
-        hi = min(hi, self.Tp)
-        if hi <= lo:
-            return
-        if self.quantized:
-            self.v8[..., lo:hi] = 128
-            self.k8[:, :, :, lo:hi] = 128
-            self.vs[..., lo:hi] = 1.0
-            self.ks[..., lo:hi] = 1.0
-        else:
-            self.v[..., lo:hi] = 0
-            self.k[:, :, :, lo:hi] = 0
-
-
-class LayerCache:
-    """`cache[i]` view with the reference's `.offset` attribute."""
-
-    def __init__(self, state, i):
-        self.state, self.i = state, i
-
-    @property
-    def offset(self):
-        return self.state.offset
-
-    @offset.setter
-    def offset(self, v):
-        self.state.offset = int(v)
-
-
-class Phi3VModel:
     def __init__(self, cfg, weights, device="cuda:0"):
-        if not torch.cuda.is_available():
-            raise RuntimeError("Phi3VModel needs a GPU: the hot path is HIP-only (no CPU fallback)")
-        ops.L.lib()                                  # fail loudly if libp3v.so is missing
-        self.cfg, self.device = cfg, torch.device(device)
+        self._init_decoder(cfg, device)
         self.vision = is_vision(cfg)
         self.w = {k: v.to(self.device, BF16).contiguous() for k, v in weights.items() if not isinstance(v, Q4Weight)}
         # 4-bit group-64 projections (MLX nn.quantize checkpoints / quantized_int4): device layout of p3v_gemv_q4
@@ -157,21 +52,12 @@ class Phi3VModel:
         self.hd = head_dim(cfg)
         if self.hd != 96:
             raise ValueError(f"decoder head_dim must be 96 (got {self.hd})")
-        self.hidden_hook = None                      # fn(layer, x [B*L, H], B, L) after every decoder layer (diagnostics)
         self.w8 = {}
         self._rope_tables = {}                                   # (B, T, factors, ..) -> (cos, sin): shared read-only (see _new_state)
         self._vit_graphs, self._vit_seen = {}, {}                # captured vision tower per crop count (clip_forward)
         self.adapters = {}                           # weight key -> (lora_a, lora_b, scale), see set_adapters
         self._lora_tmp = {}                          # decode-sized (M <= 16) adapter scratch: captured graphs point at it
         self._lora_flat = None                       # ONE grow-only scratch for prefill-sized calls (not graph-captured)
-        # A long-lived owner that may share the GPU with other streams / processes (server.py) sets this: the decode step then
-        # uses no launch that needs all of its workgroups resident at once (the fused attention + o_proj launch, the in-launch
-        # split-KV merge on grids larger than the machine) -- ADVICE r04.  One-shot generate() on an exclusive GPU keeps them.
-        self.serving = os.environ.get("P3V_SHARED_GPU", "0") == "1"
-        self.epoch = 0                               # bumped whenever captured decode graphs become stale
-        self._prefill_graphs = {}                    # (S, max_tokens) -> captured short-prompt prefill (see _prefill_captured)
-        self._prefill_seen = {}
-        self._states = weakref.WeakSet()             # every live CacheState (their graphs bake pointers into this model)
         # quantize_model=True (fp8): prompt-sized projections run W8A8 on the fp8 MFMA unless fp8_activations=False
         # (then: dequantise to a bf16 scratch + bf16 MFMA, weight-only accuracy at bf16 prefill speed)
         self.fp8_act = bool(getattr(cfg, "fp8_activations", True)) and os.environ.get("P3V_FP8_PREFILL", "mfma") != "dequant"
@@ -196,7 +82,7 @@ class Phi3VModel:
         self._deq = torch.empty(n_max, dtype=BF16, device=self.device)      # one dequantised matrix (prefill GEMM scratch)
 
     # ------------------------------------------------------------------ LoRA adapters (use_adapter=True)
-    @_on_device
+    @on_device
     def set_adapters(self, adapters):
         """Attach LoRA adapters: {"model.layers.<i>.<target>.weight": (lora_a [in,r] f32, lora_b [r,out] f32, scale)}
         (weights.resolve_adapter).  An adapted projection runs unfused: materialised RMSNorm -> frozen projection with a
@@ -330,7 +216,7 @@ class Phi3VModel:
             o=torch.empty((n * T, D), dtype=BF16, device=dev), h=torch.empty((n * T, D), dtype=BF16, device=dev),
             qkv=torch.empty((n * T, 3 * D), dtype=BF16, device=dev), f=torch.empty((n * T, I_), dtype=BF16, device=dev))
 
-    @_on_device
+    @on_device
     def clip_forward(self, pix):
         """ClipModel.__call__ (phi.py:216-221) on live crops; pix f32 [n,3,336,336] -> f32 [n,577,D]
         (row 0 = CLS, which the caller skips).
@@ -486,81 +372,6 @@ class Phi3VModel:
             m = np.asarray(mask)
             st.pad_len = torch.as_tensor((m == 0).sum(axis=1).astype(np.int32)).to(self.device)
         return st
-
-    # ------------------------------------------------------------------ slot state of the continuous-batching engine
-    @_on_device
-    def new_slot_state(self, slots, window):
-        """A cache of `slots` batch rows and `window` columns that is not tied to one prompt batch (engine.py): every row
-        has its OWN left padding and position table, so a request can be prefilled into a free row while the other rows
-        are mid-generation.  All rows start empty (pad_len = window: every key masked).  The window fixes the RoPE regime
-        of every row (phi.py:492: one choice per call from prompt + max_tokens): window <= 4096 -> short factors, beyond
-        -> long factors; the engine admits only requests that would pick the same factors alone.  With
-        `quantize_cache=True` the rows keep the int8 KV cache."""
-        st = self._new_state(slots, 0, window, None, None, shared_tables=False)
-        st.pad_len = torch.full((slots,), window, dtype=I32, device=self.device)
-        st.slots = True
-        return st
-
-    @_on_device
-    def prefill_slot(self, st, row, inputs, return_logits=False):
-        """Prefill one request (a B = 1 `processor(...)` result) -- or n requests as one batch (`collate_requests` of them:
-        equal lengths, or shorter rows left-padded inside the group) -- into the batch rows row .. row+n-1 of a slot state so
-        that every row's LAST prompt token sits in column st.offset - 1: row i gets left padding pad_i = st.offset - S_i and
-        position ids 0..S_i-1 from column pad_i on.  Keys left of pad_i (stale rows of an earlier occupant, the group's own
-        padding) are masked by pad_len.  Returns the first greedy tokens (int32 [n, 1] on the device; with return_logits also
-        the last-position logits).  Each row computes what a B = 1 run of its request computes (pad invariance)."""
-        cfg = self.cfg
-        ids = np.asarray(inputs["input_ids"])
-        ids = ids[None] if ids.ndim == 1 else ids
-        n, S = ids.shape
-        lens = np.full(n, S, dtype=np.int64)
-        if "mask" in inputs:
-            m = np.asarray(inputs["mask"]).reshape(n, S)
-            lens = m.sum(1).astype(np.int64)
-            if not all(int(m[i, S - lens[i]:].sum()) == lens[i] for i in range(n)) or lens.min() < 1:
-                raise ValueError("prefill_slot takes LEFT-padded rows")
-        win = st.offset - S                                      # first column the group's batch writes
-        if win < 0:
-            raise ValueError(f"prompt of {S} tokens does not fit left of column {st.offset}")
-        pads = torch.as_tensor(st.offset - lens, dtype=torch.int32)
-        half = self.hd // 2
-        su = cfg.rope_scaling["long_factor" if st.T > cfg.original_max_position_embeddings else "short_factor"]   # as _new_state
-        inv_freq = 1.0 / (torch.tensor(su, dtype=F32)
-                          * (torch.tensor(float(cfg.rope_theta), dtype=F32) ** (torch.arange(0, self.hd, 2, dtype=F32) / self.hd)))
-        rows = slice(row, row + n)
-        uniq = np.unique(lens)
-        for L_ in uniq:                                          # one table per distinct length
-            pos = (torch.arange(st.T, dtype=F32) - float(st.offset - L_)).clamp_min(0).to(self.device)
-            cos, sin = ops.rope_table(pos, inv_freq.to(self.device), rope_scaling_factor(cfg))
-            for i in np.nonzero(lens == L_)[0]:
-                st.cos[row + i].copy_(cos.view(st.T, half)), st.sin[row + i].copy_(sin.view(st.T, half))
-        st.pad_len[rows].copy_(pads.to(self.device))
-        view = CacheState.__new__(CacheState)                   # these rows as an n-row cache at offset `win`
-        view.__dict__.update(B=n, S=S, max_tokens=st.max_tokens, T=st.T, Tp=st.Tp, quantized=st.quantized, offset=win, graphs={},
-                             epoch=self.epoch, cos=st.cos[rows], sin=st.sin[rows], pad_len=st.pad_len[rows],
-                             fresh_rows=True)    # columns left of `win` hold nothing these rows may see (pad_len >= win)
-        if st.quantized:
-            view.__dict__.update(k8=st.k8[:, rows], v8=st.v8[:, rows], ks=st.ks[:, rows], vs=st.vs[:, rows],
-                                 k_tmp=st.k_tmp[rows], v_tmp=st.v_tmp[rows])
-        else:
-            view.__dict__.update(k=st.k[:, rows], v=st.v[:, rows])
-        kw = {k: v for k, v in inputs.items() if k in ("pixel_values", "image_sizes", "positions")}
-        logits, _ = self(input_ids=ids, cache=[LayerCache(view, i) for i in range(cfg.num_hidden_layers)], full_logits=False, **kw)
-        assert view.offset == st.offset
-        tok = ops.argmax(logits[:, -1, :].contiguous())[:, None]
-        return (tok, logits) if return_logits else tok
-
-    @_on_device
-    def decode_graph(self, st):
-        """The captured greedy step of a state (built on first use): its `tok` / `next_tok` / `d_past` device buffers."""
-        if st.epoch != self.epoch:
-            st.graphs.clear()
-            st.epoch = self.epoch
-        g = st.graphs.get("greedy")
-        if g is None:
-            g = st.graphs["greedy"] = self._build_decode_graph(st)
-            g["host_tok"] = None
-        return g
 
     # ------------------------------------------------------------------ decoder stack
     def _alloc_bufs(self, B, L):
@@ -800,21 +611,26 @@ class Phi3VModel:
         ops.kv_quantize_mlx4(st.k[i], st.v[i], st.k4[i], st.v4[i], st.k_sb[i], st.v_sb[i], L, qkv=qkv, cos_t=st.cos, sin_t=st.sin, nh=nh,
                              past=0, tab_t=st.T, tab_div=1)
 
-    # ------------------------------------------------------------------ graph-replayed greedy decode step
-    def _build_decode_graph(self, st):
-        """Capture ONE greedy decode step (embed -> 32 layers -> norm+lm_head -> argmax ->
-        bookkeeping) as a hipGraph.  All loop state lives in HBM: `tok` (next input ids),
-        `d_past` (cache length), `d_step`, `history` -- so replays need no host input and
-        a token costs one graph launch instead of ~170 kernel launches."""
-        cfg, w, B, dev = self.cfg, self.w, st.B, self.device
-        g = dict(tok=torch.zeros((B,), dtype=I32, device=dev), d_past=torch.zeros((1,), dtype=I32, device=dev),
-                 d_step=torch.zeros((1,), dtype=I32, device=dev),
-                 # the step's tokens land in PINNED HOST memory straight from `k_step_end` (one 4-byte store per row and step):
-                 # the host loop reads them after the step's event, no D2H copy node sits between two replays (api.greedy_loop)
-                 history=torch.zeros((B, max(1, st.max_tokens) + 1), dtype=I32).pin_memory(),
-                 x=torch.empty((B, cfg.hidden_size), dtype=BF16, device=dev),
-                 logits=torch.empty((B, cfg.vocab_size), dtype=BF16, device=dev),
-                 next_tok=torch.zeros((B,), dtype=I32, device=dev), ticket=torch.zeros((1,), dtype=I32, device=dev))
+    # ------------------------------------------------------------------ hooks of DecoderModel
+    def _slot_rows(self, st, row, lens):
+        half, cfg = self.hd // 2, self.cfg
+        su = cfg.rope_scaling["long_factor" if st.T > cfg.original_max_position_embeddings else "short_factor"]   # as _new_state
+        inv_freq = 1.0 / (torch.tensor(su, dtype=F32)
+                          * (torch.tensor(float(cfg.rope_theta), dtype=F32) ** (torch.arange(0, self.hd, 2, dtype=F32) / self.hd)))
+        for L_ in np.unique(lens):                               # one table per distinct length
+            pos = (torch.arange(st.T, dtype=F32) - float(st.offset - L_)).clamp_min(0).to(self.device)
+            cos, sin = ops.rope_table(pos, inv_freq.to(self.device), rope_scaling_factor(cfg))
+            for i in np.nonzero(lens == L_)[0]:
+                st.cos[row + i].copy_(cos.view(st.T, half)), st.sin[row + i].copy_(sin.view(st.T, half))
+
+    def _embed(self, ids, out=None):
+        return ops.embed_gather(ids, self.w["model.embed_tokens.weight"], out=out)
+
+    def _head(self, x, out=None, bufs=None):
+        return self._proj(x, "lm_head.weight", norm_w=self.w["model.norm.weight"], out=out)
+
+    def _step_bufs(self, st):
+        B = st.B
         bufs = self._alloc_bufs(B, 1)
         self._split_plan(bufs, B, 1, st.Tp, st.quantized, serving=getattr(st, "serving", False) or self.serving)   # one split per tile of CAPACITY
         # the cache length only grows under a captured step (greedy_step rebuilds the graph if it ever finds it below this); a
@@ -822,211 +638,38 @@ class Phi3VModel:
         bufs["past_lb"] = -1 if getattr(st, "slots", False) else int(st.offset)
         if not getattr(st, "slots", False):
             self._plan_fused_oproj(bufs, B, 1, st.Tp, st.quantized)
-        bufs["rope_cos"] = torch.empty((B, 1, self.hd // 2), dtype=F32, device=dev)
+        bufs["rope_cos"] = torch.empty((B, 1, self.hd // 2), dtype=F32, device=self.device)
         bufs["rope_sin"] = torch.empty_like(bufs["rope_cos"])
-        g["bufs"] = bufs
+        return bufs
 
-        g["amax_ws"] = torch.zeros((ops.L.GEMV_STEP_WS_BYTES // 4,), dtype=F32, device=dev)   # (its arrival counters start at zero)
+    def _step(self, g, st):
+        # the step's two ends have no launch of their own where the library folds them into the first / last projection
+        # (B = 1 on bf16, e4m3 or 4-bit weights: ops.gemv_step_begin / gemv_step_end; 129 launches per step instead of 131)
+        cfg, w, bufs = self.cfg, self.w, g["bufs"]
+        self._layers(g["x"], st, st.B, 1, 0, 1, bufs=bufs, d_past=g["d_past"],
+                     step_begin=dict(tok=g["tok"], table=w["model.embed_tokens.weight"], cos_o=bufs["rope_cos"], sin_o=bufs["rope_sin"]))
+        head = "lm_head.weight"
+        w_fold = w.get(head) if head in w else (self.w8.get(head) or self.w4.get(head))   # bf16, (e4m3, row scales) or (4-bit, scale | bias)
+        if not (w_fold is not None and head not in self.adapters and os.environ.get("P3V_STEP_FOLD", "1") != "0"
+                and ops.gemv_step_end(g["x"], w_fold, w["model.norm.weight"], cfg.rms_norm_eps, g["logits"], g["next_tok"], g["tok"],
+                                      g["history"], g["d_step"], g["d_past"], g["ticket"], g["amax_ws"])):
+            self._proj(g["x"], head, norm_w=w["model.norm.weight"], out=g["logits"], h=bufs["h"])   # (h: the norm's output buffer)
+            ops.step_end(g["logits"], g["next_tok"], g["tok"], g["history"], g["d_step"], g["d_past"], g["ticket"])
 
-        def step():
-            # (round 6) the step's two ends have no launch of their own where the library folds them into the first / last projection
-            # (B = 1 on bf16, e4m3 or 4-bit weights: ops.gemv_step_begin / gemv_step_end; 129 launches per step instead of 131)
-            self._layers(g["x"], st, B, 1, 0, 1, bufs=bufs, d_past=g["d_past"],
-                         step_begin=dict(tok=g["tok"], table=w["model.embed_tokens.weight"], cos_o=bufs["rope_cos"], sin_o=bufs["rope_sin"]))
-            head = "lm_head.weight"
-            w_fold = w.get(head) if head in w else (self.w8.get(head) or self.w4.get(head))   # bf16, (e4m3, row scales) or (4-bit, scale | bias)
-            if not (w_fold is not None and head not in self.adapters and os.environ.get("P3V_STEP_FOLD", "1") != "0"
-                    and ops.gemv_step_end(g["x"], w_fold, w["model.norm.weight"], cfg.rms_norm_eps, g["logits"], g["next_tok"], g["tok"],
-                                          g["history"], g["d_step"], g["d_past"], g["ticket"], g["amax_ws"])):
-                self._proj(g["x"], head, norm_w=w["model.norm.weight"], out=g["logits"], h=bufs["h"])   # (h: the norm's output
-                ops.step_end(g["logits"], g["next_tok"], g["tok"], g["history"], g["d_step"], g["d_past"], g["ticket"])
-        g["d_past"].fill_(st.offset)
-        g["gemm_ws"] = {}                                        # B > 16 rows: the projections are split-K GEMMs; their workspace
-        with ops.owned_gemm_workspace(g["gemm_ws"], frozen=False):   # belongs to the graph (sized here, baked in below)
-            step()                                               # warm-up run (sets func attributes, pages code in)
-        torch.cuda.synchronize()
-        graph = ops.Graph()
-        side = torch.cuda.Stream(device=dev)
-        side.wait_stream(torch.cuda.current_stream())
-        with torch.cuda.stream(side), ops.owned_gemm_workspace(g["gemm_ws"], frozen=True):
-            graph.begin()
-            step()
-            graph.end()
-        torch.cuda.current_stream().wait_stream(side)
-        g["d_step"].zero_()                                      # the warm-up run above counted as a step
-        g["graph"] = graph
-        return g
+    def _cache_token_bytes(self):
+        return 4 * self.cfg.num_hidden_layers * self.cfg.num_key_value_heads * self.hd
 
-    @_on_device
-    def greedy_prefill(self, max_tokens, **inputs):
-        """Prefill + first greedy token: `logits, cache = model(**inputs, max_tokens); argmax(logits[:, -1])`
-        (reference phi_3_vision_mlx.py:385-386).  Returns (token [B,1] int32 on the device, cache)."""
-        logits, cache = self(**inputs, max_tokens=max_tokens)
-        return ops.argmax(logits[:, -1, :].contiguous())[:, None], cache
-
-    @_on_device
-    def greedy_step(self, token, cache):
-        """One greedy decode step through the captured graph.  Equivalent to
-        `logits, cache = model(input_ids=token, cache=cache); next = argmax(logits[:, -1])`
-        (reference phi_3_vision_mlx.py:391-392).  Returns (logits [B,1,V], next_token [B,1])
-        -- views of persistent buffers, valid until the next call."""
-        st = cache[0].state
-        if st.offset + 1 > st.T:
-            raise ValueError(f"KV cache overflow: {st.offset}+1 > {st.T} (prompt + max_tokens)")
-        if st.epoch != self.epoch:                              # adapters changed since the capture: stale pointers
-            st.graphs.clear()
-            st.epoch = self.epoch
-        g = st.graphs.get("greedy")
-        if g is not None and st.offset < g["bufs"].get("past_lb", -1):   # the cache was rewound below the captured lower bound
-            g = None
-        if g is None:
-            g = st.graphs["greedy"] = self._build_decode_graph(st)
-            g["host_tok"] = None
-        if g["host_tok"] is None or token is not g["host_tok"]:
-            g["tok"].copy_(token.reshape(-1).to(self.device, I32))   # first step / caller-chosen token
-        g["d_past"].fill_(st.offset) if g.get("synced_offset") != st.offset else None
-        g["graph"].launch()
-        g["n_replays"] = g.get("n_replays", 0) + 1              # replay r wrote its token to history[:, r - 1] (while it fits)
-        st.offset += 1
-        g["synced_offset"] = st.offset
-        g["host_tok"] = g["next_tok"].view(-1, 1)
-        return g["logits"].view(st.B, 1, -1), g["host_tok"]
-
-    @_on_device
-    def __call__(self, input_ids, pixel_values=None, image_sizes=None, positions=None, cache=None, pids=None, mask=None,
-                 max_tokens=0, advance_offset=None, n_beam=1, full_logits=None):
-        """Phi3ForCausalLM.__call__ (phi.py:606-608) + Phi3F.__call__ (phi.py:576-592).
-
-        Returns (logits bf16 [B, L', V], cache).  On a prefill call (cache is None)
-        only the last position is projected through lm_head (L' = 1) unless
-        `full_logits=True`: every caller in the reference reads `logits[:, -1]`
-        of a prefill only; cached calls return all L rows."""
-        cfg, w = self.cfg, self.w
-        if torch.is_tensor(input_ids):
-            ids = input_ids.to(self.device, I32)
-        else:
-            ids = torch.as_tensor(np.asarray(input_ids).astype(np.int32)).to(self.device)
-        if ids.dim() == 1:
-            ids = ids[None]
-        ids = ids.contiguous()
-        B, L = ids.shape
-        H = cfg.hidden_size
-        prefill = cache is None
-        if prefill and pixel_values is None and B == 1 and pids is None and mask is None and n_beam == 1 and not full_logits \
-                and advance_offset is None:
-            got = self._prefill_captured(ids, L, max_tokens)
-            if got is not None:
-                return got
-        if prefill:
-            # (before the vision tower is enqueued: the host is launch-bound through the ViT's ~280 launches, so whatever it does between
-            #  the tower and the decoder -- cache allocation, its zero fill, the rotation tables -- would show as idle GPU time there)
-            st = self._new_state(B, L, max_tokens, pids, mask)
-            cache = [LayerCache(st, i) for i in range(cfg.num_hidden_layers)]
-        else:
-            st = cache[0].state
-        x = ops.embed_gather(ids.view(-1), w["model.embed_tokens.weight"])
-        if pixel_values is not None and self.vision:
-            self.vision_embed(x, pixel_values, image_sizes, positions, L)
-        past = st.offset
-        if n_beam == 1 and past + L > st.T:
-            raise ValueError(f"KV cache overflow: {past}+{L} > {st.T} (prompt + max_tokens)")
-        if full_logits is None:
-            full_logits = not prefill
-        x = self._layers(x, st, B, L, past, n_beam, last_only=not full_logits)
-        if n_beam == 1:
-            st.offset = past + L                                 # KVCache.__call__ auto-advance (phi.py:544-547)
-        if advance_offset is not None:
-            st.offset = past + advance_offset                    # phi.py:589-591
-        if not full_logits and x.shape[0] != B:
-            x = x.view(B, L, H)[:, -1, :].contiguous()
-        logits = self._proj(x, "lm_head.weight", norm_w=w["model.norm.weight"])
-        return logits.view(B, -1, cfg.vocab_size), cache
-
-    # ------------------------------------------------------------------ captured prefill of short text prompts
-    PREFILL_GRAPH_MAX_S = 512
-    PREFILL_GRAPH_ENTRIES = 4
-    PREFILL_GRAPH_MAX_CACHE_BYTES = 2 << 30                       # an entry pins its (S + max_tokens) KV cache: 393 KB per token at full size
-
-    def _prefill_captured(self, ids, S, max_tokens):
-        """Short text prompts (B = 1, 17 .. 512 tokens) are launch-bound: ~390 launches of a few microseconds each, every one paid
-        for in Python + ctypes time (4.5 ms of wall time for 3.6 ms of kernels).  A (length, max_tokens) pair seen
-        for the SECOND time is captured as ONE hipGraph over buffers the entry owns -- ids, activations, rotation tables, the KV
-        cache itself -- and later prompts of that geometry cost one 0.5 KB copy + one graph launch.  The entry's cache is LEASED to
-        the caller: every call gets its own CacheState object (a shallow copy of the entry's: same tensors, same decode graphs, its
-        own offset) and the lease IS that object -- while it is alive, through the returned cache list or through a kept
-        `cache[i].state`, a new prompt of the same geometry takes the eager path, so a caller that keeps two caches gets two caches
-        (the reference's contract).  An entry whose caller died in an unrecovered failed step is dropped (`CacheState.mark_dirty`),
-        and entries whose cache would exceed PREFILL_GRAPH_MAX_CACHE_BYTES are not made.  Bit-identical to the eager path (same
-        kernels, same order).  P3V_PREFILL_GRAPH=0 switches it off.  Returns None when not applicable."""
+    def _prefill_key(self, S, max_tokens):
         cfg = self.cfg
-        if (os.environ.get("P3V_PREFILL_GRAPH", "1") == "0" or S <= ops.L.DECODE_MAX_L or S > self.PREFILL_GRAPH_MAX_S or max_tokens < 1
-                or getattr(cfg, "use_quantized_cache", False) or self.adapters or self.hidden_hook is not None or self.w8):
-            return None                                           # (4-bit weights are captured too, round 6: their prefill is the bf16 one + a
+        if getattr(cfg, "use_quantized_cache", False) or self.adapters or self.w8:
+            return None                                           # (4-bit weights are captured too: their prefill is the bf16 one + a
                                                                   #  dequantise launch per projection into the model's own scratch)
-        if 4 * cfg.num_hidden_layers * cfg.num_key_value_heads * self.hd * (S + max_tokens + 256) > self.PREFILL_GRAPH_MAX_CACHE_BYTES:
-            return None
         # the graph bakes in the rotation tables and the weight pointers: both are part of the key (tests mutate `cfg` and swap weight
         # tensors on a live model; in-place weight updates are seen by the graph as they are by every launch)
         nl = cfg.num_hidden_layers - 1
+
         def wptr(k):
             return self.w[k].data_ptr() if k in self.w else self.w4[k][0].data_ptr()
-        key = (S, max_tokens, rope_scaling_factor(cfg), float(cfg.rope_theta), cfg.original_max_position_embeddings,
-               self.w["model.embed_tokens.weight"].data_ptr(), wptr("lm_head.weight"),
-               wptr("model.layers.0.self_attn.qkv_proj.weight"), wptr(f"model.layers.{nl}.mlp.down_proj.weight"))
-        e = self._prefill_graphs.get(key)
-        if e is None:
-            if self._prefill_seen.get(key, 0) < 1:                # first sighting: eager (one-off lengths never pay for a capture)
-                if len(self._prefill_seen) > 64:
-                    self._prefill_seen.clear()
-                self._prefill_seen[key] = 1
-                return None
-            if len(self._prefill_graphs) >= self.PREFILL_GRAPH_ENTRIES:
-                self._prefill_graphs.pop(next(iter(self._prefill_graphs)))
-            e = self._prefill_graphs[key] = self._build_prefill_graph(S, max_tokens)
-        if e["lease"] is not None and e["lease"]() is not None:    # the previous caller still holds this entry's cache
-            return None
-        if e["st"].shared["dirty"]:                               # its last caller died in a failed step: NaN rows, half-armed buffers
-            del self._prefill_graphs[key]
-            self._prefill_seen[key] = 1                           # (the next prompt of this geometry captures afresh)
-            return None
-        st = copy.copy(e["st"])                                   # this call's state: the entry's tensors and graphs, its own offset
-        self._states.add(st)
-        e["ids"].copy_(ids.view(-1), non_blocking=True)
-        st.offset = 0
-        g = st.graphs.get("greedy")
-        if g is not None:                                         # the decode graph of this cache geometry stays valid: same buffers
-            g["n_replays"], g["host_tok"], g["synced_offset"] = 0, None, None
-            g["d_step"].zero_()
-        e["graph"].launch()
-        st.offset = S
-        e["lease"] = weakref.ref(st)
-        return e["logits"].clone().view(1, 1, cfg.vocab_size), [LayerCache(st, i) for i in range(cfg.num_hidden_layers)]
-
-    def _build_prefill_graph(self, S, max_tokens):
-        cfg, w, dev = self.cfg, self.w, self.device
-        st = self._new_state(1, S, max_tokens, None, None)
-        e = dict(st=st, lease=None, ids=torch.zeros((S,), dtype=I32, device=dev), x=torch.empty((S, cfg.hidden_size), dtype=BF16, device=dev),
-                 logits=torch.empty((1, cfg.vocab_size), dtype=BF16, device=dev), bufs=self._alloc_bufs(1, S), ws={})
-
-        def run():
-            st.offset = 0
-            ops.embed_gather(e["ids"], w["model.embed_tokens.weight"], out=e["x"])
-            xl = self._layers(e["x"], st, 1, S, 0, 1, bufs=e["bufs"], last_only=True)
-            self._proj(xl.view(1, -1), "lm_head.weight", norm_w=w["model.norm.weight"], out=e["logits"])
-        with ops.owned_gemm_workspace(e["ws"], frozen=False):
-            run()                                                # warm-up (sizes the split-K workspace the graph owns)
-        torch.cuda.synchronize()
-        graph = ops.Graph()
-        side = torch.cuda.Stream(device=dev)
-        side.wait_stream(torch.cuda.current_stream())
-        with torch.cuda.stream(side), ops.owned_gemm_workspace(e["ws"], frozen=True):
-            graph.begin()
-            run()
-            graph.end()
-        torch.cuda.current_stream().wait_stream(side)
-        e["graph"] = graph
-        return e
-
-    @property
-    def layers(self):
-        return range(self.cfg.num_hidden_layers)
+        return (S, max_tokens, rope_scaling_factor(cfg), float(cfg.rope_theta), cfg.original_max_position_embeddings,
+                self.w["model.embed_tokens.weight"].data_ptr(), wptr("lm_head.weight"),
+                wptr("model.layers.0.self_attn.qkv_proj.weight"), wptr(f"model.layers.{nl}.mlp.down_proj.weight"))

@@ -11,7 +11,7 @@ import torch
 
 from . import _lib as L
 from ._lib import (EPI_BIAS, EPI_BIAS_GELU, EPI_BIAS_QGELU, EPI_BIAS_RESID_F32, EPI_F32, EPI_NONE,  # noqa: F401
-                   EPI_PATCH, EPI_RESID_BF16, EPI_SILU_MUL)
+                   EPI_PATCH, EPI_RESID_BF16, EPI_SCALE_RESID_F32, EPI_SILU_MUL)
 
 BF16, F32, I32 = torch.bfloat16, torch.float32, torch.int32
 
@@ -490,30 +490,36 @@ def hd_merge(feats, sub_gn, glb_gn, h, w, grid, C_):
     return out
 
 
+def _logits(t, name, bf16_fn, f32_fn):
+    """The entry point for a logits tensor's type (bf16, or fp32 of an fp32 model)."""
+    _chk(t, F32 if t.dtype == F32 else BF16, name)
+    return f32_fn if t.dtype == F32 else bf16_fn
+
+
 def argmax(logits2d, out=None):
-    """mx.argmax(logits[:, -1, :]) (phi_3_vision_mlx.py:386): bf16 rows, first max wins."""
-    _chk(logits2d, BF16, "logits")
+    """mx.argmax(logits[:, -1, :]) (phi_3_vision_mlx.py:386): bf16 or fp32 rows, first max wins."""
+    fn = _logits(logits2d, "logits", L.lib().p3v_argmax, L.lib().p3v_argmax_f32)
     rows, n = logits2d.shape
     out = torch.empty((rows,), dtype=I32, device=logits2d.device) if out is None else out
-    L.check(L.lib().p3v_argmax(_p(logits2d), _p(out), rows, n, n, _stream()), "argmax")
+    L.check(fn(_p(logits2d), _p(out), rows, n, n, _stream()), "argmax")
     return out
 
 
 def log_softmax(x):
-    """nn.log_softmax over the last axis: x - bf16(logsumexp(x)), rounded to bf16 (the reference's composite)."""
-    _chk(x, BF16, "x")
+    """nn.log_softmax over the last axis: x - bf16(logsumexp(x)), rounded to bf16 (the reference's composite; fp32 rows: unrounded)."""
+    fn = _logits(x, "x", L.lib().p3v_log_softmax, L.lib().p3v_log_softmax_f32)
     n = x.shape[-1]
     y = torch.empty_like(x)
-    L.check(L.lib().p3v_log_softmax(_p(x), _p(y), x.numel() // n, n, _stream()), "log_softmax")
+    L.check(fn(_p(x), _p(y), x.numel() // n, n, _stream()), "log_softmax")
     return y
 
 
 def topk(x2d, k):
     """k largest per row ordered by (-value, index); replaces mx.argpartition (Q9)."""
-    _chk(x2d, BF16, "x")
+    fn = _logits(x2d, "x", L.lib().p3v_topk, L.lib().p3v_topk_f32)
     rows, n = x2d.shape
     out = torch.empty((rows, k), dtype=I32, device=x2d.device)
-    L.check(L.lib().p3v_topk(_p(x2d), _p(out), rows, n, k, n, _stream()), "topk")
+    L.check(fn(_p(x2d), _p(out), rows, n, k, n, _stream()), "topk")
     return out
 
 
@@ -589,8 +595,108 @@ def step_begin(tok, table, x_out, cos_t, sin_t, d_past, cos_out, sin_out, zero_b
 def step_end(logits, next_tok, tok, history, d_step, d_past, ticket):
     """Tail of a replayed greedy step: argmax + history/tok bookkeeping + counters (one launch)."""
     B, n = logits.shape[0], logits.shape[-1]
-    L.check(L.lib().p3v_step_end(_p(logits), _p(next_tok), _p(tok), _p(history), _p(d_step), _p(d_past), _p(ticket), B, n,
+    fn = _logits(logits, "logits", L.lib().p3v_step_end, L.lib().p3v_step_end_f32)
+    L.check(fn(_p(logits), _p(next_tok), _p(tok), _p(history), _p(d_step), _p(d_past), _p(ticket), B, n,
                                  history.shape[1], _stream()), "step_end")
+
+
+# ---------------------------------------------------------------- layered decoders (include/p3v.h)
+def embed_scale(ids, table, scale, out=None):
+    """x fp32 [n, H] = table[id] * scale."""
+    _chk(ids, I32, "ids"), _chk(table, BF16, "table")
+    V, H = table.shape
+    out = torch.empty((ids.numel(), H), dtype=F32, device=table.device) if out is None else out
+    L.check(L.lib().p3v_embed_scale(_p(ids), _p(table), _p(out), ids.numel(), H, V, float(scale), _stream()), "embed_scale")
+    return out
+
+
+def dyt(x, norm, out, B, Lq, shift=None, hist=None, past=0, d_past=None, pad_len=None):
+    """Dynamic tanh of the fp32 residual rows x [B*L, H]: norm = (alpha, w, b) -> out (bf16 or fp32 rows).  shift (bf16 [H]): token shift
+    behind it, the token before a call's first one taken from (and the call's last ones stored in) hist [B, R, H] fp32."""
+    alpha, w, b = norm
+    _chk(x, F32, "x"), _chk(w, BF16, "w"), _chk(b, BF16, "b"), _chk(out, F32 if out.dtype == F32 else BF16, "out")
+    H = x.shape[-1]
+    if x.numel() < B * Lq * H or out.numel() < B * Lq * H or w.numel() != H or b.numel() != H:
+        raise ValueError(f"dyt: shapes {tuple(x.shape)}, {tuple(w.shape)} -> {tuple(out.shape)} for {B} x {Lq} rows")
+    if shift is not None:
+        _chk(shift, BF16, "shift"), _chk(hist, F32, "hist")
+        if shift.numel() != H or hist.shape[0] != B or hist.shape[2] != H:
+            raise ValueError(f"dyt: shift {tuple(shift.shape)}, history {tuple(hist.shape)}")
+    args = L.DytArgs(_p(x), _p(w), _p(b), _p(shift), _p(hist) if shift is not None else 0, _p(pad_len), _p(d_past), float(alpha),
+                     int(past), hist.shape[1] if shift is not None else 0, B, Lq, H)
+    L.check(L.lib().p3v_dyt(C.byref(args), _p(out), int(out.dtype == F32), _stream()), "dyt")
+    return out
+
+
+def project(x, w, epilogue=EPI_NONE, resid=None, col_scale=None, out=None):
+    """One projection of a layered decoder, x [M, K] bf16 or fp32: the weight-streaming GEMV, the MFMA GEMM, or -- fp32 rows, and sizes
+    those do not take -- the fp32-arithmetic kernel of every size."""
+    f32 = x.dtype == F32
+    _chk(x, F32 if f32 else BF16, "x"), _chk(w, BF16, "w")
+    M, K = x.shape
+    N = w.shape[0] // 2 if epilogue == EPI_SILU_MUL else w.shape[0]
+    if w.shape[1] != K:
+        raise ValueError(f"project: K mismatch {tuple(x.shape)} x {tuple(w.shape)}")
+    if out is None:
+        out = torch.empty((M, N), dtype=F32 if f32 or epilogue in (EPI_F32, EPI_SCALE_RESID_F32) else BF16, device=x.device)
+    if tuple(out.shape) != (M, N) or (resid is not None and tuple(resid.shape) != (M, N)) or (col_scale is not None and col_scale.numel() != N):
+        raise ValueError(f"project: output {tuple(out.shape)} for {M} x {N}")
+    scaled = epilogue == EPI_SCALE_RESID_F32
+    if scaled:
+        _chk(resid, F32, "resid"), _chk(col_scale, BF16, "col_scale"), _chk(out, F32, "out")
+    if not f32 and not scaled and K % 8 == 0 and out.is_contiguous():
+        if M <= 8 or (M <= GEMV_MAX_M and K % 512 == 0):
+            return gemv(x, w, epilogue, resid=resid, out=out)
+        if K % 64 == 0 and N % 8 == 0:
+            return gemm(x, w, epilogue, resid=resid, out=out)
+    args = L.GemmArgs(_p(x), _p(w), _p(out), 0, _p(resid), 0, M, N, K, x.stride(0), w.stride(0), out.stride(0), epilogue, 0, 0, 0, _p(col_scale))
+    L.check(L.lib().p3v_gemm_any(C.byref(args), int(f32), _stream()), "gemm_any")
+    return out
+
+
+def mix_plan(B, Lq, H, G, dim, vdim, n_keys, dtype):
+    """Key splits of a mixed-head attention call (0: the any-size kernel); n_keys = cache capacity for one-token calls, past + L otherwise."""
+    return int(L.lib().p3v_attn_mix_plan(B, Lq, H, G, dim, vdim, int(n_keys), int(dtype == F32)))
+
+
+def mix_ws_bytes(B, Lq, H, vdim, n_split):
+    return int(L.lib().p3v_attn_mix_ws_bytes(B, Lq, H, vdim, n_split)) if n_split > 0 else 0
+
+
+def attention_mixed(qkv, q, k, v, out, norms, talk, sink, B, Lq, H, G, dim, vdim, eps, scale, past, v_first=None, vmix=0.0, pad_len=None,
+                    d_past=None, ws=None, n_split=0):
+    """Head split + whole-projection q / k norms + value mixing + cache append + attention with mixed heads, sink and output gate
+    (include/p3v.h: p3v_mix_args_t).  qkv [B*L, >= H dim + G dim + G vdim + H] (bf16 or fp32), caches k / v as LayeredCacheState keeps
+    them, out [B*L, H vdim]; v_first [B*L, >= G vdim] view: the first value-mixing layer's own values of these tokens."""
+    f32 = qkv.dtype == F32
+    for t, n in ((qkv, "qkv"), (q, "q"), (k, "k"), (v, "v"), (out, "out")):
+        _chk(t, F32 if f32 else BF16, n)
+    for t, n in ((norms[0], "q_norm"), (norms[1], "k_norm"), (talk, "talk"), (sink, "sink")):
+        _chk(t, BF16, n)
+    dimp, vdimp, Tp, ld = k.shape[3], v.shape[3], k.shape[2], qkv.shape[1]
+    n_qkv = H * dim + G * (dim + vdim)
+    if (tuple(k.shape[:2]) != (B, G) or tuple(v.shape) != (B, G, Tp // 16, vdimp, 16) or qkv.shape[0] != B * Lq or ld < n_qkv + H
+            or q.numel() < B * H * Lq * dimp or out.numel() < B * Lq * H * vdim or norms[0].numel() != H * dim or norms[1].numel() != G * dim
+            or tuple(talk.shape) != (H, H) or sink.numel() != H or (pad_len is not None and pad_len.numel() != B)):
+        raise ValueError(f"attention_mixed: shapes qkv {tuple(qkv.shape)}, k {tuple(k.shape)}, v {tuple(v.shape)}, out {tuple(out.shape)}")
+    if v_first is not None and (v_first.dtype != qkv.dtype or tuple(v_first.shape) != (B * Lq, G * vdim) or v_first.stride(1) != 1):
+        raise ValueError("attention_mixed: v_first is a [B*L, G vdim] row view")
+    if n_split > 0 and (n_split > 1 or Lq == 1) and (ws is None or ws.numel() * ws.element_size() < mix_ws_bytes(B, Lq, H, vdim, n_split)):
+        raise ValueError("attention_mixed: workspace smaller than mix_ws_bytes")
+    if d_past is None and past + Lq > Tp:
+        raise ValueError(f"attention_mixed: columns {past} + {Lq} > {Tp}")
+    gate = qkv[:, n_qkv:]
+    args = L.MixArgs(_p(qkv), _p(norms[0]), _p(norms[1]), _p(v_first), _p(q), _p(k), _p(v), _p(talk), _p(sink), _p(gate), _p(out), _p(ws),
+                     _p(pad_len), _p(d_past), float(eps), float(vmix), float(scale), B, Lq, H, G, dim, vdim, dimp, vdimp, ld,
+                     0 if v_first is None else v_first.stride(0), int(past), Tp, int(n_split), int(f32))
+    if Lq == 1 and n_split > 0:
+        rc = L.lib().p3v_attn_mix_decode(C.byref(args), _stream())
+        if rc != L.ERR_UNSUPPORTED:
+            L.check(rc, "attn_mix_decode")
+            return out
+    L.check(L.lib().p3v_qkv_heads(C.byref(args), _stream()), "qkv_heads")
+    L.check(L.lib().p3v_attn_mix(C.byref(args), _stream()), "attn_mix")
+    return out
 
 
 def store_token(tok, history, d_step, tok_next=None):

@@ -45,18 +45,24 @@ class ByteTokenizer:
     SPECIALS = {"<|endoftext|>": 32000, "<|assistant|>": 32001, "<|system|>": 32006,
                 "<|end|>": 32007, "<|user|>": 32010}
 
-    def __init__(self):
+    def __init__(self, vocab_size=None):
+        """vocab_size: a vocabulary too small for the chat markers spells them out as bytes and takes id 2 as the prefix token."""
+        self.vocab_size = vocab_size
+        if vocab_size is not None and vocab_size <= max(self.SPECIALS.values()):
+            self.SPECIALS, self.PREFIX = {}, 2
         self._inv = {v: k for k, v in self.SPECIALS.items()}
-        self._split = re.compile("(" + "|".join(re.escape(k) for k in self.SPECIALS) + ")")
+        self._split = re.compile("(" + "|".join(re.escape(k) for k in self.SPECIALS) + ")") if self.SPECIALS else None
 
     def encode(self, text, add_special_tokens=True):
         ids = [self.BOS] if add_special_tokens else []
         ids.append(self.PREFIX)
-        for part in self._split.split(text):
+        for part in self._split.split(text) if self._split else [text]:
             if part in self.SPECIALS:
                 ids.append(self.SPECIALS[part])
             else:
                 ids.extend(3 + b for b in part.encode("utf-8"))
+        if self.vocab_size is not None and max(ids) >= self.vocab_size:
+            raise ValueError(f"token id {max(ids)} is outside the vocabulary of {self.vocab_size}: the model directory needs a tokenizer")
         return ids
 
     def __call__(self, texts, add_special_tokens=True):
@@ -86,7 +92,7 @@ class ByteTokenizer:
         return [self.decode(s, skip_special_tokens) for s in seqs]
 
 
-def load_tokenizer(local_dir):
+def load_tokenizer(local_dir, vocab_size=None):
     """`AutoTokenizer.from_pretrained(local_dir)` as the reference does
     (phi.py:230) when tokenizer files exist; otherwise the byte fallback."""
     has_files = local_dir is not None and any(
@@ -94,7 +100,7 @@ def load_tokenizer(local_dir):
     if has_files:
         from transformers import AutoTokenizer
         return AutoTokenizer.from_pretrained(local_dir)
-    return ByteTokenizer()
+    return ByteTokenizer(vocab_size)
 
 
 # ---------------------------------------------------------------------------
@@ -122,6 +128,18 @@ class Phi3FProcessor:
     def __call__(self, texts, images=None):
         if images is not None:
             print("WARNING: You are using phi3_mini_128k. Use phi3_v for VLM tasks.")
+        return self._tokenize(texts)
+
+
+class TextProcessor(Phi3FProcessor):
+    """Text requests of a model whose vocabulary size its config gives; the tokenizer of the model directory, or bytes."""
+
+    def __init__(self, local_dir=None, return_mx=True, tokenizer=None, vocab_size=None):
+        super().__init__(local_dir, return_mx, tokenizer if tokenizer is not None else load_tokenizer(local_dir, vocab_size))
+
+    def __call__(self, texts, images=None):
+        if images is not None:
+            raise ValueError("a text model takes no images")
         return self._tokenize(texts)
 
 

@@ -277,16 +277,18 @@ def serve_continuous(engine, port=8000, host="127.0.0.1", image_policy=None, **k
 
 
 def run(port=8000, synthetic=False, blind_model=False, merge=False, continuous=False, host="127.0.0.1", image_policy=None,
-        long_window=0, slots=8):
+        long_window=0, slots=8, model_path=None, dtype=None):
     from .api import _apply_chat_template, generate, load
-    preload = load(blind_model=blind_model, synthetic=synthetic or None)
+    preload = load(blind_model=blind_model, synthetic=synthetic or None, model_path=model_path, **({"dtype": dtype} if dtype else {}))
     processor = preload[1]
     preload[0].serving = True            # a server does not own the GPU: no launch that needs its whole grid resident at once (model.py)
     if continuous:
         import torch.distributed as dist
         from .engine import ContinuousEngine, RegimeRouter
-        eng = ContinuousEngine(*preload, slots=slots)                 # requests with prompt + max_tokens <= 4096 (short RoPE factors)
-        if long_window > 4096:                                       # + one engine for the long-RoPE regime (phi.py:492)
+        regimes = getattr(preload[0], "rope_regimes", True)
+        window = {} if regimes or not long_window else {"window": long_window}
+        eng = ContinuousEngine(*preload, slots=slots, **window)       # requests with prompt + max_tokens <= 4096 (short RoPE factors)
+        if regimes and long_window > 4096:                                       # + one engine for the long-RoPE regime (phi.py:492)
             eng = RegimeRouter([eng, ContinuousEngine(*preload, slots=max(1, slots // 2), window=long_window)])
         world = dist.get_world_size() if dist.is_available() and dist.is_initialized() else 1
         front = None
@@ -335,6 +337,8 @@ if __name__ == "__main__":
     ap.add_argument("--port", type=int, default=8000)
     ap.add_argument("--synthetic", action="store_true", help="seeded random weights instead of models/phi3_v")
     ap.add_argument("--tiny", action="store_true", help="with --synthetic: the 2-layer test model (smoke tests)")
+    ap.add_argument("--model", default=None, help="model directory (config.json + *.safetensors) of any supported architecture")
+    ap.add_argument("--dtype", default=None, choices=("bfloat16", "float32"), help="activation type (float32: layered decoders only)")
     ap.add_argument("--blind", action="store_true", help="text-only Phi-3-mini-128K")
     ap.add_argument("--merge", action="store_true", help="fold concurrent same-budget requests into one batched generate (opt-in)")
     ap.add_argument("--continuous", action="store_true", help="continuous batching engine (requests join / leave between decode steps)")
@@ -355,4 +359,5 @@ if __name__ == "__main__":
         if torch.cuda.is_available():
             torch.cuda.set_device(int(os.environ.get("LOCAL_RANK", "0")) % torch.cuda.device_count())   # (fewer GPUs than ranks: shared)
         dist.init_process_group("gloo")                          # requests and token lists only: host memory (fleet.py)
-    run(a.port, "tiny" if a.synthetic and a.tiny else a.synthetic, a.blind, a.merge, a.continuous, a.host, ImagePolicy(a.image_dir, a.image_host), a.long_window, a.slots)
+    run(a.port, "tiny" if a.synthetic and a.tiny else a.synthetic, a.blind, a.merge, a.continuous, a.host, ImagePolicy(a.image_dir, a.image_host), a.long_window, a.slots,
+        a.model, a.dtype)

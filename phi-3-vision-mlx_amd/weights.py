@@ -15,6 +15,7 @@ import zlib
 import torch
 
 from .config import is_vision
+from .registry import family
 
 _M32 = 0xFFFFFFFF
 
@@ -60,6 +61,36 @@ def row_exponents(n_rows, seed, spread, device="cpu"):
 
 
 def weight_specs(cfg):
+    """[(name, shape, kind)] of every tensor of the model (its family's table; kinds: _KIND)."""
+    return family(cfg).weight_specs(cfg)
+
+
+def layered_weight_specs(cfg):
+    """The tensors of a layered decoder (config.LayerSpec)."""
+    D, V = cfg.hidden_size, cfg.vocab_size
+    first_v = next((i for i, s in enumerate(cfg.layers) if s.mixer.v_mix), None)
+
+    def norm(name):
+        return [(name, (D,), "norm"), (name + ".b", (D,), "bias"), (name + ".alpha", (), "alpha")]
+    specs = [("embed", (V, D), "embed")]
+    for i, s in enumerate(cfg.layers):
+        p, m = f"l{i}.", s.mixer
+        H, G = m.heads, m.kv_heads
+        specs += norm(p + "norm1")
+        specs += [(p + "mix.q", (H * m.dim, D), "matrix"), (p + "mix.k", (G * m.dim, D), "matrix"), (p + "mix.v", (G * m.vdim, D), "matrix"),
+                  (p + "mix.q.norm", (H * m.dim,), "norm"), (p + "mix.k.norm", (G * m.dim,), "norm"),
+                  (p + "mix.talk", (H, H), "talk"), (p + "mix.sink", (H,), "sink"), (p + "mix.g", (H, D), "matrix"),
+                  (p + "mix.o", (D, H * m.vdim), "matrix"), (p + "ls1", (D,), "norm"), (p + "shift", (D,), "shift")]
+        if m.v_mix and i != first_v:                             # (the first such layer blends nothing in: a tensor of it is not read)
+            specs.append((p + "mix.vmix", (), "alpha"))
+        if s.mlp is not None:
+            specs += norm(p + "norm2")
+            specs += [(p + "mlp.gate", (s.mlp.ff, D), "matrix"), (p + "mlp.up", (s.mlp.ff, D), "matrix"), (p + "mlp.down", (D, s.mlp.ff), "matrix"),
+                      (p + "ls2", (D,), "norm")]
+    return specs + norm("final.norm") + [("head", (V, D), "matrix")]
+
+
+def phi3_weight_specs(cfg):
     """[(name, shape, kind)] in HF naming; kind in {matrix, norm, bias, embed, gn}."""
     H, I, V = cfg.hidden_size, cfg.intermediate_size, cfg.vocab_size
     nh, nkv = cfg.num_attention_heads, cfg.num_key_value_heads
@@ -113,6 +144,7 @@ def weight_specs(cfg):
 _KIND = {  # kind -> (std, mean)
     "matrix": (0.02, 0.0), "embed": (0.02, 0.0), "bias": (0.02, 0.0),
     "gn": (0.02, 0.0), "norm": (0.05, 1.0),
+    "alpha": (0.1, 0.6), "sink": (0.5, 1.0), "shift": (0.2, 0.4), "talk": (0.1, 0.0),     # ("talk": around the identity)
 }
 
 
@@ -124,7 +156,8 @@ def synth_tensor(name, shape, kind, seed=0, device="cpu", std_scale=1.0):
     if kind in ("matrix", "embed"):
         std = std * std_scale
     sd = (zlib.crc32(name.encode()) ^ (seed * 0x85EBCA6B)) & _M32
-    return synth_values(n, sd, std, mean, device=device).reshape(shape)
+    t = synth_values(n, sd, std, mean, device=device).reshape(shape)
+    return t + torch.eye(shape[0], dtype=t.dtype, device=device) if kind == "talk" else t
 
 
 def peaked_lm_head(w, spread, head_seed=0):
@@ -241,9 +274,14 @@ def load_safetensors_dir(model_path, cfg, device="cpu"):
         if "patch_embedding.weight" in k and getattr(cfg, "sanitized", False):
             t = t.permute(0, 3, 1, 2).contiguous()
         out[k] = t.to(torch.bfloat16).to(device)
-    missing = [n for n, _, _ in weight_specs(cfg) if n not in out]
+    specs = weight_specs(cfg)
+    missing = [n for n, _, _ in specs if n not in out]
     if missing:
         raise KeyError(f"weights missing from {model_path}: {missing[:4]}{'...' if len(missing) > 4 else ''}")
+    if family(cfg).layered:
+        wrong = [(n, tuple(out[n].shape), s) for n, s, _ in specs if tuple(out[n].shape) != tuple(s)]
+        if wrong:
+            raise ValueError(f"weights of other shapes than the config's in {model_path}: {wrong[:4]}")
     return out
 
 
