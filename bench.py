@@ -49,6 +49,8 @@ def parse():
     ap.add_argument("--config4", action="store_true", help="BASELINE configs[3]: 8 mixed image+text requests per GPU, batched (B = 8)")
     ap.add_argument("--config5", action="store_true", help="BASELINE configs[4]: fp8 (e4m3) weights, W8A8 prefill on the fp8 MFMA, int8 KV cache")
     ap.add_argument("--fp8-weight-only", action="store_true", help="with --config5: fp8_activations=False (dequantise + bf16 MFMA prefill)")
+    ap.add_argument("--layered", action="store_true", help="the layered text decoders (Pelalix layers of realistic sizes, random weights) beside "
+                    "Phi-3 layers of equal size: prefill and decode throughput; its own JSON line instead of the headline one")
     ap.add_argument("--tiny", action="store_true", help="tiny config (debug only; the result is NOT the headline metric)")
     return ap.parse_args()
 
@@ -266,8 +268,82 @@ def other_configs(model, processor, dev, args):
     return out
 
 
+LAYERED_SIZES = [(3072, 32, 32, 96, 8192), (3072, 32, 8, 96, 8192), (1536, 16, 4, 96, 4096)]     # width, heads, kv heads, head size, ff
+LAYERED_LAYERS, LAYERED_VOCAB = 8, 32064
+
+
+def layered_config_dict(width, heads, kv, dim, ff, layers=LAYERED_LAYERS):
+    """A Pelalix config with the layer sizes of a Phi-3 decoder."""
+    layer = {"type": "attention", "mlp": {"kind": "dense", "ff": ff},
+             "mixer": {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "v_mix": True}}
+    return {"architecture": "Pelalix", "width": width, "vocab": LAYERED_VOCAB, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0}, "layers": [layer] * layers}
+
+
+def layered_run(model, prompts, decodes, steps, reps=5):
+    """{prompt length: (ms, tokens/s)} of the whole prompt call and {(batch, context): (ms per step, tokens/s)} of the captured greedy step."""
+    import numpy as np
+    import torch
+    from phi_3_vision_mlx_amd import ops
+    out = {"prefill": {}, "decode": {}}
+    rng = np.random.default_rng(0)
+    for S in prompts:
+        ids, ms = rng.integers(3, 32000, (1, S)), []
+        for rep in range(reps + 2):
+            torch.cuda.synchronize()
+            t0 = time.perf_counter()
+            logits, cache = model(input_ids=ids, max_tokens=8)
+            ops.argmax(logits[:, -1, :].contiguous()).tolist()
+            ms.append((time.perf_counter() - t0) * 1e3)
+            del logits, cache
+        t = float(np.median(ms[2:]))
+        out["prefill"][str(S)] = {"ms": round(t, 3), "tokens_per_s": round(S / t * 1e3, 1)}
+        print("layered: prefill", S, out["prefill"][str(S)], file=sys.stderr, flush=True)
+    for B, S in decodes:
+        logits, cache = model(input_ids=rng.integers(3, 32000, (B, S)), max_tokens=4 * steps + 16)
+        tok = ops.argmax(logits[:, -1, :].contiguous())[:, None]
+        ts = []
+        for rep in range(4):                                      # (the first region warms up and captures)
+            torch.cuda.synchronize()
+            t0 = time.perf_counter()
+            for _ in range(steps):
+                _, tok = model.greedy_step(tok, cache)
+            torch.cuda.synchronize()
+            ts.append((time.perf_counter() - t0) / steps * 1e3)
+        t = float(np.median(ts[1:]))
+        out["decode"][f"B{B}@{S}"] = {"ms_per_step": round(t, 4), "tokens_per_s": round(B / t * 1e3, 1)}
+        print("layered: decode", B, S, out["decode"][f"B{B}@{S}"], file=sys.stderr, flush=True)
+        del cache
+    return out
+
+
+def bench_layered(args):
+    import torch
+    from phi_3_vision_mlx_amd.api import load_synthetic
+    from phi_3_vision_mlx_amd.config import phi3v_config_dict
+    torch.cuda.set_device(0)
+    prompts, decodes = (512, 2048, 8192), ((1, 512), (1, 2048), (1, 8192), (8, 2048))
+    rows = []
+    for width, heads, kv, dim, ff in LAYERED_SIZES:
+        row = {"width": width, "heads": heads, "kv_heads": kv, "head_size": dim, "ff": ff, "layers": LAYERED_LAYERS, "vocab": LAYERED_VOCAB}
+        phi = dict(phi3v_config_dict(vision=False), hidden_size=width, num_attention_heads=heads, num_key_value_heads=kv, intermediate_size=ff,
+                   num_hidden_layers=LAYERED_LAYERS)
+        for name, cfg in (("pelalix", layered_config_dict(width, heads, kv, dim, ff)), ("phi3", phi)):
+            model, _ = load_synthetic(config=cfg, device="cuda:0")
+            print("layered:", name, width, heads, kv, file=sys.stderr, flush=True)
+            row[name] = layered_run(model, prompts, decodes, args.steps if args.steps != 128 else 48)
+            del model
+            torch.cuda.empty_cache()
+        row["pelalix_over_phi3_time"] = {
+            k: {s: round(row["pelalix"][k][s][f] / row["phi3"][k][s][f], 3) for s in row["phi3"][k]} for k, f in (("prefill", "ms"), ("decode", "ms_per_step"))}
+        rows.append(row)
+    print(json.dumps({"metric": "layered decoders: prefill ms and decode ms per step beside Phi-3 layers of equal size", "dtype": "bf16",
+                      "data": "synthetic", "higher_is_better": False, "sizes": rows}), flush=True)
+
+
 def main():
     args = parse()
+    if args.layered:
+        return bench_layered(args)
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
         spawn_ranks(args)                                         # does not return
     import numpy as np

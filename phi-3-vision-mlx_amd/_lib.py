@@ -39,7 +39,7 @@ class QkvSplit(C.Structure):
 
 class GemvArgs(C.Structure):
     _fields_ = [("x", vp), ("W", vp), ("out", vp), ("resid", vp), ("norm_w", vp), ("norm_eps", f32),
-                ("M", i32), ("N", i32), ("K", i32), ("epilogue", i32)]
+                ("M", i32), ("N", i32), ("K", i32), ("epilogue", i32), ("col_scale", vp)]
 
 
 class GemvStep(C.Structure):
@@ -158,6 +158,7 @@ SIGNATURES = {
     "p3v_step_end": (i32, [vp, vp, vp, vp, vp, vp, vp, i32, i32, i32, vp]),
     "p3v_embed_scale": (i32, [vp, vp, vp, i32, i32, i32, f32, vp]),
     "p3v_dyt": (i32, [C.POINTER(DytArgs), vp, i32, vp]),
+    "p3v_gemv_dyt": (i32, [C.POINTER(GemvArgs), C.POINTER(DytArgs), vp]),
     "p3v_gemm_any": (i32, [C.POINTER(GemmArgs), i32, vp]),
     "p3v_qkv_heads": (i32, [C.POINTER(MixArgs), vp]),
     "p3v_attn_mix": (i32, [C.POINTER(MixArgs), vp]),

@@ -237,7 +237,7 @@ __global__ void __launch_bounds__(256, 2) k_gemm(GemmP p) {
     if (p.bias && n < p.N) bw = *(const u32x2_t*)(p.bias + n);
     bias[j][0] = bf16lo(bw[0]), bias[j][1] = bf16hi(bw[0]), bias[j][2] = bf16lo(bw[1]), bias[j][3] = bf16hi(bw[1]);
   }
-  if (EPI == P3V_EPI_BIAS_RESID_F32 || EPI == P3V_EPI_F32 || EPI == P3V_EPI_PATCH) {
+  if (EPI == P3V_EPI_BIAS_RESID_F32 || EPI == P3V_EPI_F32 || EPI == P3V_EPI_PATCH || EPI == P3V_EPI_SCALE_RESID_F32) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int m = mrow0 + i * 16;
@@ -248,7 +248,9 @@ __global__ void __launch_bounds__(256, 2) k_gemm(GemmP p) {
           const size_t o = (size_t)m * p.ldo + n;
           size_t oo = o;
           float4 v = make_float4(acc[i][j][0] + bias[j][0], acc[i][j][1] + bias[j][1], acc[i][j][2] + bias[j][2], acc[i][j][3] + bias[j][3]);
-          if (EPI == P3V_EPI_BIAS_RESID_F32) {
+          if (EPI == P3V_EPI_SCALE_RESID_F32)                  // (`bias` carries the per-column scale)
+            v = make_float4(acc[i][j][0] * bias[j][0], acc[i][j][1] * bias[j][1], acc[i][j][2] * bias[j][2], acc[i][j][3] * bias[j][3]);
+          if (EPI == P3V_EPI_BIAS_RESID_F32 || EPI == P3V_EPI_SCALE_RESID_F32) {
             const float4 r4 = *(const float4*)((const float*)p.resid + o);
             v.x += r4.x, v.y += r4.y, v.z += r4.z, v.w += r4.w;
           } else if (EPI == P3V_EPI_PATCH) {
@@ -359,7 +361,7 @@ static int gemm_big_rows(const p3v_gemm_args_t* a) {
 // and applies the epilogue.  Without a workspace of that size the shape runs on the one-pass kernels.
 template <int EPI>
 __global__ void __launch_bounds__(256) k_splitk_reduce(const float* __restrict__ part, void* __restrict__ out, const void* __restrict__ resid,
-                                                       int M, int N, int ldp, int ldo, int S) {
+                                                       const bf16_t* __restrict__ col_scale, int M, int N, int ldp, int ldo, int S) {
   constexpr bool SILU = EPI == P3V_EPI_SILU_MUL;             // part holds [gate | up] columns (2N), out N columns
   const int per_row = N / 8;
   const long i = (long)blockIdx.x * 256 + threadIdx.x;
@@ -387,6 +389,15 @@ __global__ void __launch_bounds__(256) k_splitk_reduce(const float* __restrict__
     load8_bf16((const bf16_t*)resid + o, r);
 #pragma unroll
     for (int e = 0; e < 8; ++e) v[e] = r[e] + bf16_round(v[e]);
+  }
+  if (EPI == P3V_EPI_SCALE_RESID_F32) {
+    float c[8];
+    load8_bf16(col_scale + n, c);
+    const float* r = (const float*)resid + o;
+    const float4 r0 = *(const float4*)r, r1 = *(const float4*)(r + 4);
+    *(float4*)((float*)out + o) = make_float4(r0.x + c[0] * v[0], r0.y + c[1] * v[1], r0.z + c[2] * v[2], r0.w + c[3] * v[3]);
+    *(float4*)((float*)out + o + 4) = make_float4(r1.x + c[4] * v[4], r1.y + c[5] * v[5], r1.z + c[6] * v[6], r1.w + c[7] * v[7]);
+    return;
   }
   store8_bf16((bf16_t*)out + o, v);
 }
@@ -456,7 +467,7 @@ static int splitk_slices(int M, int N, int K, int epilogue) {
   if (t.gemm_no_splitk || M <= 16 || M > t.gemm_splitk_max_m /* beyond, every projection has >= 256 tiles anyway */ ||
       N % 128 || K % 512)
     return 1;
-  if (epilogue != P3V_EPI_NONE && epilogue != P3V_EPI_RESID_BF16 && !silu) return 1;
+  if (epilogue != P3V_EPI_NONE && epilogue != P3V_EPI_RESID_BF16 && epilogue != P3V_EPI_SCALE_RESID_F32 && !silu) return 1;
   const int w_rows = silu ? 2 * N : N;                        // SiLU: [gate; up] taken as 2N plain output columns
   const int tiles = p3v_cdiv(M, BM) * (w_rows / BN);
   int S = 1;
@@ -500,10 +511,12 @@ int p3v_splitk_reduce(const float* part, const p3v_gemm_args_t* a, int S, hipStr
   const int w_rows = silu ? 2 * a->N : a->N;
   const long items = (long)a->M * (a->N / 8);
   const dim3 grid((unsigned)p3v_cdiv(items, 256));
-  if (silu) hipLaunchKernelGGL(k_splitk_reduce<P3V_EPI_SILU_MUL>, grid, dim3(256), 0, s, part, a->out, a->resid, a->M, a->N, w_rows, a->ldo, S);
+  if (silu) hipLaunchKernelGGL(k_splitk_reduce<P3V_EPI_SILU_MUL>, grid, dim3(256), 0, s, part, a->out, a->resid, a->col_scale, a->M, a->N, w_rows, a->ldo, S);
+  else if (a->epilogue == P3V_EPI_SCALE_RESID_F32)
+    hipLaunchKernelGGL(k_splitk_reduce<P3V_EPI_SCALE_RESID_F32>, grid, dim3(256), 0, s, part, a->out, a->resid, a->col_scale, a->M, a->N, w_rows, a->ldo, S);
   else if (a->epilogue == P3V_EPI_RESID_BF16)
-    hipLaunchKernelGGL(k_splitk_reduce<P3V_EPI_RESID_BF16>, grid, dim3(256), 0, s, part, a->out, a->resid, a->M, a->N, w_rows, a->ldo, S);
-  else hipLaunchKernelGGL(k_splitk_reduce<P3V_EPI_NONE>, grid, dim3(256), 0, s, part, a->out, a->resid, a->M, a->N, w_rows, a->ldo, S);
+    hipLaunchKernelGGL(k_splitk_reduce<P3V_EPI_RESID_BF16>, grid, dim3(256), 0, s, part, a->out, a->resid, a->col_scale, a->M, a->N, w_rows, a->ldo, S);
+  else hipLaunchKernelGGL(k_splitk_reduce<P3V_EPI_NONE>, grid, dim3(256), 0, s, part, a->out, a->resid, a->col_scale, a->M, a->N, w_rows, a->ldo, S);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
 }
@@ -531,7 +544,8 @@ extern "C" int p3v_gemm(const p3v_gemm_args_t* a, void* stream) {
     return P3V_ERR_ARG;
   if ((a->epilogue == P3V_EPI_BIAS_RESID_F32 || a->epilogue == P3V_EPI_RESID_BF16) && !a->resid) return P3V_ERR_ARG;
   if (a->epilogue == P3V_EPI_PATCH && (!a->pos || a->patches_per_img <= 0)) return P3V_ERR_ARG;
-  if (a->epilogue < 0 || a->epilogue > P3V_EPI_F32) return P3V_ERR_ARG;
+  if (a->epilogue < 0 || a->epilogue > P3V_EPI_SCALE_RESID_F32) return P3V_ERR_ARG;
+  if (a->epilogue == P3V_EPI_SCALE_RESID_F32 && (!a->resid || !a->col_scale || ((uintptr_t)a->col_scale & 15) || a->bias)) return P3V_ERR_ARG;
   if (a->M == 0) return P3V_OK;
   {                                                            // operands are addressed with 32-bit byte offsets (buffer loads)
     const size_t w_rows = (size_t)a->N * (a->epilogue == P3V_EPI_SILU_MUL ? 2 : 1);
@@ -553,7 +567,7 @@ extern "C" int p3v_gemm(const p3v_gemm_args_t* a, void* stream) {
     top.M = rows_big;
     const int rc = p3v_gemm256_try(&top, s);
     if (rc == P3V_OK && rows_big < a->M) {
-      const bool f32_out = a->epilogue == P3V_EPI_BIAS_RESID_F32 || a->epilogue == P3V_EPI_F32;
+      const bool f32_out = a->epilogue == P3V_EPI_BIAS_RESID_F32 || a->epilogue == P3V_EPI_F32 || a->epilogue == P3V_EPI_SCALE_RESID_F32;
       const size_t out_row = (size_t)a->ldo * (f32_out ? 4 : 2);
       p3v_gemm_args_t rest = *a;
       rest.M = a->M - rows_big;
@@ -568,7 +582,7 @@ extern "C" int p3v_gemm(const p3v_gemm_args_t* a, void* stream) {
 }
 
 static int gemm128(const p3v_gemm_args_t* a, hipStream_t s) {
-  const GemmP p = {a->A, a->W, a->out, a->bias, a->resid, a->pos,
+  const GemmP p = {a->A, a->W, a->out, a->epilogue == P3V_EPI_SCALE_RESID_F32 ? a->col_scale : a->bias, a->resid, a->pos,
                    a->M, a->N, a->K, a->lda, a->ldw, a->ldo, a->patches_per_img, 0, {}};
   switch (a->epilogue) {
     case P3V_EPI_NONE: return launch_gemm<P3V_EPI_NONE>(p, s);
@@ -580,6 +594,7 @@ static int gemm128(const p3v_gemm_args_t* a, hipStream_t s) {
     case P3V_EPI_SILU_MUL: return launch_gemm<P3V_EPI_SILU_MUL>(p, s);
     case P3V_EPI_PATCH: return launch_gemm<P3V_EPI_PATCH>(p, s);
     case P3V_EPI_F32: return launch_gemm<P3V_EPI_F32>(p, s);
+    case P3V_EPI_SCALE_RESID_F32: return launch_gemm<P3V_EPI_SCALE_RESID_F32>(p, s);
     default: return P3V_ERR_ARG;
   }
 }

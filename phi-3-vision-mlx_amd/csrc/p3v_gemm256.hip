@@ -311,7 +311,7 @@ int p3v_gemm256_try(const p3v_gemm_args_t* a, hipStream_t s) {
   if (a->N % n_tile || a->K % TK || a->epilogue == P3V_EPI_PATCH) return P3V_ERR_UNSUPPORTED;
   const size_t w_rows = (size_t)a->N * (a->epilogue == P3V_EPI_SILU_MUL ? 2 : 1);
   if (w_rows * a->ldw * 2 >= ((size_t)1 << 32) || (size_t)256 * a->lda * 2 >= ((size_t)1 << 31)) return P3V_ERR_UNSUPPORTED;  // 32-bit buffer offsets
-  const Gemm256P p = {a->A, a->W, a->out, a->bias, a->resid, a->M, a->N, a->K, a->lda, a->ldw, a->ldo, {}};
+  const Gemm256P p = {a->A, a->W, a->out, a->epilogue == P3V_EPI_SCALE_RESID_F32 ? a->col_scale : a->bias, a->resid, a->M, a->N, a->K, a->lda, a->ldw, a->ldo, {}};
   switch (a->epilogue) {
     case P3V_EPI_NONE: return launch_gemm256<P3V_EPI_NONE>(p, s);
     case P3V_EPI_BIAS: return launch_gemm256<P3V_EPI_BIAS>(p, s);
@@ -321,6 +321,7 @@ int p3v_gemm256_try(const p3v_gemm_args_t* a, hipStream_t s) {
     case P3V_EPI_RESID_BF16: return launch_gemm256<P3V_EPI_RESID_BF16>(p, s);
     case P3V_EPI_SILU_MUL: return launch_gemm256<P3V_EPI_SILU_MUL>(p, s);
     case P3V_EPI_F32: return launch_gemm256<P3V_EPI_F32>(p, s);
+    case P3V_EPI_SCALE_RESID_F32: return launch_gemm256<P3V_EPI_SCALE_RESID_F32>(p, s);
     default: return P3V_ERR_UNSUPPORTED;
   }
 }

@@ -66,7 +66,7 @@ __device__ __forceinline__ void gemm256_epilogue(const Gemm256P& p, f32x4_t (&ac
       const int m = mrow0 + i * 16;
       if (m < p.M && n < p.N) *(u32x4_t*)((bf16_t*)p.out + (size_t)m * p.ldo + n) = w;
     }
-  } else if (EPI == P3V_EPI_BIAS_RESID_F32 || EPI == P3V_EPI_F32) {
+  } else if (EPI == P3V_EPI_BIAS_RESID_F32 || EPI == P3V_EPI_F32 || EPI == P3V_EPI_SCALE_RESID_F32) {
     float bias[4][4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
@@ -84,7 +84,9 @@ __device__ __forceinline__ void gemm256_epilogue(const Gemm256P& p, f32x4_t (&ac
         if (m < p.M && n < p.N) {
           const size_t o = (size_t)m * p.ldo + n;
           float4 v = make_float4(acc[i][j][0] + bias[j][0], acc[i][j][1] + bias[j][1], acc[i][j][2] + bias[j][2], acc[i][j][3] + bias[j][3]);
-          if (EPI == P3V_EPI_BIAS_RESID_F32) {
+          if (EPI == P3V_EPI_SCALE_RESID_F32)                  // (`bias` carries the per-column scale)
+            v = make_float4(acc[i][j][0] * bias[j][0], acc[i][j][1] * bias[j][1], acc[i][j][2] * bias[j][2], acc[i][j][3] * bias[j][3]);
+          if (EPI == P3V_EPI_BIAS_RESID_F32 || EPI == P3V_EPI_SCALE_RESID_F32) {
             const float4 r4 = *(const float4*)((const float*)p.resid + o);
             v.x += r4.x, v.y += r4.y, v.z += r4.z, v.w += r4.w;
           }

@@ -167,8 +167,10 @@ static RowsPlan rows_plan(int M, int N, int K, int epilogue) {
   const bool silu = epilogue == P3V_EPI_SILU_MUL;
   RowsPlan none = {0, 0, 0};
   if (!t.gemm_rows || M <= 8 || M > 32 || N % (silu ? 8 : 16)) return none;
-  if (epilogue != P3V_EPI_NONE && epilogue != P3V_EPI_RESID_BF16 && !silu) return none;
+  const bool scaled = epilogue == P3V_EPI_SCALE_RESID_F32;                         // (its epilogue is the reduction launch's)
+  if (epilogue != P3V_EPI_NONE && epilogue != P3V_EPI_RESID_BF16 && !scaled && !silu) return none;
   const int n_sets = N / (silu ? 8 : 16);
+  if (K == 3072 && scaled && n_sets >= 512) return none;
   if (K == 3072) return n_sets >= 512 ? RowsPlan{1, 4, 3} : RowsPlan{4, 3, 1};     // qkv / gate_up in one pass; o_proj: 4 slices of 768
   if (K == 8192) return RowsPlan{4, 4, 2};                                          // down: 4 slices of 2048
   return none;

@@ -67,6 +67,7 @@ __device__ __forceinline__ void sk_wait_stages(int n) {
 struct SkinnyP {
   const bf16_t* A; const bf16_t* W; void* out; const void* resid;
   int M, N, K, lda, ldw, ldo;      // N = output columns (SiLU: W holds 2N rows, gate rows then up rows)
+  const bf16_t* col_scale;         // P3V_EPI_SCALE_RESID_F32
   int kslice;                      // 0: one pass with the epilogue; else K columns per slice, fp32 partials
   QkvP q;                          // P3V_EPI_QKV only (p3v_gemm_qkv.h): head split + rotation + KV append in the epilogue
 };
@@ -272,6 +273,24 @@ __global__ void __launch_bounds__(512, 1) k_gemm_skinny(SkinnyP p) {
     }
     return;
   }
+  if constexpr (EPI == P3V_EPI_SCALE_RESID_F32) {
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      const int m = mrow0 + i * 16;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int n = n0 + wc * 64 + j * 16 + fq * 4;
+        if (m < p.M && n < p.N) {
+          const size_t o = (size_t)m * p.ldo + n;
+          const u32x2_t c = *(const u32x2_t*)(p.col_scale + n);
+          const float4 r4 = *(const float4*)((const float*)p.resid + o);
+          *(float4*)((float*)p.out + o) = make_float4(r4.x + acc[i][j][0] * bf16lo(c[0]), r4.y + acc[i][j][1] * bf16hi(c[0]),
+                                                      r4.z + acc[i][j][2] * bf16lo(c[1]), r4.w + acc[i][j][3] * bf16hi(c[1]));
+        }
+      }
+    }
+    return;
+  }
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int m = mrow0 + i * 16;
@@ -316,7 +335,7 @@ static int sk_slices(int M, int N, int K, int epilogue) {
   const P3vTuning& t = p3v_tuning();
   const bool silu = epilogue == P3V_EPI_SILU_MUL;
   if (t.gemm_no_skinny || M <= 8 || M > t.gemm_skinny_max_m || K % SK_BK || N % (silu ? 32 : 64)) return 0;
-  if (epilogue != P3V_EPI_NONE && epilogue != P3V_EPI_RESID_BF16 && !silu) return 0;
+  if (epilogue != P3V_EPI_NONE && epilogue != P3V_EPI_RESID_BF16 && epilogue != P3V_EPI_SCALE_RESID_F32 && !silu) return 0;
   const int tiles = p3v_cdiv(M, SK_BM) * ((silu ? 2 * N : N) / SK_TN);
   if (t.gemm_skinny_s > 0) return K % (t.gemm_skinny_s * SK_BK) ? 1 : t.gemm_skinny_s;
   int best = 1;
@@ -366,7 +385,7 @@ int p3v_gemm_skinny_partials(const p3v_gemm_args_t* a, int* S_out, hipStream_t s
   if (S <= 1 || !a->ws || a->ws_bytes < (int64_t)S * a->M * w_rows * 4) return P3V_ERR_UNSUPPORTED;
   if ((uintptr_t)a->ws & 15) return P3V_ERR_ARG;
   *S_out = S;
-  const SkinnyP p = {a->A, a->W, a->ws, a->resid, a->M, a->N, a->K, a->lda, a->ldw, a->ldo, a->K / S, {}};
+  const SkinnyP p = {a->A, a->W, a->ws, a->resid, a->M, a->N, a->K, a->lda, a->ldw, a->ldo, a->col_scale, a->K / S, {}};
   if (silu) return launch_skinny<P3V_EPI_SILU_MUL>(p, S, s);
   if (a->epilogue == P3V_EPI_RESID_BF16) return launch_skinny<P3V_EPI_RESID_BF16>(p, S, s);
   return launch_skinny<P3V_EPI_NONE>(p, S, s);
@@ -385,7 +404,8 @@ int p3v_gemm_skinny_try(const p3v_gemm_args_t* a, hipStream_t s) {
   if (rc == P3V_OK) return p3v_splitk_reduce((const float*)a->ws, a, S, s);
   if (rc != P3V_ERR_UNSUPPORTED) return rc;
   if (sk_slices(a->M, a->N, a->K, a->epilogue) == 0) return P3V_ERR_UNSUPPORTED;   // (a rows shape whose slices found no workspace and that the tile kernel does not take)
-  const SkinnyP p = {a->A, a->W, a->out, a->resid, a->M, a->N, a->K, a->lda, a->ldw, a->ldo, 0, {}};
+  const SkinnyP p = {a->A, a->W, a->out, a->resid, a->M, a->N, a->K, a->lda, a->ldw, a->ldo, a->col_scale, 0, {}};
+  if (a->epilogue == P3V_EPI_SCALE_RESID_F32) return launch_skinny<P3V_EPI_SCALE_RESID_F32>(p, 1, s);
   if (a->epilogue == P3V_EPI_SILU_MUL) return launch_skinny<P3V_EPI_SILU_MUL>(p, 1, s);
   if (a->epilogue == P3V_EPI_RESID_BF16) return launch_skinny<P3V_EPI_RESID_BF16>(p, 1, s);
   return launch_skinny<P3V_EPI_NONE>(p, 1, s);
@@ -404,7 +424,7 @@ int p3v_gemm_skinny_qkv(const p3v_gemm_args_t* a, const QkvP& q, hipStream_t s) 
       return P3V_ERR_HIP;
     attr_set = true;
   }
-  const SkinnyP p = {a->A, a->W, nullptr, nullptr, a->M, a->N, a->K, a->lda, a->ldw, 0, 0, q};
+  const SkinnyP p = {a->A, a->W, nullptr, nullptr, a->M, a->N, a->K, a->lda, a->ldw, 0, nullptr, 0, q};
   const int mt = p3v_cdiv(a->M, SK_BM), tiles = ((q.nh + q.nkv) * q.hd / 64) * mt + (q.nkv * q.hd / SK_BM) * p3v_cdiv(a->M, 64);
   hipLaunchKernelGGL((k_gemm_skinny<P3V_EPI_QKV, false, SK_TN>), dim3(tiles), dim3(512), SkCfg<SK_TN>::LDS, s, p);
   P3V_CHECK_LAUNCH();

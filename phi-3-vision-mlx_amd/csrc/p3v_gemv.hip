@@ -101,6 +101,8 @@ __global__ void __launch_bounds__(256) k_gemv(GemvP p) {
             const float v = h ? a1[m] : a0[m];
             const size_t o = (size_t)m * p.N + (h ? r1 : r0);
             if (p.epi == P3V_EPI_F32) ((float*)p.out)[o] = v;
+            else if (p.epi == P3V_EPI_SCALE_RESID_F32)
+              ((float*)p.out)[o] = ((const float*)p.resid)[o] + bf16_to_f32(p.col_scale[h ? r1 : r0]) * v;
             else if (p.epi == P3V_EPI_RESID_BF16)
               ((bf16_t*)p.out)[o] = f32_to_bf16(bf16_to_f32(p.resid[o]) + bf16_round(v));
             else ((bf16_t*)p.out)[o] = f32_to_bf16(v);
@@ -157,6 +159,13 @@ __global__ void __launch_bounds__(256) k_gemv3(GemvP p, int units_per_wave, int 
   GMARK(1);
 }
 
+template <int NST, int CH, int VAR>
+__global__ void __launch_bounds__(256) k_gemv3_layered(GemvP p, int units_per_wave, int wpw) {
+  extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
+  __shared__ float red[8];
+  gemv3_body<1, NST, CH, STEP_NONE, VAR>(p, units_per_wave, blockIdx.x, smem, red, wpw);
+}
+
 template <int MT, int NST, int CH, int STEP>
 __global__ void __launch_bounds__(256) k_gemv3_step(GemvP p, int units_per_wave, int wpw, GemvStepP sp) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
@@ -164,7 +173,7 @@ __global__ void __launch_bounds__(256) k_gemv3_step(GemvP p, int units_per_wave,
   gemv3_body<MT, NST, CH, STEP>(p, units_per_wave, blockIdx.x, smem, red, wpw, &sp);
 }
 
-template <int MT, int NST, int CH, int STEP = STEP_NONE>
+template <int MT, int NST, int CH, int STEP = STEP_NONE, int VAR = 0>
 static int launch_gemv3(const GemvP& p, hipStream_t s, const GemvStepP* sp = nullptr) {
   static int n_cu = 0;
   if (!n_cu) {
@@ -185,7 +194,9 @@ static int launch_gemv3(const GemvP& p, hipStream_t s, const GemvStepP* sp = nul
       return P3V_ERR_HIP;
     attr_set = true;
   }
-  if constexpr (STEP != STEP_NONE) {
+  if constexpr (VAR != 0) {
+    hipLaunchKernelGGL((k_gemv3_layered<NST, CH, VAR>), dim3(p3v_cdiv(waves, wpw_)), dim3(256), lds, s, p, upw, wpw_);
+  } else if constexpr (STEP != STEP_NONE) {
     if (p3v_cdiv(waves, wpw_) > P3V_GEMV_STEP_MAX_WG) return P3V_ERR_UNSUPPORTED;      // (amax_ws holds one candidate per workgroup and row)
     hipLaunchKernelGGL((k_gemv3_step<MT, NST, CH, STEP>), dim3(p3v_cdiv(waves, wpw_)), dim3(256), lds, s, p, upw, wpw_, *sp);
   } else {
@@ -286,6 +297,8 @@ __global__ void __launch_bounds__(256) k_gemv_mfma(GemvP p) {
       ((bf16_t*)p.out)[o] = f32_to_bf16(bf16_round(gt * bf16_round(1.f / (1.f + __expf(-gt)))) * up);
     } else if (p.epi == P3V_EPI_F32) {
       ((float*)p.out)[o] = v0;
+    } else if (p.epi == P3V_EPI_SCALE_RESID_F32) {
+      ((float*)p.out)[o] = ((const float*)p.resid)[o] + bf16_to_f32(p.col_scale[n]) * v0;
     } else if (p.epi == P3V_EPI_RESID_BF16) {
       ((bf16_t*)p.out)[o] = f32_to_bf16(bf16_to_f32(p.resid[o]) + bf16_round(v0));
     } else {
@@ -337,7 +350,7 @@ extern "C" int p3v_gemv_timing_read(long long* out, int n) {
 // first MFMA (that pass took 3 us; the sums are exchanged by the barrier the partials need anyway).  (Two slices in
 // flight per wave -- tried: the 32 extra load instructions block the wave in issue while the queues are full and the
 // prologue behind them gets later, not earlier.)
-template <bool SILU, int NW, int NST>
+template <bool SILU, int NW, int NST, bool SCALED = false>
 __global__ void __launch_bounds__(NW * 64) k_gemv_mfma8(GemvP p, int n_sets) {
   constexpr int KQ = NST * 256, K = KQ * NW, XS = K * 2 + 64, NCH = KQ / 8;     // slice elements, LDS row stride (bytes), slice chunks
   constexpr int ROWS = SILU ? 8 : 16;                                            // output columns per set
@@ -449,6 +462,11 @@ __global__ void __launch_bounds__(NW * 64) k_gemv_mfma8(GemvP p, int n_sets) {
     const bool e_live = tid < (SILU ? 64 : 128) && e_m < p.M && e_n < p.N;
     const size_t e_o = (size_t)e_m * p.N + e_n;
     const bool e_has = !SILU && p.epi == P3V_EPI_RESID_BF16;
+    float e_rf = 0.f, e_ls = 0.f;                                                // SCALED: fp32 residual, column scale
+    if constexpr (SCALED) {
+      e_rf = ((const float*)p.resid)[e_live ? e_o : 0];
+      e_ls = bf16_to_f32(p.col_scale[e_live ? e_n : 0]);
+    }
     uint32_t e_res = (e_has ? p.resid : p.x)[e_has && e_live ? e_o : 0];
     f32x4_t acc0 = {0.f, 0.f, 0.f, 0.f}, acc1 = {0.f, 0.f, 0.f, 0.f};
     auto step = [&](auto stc) {
@@ -500,7 +518,9 @@ __global__ void __launch_bounds__(NW * 64) k_gemv_mfma8(GemvP p, int n_sets) {
           v1 *= r;
         }
         const size_t o = e_o;
-        if (SILU) {
+        if constexpr (SCALED) {
+          ((float*)p.out)[o] = e_rf + e_ls * v0;
+        } else if (SILU) {
           const float gt = bf16_round(v0), up = bf16_round(v1);
           ((bf16_t*)p.out)[o] = f32_to_bf16(bf16_round(gt * bf16_round(1.f / (1.f + __expf(-gt)))) * up);
         } else if (p.epi == P3V_EPI_F32) {
@@ -520,12 +540,12 @@ __global__ void __launch_bounds__(NW * 64) k_gemv_mfma8(GemvP p, int n_sets) {
   do_set(IC0{}, std::false_type{});
 }
 
-template <bool SILU, int NW, int NST>
+template <bool SILU, int NW, int NST, bool SCALED = false>
 static int launch_gemv_mfma8(const GemvP& p, hipStream_t s) {
   const size_t lds = (size_t)8 * (p.K * 2 + 64);
   static bool attr_set = false;
   if (!attr_set && lds > 40 * 1024) {
-    if (hipFuncSetAttribute((const void*)k_gemv_mfma8<SILU, NW, NST>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 8704) != hipSuccess)
+    if (hipFuncSetAttribute((const void*)k_gemv_mfma8<SILU, NW, NST, SCALED>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 8704) != hipSuccess)
       return P3V_ERR_HIP;
     attr_set = true;
   }
@@ -533,7 +553,7 @@ static int launch_gemv_mfma8(const GemvP& p, hipStream_t s) {
   // (576 sets -> 192 x 3, 1024 -> 256 x 4, 2004 -> 251 x 8, 192 -> 192 x 1)
   const int max_wg = p3v_tuning().gemv8_wgs;
   const int n_sets = p3v_cdiv(p.N, SILU ? 8 : 16), per = p3v_cdiv(n_sets, max_wg), grid = p3v_cdiv(n_sets, per);
-  hipLaunchKernelGGL((k_gemv_mfma8<SILU, NW, NST>), dim3(grid), dim3(NW * 64), lds, s, p, n_sets);
+  hipLaunchKernelGGL((k_gemv_mfma8<SILU, NW, NST, SCALED>), dim3(grid), dim3(NW * 64), lds, s, p, n_sets);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
 }
@@ -574,19 +594,59 @@ extern "C" int p3v_gemv_step(const p3v_gemv_args_t* a, const p3v_gemv_step_t* st
   return begin ? launch_gemv3<1, 4, 4, STEP_BEGIN>(p, s, &sp) : launch_gemv3<1, 4, 4, STEP_END>(p, s, &sp);
 }
 
+// the one-row streaming kernel in its layered variants; P3V_ERR_UNSUPPORTED (nothing launched) for other shapes
+template <int VAR>
+static int gemv3_layered(const GemvP& p, hipStream_t s) {
+  if (p.M != 1 || p.N % 2 || p3v_tuning().gemv_variant != 3) return P3V_ERR_UNSUPPORTED;
+  switch (p.K) {
+    case 1024: return launch_gemv3<1, 1, 2, STEP_NONE, VAR>(p, s);
+    case 2048: return launch_gemv3<1, 1, 4, STEP_NONE, VAR>(p, s);
+    case 3072: return launch_gemv3<1, 1, 6, STEP_NONE, VAR>(p, s);
+    case 4096: return launch_gemv3<1, 2, 4, STEP_NONE, VAR>(p, s);
+    case 8192: return launch_gemv3<1, 4, 4, STEP_NONE, VAR>(p, s);
+    default: return P3V_ERR_UNSUPPORTED;
+  }
+}
+
+extern "C" int p3v_gemv_dyt(const p3v_gemv_args_t* a, const p3v_dyt_args_t* d, void* stream) {
+  if (!a || !d || !a->W || !a->out || a->M <= 0 || a->N <= 0 || a->K <= 0) return P3V_ERR_ARG;
+  if (!d->x || !d->w || !d->b || d->B != a->M || d->L != 1 || d->H != a->K) return P3V_ERR_ARG;
+  if (d->mu && (!d->hist || d->hist_rows < 2 || (!d->d_past && d->past < 0))) return P3V_ERR_ARG;
+  if (a->M != 1 || (a->epilogue != P3V_EPI_NONE && a->epilogue != P3V_EPI_SILU_MUL)) return P3V_ERR_UNSUPPORTED;
+  if (((uintptr_t)d->x | (uintptr_t)d->w | (uintptr_t)d->b | (uintptr_t)d->mu | (uintptr_t)d->hist | (uintptr_t)a->W) & 15) return P3V_ERR_UNSUPPORTED;
+  const GemvP p = {nullptr, a->W, a->out, nullptr, nullptr, 0.f, a->M, a->N, a->K, a->epilogue,
+                   a->epilogue == P3V_EPI_SILU_MUL ? a->N : (a->N + 1) / 2, nullptr, dyt_params(d)};
+  return gemv3_layered<GEMV_DYT>(p, (hipStream_t)stream);
+}
+
 extern "C" int p3v_gemv(const p3v_gemv_args_t* a, void* stream) {
   if (!a || !a->x || !a->W || !a->out) return P3V_ERR_ARG;
   if (a->M <= 0 || a->M > 16 || a->N <= 0 || a->K <= 0 || a->K % 8) return P3V_ERR_ARG;
   if (a->epilogue != P3V_EPI_NONE && a->epilogue != P3V_EPI_RESID_BF16 && a->epilogue != P3V_EPI_SILU_MUL &&
-      a->epilogue != P3V_EPI_F32)
+      a->epilogue != P3V_EPI_F32 && a->epilogue != P3V_EPI_SCALE_RESID_F32)
     return P3V_ERR_UNSUPPORTED;
   if (a->epilogue == P3V_EPI_RESID_BF16 && !a->resid) return P3V_ERR_ARG;
+  const bool scaled = a->epilogue == P3V_EPI_SCALE_RESID_F32;
+  if (scaled && (!a->resid || !a->col_scale)) return P3V_ERR_ARG;
   const int mt = a->M <= 1 ? 1 : a->M <= 2 ? 2 : a->M <= 4 ? 4 : 8;
   GemvP p = {a->x, a->W, a->out, a->resid, a->norm_w, a->norm_eps, a->M, a->N, a->K, a->epilogue,
-             a->epilogue == P3V_EPI_SILU_MUL ? a->N : (a->N + 1) / 2};
+             a->epilogue == P3V_EPI_SILU_MUL ? a->N : (a->N + 1) / 2, a->col_scale, {}};
   hipStream_t s = (hipStream_t)stream;
+  if (scaled) {
+    const int rc = gemv3_layered<GEMV_SCALED>(p, s);
+    if (rc != P3V_ERR_UNSUPPORTED) return rc;
+    if (p3v_tuning().gemv_mfma8 && a->M >= 2 && a->M <= 8)
+      switch (a->K) {
+        case 1024: return launch_gemv_mfma8<false, 4, 1, true>(p, s);
+        case 2048: return launch_gemv_mfma8<false, 4, 2, true>(p, s);
+        case 3072: return launch_gemv_mfma8<false, 4, 3, true>(p, s);
+        case 4096: return launch_gemv_mfma8<false, 8, 2, true>(p, s);
+        case 8192: return launch_gemv_mfma8<false, 8, 4, true>(p, s);
+        default: break;
+      }
+  }
   const int variant = p3v_tuning().gemv_variant;       // 1: generic kernel only; 3: streaming kernel where it applies
-  if (variant == 3 && mt == 1 && a->N % 2 == 0 && (a->K == 3072 || a->K == 8192)) {
+  if (variant == 3 && mt == 1 && !scaled && a->N % 2 == 0 && (a->K == 3072 || a->K == 8192)) {
     if (a->K == 3072) return launch_gemv3<1, 1, 6>(p, s);
     return launch_gemv3<1, 4, 4>(p, s);                  // 8192 = 4 stages x 4 chunks: keeps 2 waves/SIMD resident
   }
@@ -599,13 +659,13 @@ extern "C" int p3v_gemv(const p3v_gemv_args_t* a, void* stream) {
   // at ctx 2531, B = 2 / 3 / 4: 2.08 / 2.43 / 2.66 ms with the MT-row streaming kernel, 1.99 / 2.16 / 2.35 with this one);
   // P3V_GEMV8_MIN=5 restores the round-1 split
   const int rows8_min = p3v_tuning().gemv8_min;
-  if (rows_variant && variant == 3 && a->M >= 2 && a->M <= 4 && a->M < rows8_min && a->N % 2 == 0 && a->epilogue != P3V_EPI_F32 &&
+  if (rows_variant && variant == 3 && a->M >= 2 && a->M <= 4 && a->M < rows8_min && a->N % 2 == 0 && a->epilogue != P3V_EPI_F32 && !scaled &&
       (a->K == 3072 || a->K == 8192)) {
     if (a->K == 3072) return mt == 2 ? launch_gemv3<2, 1, 6>(p, s) : launch_gemv3<4, 1, 6>(p, s);
     return mt == 2 ? launch_gemv3<2, 4, 4>(p, s) : launch_gemv3<4, 4, 4>(p, s);
   }
   const int rows8 = p3v_tuning().gemv_mfma8;
-  if (rows8 && a->M >= rows8_min && a->M <= 8) {
+  if (rows8 && !scaled && a->M >= rows8_min && a->M <= 8) {
     const bool silu = a->epilogue == P3V_EPI_SILU_MUL;
     switch (a->K) {                                      // K = NW waves x NST stages x 256
       case 1024: return silu ? launch_gemv_mfma8<true, 4, 1>(p, s) : launch_gemv_mfma8<false, 4, 1>(p, s);

@@ -4,13 +4,18 @@
 #pragma once
 #include <type_traits>
 
-#include "p3v_common.h"
+#include "p3v_layered.h"
 
 struct GemvP {
   const bf16_t* x; const bf16_t* W; void* out; const bf16_t* resid; const bf16_t* norm_w;
   float eps;
   int M, N, K, epi, units;
+  const bf16_t* col_scale;               // P3V_EPI_SCALE_RESID_F32 (resid and out are fp32 then)
+  DytP dyt;                              // GEMV_DYT: dyt.x (fp32) in place of x
 };
+// Variants of the one-row body for the layered decoders (fp32 residual stream): GEMV_DYT = the input row is a dynamic tanh (+ token
+// shift) of the residual row, computed while the first weights are on their way; GEMV_SCALED = out = resid + col_scale * acc in fp32.
+enum { GEMV_DYT = 1, GEMV_SCALED = 2 };
 
 // 8 bf16 x 8 bf16 -> fp32 accumulate on v_dot2c_f32_bf16 (two products per instruction straight from the packed
 // operands): 4 VALU instructions per 16-byte weight chunk instead of 8 unpacks + 8 FMAs -- the GEMV's VALU pipe was
@@ -147,7 +152,7 @@ __device__ __forceinline__ void gemv_step_end_tail(const GemvStepP* sp, const Ar
 // wpw: waves of the 4-wave workgroup that take rows (4, or 3: wave 3 then only helps with the prologue).  1536 streaming waves
 // (qkv, o_proj, down) as 384 four-wave workgroups put two workgroups on half of the CUs and one on the others, and the launch
 // lasts as long as the doubly loaded CUs; 512 workgroups x 3 waves load every CU alike (tools/gemv_timeline.py).
-template <int MT, int NST, int CH, int STEP = STEP_NONE>
+template <int MT, int NST, int CH, int STEP = STEP_NONE, int VAR = 0>
 __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, int bx, unsigned char* smem, float* red, int wpw = 4,
                                            const GemvStepP* sp = nullptr) {
   constexpr int CHUNKS = NST * CH * 64;                 // 16-byte chunks per row (K = 8 * CHUNKS)
@@ -161,6 +166,27 @@ __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, i
   const int n_st = (u_end - u_begin) * NST;
 
   // ---- 1. x / norm-weight loads (oldest in the queue)
+  constexpr bool DYT = (VAR & GEMV_DYT) != 0, SCALED = (VAR & GEMV_SCALED) != 0;
+  static_assert(VAR == 0 || (MT == 1 && STEP == STEP_NONE), "one-row variants");
+  float4 dx[XC][2], dh[XC][2];                           // GEMV_DYT: residual chunk, the token before's unshifted input
+  u32x4_t db[XC], dm[XC];
+  int d_pos = 0;
+  bool d_prev = false;
+  if constexpr (DYT) {
+    if (p.dyt.mu) {
+      d_pos = p.dyt.d_past ? *p.dyt.d_past : p.dyt.past;
+      d_prev = d_pos > (p.dyt.pad_len ? p.dyt.pad_len[0] : 0);
+    }
+    const float* hrow = p.dyt.mu ? p.dyt.hist + (size_t)((d_pos + p.dyt.R - 1) % p.dyt.R) * (CHUNKS * 8) : p.dyt.x;
+#pragma unroll
+    for (int k = 0; k < XC; ++k) {
+      const int c = min(tid + k * 256, CHUNKS - 1);
+      dx[k][0] = ((const float4*)p.dyt.x)[2 * c], dx[k][1] = ((const float4*)p.dyt.x)[2 * c + 1];
+      dh[k][0] = ((const float4*)hrow)[2 * c], dh[k][1] = ((const float4*)hrow)[2 * c + 1];
+      db[k] = ((const u32x4_t*)p.dyt.b)[c];
+      dm[k] = ((const u32x4_t*)(p.dyt.mu ? p.dyt.mu : p.dyt.b))[c];
+    }
+  }
   u32x4_t xv[MT][XC], gv[XC];
   const bf16_t* xrow[MT];
 #pragma unroll
@@ -177,13 +203,16 @@ __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, i
   for (int k = 0; k < XC; ++k) {
     const int c = min(tid + k * 256, CHUNKS - 1);
 #pragma unroll
-    for (int m = 0; m < MT; ++m) xv[m][k] = ((const u32x4_t*)xrow[m])[c];
-    gv[k] = p.norm_w ? ((const u32x4_t*)p.norm_w)[c] : (u32x4_t){0, 0, 0, 0};
+    for (int m = 0; m < MT; ++m)
+      if constexpr (!DYT) xv[m][k] = ((const u32x4_t*)xrow[m])[c];
+    if constexpr (DYT) gv[k] = ((const u32x4_t*)p.dyt.w)[c];
+    else gv[k] = p.norm_w ? ((const u32x4_t*)p.norm_w)[c] : (u32x4_t){0, 0, 0, 0};
   }
 
   // ---- 2. weight pipeline state
   u32x4_t wbuf[2][2][CH];
   uint32_t rbuf[2][MT];                                  // residual pair (2 bf16) of the row pair, per x row
+  float2 fbuf[2];                                        // GEMV_SCALED: the fp32 residual pair, rbuf its column scales
   auto issue = [&](int gs, auto bufc) {
     constexpr int buf = decltype(bufc)::value;
     const int u = min(u_begin + gs / NST, p.units - 1), s = gs % NST;
@@ -196,8 +225,12 @@ __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, i
       wbuf[buf][0][j] = __builtin_nontemporal_load(w0 + j * 64);
       wbuf[buf][1][j] = __builtin_nontemporal_load(w1 + j * 64);
     }
+    if constexpr (SCALED) {
+      fbuf[buf] = *(const float2*)((const float*)p.resid + 2 * u);
+      rbuf[buf][0] = *(const uint32_t*)(p.col_scale + 2 * u);
+    }
 #pragma unroll
-    for (int m = 0; m < MT; ++m) {                       // 4-byte aligned: r0 = 2u is even, N is even on this path
+    for (int m = 0; m < (SCALED ? 0 : MT); ++m) {        // 4-byte aligned: r0 = 2u is even, N is even on this path
       const bf16_t* rp = p.resid + (size_t)min(m, p.M - 1) * p.N + 2 * u;
       rbuf[buf][m] = !has_res ? 0u : *(const uint32_t*)rp;
     }
@@ -205,8 +238,32 @@ __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, i
   if (n_st > 0) issue(0, IC0{});
 
   // ---- 3. RMSNorm prologue (waits for the x loads only) -> LDS
+  if constexpr (DYT) {
+    const float al = p.dyt.alpha;
 #pragma unroll
-  for (int m = 0; m < MT; ++m) {
+    for (int k = 0; k < XC; ++k) {
+      const int c = tid + k * 256;
+      if (c < CHUNKS) {
+        const float xe[8] = {dx[k][0].x, dx[k][0].y, dx[k][0].z, dx[k][0].w, dx[k][1].x, dx[k][1].y, dx[k][1].z, dx[k][1].w};
+        const float pe[8] = {dh[k][0].x, dh[k][0].y, dh[k][0].z, dh[k][0].w, dh[k][1].x, dh[k][1].y, dh[k][1].z, dh[k][1].w};
+        float h[8], s[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          const float g = j & 1 ? bf16hi(gv[k][j >> 1]) : bf16lo(gv[k][j >> 1]), b = j & 1 ? bf16hi(db[k][j >> 1]) : bf16lo(db[k][j >> 1]);
+          h[j] = tanhf(xe[j] * al) * g + b;
+          const float mu = j & 1 ? bf16hi(dm[k][j >> 1]) : bf16lo(dm[k][j >> 1]);
+          s[j] = p.dyt.mu ? h[j] + ((d_prev ? pe[j] : 0.f) - h[j]) * mu : h[j];
+        }
+        xs[c] = (u32x4_t){pack_bf16x2(s[0], s[1]), pack_bf16x2(s[2], s[3]), pack_bf16x2(s[4], s[5]), pack_bf16x2(s[6], s[7])};
+        if (p.dyt.mu && bx == 0) {                        // (another slot than the one every workgroup reads: R >= 2)
+          float4* hw = (float4*)(p.dyt.hist + (size_t)(d_pos % p.dyt.R) * (CHUNKS * 8)) + 2 * c;
+          hw[0] = make_float4(h[0], h[1], h[2], h[3]), hw[1] = make_float4(h[4], h[5], h[6], h[7]);
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int m = 0; m < (DYT ? 0 : MT); ++m) {
     float r = 1.f;
     if (p.norm_w) {
       float ss = 0.f;
@@ -268,7 +325,9 @@ __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, i
 #pragma unroll
         for (int m = 0; m < MT; ++m) {
           if (m < p.M) {
-            if (silu) {
+            if constexpr (SCALED) {
+              *(float2*)((float*)p.out + 2 * u) = make_float2(fbuf[buf].x + bf16lo(rbuf[buf][0]) * a0[0], fbuf[buf].y + bf16hi(rbuf[buf][0]) * a1[0]);
+            } else if (silu) {
               const float g = bf16_round(a0[m]), up = bf16_round(a1[m]);
               const float sg = bf16_round(g * bf16_round(1.f / (1.f + __expf(-g))));
               bf16_t* dst = (bf16_t*)p.out + (size_t)m * p.N + u;

@@ -95,8 +95,9 @@ class LayeredModel(DecoderModel):
 
     def _head(self, x, out=None, bufs=None):
         h = bufs["h"][:x.shape[0]] if bufs is not None else torch.empty(x.shape, dtype=self.act_dtype, device=x.device)
-        ops.dyt(x, self.final_norm, h, x.shape[0], 1)
-        return ops.project(h, self.head, EPI_NONE, out=out)
+        if out is None:
+            out = torch.empty((x.shape[0], self.cfg.vocab_size), dtype=self.act_dtype, device=x.device)
+        return ops.project_dyt(x, self.final_norm, self.head, h, EPI_NONE, out=out, B=x.shape[0])
 
     def _layers(self, x, st, B, L, past, n_beam, bufs=None, d_past=None, last_only=False):
         """The stack on x fp32 [B*L, width], in place.  last_only: the last layer's residual branches run on the B last rows alone;
@@ -112,8 +113,8 @@ class LayeredModel(DecoderModel):
             n_o = m.heads * m.vdim
             h, o = bufs["h"], bufs["o"][:M * n_o].view(M, n_o)
             qkv = bufs["qkv_first"] if i == self.first_v else bufs["qkv"][:M * ly.qkvg.shape[0]].view(M, -1)
-            ops.dyt(x, ly.norm1, h, B, L, shift=ly.shift, hist=st.shift[i], past=past, d_past=d_past, pad_len=st.pad_len)
-            ops.project(h, ly.qkvg, out=qkv)
+            ops.project_dyt(x, ly.norm1, ly.qkvg, h, out=qkv, B=B, Lq=L, shift=ly.shift, hist=st.shift[i], past=past, d_past=d_past,
+                            pad_len=st.pad_len)
             ops.attention_mixed(qkv, bufs["q"], st.k[i], st.v[i], o, ly.norms, ly.talk, ly.sink, B, L, m.heads, m.kv_heads, m.dim, m.vdim, eps,
                                 m.scale, past, v_first=v_first if m.v_mix else None, vmix=ly.vmix, pad_len=st.pad_len, d_past=d_past,
                                 ws=bufs["mix_ws"], n_split=bufs["n_split"][i])
@@ -126,8 +127,7 @@ class LayeredModel(DecoderModel):
             if ly.mlp:
                 ff = ly.spec.mlp.ff
                 h, a = h[:rows], bufs["a"][:rows * ff].view(rows, ff)
-                ops.dyt(x, ly.norm2, h, rows, 1)
-                ops.project(h, ly.gate_up, EPI_SILU_MUL, out=a)
+                ops.project_dyt(x, ly.norm2, ly.gate_up, h, EPI_SILU_MUL, out=a, B=rows)
                 ops.project(a, ly.down, EPI_SCALE_RESID_F32, resid=x, col_scale=ly.ls2, out=x)
             if self.hidden_hook is not None:
                 self.hidden_hook(i, x, B, rows // B)

@@ -113,20 +113,21 @@ def _gemm_workspace(device, nbytes):
     return buf
 
 
-def gemm(a, w, epilogue=EPI_NONE, bias=None, resid=None, out=None, n_out=None, pos=None, patches_per_img=0, ldo=None):
+def gemm(a, w, epilogue=EPI_NONE, bias=None, resid=None, out=None, n_out=None, pos=None, patches_per_img=0, ldo=None,
+         col_scale=None):
     """nn.Linear / patch conv: out[M,N] = a[M,K] @ w[N,K]^T (+ epilogue), bf16 MFMA."""
     _chk(a, BF16, "a"), _chk(w, BF16, "w")
     M, K = a.shape
     N = n_out if n_out is not None else (w.shape[0] // 2 if epilogue == EPI_SILU_MUL else w.shape[0])
     if w.shape[1] != K:
         raise ValueError(f"gemm: K mismatch {a.shape} x {w.shape}")
-    f32_out = epilogue in (EPI_BIAS_RESID_F32, EPI_PATCH, EPI_F32)
+    f32_out = epilogue in (EPI_BIAS_RESID_F32, EPI_PATCH, EPI_F32, EPI_SCALE_RESID_F32)
     if out is None:
         out = torch.empty((M, N), dtype=F32 if f32_out else BF16, device=a.device)
     ws_bytes = L.lib().p3v_gemm_ws_bytes(M, N, K, epilogue)
     ws = _gemm_workspace(a.device, ws_bytes) if ws_bytes else None
     args = L.GemmArgs(_p(a), _p(w), _p(out), _p(bias), _p(resid), _p(pos), M, N, K, a.stride(0), w.stride(0),
-                      ldo if ldo is not None else N, epilogue, patches_per_img, _p(ws), ws.numel() if ws is not None else 0)
+                      ldo if ldo is not None else N, epilogue, patches_per_img, _p(ws), ws.numel() if ws is not None else 0, _p(col_scale))
     L.check(L.lib().p3v_gemm(C.byref(args), _stream()), "gemm")
     return out
 
@@ -158,14 +159,14 @@ def gemm_resid_norm(a, w, resid, norm_w, eps, normed, out=None):
 GEMV_MAX_M = 16
 
 
-def gemv(x, w, epilogue=EPI_NONE, resid=None, norm_w=None, norm_eps=0.0, out=None):
+def gemv(x, w, epilogue=EPI_NONE, resid=None, norm_w=None, norm_eps=0.0, out=None, col_scale=None):
     """Skinny nn.Linear for decode (M<=16) with optional fused RMSNorm / epilogue."""
     _chk(x, BF16, "x"), _chk(w, BF16, "w")
     M, K = x.shape
     N = w.shape[0] // 2 if epilogue == EPI_SILU_MUL else w.shape[0]
     if out is None:
-        out = torch.empty((M, N), dtype=F32 if epilogue == EPI_F32 else BF16, device=x.device)
-    args = L.GemvArgs(_p(x), _p(w), _p(out), _p(resid), _p(norm_w), float(norm_eps), M, N, K, epilogue)
+        out = torch.empty((M, N), dtype=F32 if epilogue in (EPI_F32, EPI_SCALE_RESID_F32) else BF16, device=x.device)
+    args = L.GemvArgs(_p(x), _p(w), _p(out), _p(resid), _p(norm_w), float(norm_eps), M, N, K, epilogue, _p(col_scale))
     L.check(L.lib().p3v_gemv(C.byref(args), _stream()), "gemv")
     return out
 
@@ -613,19 +614,44 @@ def embed_scale(ids, table, scale, out=None):
 def dyt(x, norm, out, B, Lq, shift=None, hist=None, past=0, d_past=None, pad_len=None):
     """Dynamic tanh of the fp32 residual rows x [B*L, H]: norm = (alpha, w, b) -> out (bf16 or fp32 rows).  shift (bf16 [H]): token shift
     behind it, the token before a call's first one taken from (and the call's last ones stored in) hist [B, R, H] fp32."""
+    args = _dyt_args(x, norm, B, Lq, shift, hist, past, d_past, pad_len)
+    _chk(out, F32 if out.dtype == F32 else BF16, "out")
+    if out.numel() < B * Lq * x.shape[-1]:
+        raise ValueError(f"dyt: output {tuple(out.shape)} for {B} x {Lq} rows")
+    L.check(L.lib().p3v_dyt(C.byref(args), _p(out), int(out.dtype == F32), _stream()), "dyt")
+    return out
+
+
+def _dyt_args(x, norm, B, Lq, shift, hist, past, d_past, pad_len):
     alpha, w, b = norm
-    _chk(x, F32, "x"), _chk(w, BF16, "w"), _chk(b, BF16, "b"), _chk(out, F32 if out.dtype == F32 else BF16, "out")
+    _chk(x, F32, "x"), _chk(w, BF16, "w"), _chk(b, BF16, "b")
     H = x.shape[-1]
-    if x.numel() < B * Lq * H or out.numel() < B * Lq * H or w.numel() != H or b.numel() != H:
-        raise ValueError(f"dyt: shapes {tuple(x.shape)}, {tuple(w.shape)} -> {tuple(out.shape)} for {B} x {Lq} rows")
+    if x.numel() < B * Lq * H or w.numel() != H or b.numel() != H or (pad_len is not None and pad_len.numel() != B):
+        raise ValueError(f"dyt: shapes {tuple(x.shape)}, {tuple(w.shape)} for {B} x {Lq} rows")
     if shift is not None:
         _chk(shift, BF16, "shift"), _chk(hist, F32, "hist")
         if shift.numel() != H or hist.shape[0] != B or hist.shape[2] != H:
             raise ValueError(f"dyt: shift {tuple(shift.shape)}, history {tuple(hist.shape)}")
-    args = L.DytArgs(_p(x), _p(w), _p(b), _p(shift), _p(hist) if shift is not None else 0, _p(pad_len), _p(d_past), float(alpha),
+    return L.DytArgs(_p(x), _p(w), _p(b), _p(shift), _p(hist) if shift is not None else 0, _p(pad_len), _p(d_past), float(alpha),
                      int(past), hist.shape[1] if shift is not None else 0, B, Lq, H)
-    L.check(L.lib().p3v_dyt(C.byref(args), _p(out), int(out.dtype == F32), _stream()), "dyt")
-    return out
+
+
+def project_dyt(x, norm, w, h, epilogue=EPI_NONE, out=None, B=1, Lq=1, **shift):
+    """project(dyt(x)): one launch for a single bf16 row of a width the streaming kernel takes, else the two (h: their scratch rows)."""
+    M, H = B * Lq, x.shape[-1]
+    if M == 1 and h.dtype == BF16 and out is not None:
+        _chk(w, BF16, "w"), _chk(out, BF16, "out")
+        N = w.shape[0] // 2 if epilogue == EPI_SILU_MUL else w.shape[0]
+        if w.shape[1] != H or out.numel() != N:
+            raise ValueError(f"project_dyt: {tuple(w.shape)} on rows of {H} -> {tuple(out.shape)}")
+        d = _dyt_args(x, norm, 1, 1, **{**dict(shift=None, hist=None, past=0, d_past=None, pad_len=None), **shift})
+        args = L.GemvArgs(0, _p(w), _p(out), 0, 0, 0.0, 1, N, H, epilogue, 0)
+        rc = L.lib().p3v_gemv_dyt(C.byref(args), C.byref(d), _stream())
+        if rc != L.ERR_UNSUPPORTED:
+            L.check(rc, "gemv_dyt")
+            return out
+    dyt(x, norm, h, B, Lq, **shift)
+    return project(h[:M], w, epilogue, out=out)
 
 
 def project(x, w, epilogue=EPI_NONE, resid=None, col_scale=None, out=None):
@@ -644,11 +670,11 @@ def project(x, w, epilogue=EPI_NONE, resid=None, col_scale=None, out=None):
     scaled = epilogue == EPI_SCALE_RESID_F32
     if scaled:
         _chk(resid, F32, "resid"), _chk(col_scale, BF16, "col_scale"), _chk(out, F32, "out")
-    if not f32 and not scaled and K % 8 == 0 and out.is_contiguous():
-        if M <= 8 or (M <= GEMV_MAX_M and K % 512 == 0):
-            return gemv(x, w, epilogue, resid=resid, out=out)
+    if not f32 and K % 8 == 0 and x.is_contiguous() and out.is_contiguous():
+        if M <= 8 and (1 << (M - 1).bit_length()) * K * 2 <= 160 * 1024 - 256:     # (the rows of x in a workgroup's LDS)
+            return gemv(x, w, epilogue, resid=resid, out=out, col_scale=col_scale)
         if K % 64 == 0 and N % 8 == 0:
-            return gemm(x, w, epilogue, resid=resid, out=out)
+            return gemm(x, w, epilogue, resid=resid, out=out, col_scale=col_scale)
     args = L.GemmArgs(_p(x), _p(w), _p(out), 0, _p(resid), 0, M, N, K, x.stride(0), w.stride(0), out.stride(0), epilogue, 0, 0, 0, _p(col_scale))
     L.check(L.lib().p3v_gemm_any(C.byref(args), int(f32), _stream()), "gemm_any")
     return out
