@@ -462,7 +462,7 @@ int p3v_gemm_any(const p3v_gemm_args_t* args /* host */, int a_f32, void* stream
  *   v = value, or with v_first (row stride ld_first) (1 - vmix) value + vmix v_first
  *   s_h = scale sum_g talk[h, g] (q_g . k_g);  p = softmax of s over the keys pad_len[b] .. own position with exp(sink_h) added to the
  *   denominator;  out row = sigmoid(gate_h) sum p v.
- * Caches: k [B, G, Tp, dimp], v [B, G, Tp/16, vdimp, 16] (dimp % 32 == 0, vdimp % 16 == 0, the padding zero), Tp % 32 == 0.
+ * Caches: k [B, G, Tp, dimp], v [B, G, Tp/16, vdimp, 16] (dimp % 32 == 0, vdimp % 32 == 0, the padding zero), Tp % 32 == 0.
  * p3v_qkv_heads writes q [B, H, L, dimp] and appends k, v; p3v_attn_mix attends from q over the cache (new tokens included);
  * p3v_attn_mix_decode does both for L = 1 (P3V_ERR_UNSUPPORTED: run the two).  n_split from p3v_attn_mix_plan (0: the any-size kernel),
  * ws of p3v_attn_mix_ws_bytes.  n_keys of the plan: the cache capacity for L = 1, past + L otherwise. */

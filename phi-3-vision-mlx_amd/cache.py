@@ -133,7 +133,7 @@ def round_up(n, m):
 class LayeredCacheState(CacheState):
     """State of a layered decoder (config.LayerSpec): per layer its own key / value sizes, in the layout of the mixed-head attention
 
-        k[i]     [B, G, Tp, dimp]             dimp = dim rounded up to 32, vdimp = vdim rounded up to 16, the padding zero
+        k[i]     [B, G, Tp, dimp]             dimp = dim rounded up to 32, vdimp = vdim rounded up to 32, the padding zero
         v[i]     [B, G, Tp / 16, vdimp, 16]
         shift[i] [B, R, width] fp32           the mixer's unshifted inputs of the last R columns (column c in row c % R)
 
@@ -152,7 +152,7 @@ class LayeredCacheState(CacheState):
         for ly in cfg.layers:
             m = ly.mixer
             self.k.append(torch.zeros((B, m.kv_heads, self.Tp, round_up(m.dim, 32)), dtype=dt, device=device))
-            self.v.append(torch.zeros((B, m.kv_heads, self.Tp // 16, round_up(m.vdim, 16), 16), dtype=dt, device=device))
+            self.v.append(torch.zeros((B, m.kv_heads, self.Tp // 16, round_up(m.vdim, 32), 16), dtype=dt, device=device))
             self.shift.append(torch.zeros((B, self.R, cfg.hidden_size), dtype=F32, device=device))
         self._loop_state()
 

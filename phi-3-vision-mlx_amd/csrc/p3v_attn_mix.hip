@@ -5,7 +5,7 @@
 //   K cache [B, G, Tp, dimp]            rows of keys: a row is an MFMA fragment (dimp: dim rounded up to 32, zeros behind)
 //   V cache [B, G, Tp / 16, vdimp, 16]  blocks of 16 keys, value dimension by value dimension: the PV product reads 8 consecutive
 //                                       keys of one dimension per lane (16 bytes, whole 512-byte runs per wave) and a 16-key tile of
-//                                       the decode step is contiguous (vdimp: vdim rounded up to 16)
+//                                       the decode step is contiguous (vdimp: vdim rounded up to 32)
 //
 // Scores, their mixing and the softmax are fp32.  The mixing runs on the bf16 matrix cores WITHOUT losing fp32: talk is bf16 data, and
 // a score is split into three bf16 terms whose sum is the fp32 value, so that every product is exact and only the fp32 accumulation
@@ -18,6 +18,12 @@
 
 typedef __attribute__((ext_vector_type(2))) float f32x2_t;
 
+// workgroup barrier for LDS data only: global loads stay in flight across it (__syncthreads would wait for them)
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
 __device__ __forceinline__ float row16_max(float v) {
   v = fmaxf(v, P3V_DPP_F32(v, 0xB1));
   v = fmaxf(v, P3V_DPP_F32(v, 0x4E));
@@ -43,7 +49,10 @@ __device__ __forceinline__ float* ws_o(float* ws, const AttnMixP& p, size_t rows
 // and output accumulators stay in registers, K / V fragments come straight from the cache: no other wave of the workgroup needs
 // them) and queries 2w, 2w + 1 of ALL heads in the mixing and the softmax; the two views meet in LDS:
 //   S  [16 q][32 keys][heads] fp32 (+ padding: both the writes of HW heads and the reads of 8 heads per lane are conflict-free)
-//   P  [heads][16 q][32 keys] bf16,  AL [heads][16 q] rescale factors
+//   P  [heads][16 q][32 keys] bf16,  AL [heads][16 q] rescale factors,  MM [heads][16 q] running maxima
+// The softmax's sum rides in the second product as one more value dimension (a row of ones).  The value fragments of a tile are
+// requested ahead of its mixing and the next tile's key fragments ahead of the second product; the barriers wait for LDS only.
+// SHARED: the heads of a wave share one key / value head (else every head loads its own fragments, one head ahead).
 template <int HW> struct MixCfg {
   static constexpr int HP = 8 * HW, HS = HP + 4, QS = 32 * HS + 4;      // heads padded, S strides (floats): key, query
   static constexpr int PQ = 40, PH = 16 * PQ + 8;                        // P strides (bf16): query, head
@@ -52,32 +61,39 @@ template <int HW> struct MixCfg {
   static constexpr int LDS = S_BYTES + P_BYTES + 2 * A_BYTES;
 };
 
-template <int HW, int DC>
+template <int HW, int DC, int VC, bool SHARED>
 __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
   typedef MixCfg<HW> C;
+  constexpr int NB = SHARED ? 1 : 2;                                     // fragment buffers
+  constexpr int QU = HW == 4 && DC + VC >= 5 ? 1 : 2;                    // queries of the mixing side by side
+  constexpr bool Q_REG = HW < 4 || DC + VC < 8;                          // else the query fragments are read again for every key tile
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   float* S = (float*)smem;
   bf16_t* P = (bf16_t*)(smem + C::S_BYTES);
   float* AL = (float*)(smem + C::S_BYTES + C::P_BYTES);
-  float* LS = AL + C::HP * 16;
+  float* MM = AL + C::HP * 16;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lc = lane & 15, lg = lane >> 4;
   const int n_qt = (p.L + 15) >> 4, qt = n_qt - 1 - (int)blockIdx.x, split = blockIdx.y, b = blockIdx.z;   // longest rows first
   const int q0 = qt * 16, per = p.H / p.G, past = p.d_past ? *p.d_past : p.past, first = p.pad_len ? p.pad_len[b] : 0;
   const int last = past + min(q0 + 15, p.L - 1);                         // last key any query of the tile sees
-  const int t_lo = first >> 5, t_hi = (last >> 5) + 1;
-  const int chunk = max(1, (t_hi - t_lo + p.n_split - 1) / p.n_split);
-  const int t0 = t_lo + split * chunk, t1 = min(t_hi, t0 + chunk);
-  const int dc = p.dimp >> 5, nvt = p.vdimp >> 4;
+  // key tiles of this split: the same for every query tile, so that the workgroups an XCD runs together walk the same keys (its L2
+  // then serves all but the first); splits beyond a query tile's keys have nothing to do and nobody reads their partials
+  const int t0 = max(first >> 5, split * p.tiles_per_split), t1 = min((last >> 5) + 1, (split + 1) * p.tiles_per_split);
+  if (split * p.tiles_per_split > last >> 5) return;
+  constexpr int NV = 2 * VC;                                             // 16-dimension blocks of a value (dimp = 32 DC, vdimp = 32 VC)
   const float sc = p.scale * LOG2E;
 
   // Q fragments (B operand: column = query, 8 consecutive dimensions)
-  bf16x8_t qf[HW][DC];
-#pragma unroll
-  for (int i = 0; i < HW; ++i) {
+  bf16x8_t qf[Q_REG ? HW : 1][DC];
+  auto load_q = [&](int i) {
     const int h = min(wave * HW + i, p.H - 1);
     const bf16_t* qr = (const bf16_t*)p.q + (((size_t)b * p.H + h) * p.L + min(q0 + lc, p.L - 1)) * p.dimp + lg * 8;
 #pragma unroll
-    for (int c = 0; c < DC; ++c) qf[i][c] = *(const bf16x8_t*)(qr + (c < dc ? c : 0) * 32);
+    for (int c = 0; c < DC; ++c) qf[Q_REG ? i : 0][c] = *(const bf16x8_t*)(qr + c * 32);
+  };
+  if constexpr (Q_REG) {
+#pragma unroll
+    for (int i = 0; i < HW; ++i) load_q(i);
   }
   // talk fragments (A operand: row = mixed head, 8 consecutive raw heads), zero beyond H
   bf16x8_t tf[C::HM];
@@ -92,48 +108,55 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
     }
     tf[m] = __builtin_bit_cast(bf16x8_t, w);
   }
-  f32x4_t o[HW][2 * DC];
+  const u32x4_t ones_w = {0x3f803f80u, 0x3f803f80u, 0x3f803f80u, 0x3f803f80u};
+  const bf16x8_t ones = __builtin_bit_cast(bf16x8_t, ones_w);
+  f32x4_t o[HW][NV], ol[HW];                                         // outputs; the row of ones: softmax sums
 #pragma unroll
-  for (int i = 0; i < HW; ++i)
+  for (int i = 0; i < HW; ++i) {
+    ol[i] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int d = 0; d < 2 * DC; ++d) o[i][d] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-  float mr[2][C::HM][4], lr[2][C::HM][4];                                // running max / per-lane sum of (query 2w + qi, head 16 m + 4 lg + r)
-#pragma unroll
-  for (int qi = 0; qi < 2; ++qi)
-#pragma unroll
-    for (int m = 0; m < C::HM; ++m)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) mr[qi][m][r] = MIX_NEG, lr[qi][m][r] = 0.f;
+    for (int d = 0; d < NV; ++d) o[i][d] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+  }
+  for (int i = tid; i < C::HP * 16; i += 512) MM[i] = MIX_NEG;
+  lds_barrier();
 
-  const bf16_t* kb = (const bf16_t*)p.k + (size_t)b * p.G * p.Tp * p.dimp + (size_t)lc * p.dimp + lg * 8;
-  const bf16_t* vb = (const bf16_t*)p.v + (size_t)b * p.G * p.Tp * p.vdimp + ((size_t)(lg >> 1) * p.vdimp + lc) * 16 + (lg & 1) * 8;
+  const bf16_t* kb = (const bf16_t*)p.k + (size_t)b * p.G * p.Tp * p.dimp;
+  const bf16_t* vb = (const bf16_t*)p.v + (size_t)b * p.G * p.Tp * p.vdimp;
+  const uint32_t k_lane = (uint32_t)(lc * p.dimp + lg * 8), v_lane = (uint32_t)(((lg >> 1) * p.vdimp + lc) * 16 + (lg & 1) * 8);
   const bool active = wave * HW < p.H;
+  bf16x8_t kf[NB][2][DC], vf[NB][NV];
+  auto load_k = [&](int t, int i) {
+    const int g = min(wave * HW + i, p.H - 1) / per, bf = SHARED ? 0 : i & 1;
+    const bf16_t* kr = kb + ((size_t)g * p.Tp + t * 32) * p.dimp + k_lane;
+#pragma unroll
+    for (int c = 0; c < DC; ++c)
+      kf[bf][0][c] = *(const bf16x8_t*)(kr + c * 32), kf[bf][1][c] = *(const bf16x8_t*)(kr + (size_t)16 * p.dimp + c * 32);
+  };
+  auto load_v = [&](int t, int i) {
+    const int g = min(wave * HW + i, p.H - 1) / per, bf = SHARED ? 0 : i & 1;
+    const bf16_t* vr = vb + ((size_t)g * (p.Tp >> 4) + t * 2) * p.vdimp * 16 + v_lane;
+#pragma unroll
+    for (int d = 0; d < NV; ++d)
+      vf[bf][d] = *(const bf16x8_t*)(vr + d * 256);
+  };
+  if (active && t0 < t1) load_k(t0, 0);
 
   for (int t = t0; t < t1; ++t) {
     // ---- raw scores of this wave's heads -> S
     if (active) {
       f32x4_t s[HW][2];
 #pragma unroll
-      for (int i = 0; i < HW; ++i) s[i][0] = s[i][1] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-      bf16x8_t kf[2][DC];
-#pragma unroll
       for (int i = 0; i < HW; ++i) {
-        const int h = min(wave * HW + i, p.H - 1), g = h / per;
-        if (i == 0 || g != min(wave * HW + i - 1, p.H - 1) / per) {
-          const bf16_t* kr = kb + ((size_t)g * p.Tp + t * 32) * p.dimp;
-#pragma unroll
-          for (int c = 0; c < DC; ++c)
-            if (c < dc) {
-              kf[0][c] = *(const bf16x8_t*)(kr + c * 32);
-              kf[1][c] = *(const bf16x8_t*)(kr + (size_t)16 * p.dimp + c * 32);
-            }
-        }
+        s[i][0] = s[i][1] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+        if (!SHARED && i + 1 < HW) load_k(t, i + 1);
+        if constexpr (!Q_REG) load_q(i);
 #pragma unroll
         for (int c = 0; c < DC; ++c)
-          if (c < dc) {
-            s[i][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[0][c], qf[i][c], s[i][0], 0, 0, 0);
-            s[i][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[1][c], qf[i][c], s[i][1], 0, 0, 0);
+          {
+            s[i][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[SHARED ? 0 : i & 1][0][c], qf[Q_REG ? i : 0][c], s[i][0], 0, 0, 0);
+            s[i][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[SHARED ? 0 : i & 1][1][c], qf[Q_REG ? i : 0][c], s[i][1], 0, 0, 0);
           }
+        if (HW > 1) __builtin_amdgcn_sched_barrier(0);
       }
 #pragma unroll
       for (int kt = 0; kt < 2; ++kt)
@@ -144,11 +167,12 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
           else if constexpr (HW == 2) *(f32x2_t*)dst = (f32x2_t){s[0][kt][r], s[1][kt][r]};
           else *dst = s[0][kt][r];
         }
+      load_v(t, 0);
     }
-    __syncthreads();
+    lds_barrier();
 
     // ---- mixing + softmax of queries 2w, 2w + 1, all heads
-#pragma unroll
+#pragma unroll QU
     for (int qi = 0; qi < 2; ++qi) {
       const int q = 2 * wave + qi, qpos = past + q0 + q;
       f32x4_t mx[C::HM][2];
@@ -190,67 +214,42 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
       for (int m = 0; m < C::HM; ++m)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float s0 = live0 ? mx[m][0][r] * sc : -INFINITY, s1 = live1 ? mx[m][1][r] * sc : -INFINITY;
-          const float mn = fmaxf(mr[qi][m][r], row16_max(fmaxf(s0, s1)));
-          const float al = __builtin_amdgcn_exp2f(mr[qi][m][r] - mn), p0 = __builtin_amdgcn_exp2f(s0 - mn), p1 = __builtin_amdgcn_exp2f(s1 - mn);
-          mr[qi][m][r] = mn;
-          lr[qi][m][r] = lr[qi][m][r] * al + (p0 + p1);
           const int h = m * 16 + lg * 4 + r;
-          if (h < C::HP) {
+          if (C::HP >= 16 || lg < 2) {
+            const float s0 = live0 ? mx[m][0][r] * sc : -INFINITY, s1 = live1 ? mx[m][1][r] * sc : -INFINITY;
+            const float mo = MM[h * 16 + q], mn = fmaxf(mo, row16_max(fmaxf(s0, s1)));
+            const float p0 = __builtin_amdgcn_exp2f(s0 - mn), p1 = __builtin_amdgcn_exp2f(s1 - mn);
             bf16_t* dst = P + h * C::PH + q * C::PQ + lc;
             dst[0] = f32_to_bf16(p0), dst[16] = f32_to_bf16(p1);
-            if (lc == 0) AL[h * 16 + q] = al;
+            if (lc == 0) AL[h * 16 + q] = __builtin_amdgcn_exp2f(mo - mn), MM[h * 16 + q] = mn;
           }
         }
     }
-    __syncthreads();
+    lds_barrier();
 
     // ---- O^T += V^T P^T of this wave's heads
     if (active) {
-      bf16x8_t vf[2 * DC];
+      load_k(min(t + 1, t1 - 1), 0);
 #pragma unroll
       for (int i = 0; i < HW; ++i) {
-        const int h = min(wave * HW + i, p.H - 1), g = h / per;
-        if (i == 0 || g != min(wave * HW + i - 1, p.H - 1) / per) {
-          const bf16_t* vr = vb + ((size_t)g * (p.Tp >> 4) + t * 2) * p.vdimp * 16;
-#pragma unroll
-          for (int d = 0; d < 2 * DC; ++d)
-            if (d < nvt) vf[d] = *(const bf16x8_t*)(vr + d * 256);
-        }
+        const int h = min(wave * HW + i, p.H - 1);
+        if (!SHARED && i + 1 < HW) load_v(t, i + 1);
         const bf16x8_t pf = *(const bf16x8_t*)(P + h * C::PH + lc * C::PQ + lg * 8);
         const float al = AL[h * 16 + lc];
+        if (__builtin_amdgcn_ballot_w64(al != 1.f)) {                    // (a maximum moved; rare behind a sequence's first tiles)
+          ol[i] *= al;
 #pragma unroll
-        for (int d = 0; d < 2 * DC; ++d)
-          if (d < nvt) {
-            o[i][d] *= al;
-            o[i][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[d], pf, o[i][d], 0, 0, 0);
-          }
+          for (int d = 0; d < NV; ++d) o[i][d] *= al;
+        }
+        ol[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf, ol[i], 0, 0, 0);
+#pragma unroll
+        for (int d = 0; d < NV; ++d)
+          o[i][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[SHARED ? 0 : i & 1][d], pf, o[i][d], 0, 0, 0);
+        if (HW > 1) __builtin_amdgcn_sched_barrier(0);                   // (one head's operands at a time: the registers are full)
       }
     }
   }
 
-  // ---- the softmax side hands its sums (and maxima) to the head side
-#pragma unroll
-  for (int qi = 0; qi < 2; ++qi)
-#pragma unroll
-    for (int m = 0; m < C::HM; ++m)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int h = m * 16 + lg * 4 + r;
-        const float l = row16_sum(lr[qi][m][r]);
-        if (lc == 0 && h < C::HP) LS[h * 16 + 2 * wave + qi] = l;
-      }
-  __syncthreads();                                                       // (AL of the last tile has been read by every wave)
-#pragma unroll
-  for (int qi = 0; qi < 2; ++qi)
-#pragma unroll
-    for (int m = 0; m < C::HM; ++m)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int h = m * 16 + lg * 4 + r;
-        if (lc == 0 && h < C::HP) AL[h * 16 + 2 * wave + qi] = mr[qi][m][r];
-      }
-  __syncthreads();
   const int row_q = q0 + lc;
   if (!active || row_q >= p.L) return;
   const size_t row = (size_t)b * p.L + row_q, rows = (size_t)p.B * p.L;
@@ -258,17 +257,17 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
   for (int i = 0; i < HW; ++i) {
     const int h = wave * HW + i;
     if (h >= p.H) continue;
-    const float m = AL[h * 16 + lc], l = LS[h * 16 + lc];
+    const float m = MM[h * 16 + lc], l = ol[i][0];
     float f = 1.f;
     if (p.n_split == 1) {
-      const float sk = bf16_to_f32(p.sink[h]) * LOG2E, mm = fmaxf(m, sk);
-      f = __builtin_amdgcn_exp2f(m - mm) / (l * __builtin_amdgcn_exp2f(m - mm) + __builtin_amdgcn_exp2f(sk - mm)) * gate_of((const bf16_t*)p.gate + row * p.ld + h);
+      const float sk = bf16_to_f32(p.sink[h]) * LOG2E, mm = fmaxf(m, sk), e = __builtin_amdgcn_exp2f(m - mm);
+      f = e / (l * e + __builtin_amdgcn_exp2f(sk - mm)) * gate_of((const bf16_t*)p.gate + row * p.ld + h);
     } else if (lg == 0) {
       *(f32x2_t*)(ws_ml(p.ws, p, row, split) + h * 2) = (f32x2_t){m, l};
     }
 #pragma unroll
-    for (int d = 0; d < 2 * DC; ++d)
-      if (d < nvt) {
+    for (int d = 0; d < NV; ++d)
+      {
         const int dd = d * 16 + lg * 4;
         if (p.n_split == 1) {
           bf16_t* dst = (bf16_t*)p.out + row * p.H * p.vdim + (size_t)h * p.vdim + dd;
@@ -281,9 +280,13 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
           }
         } else {
           float* dst = ws_o(p.ws, p, rows, row, split) + (size_t)h * p.vdim + dd;
+          if (p.vdim % 4 == 0) {
+            if (dd < p.vdim) *(float4*)dst = make_float4(o[i][d][0], o[i][d][1], o[i][d][2], o[i][d][3]);
+          } else {
 #pragma unroll
-          for (int r = 0; r < 4; ++r)
-            if (dd + r < p.vdim) dst[r] = o[i][d][r];
+            for (int r = 0; r < 4; ++r)
+              if (dd + r < p.vdim) dst[r] = o[i][d][r];
+          }
         }
       }
   }
@@ -293,10 +296,10 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
 // A workgroup takes a run of 16-key tiles of one sequence, all heads: the query's whole-projection norm is recomputed in every
 // workgroup (a few KB), the workgroup whose run holds the new position also normalises and appends the new key and mixes and appends
 // the new value.  Partials of the runs are merged by k_attn_mix_combine.
-template <int DC, int NP>
+template <int GW, int DC, int NP>
 __global__ void __launch_bounds__(512) k_attn_mix_decode(QkvHeadsP hp, AttnMixP p) {
   constexpr int SS = 20;                                                 // S / P row stride (floats)
-  __shared__ float S[MIX_MAX_H * SS], P[MIX_MAX_H * SS], talk[MIX_MAX_H * (MIX_MAX_H + 1)], AL[MIX_MAX_H], red[16];
+  __shared__ float S[MIX_MAX_H * SS], P[MIX_MAX_H * SS], talk[MIX_MAX_H * (MIX_MAX_H + 1)], AL[MIX_MAX_H], red[2][8];
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   bf16_t* qs = (bf16_t*)smem;                                            // [H][dimp] normalised query
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lc = lane & 15, lg = lane >> 4;
@@ -305,7 +308,7 @@ __global__ void __launch_bounds__(512) k_attn_mix_decode(QkvHeadsP hp, AttnMixP 
   const int t_first = split * p.tiles_per_split, own = past >> 4;
   if (t_first > own) return;                                             // beyond the live keys: the merge does not look here
   const int t_begin = max(t_first, first >> 4), t_end = min(t_first + p.tiles_per_split, own + 1);
-  const bool owner = own < t_end;
+  const bool owner = own < t_first + p.tiles_per_split;
   const int nq = p.H * p.dim, nk = p.G * p.dim, nv = p.G * p.vdim;
   const bf16_t* row = (const bf16_t*)hp.qkv + (size_t)b * hp.ld;
   float* ml = ws_ml(p.ws, p, b, split);
@@ -314,76 +317,97 @@ __global__ void __launch_bounds__(512) k_attn_mix_decode(QkvHeadsP hp, AttnMixP 
     if (!owner) return;                                                  // an idle batch row still appends: its cache stays finite
   }
 
+  // ---- keys and values of the first tile are requested before anything else (by the workgroup of the new position behind its append)
+  // (GW kv heads per wave; a wave beyond the last one repeats it: same loads, same scores)
+  const float sc = p.scale * LOG2E;
+  const bf16_t* kb = (const bf16_t*)p.k + ((size_t)b * p.G * p.Tp + lc) * p.dimp + lg * 8;
+  bf16x8_t kf[GW][DC];
+  auto load_k = [&](int t) {
+#pragma unroll
+    for (int i = 0; i < GW; ++i) {
+      const bf16_t* kr = kb + ((size_t)min(wave * GW + i, p.G - 1) * p.Tp + t * 16) * p.dimp;
+#pragma unroll
+      for (int c = 0; c < DC; ++c) kf[i][c] = *(const bf16x8_t*)(kr + c * 32);
+    }
+  };
+  u32x4_t vv[NP][2];
+  int vh[NP];
+  uint32_t vo[NP];
+#pragma unroll
+  for (int j = 0; j < NP; ++j) {
+    const int i = min(tid + 512 * j, p.H * p.vdim - 1), h = i / p.vdim, d = i - h * p.vdim, g = h / per;
+    vh[j] = h;
+    vo[j] = (uint32_t)(g * (p.Tp >> 4) * p.vdimp + d) * 2;               // 16-byte units inside the sequence's cache
+  }
+  const u32x4_t* vb = (const u32x4_t*)p.v + (size_t)b * p.G * (p.Tp >> 4) * p.vdimp * 2;
+  auto load_v = [&](int t) {
+#pragma unroll
+    for (int j = 0; j < NP; ++j) {
+      const u32x4_t* vr = vb + vo[j] + (uint32_t)t * (uint32_t)(p.vdimp * 2);
+      vv[j][0] = vr[0], vv[j][1] = vr[1];
+    }
+  };
+  const bool live = t_begin < t_end;
   // ---- query (and key) norm
   float sq = 0.f, sk = 0.f;
+#pragma unroll 1
   for (int e = tid; e < nq; e += 512) { const float v = bf16_to_f32(row[e]); sq += v * v; }
   if (owner)
+#pragma unroll 1
     for (int e = tid; e < nk; e += 512) { const float v = bf16_to_f32(row[nq + e]); sk += v * v; }
+  if (!owner) load_k(t_begin), load_v(t_begin);
+#pragma unroll 1
   for (int e = tid; e < p.H * p.H; e += 512) { const int h = e / p.H; talk[h * (MIX_MAX_H + 1) + e - h * p.H] = bf16_to_f32(p.talk[e]); }
-  const float rq = 1.f / sqrtf(block_sum(sq, red) / (float)nq + hp.eps), rk = 1.f / sqrtf(block_sum(sk, red) / (float)nk + hp.eps);
+  sq = wave_sum(sq), sk = wave_sum(sk);
+  if (lane == 0) red[0][wave] = sq, red[1][wave] = sk;
+  lds_barrier();                     // (not __syncthreads: the tile's loads stay in flight)
+  sq = sk = 0.f;
+#pragma unroll
+  for (int w = 0; w < 8; ++w) sq += red[0][w], sk += red[1][w];
+  const float rq = 1.f / sqrtf(sq / (float)nq + hp.eps), rk = 1.f / sqrtf(sk / (float)nk + hp.eps);
+#pragma unroll 1
   for (int e = tid; e < p.H * p.dimp; e += 512) {
     const int h = e / p.dimp, d = e - h * p.dimp;
     qs[e] = d < p.dim ? f32_to_bf16(bf16_to_f32(row[h * p.dim + d]) * rq * bf16_to_f32(hp.q_norm[h * p.dim + d])) : (bf16_t)0;
   }
   if (owner) {
+#pragma unroll 1
     for (int e = tid; e < nk; e += 512) {
       const int g = e / p.dim, d = e - g * p.dim;
       ((bf16_t*)hp.k)[(((size_t)b * p.G + g) * p.Tp + past) * p.dimp + d] = f32_to_bf16(bf16_to_f32(row[nq + e]) * rk * bf16_to_f32(hp.k_norm[e]));
     }
+#pragma unroll 1
     for (int e = tid; e < nv; e += 512) {
       const int g = e / p.vdim, d = e - g * p.vdim;
       float v = bf16_to_f32(row[nq + nk + e]);
       if (hp.v_first) v = (1.f - hp.vmix) * v + hp.vmix * bf16_to_f32(((const bf16_t*)hp.v_first)[(size_t)b * hp.ld_first + e]);
       ((bf16_t*)hp.v)[((((size_t)b * p.G + g) * (p.Tp >> 4) + own) * p.vdimp + d) * 16 + (past & 15)] = f32_to_bf16(v);
     }
+    __syncthreads();                                                     // (the stores have to be visible to the whole workgroup)
   }
-  __syncthreads();                                                       // the query is in LDS, the new key / value in the cache
-  if (t_begin >= t_end) return;
+  lds_barrier();                     // the query (and the new key / value) is in LDS
+  if (!live) return;
+  if (owner) load_k(t_begin), load_v(t_begin);
 
-  const int dc = p.dimp >> 5, gw = (p.G + 7) >> 3;                       // kv heads per wave
-  const float sc = p.scale * LOG2E;
-  const bf16_t* kb = (const bf16_t*)p.k + ((size_t)b * p.G * p.Tp + lc) * p.dimp + lg * 8;
   float acc[NP];
 #pragma unroll
   for (int j = 0; j < NP; ++j) acc[j] = 0.f;
   float m_run = MIX_NEG, l_run = 0.f;                                    // of head tid >> 4 (replicated over its 16 keys' threads)
-  bf16x8_t kf[4][DC];
-  auto load_k = [&](int t) {
-#pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (i < gw && wave * gw + i < p.G) {
-        const bf16_t* kr = kb + ((size_t)(wave * gw + i) * p.Tp + t * 16) * p.dimp;
-#pragma unroll
-        for (int c = 0; c < DC; ++c)
-          if (c < dc) kf[i][c] = *(const bf16x8_t*)(kr + c * 32);
-      }
-  };
-  load_k(t_begin);
   for (int t = t_begin; t < t_end; ++t) {
-    // ---- value rows of this tile: requested now, used after the softmax
-    u32x4_t vv[NP][2];
-#pragma unroll
-    for (int j = 0; j < NP; ++j) {
-      const int i = min(tid + 512 * j, p.H * p.vdim - 1), h = i / p.vdim, d = i - h * p.vdim;
-      const u32x4_t* vr = (const u32x4_t*)((const bf16_t*)p.v + ((((size_t)b * p.G + h / per) * (p.Tp >> 4) + t) * p.vdimp + d) * 16);
-      vv[j][0] = vr[0], vv[j][1] = vr[1];
-    }
     // ---- raw scores: rows = keys, columns = the query heads of a kv head
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (i < gw && wave * gw + i < p.G) {
-        const int g = wave * gw + i;
-        f32x4_t s = {0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < GW; ++i) {
+      const int g = min(wave * GW + i, p.G - 1);
+      f32x4_t s = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int c = 0; c < DC; ++c)
-          if (c < dc) {
-            const bf16x8_t qf = *(const bf16x8_t*)(qs + (size_t)(g * per + min(lc, per - 1)) * p.dimp + c * 32 + lg * 8);
-            s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i][c], qf, s, 0, 0, 0);
-          }
-        if (lc < per) *(float4*)(S + (g * per + lc) * SS + lg * 4) = make_float4(s[0], s[1], s[2], s[3]);
+      for (int c = 0; c < DC; ++c) {
+        const bf16x8_t qf = *(const bf16x8_t*)(qs + (size_t)(g * per + min(lc, per - 1)) * p.dimp + c * 32 + lg * 8);
+        s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[i][c], qf, s, 0, 0, 0);
       }
+      if (lc < per) *(float4*)(S + (g * per + lc) * SS + lg * 4) = make_float4(s[0], s[1], s[2], s[3]);
+    }
     if (t + 1 < t_end) load_k(t + 1);
-    __syncthreads();
+    lds_barrier();
     // ---- mixing + softmax: thread = (head, key)
     {
       const int h = tid >> 4, key = t * 16 + lc;
@@ -398,21 +422,21 @@ __global__ void __launch_bounds__(512) k_attn_mix_decode(QkvHeadsP hp, AttnMixP 
         if (lc == 0) AL[h] = al;
       }
     }
-    __syncthreads();
+    lds_barrier();
 #pragma unroll
     for (int j = 0; j < NP; ++j) {
-      const int i = min(tid + 512 * j, p.H * p.vdim - 1), h = i / p.vdim;
-      const float* pr = P + h * SS;
-      float a = acc[j] * AL[h];
+      const float4* pr = (const float4*)(P + vh[j] * SS);
+      float a = acc[j] * AL[vh[j]];
 #pragma unroll
-      for (int u = 0; u < 2; ++u)
-#pragma unroll
-        for (int w = 0; w < 4; ++w) {
-          a = fmaf(pr[u * 8 + 2 * w], bf16lo(vv[j][u][w]), a);
-          a = fmaf(pr[u * 8 + 2 * w + 1], bf16hi(vv[j][u][w]), a);
-        }
+      for (int u = 0; u < 4; ++u) {
+        const float4 q = pr[u];
+        const uint32_t w0 = vv[j][u >> 1][(u & 1) * 2], w1 = vv[j][u >> 1][(u & 1) * 2 + 1];
+        a = fmaf(q.x, bf16lo(w0), a), a = fmaf(q.y, bf16hi(w0), a), a = fmaf(q.z, bf16lo(w1), a), a = fmaf(q.w, bf16hi(w1), a);
+      }
+      asm volatile("" : "+v"(a));                                        // (here, not sunk behind the branch below with every operand kept)
       acc[j] = a;
     }
+    if (t + 1 < t_end) load_v(t + 1);
   }
   if (lc == 0 && (tid >> 4) < p.H) *(f32x2_t*)(ml + 2 * (tid >> 4)) = (f32x2_t){m_run, l_run};
   float* od = ws_o(p.ws, p, p.B, b, split);
@@ -422,39 +446,93 @@ __global__ void __launch_bounds__(512) k_attn_mix_decode(QkvHeadsP hp, AttnMixP 
 }
 
 // ---------------------------------------------------------------- merge of the splits + sink + output gate
-__global__ void __launch_bounds__(256) k_attn_mix_combine(AttnMixP p) {
-  __shared__ float red[16], part[256];
+// splits of `row` that were written: those that begin at or before its last live key tile
+__device__ __forceinline__ int live_splits(const AttnMixP& p, size_t row, int shift) {
+  const int past = p.d_past ? *p.d_past : p.past, l = (int)(row % p.L), last = past + min((l & ~15) + 15, p.L - 1);
+  return min(p.n_split, (last >> shift) / p.tiles_per_split + 1);
+}
+// one token per sequence: many splits, few rows -- a workgroup per (head, row), groups of threads share the splits
+#define MIX_MAX_SPLIT 1024
+__global__ void __launch_bounds__(512) k_attn_mix_combine(AttnMixP p) {
+  __shared__ float red[16], part[512], wt[MIX_MAX_SPLIT];
   const int h = blockIdx.x, tid = threadIdx.x;
   const size_t row = blockIdx.y, rows = (size_t)p.B * p.L;
-  int n = p.n_split;
-  if (p.tiles_per_split) {                                               // decode: only the runs that reach into the live keys were written
-    const int past = p.d_past ? *p.d_past : p.past;
-    n = min(n, (past >> 4) / p.tiles_per_split + 1);
-  }
+  const int n = live_splits(p, row, 4);
   const float sk = bf16_to_f32(p.sink[h]) * LOG2E;
-  float m = sk;
-  for (int s = tid; s < n; s += 256) m = fmaxf(m, ws_ml(p.ws, p, row, s)[2 * h]);
+  float m = sk, lm[MIX_MAX_SPLIT / 512], ll[MIX_MAX_SPLIT / 512];
+#pragma unroll
+  for (int i = 0; i < MIX_MAX_SPLIT / 512; ++i) {
+    const int s = tid + 512 * i;
+    lm[i] = MIX_NEG, ll[i] = 0.f;
+    if (s < n) { const f32x2_t q = *(const f32x2_t*)(ws_ml(p.ws, p, row, s) + 2 * h); lm[i] = q[0], ll[i] = q[1]; }
+    m = fmaxf(m, lm[i]);
+  }
   m = block_max(m, red);
   float l = 0.f;
-  for (int s = tid; s < n; s += 256) { const float* q = ws_ml(p.ws, p, row, s) + 2 * h; l += q[1] * __builtin_amdgcn_exp2f(q[0] - m); }
+#pragma unroll
+  for (int i = 0; i < MIX_MAX_SPLIT / 512; ++i) {
+    const float w = __builtin_amdgcn_exp2f(lm[i] - m);
+    wt[tid + 512 * i] = lm[i] > 0.5f * MIX_NEG ? w : -1.f;               // (-1: a split of padding, whose outputs were not written)
+    l += ll[i] * w;
+  }
   l = block_sum(l, red) + __builtin_amdgcn_exp2f(sk - m);
   const float f = gate_of((const bf16_t*)p.gate + row * p.ld + h) / l;
-  const int vw = p.vdim <= 32 ? 32 : p.vdim <= 64 ? 64 : p.vdim <= 128 ? 128 : 256, ng = 256 / vw, grp = tid / vw;
-  for (int d0 = 0; d0 < p.vdim; d0 += vw) {
-    const int d = d0 + tid - grp * vw;
-    float a = 0.f;
-    if (d < p.vdim)
-#pragma unroll 4
-      for (int s = grp; s < n; s += ng) {
-        const float ms = ws_ml(p.ws, p, row, s)[2 * h];
-        if (ms > 0.5f * MIX_NEG) a = fmaf(__builtin_amdgcn_exp2f(ms - m), ws_o(p.ws, p, rows, row, s)[(size_t)h * p.vdim + d], a);
+  const int vw = p.vdim <= 32 ? 32 : p.vdim <= 64 ? 64 : 128, ng = 512 / vw, grp = tid / vw, d = tid - grp * vw;
+  float a = 0.f;
+  if (d < p.vdim) {
+    const float* o = ws_o(p.ws, p, rows, row, 0) + (size_t)h * p.vdim + d;
+    const size_t step = (size_t)p.H * p.vdim;
+#pragma unroll 8
+    for (int s = grp; s < n; s += ng) {
+      const float w = wt[s], v = o[s * step];
+      a = w >= 0.f ? fmaf(w, v, a) : a;
+    }
+  }
+  part[tid] = a;
+  __syncthreads();
+  if (grp == 0 && d < p.vdim) {
+    for (int g = 1; g < ng; ++g) a += part[g * vw + tid];
+    ((bf16_t*)p.out)[row * p.H * p.vdim + (size_t)h * p.vdim + d] = f32_to_bf16(a * f);
+  }
+}
+// prompts: few splits, many rows -- a workgroup per row
+#define MIX_MAX_ROW_SPLIT 16
+__global__ void __launch_bounds__(256) k_attn_mix_combine_rows(AttnMixP p) {
+  __shared__ float wt[MIX_MAX_H][MIX_MAX_ROW_SPLIT];
+  const size_t row = blockIdx.x, rows = (size_t)p.B * p.L;
+  const int tid = threadIdx.x, n = live_splits(p, row, 5);
+  if (tid < p.H) {
+    const float sk = bf16_to_f32(p.sink[tid]) * LOG2E;
+    float m = sk;
+    for (int s = 0; s < n; ++s) m = fmaxf(m, ws_ml(p.ws, p, row, s)[2 * tid]);
+    float l = __builtin_amdgcn_exp2f(sk - m);
+    for (int s = 0; s < n; ++s) {
+      const float* q = ws_ml(p.ws, p, row, s) + 2 * tid;
+      l += q[1] * __builtin_amdgcn_exp2f(q[0] - m);
+    }
+    const float f = gate_of((const bf16_t*)p.gate + row * p.ld + tid) / l;
+    for (int s = 0; s < n; ++s) wt[tid][s] = f * __builtin_amdgcn_exp2f(ws_ml(p.ws, p, row, s)[2 * tid] - m);
+  }
+  __syncthreads();
+  const size_t step = (size_t)p.H * p.vdim;
+  const float* o = ws_o(p.ws, p, rows, row, 0);
+  bf16_t* out = (bf16_t*)p.out + row * step;
+  if (p.vdim % 4 == 0) {
+    for (int e = tid * 4; e < p.H * p.vdim; e += 1024) {
+      const int h = e / p.vdim;
+      float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
+      for (int s = 0; s < n; ++s) {
+        const float4 v = *(const float4*)(o + s * step + e);
+        const float w = wt[h][s];
+        a.x = fmaf(w, v.x, a.x), a.y = fmaf(w, v.y, a.y), a.z = fmaf(w, v.z, a.z), a.w = fmaf(w, v.w, a.w);
       }
-    __syncthreads();
-    part[tid] = a;
-    __syncthreads();
-    if (grp == 0 && d < p.vdim) {
-      for (int g = 1; g < ng; ++g) a += part[g * vw + tid];
-      ((bf16_t*)p.out)[row * p.H * p.vdim + (size_t)h * p.vdim + d] = f32_to_bf16(a * f);
+      *(u32x2_t*)(out + e) = (u32x2_t){pack_bf16x2(a.x, a.y), pack_bf16x2(a.z, a.w)};
+    }
+  } else {
+    for (int e = tid; e < p.H * p.vdim; e += 256) {
+      float a = 0.f;
+      for (int s = 0; s < n; ++s) a = fmaf(wt[e / p.vdim][s], o[s * step + e], a);
+      out[e] = f32_to_bf16(a);
     }
   }
 }
@@ -467,9 +545,12 @@ static bool mix_fast(int H, int G, int dim, int vdim, int f32) {
 extern "C" int p3v_attn_mix_plan(int B, int L, int H, int G, int dim, int vdim, int n_keys, int f32) {
   if (B <= 0 || L <= 0 || H <= 0 || G <= 0 || n_keys <= 0 || !mix_fast(H, G, dim, vdim, f32)) return 0;
   const int want = p3v_tuning().mix_wgs;
-  if (L == 1) return max(1, min(p3v_cdiv(n_keys, 16), (want > 0 ? want : 512) / B));
+  if (L == 1) {                                                          // about one workgroup per CU, runs of equal length
+    const int tiles = p3v_cdiv(n_keys, 16), per = p3v_cdiv(tiles, max(1, (want > 0 ? want : 256) / B));
+    return min(p3v_cdiv(tiles, per), MIX_MAX_SPLIT);
+  }
   const int qt = p3v_cdiv(L, 16) * B, tiles = p3v_cdiv(n_keys, 32);
-  return max(1, min(min(16, p3v_cdiv(want > 0 ? want : 320, qt)), tiles / 4));
+  return max(1, min(min(MIX_MAX_ROW_SPLIT, p3v_cdiv(want > 0 ? want : 320, qt)), tiles / 4));
 }
 
 extern "C" int64_t p3v_attn_mix_ws_bytes(int B, int L, int H, int vdim, int n_split) {
@@ -478,30 +559,39 @@ extern "C" int64_t p3v_attn_mix_ws_bytes(int B, int L, int H, int vdim, int n_sp
 }
 
 static int mix_combine(const AttnMixP& p, hipStream_t s) {
-  hipLaunchKernelGGL(k_attn_mix_combine, dim3(p.H, p.B * p.L), dim3(256), 0, s, p);
+  if (p.L == 1) hipLaunchKernelGGL(k_attn_mix_combine, dim3(p.H, p.B), dim3(512), 0, s, p);
+  else hipLaunchKernelGGL(k_attn_mix_combine_rows, dim3(p.B * p.L), dim3(256), 0, s, p);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
 }
 
-template <int HW, int DC>
+template <int HW, int DC, int VC, bool SHARED>
 static int launch_prefill(const AttnMixP& p, hipStream_t s) {
   static bool attr_set = false;
   if (!attr_set) {
-    if (hipFuncSetAttribute((const void*)k_attn_mix_prefill<HW, DC>, hipFuncAttributeMaxDynamicSharedMemorySize, MixCfg<HW>::LDS) != hipSuccess) return P3V_ERR_HIP;
+    if (hipFuncSetAttribute((const void*)k_attn_mix_prefill<HW, DC, VC, SHARED>, hipFuncAttributeMaxDynamicSharedMemorySize, MixCfg<HW>::LDS) != hipSuccess) return P3V_ERR_HIP;
     attr_set = true;
   }
-  hipLaunchKernelGGL((k_attn_mix_prefill<HW, DC>), dim3(p3v_cdiv(p.L, 16), p.n_split, p.B), dim3(512), MixCfg<HW>::LDS, s, p);
+  hipLaunchKernelGGL((k_attn_mix_prefill<HW, DC, VC, SHARED>), dim3(p3v_cdiv(p.L, 16), p.n_split, p.B), dim3(512), MixCfg<HW>::LDS, s, p);
   P3V_CHECK_LAUNCH();
   return p.n_split > 1 ? mix_combine(p, s) : P3V_OK;
 }
-template <int HW>
+template <int HW, bool SHARED, int DC>
+static int prefill_vc(const AttnMixP& p, hipStream_t s) {
+  switch (p.vdimp / 32) {
+    case 1: return launch_prefill<HW, DC, 1, SHARED>(p, s);
+    case 2: return launch_prefill<HW, DC, 2, SHARED>(p, s);
+    case 3: return launch_prefill<HW, DC, 3, SHARED>(p, s);
+    default: return launch_prefill<HW, DC, 4, SHARED>(p, s);
+  }
+}
+template <int HW, bool SHARED>
 static int prefill_dc(const AttnMixP& p, hipStream_t s) {
-  const int dc = max(p.dimp / 32, p3v_cdiv(p.vdimp, 32));
-  switch (dc) {
-    case 1: return launch_prefill<HW, 1>(p, s);
-    case 2: return launch_prefill<HW, 2>(p, s);
-    case 3: return launch_prefill<HW, 3>(p, s);
-    default: return launch_prefill<HW, 4>(p, s);
+  switch (p.dimp / 32) {
+    case 1: return prefill_vc<HW, SHARED, 1>(p, s);
+    case 2: return prefill_vc<HW, SHARED, 2>(p, s);
+    case 3: return prefill_vc<HW, SHARED, 3>(p, s);
+    default: return prefill_vc<HW, SHARED, 4>(p, s);
   }
 }
 
@@ -510,40 +600,51 @@ extern "C" int p3v_attn_mix(const p3v_mix_args_t* a, void* stream) {
   if (rc != P3V_OK) return rc;
   if (!a->q || !a->talk || !a->sink || !a->gate || !a->out || a->n_split < 0) return P3V_ERR_ARG;
   hipStream_t s = (hipStream_t)stream;
-  if (a->n_split == 0 || !mix_fast(a->H, a->G, a->dim, a->vdim, a->f32)) return p3v_attn_mix_any(a, s);
-  if (a->n_split > 1 && !a->ws) return P3V_ERR_ARG;
-  const AttnMixP p = attn_mix_params(a);
-  return p.H <= 8 ? prefill_dc<1>(p, s) : p.H <= 16 ? prefill_dc<2>(p, s) : prefill_dc<4>(p, s);
+  if (a->n_split == 0 || a->vdimp > 128 || a->dimp > 128 || !mix_fast(a->H, a->G, a->dim, a->vdim, a->f32)) return p3v_attn_mix_any(a, s);
+  if (a->n_split > 1 && (!a->ws || a->n_split > MIX_MAX_ROW_SPLIT)) return P3V_ERR_ARG;
+  AttnMixP p = attn_mix_params(a);
+  // (the position may be a device value: the splits then cover the capacity)
+  p.tiles_per_split = p3v_cdiv(p3v_cdiv(a->d_past ? a->Tp : a->past + a->L, 32), a->n_split);
+  if (p.n_split > 1 && p.L == 1) return P3V_ERR_ARG;                     // (k_attn_mix_combine's splits are 16-key tiles)
+  const int per = p.H / p.G;                                             // query heads of a key / value head
+  if (p.H <= 8) return prefill_dc<1, true>(p, s);
+  if (p.H <= 16) return per % 2 ? prefill_dc<2, false>(p, s) : prefill_dc<2, true>(p, s);
+  return per % 4 ? prefill_dc<4, false>(p, s) : prefill_dc<4, true>(p, s);
 }
 
-template <int DC, int NP>
+template <int GW, int DC, int NP>
 static int launch_decode(const QkvHeadsP& hp, const AttnMixP& p, hipStream_t s) {
-  hipLaunchKernelGGL((k_attn_mix_decode<DC, NP>), dim3(p.n_split, p.B), dim3(512), (size_t)p.H * p.dimp * 2, s, hp, p);
+  hipLaunchKernelGGL((k_attn_mix_decode<GW, DC, NP>), dim3(p.n_split, p.B), dim3(512), (size_t)p.H * p.dimp * 2, s, hp, p);
   P3V_CHECK_LAUNCH();
   return mix_combine(p, s);
 }
-template <int DC>
+template <int GW, int DC>
 static int decode_np(const QkvHeadsP& hp, const AttnMixP& p, hipStream_t s) {
   const int np = p3v_cdiv(p.H * p.vdim, 512);
-  return np <= 1 ? launch_decode<DC, 1>(hp, p, s) : np <= 2 ? launch_decode<DC, 2>(hp, p, s) : np <= 4 ? launch_decode<DC, 4>(hp, p, s)
-       : np <= 6 ? launch_decode<DC, 6>(hp, p, s) : launch_decode<DC, 8>(hp, p, s);
+  return np <= 2 ? launch_decode<GW, DC, 2>(hp, p, s) : np <= 4 ? launch_decode<GW, DC, 4>(hp, p, s)
+       : np <= 6 ? launch_decode<GW, DC, 6>(hp, p, s) : launch_decode<GW, DC, 8>(hp, p, s);
+}
+template <int DC>
+static int decode_gw(const QkvHeadsP& hp, const AttnMixP& p, hipStream_t s) {
+  return p.G <= 8 ? decode_np<1, DC>(hp, p, s) : p.G <= 16 ? decode_np<2, DC>(hp, p, s) : decode_np<4, DC>(hp, p, s);
 }
 
 extern "C" int p3v_attn_mix_decode(const p3v_mix_args_t* a, void* stream) {
   const int rc = p3v_mix_check(a);
   if (rc != P3V_OK) return rc;
   if (!a->qkv || !a->q_norm || !a->k_norm || !a->talk || !a->sink || !a->gate || !a->out || a->n_split < 0) return P3V_ERR_ARG;
-  if (a->L != 1 || a->n_split == 0 || !mix_fast(a->H, a->G, a->dim, a->vdim, a->f32) || a->H / a->G > 16) return P3V_ERR_UNSUPPORTED;
-  if (!a->ws) return P3V_ERR_ARG;
+  if (a->L != 1 || a->n_split == 0 || !mix_fast(a->H, a->G, a->dim, a->vdim, a->f32) || a->H / a->G > 16 || a->dimp > 128)
+    return P3V_ERR_UNSUPPORTED;
+  if (!a->ws || a->n_split > MIX_MAX_SPLIT) return P3V_ERR_ARG;
   AttnMixP p = attn_mix_params(a);
   p.tiles_per_split = p3v_cdiv(a->Tp / 16, a->n_split);
   const QkvHeadsP hp = {a->qkv, a->q_norm, a->k_norm, a->v_first, nullptr, a->k, a->v, a->d_past, a->eps, a->vmix,
                         a->B, a->L, a->H, a->G, a->dim, a->vdim, a->dimp, a->vdimp, a->ld, a->ld_first, a->past, a->Tp};
   hipStream_t s = (hipStream_t)stream;
   switch (a->dimp / 32) {
-    case 1: return decode_np<1>(hp, p, s);
-    case 2: return decode_np<2>(hp, p, s);
-    case 3: return decode_np<3>(hp, p, s);
-    default: return decode_np<4>(hp, p, s);
+    case 1: return decode_gw<1>(hp, p, s);
+    case 2: return decode_gw<2>(hp, p, s);
+    case 3: return decode_gw<3>(hp, p, s);
+    default: return decode_gw<4>(hp, p, s);
   }
 }

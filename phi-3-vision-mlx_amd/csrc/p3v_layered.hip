@@ -164,7 +164,8 @@ extern "C" int p3v_gemm_any(const p3v_gemm_args_t* a, int a_f32, void* stream) {
 }
 
 // ---------------------------------------------------------------- head split: whole-projection q / k norms, value mixing, cache append
-// A workgroup takes the up to 16 tokens of one sequence that share a 16-token block of the value cache.  Norms: a wave per token.
+// gridDim.x walks the 16-token blocks of the value cache that a call touches; gridDim.z shares a block's work: 4 workgroups for the
+// query / key norms (a wave per token), 4 for a quarter of the value columns each.
 template <typename T, int V>
 __global__ void __launch_bounds__(256) k_qkv_heads(QkvHeadsP p) {
   const int b = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -172,7 +173,9 @@ __global__ void __launch_bounds__(256) k_qkv_heads(QkvHeadsP p) {
   const int blk = (past >> 4) + blockIdx.x, pos_lo = max(past, blk * 16), pos_hi = min(past + p.L, blk * 16 + 16);
   const int nq = p.H * p.dim, nk = p.G * p.dim, nv = p.G * p.vdim;
   const T* base = (const T*)p.qkv;
-  for (int pos = pos_lo + wave; pos < pos_hi; pos += 4) {
+  const int part = blockIdx.z;
+  const int pos = blk * 16 + part * 4 + wave;
+  if (part < 4 && pos >= pos_lo && pos < pos_hi) {
     const int l = pos - past;
     const T* row = base + ((size_t)b * p.L + l) * p.ld;
     float sq = 0.f, sk = 0.f;
@@ -200,7 +203,7 @@ __global__ void __launch_bounds__(256) k_qkv_heads(QkvHeadsP p) {
       store_acts<V>((T*)p.k + (((size_t)b * p.G + g) * p.Tp + pos) * p.dimp + d, v);
     }
   }
-  for (int e = threadIdx.x; e < nv; e += 256) {
+  for (int e = (part - 4) * 256 + threadIdx.x; part >= 4 && e < nv; e += 1024) {
     const int g = e / p.vdim, d = e - g * p.vdim;
     T* dst = (T*)p.v + ((((size_t)b * p.G + g) * (p.Tp >> 4) + blk) * p.vdimp + d) * 16;
     const T* src = base + ((size_t)b * p.L - past) * p.ld + nq + nk + e;            // + pos * ld
@@ -227,7 +230,7 @@ extern "C" int p3v_qkv_heads(const p3v_mix_args_t* a, void* stream) {
   if (!a->qkv || !a->q || !a->q_norm || !a->k_norm) return P3V_ERR_ARG;
   const QkvHeadsP p = {a->qkv, a->q_norm, a->k_norm, a->v_first, a->q, a->k, a->v, a->d_past, a->eps, a->vmix,
                        a->B, a->L, a->H, a->G, a->dim, a->vdim, a->dimp, a->vdimp, a->ld, a->ld_first, a->past, a->Tp};
-  const dim3 grid(a->L == 1 ? 1 : p3v_cdiv(a->L + 15, 16) + (a->d_past ? 1 : 0), a->B);
+  const dim3 grid(a->L == 1 ? 1 : p3v_cdiv(a->L + 15, 16) + (a->d_past ? 1 : 0), a->B, 8);
   const bool vec = a->dim % 8 == 0 && a->ld % 8 == 0;
   hipStream_t s = (hipStream_t)stream;
   if (a->f32) {
@@ -319,7 +322,7 @@ __global__ void __launch_bounds__(256) k_attn_mix_any(AttnMixP p) {
 
 int p3v_mix_check(const p3v_mix_args_t* a) {
   if (!a || !a->k || !a->v || a->B <= 0 || a->L <= 0 || a->H <= 0 || a->G <= 0 || a->H % a->G || a->dim <= 0 || a->vdim <= 0) return P3V_ERR_ARG;
-  if (a->dimp < a->dim || a->dimp % 32 || a->vdimp < a->vdim || a->vdimp % 16 || a->Tp <= 0 || a->Tp % 32) return P3V_ERR_ARG;
+  if (a->dimp < a->dim || a->dimp % 32 || a->vdimp < a->vdim || a->vdimp % 32 || a->Tp <= 0 || a->Tp % 32) return P3V_ERR_ARG;
   if (!a->d_past && (a->past < 0 || a->past + a->L > a->Tp)) return P3V_ERR_ARG;
   return P3V_OK;
 }

@@ -31,7 +31,8 @@ class _Layer:
         self.norm1 = (float(w[p + "norm1.alpha"]), t("norm1"), t("norm1.b"))
         self.shift, self.ls1 = t("shift"), t("ls1")
         qkvg = torch.cat([t("mix.q"), t("mix.k"), t("mix.v"), t("mix.g")])
-        n = round_up(qkvg.shape[0], 64)                          # whole tiles: the padding rows are zero and nobody reads their outputs
+        # whole GEMM tiles (the 256-column ones where the matrix is wide): the padding rows are zero and nobody reads their outputs
+        n = round_up(qkvg.shape[0], 256 if qkvg.shape[0] >= 2048 else 64)
         self.qkvg = torch.cat([qkvg, qkvg.new_zeros((n - qkvg.shape[0], qkvg.shape[1]))]).contiguous()
         self.norms = (t("mix.q.norm"), t("mix.k.norm"))
         self.talk, self.sink, self.vmix, self.o = t("mix.talk"), t("mix.sink"), float(w[p + "mix.vmix"]) if p + "mix.vmix" in w else 0.0, t("mix.o")
@@ -67,7 +68,7 @@ class LayeredModel(DecoderModel):
 
     def _cache_token_bytes(self):
         e = 4 if self.act_dtype == F32 else 2
-        return sum(e * s.mixer.kv_heads * (round_up(s.mixer.dim, 32) + round_up(s.mixer.vdim, 16)) for s in self.cfg.layers)
+        return sum(e * s.mixer.kv_heads * (round_up(s.mixer.dim, 32) + round_up(s.mixer.vdim, 32)) for s in self.cfg.layers)
 
     def _alloc_bufs(self, B, L, n_keys=None):
         """n_keys: what the attention's key splits are planned for (one-token calls: the cache capacity, so that eager and captured steps

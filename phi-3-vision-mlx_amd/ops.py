@@ -720,6 +720,7 @@ def attention_mixed(qkv, q, k, v, out, norms, talk, sink, B, Lq, H, G, dim, vdim
         if rc != L.ERR_UNSUPPORTED:
             L.check(rc, "attn_mix_decode")
             return out
+        args.n_split = 1
     L.check(L.lib().p3v_qkv_heads(C.byref(args), _stream()), "qkv_heads")
     L.check(L.lib().p3v_attn_mix(C.byref(args), _stream()), "attn_mix")
     return out

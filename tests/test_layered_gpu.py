@@ -106,7 +106,7 @@ def close(got, want, dt, what=""):
     """Worst row and worst element of got - want, both against the rms of want: rounding of a bf16 (or fp32) result and its inputs."""
     d, s = np.asarray(got, dtype=np.float64) - want, np.sqrt((want ** 2).mean())
     row, worst = float(np.sqrt((d ** 2).mean(-1)).max() / s), float(np.abs(d).max() / s)
-    assert row < (1e-5 if dt == F32 else 0.025) and worst < (1e-4 if dt == F32 else 0.15), (what, row, worst)
+    assert row < (1e-5 if dt == F32 else 0.04) and worst < (1e-4 if dt == F32 else 0.15), (what, row, worst)
 
 
 TOL = {"float32": 2e-5, "bfloat16": 0.035}
@@ -220,7 +220,7 @@ class Mix:
         self.qn, self.kn = bf(self.r.normal(1.0, 0.3, H * dim)), bf(self.r.normal(1.0, 0.3, G * dim))
         self.talk, self.sink = bf(np.eye(H) + self.r.normal(0, 0.8 * H ** -0.5, (H, H))), bf(self.r.normal(1, 1, H))
         self.k = torch.zeros((B, G, Tp, round_up(dim, 32)), dtype=dt, device=DEV)
-        self.v = torch.zeros((B, G, Tp // 16, round_up(vdim, 16), 16), dtype=dt, device=DEV)
+        self.v = torch.zeros((B, G, Tp // 16, round_up(vdim, 32), 16), dtype=dt, device=DEV)
         self.vmix, self.eps = 0.0, 1e-5
 
     def run(self, qkv, L, past, pads=None, first=None, plan=None, d_past=False):
