@@ -57,8 +57,8 @@ template <int HW> struct MixCfg {
   static constexpr int HP = 8 * HW, HS = HP + 4, QS = 32 * HS + 4;      // heads padded, S strides (floats): key, query
   static constexpr int PQ = 40, PH = 16 * PQ + 8;                        // P strides (bf16): query, head
   static constexpr int HM = (HP + 15) / 16;                              // 16-head row blocks of the mixing
-  static constexpr int S_BYTES = 16 * QS * 4, P_BYTES = HP * PH * 2, A_BYTES = HP * 16 * 4;
-  static constexpr int LDS = S_BYTES + P_BYTES + 2 * A_BYTES;
+  static constexpr int S_BYTES = 16 * QS * 4, P_BYTES = HP * PH * 2, A_BYTES = HM * 16 * 16 * 4;
+  static constexpr int LDS = S_BYTES + P_BYTES + 2 * A_BYTES + HM * 1024 + (HW == 4 ? 8 * 4096 : 0);
 };
 
 template <int HW, int DC, int VC, bool SHARED>
@@ -66,12 +66,13 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
   typedef MixCfg<HW> C;
   constexpr int NB = SHARED ? 1 : 2;                                     // fragment buffers
   constexpr int QU = HW == 4 && DC + VC >= 5 ? 1 : 2;                    // queries of the mixing side by side
-  constexpr bool Q_REG = HW < 4 || DC + VC < 8;                          // else the query fragments are read again for every key tile
+  constexpr bool Q_REG = HW < 4 || DC + VC <= 6;                         // else the query fragments are read again for every key tile
+  constexpr bool Q_LDS = HW == 4 && DC + VC == 6;                        // the last head's wait in LDS
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   float* S = (float*)smem;
   bf16_t* P = (bf16_t*)(smem + C::S_BYTES);
   float* AL = (float*)(smem + C::S_BYTES + C::P_BYTES);
-  float* MM = AL + C::HP * 16;
+  float* MM = AL + C::HM * 256;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lc = lane & 15, lg = lane >> 4;
   const int n_qt = (p.L + 15) >> 4, qt = n_qt - 1 - (int)blockIdx.x, split = blockIdx.y, b = blockIdx.z;   // longest rows first
   const int q0 = qt * 16, per = p.H / p.G, past = p.d_past ? *p.d_past : p.past, first = p.pad_len ? p.pad_len[b] : 0;
@@ -81,43 +82,45 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
   const int t0 = max(first >> 5, split * p.tiles_per_split), t1 = min((last >> 5) + 1, (split + 1) * p.tiles_per_split);
   if (split * p.tiles_per_split > last >> 5) return;
   constexpr int NV = 2 * VC;                                             // 16-dimension blocks of a value (dimp = 32 DC, vdimp = 32 VC)
-  const float sc = p.scale * LOG2E;
+  const float sc = fabsf(p.scale) * LOG2E;                               // (a negative scale's sign goes into talk: the row maxima then scale)
+  const uint32_t flip = p.scale < 0.f ? 0x8000u : 0u;
 
   // Q fragments (B operand: column = query, 8 consecutive dimensions)
+  u32x4_t* QL = (u32x4_t*)(MM + C::HM * 256) + C::HM * 64 + wave * (4 * 64) + lane;
   bf16x8_t qf[Q_REG ? HW : 1][DC];
   auto load_q = [&](int i) {
     const int h = min(wave * HW + i, p.H - 1);
     const bf16_t* qr = (const bf16_t*)p.q + (((size_t)b * p.H + h) * p.L + min(q0 + lc, p.L - 1)) * p.dimp + lg * 8;
 #pragma unroll
-    for (int c = 0; c < DC; ++c) qf[Q_REG ? i : 0][c] = *(const bf16x8_t*)(qr + c * 32);
+    for (int c = 0; c < DC; ++c) {
+      const bf16x8_t v = *(const bf16x8_t*)(qr + c * 32);
+      if (Q_LDS && i == HW - 1) QL[c * 64] = __builtin_bit_cast(u32x4_t, v);
+      else qf[Q_REG ? i : 0][c] = v;
+    }
   };
   if constexpr (Q_REG) {
 #pragma unroll
     for (int i = 0; i < HW; ++i) load_q(i);
   }
-  // talk fragments (A operand: row = mixed head, 8 consecutive raw heads), zero beyond H
-  bf16x8_t tf[C::HM];
-#pragma unroll
-  for (int m = 0; m < C::HM; ++m) {
+  // talk fragments (A operand: row = mixed head, 8 consecutive raw heads), zero beyond H; kept in LDS
+  u32x4_t* TF = (u32x4_t*)(MM + C::HM * 256);
+  for (int m = wave; m < C::HM; m += 8) {
     u32x4_t w = {0u, 0u, 0u, 0u};
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
       const int h = m * 16 + lc, g = lg * 8 + j;
-      const uint32_t v = h < p.H && g < p.H ? p.talk[h * p.H + g] : 0;
+      const uint32_t v = h < p.H && g < p.H ? p.talk[h * p.H + g] ^ flip : 0;
       w[j >> 1] |= v << (16 * (j & 1));
     }
-    tf[m] = __builtin_bit_cast(bf16x8_t, w);
+    TF[m * 64 + lane] = w;
   }
-  const u32x4_t ones_w = {0x3f803f80u, 0x3f803f80u, 0x3f803f80u, 0x3f803f80u};
-  const bf16x8_t ones = __builtin_bit_cast(bf16x8_t, ones_w);
-  f32x4_t o[HW][NV], ol[HW];                                         // outputs; the row of ones: softmax sums
+  f32x4_t o[HW][NV], ol = {0.f, 0.f, 0.f, 0.f};                          // outputs; softmax sums (row i: head i of the wave)
 #pragma unroll
   for (int i = 0; i < HW; ++i) {
-    ol[i] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int d = 0; d < NV; ++d) o[i][d] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
   }
-  for (int i = tid; i < C::HP * 16; i += 512) MM[i] = MIX_NEG;
+  for (int i = tid; i < C::HM * 256; i += 512) MM[i] = MIX_NEG;
   lds_barrier();
 
   const bf16_t* kb = (const bf16_t*)p.k + (size_t)b * p.G * p.Tp * p.dimp;
@@ -127,17 +130,18 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
   bf16x8_t kf[NB][2][DC], vf[NB][NV];
   auto load_k = [&](int t, int i) {
     const int g = min(wave * HW + i, p.H - 1) / per, bf = SHARED ? 0 : i & 1;
-    const bf16_t* kr = kb + ((size_t)g * p.Tp + t * 32) * p.dimp + k_lane;
+    const bf16_t *k0 = kb + ((size_t)g * p.Tp + t * 32) * p.dimp, *k1 = k0 + (size_t)16 * p.dimp;
+    asm volatile("" : "+s"(k0), "+s"(k1));                               // (scalar bases + one 32-bit lane offset: no 64-bit lane addresses)
 #pragma unroll
-    for (int c = 0; c < DC; ++c)
-      kf[bf][0][c] = *(const bf16x8_t*)(kr + c * 32), kf[bf][1][c] = *(const bf16x8_t*)(kr + (size_t)16 * p.dimp + c * 32);
+    for (int c = 0; c < DC; ++c) kf[bf][0][c] = *(const bf16x8_t*)(k0 + k_lane + c * 32), kf[bf][1][c] = *(const bf16x8_t*)(k1 + k_lane + c * 32);
   };
   auto load_v = [&](int t, int i) {
     const int g = min(wave * HW + i, p.H - 1) / per, bf = SHARED ? 0 : i & 1;
-    const bf16_t* vr = vb + ((size_t)g * (p.Tp >> 4) + t * 2) * p.vdimp * 16 + v_lane;
+    const bf16_t* vr = vb + ((size_t)g * (p.Tp >> 4) + t * 2) * p.vdimp * 16;
+    asm volatile("" : "+s"(vr));
 #pragma unroll
     for (int d = 0; d < NV; ++d)
-      vf[bf][d] = *(const bf16x8_t*)(vr + d * 256);
+      vf[bf][d] = *(const bf16x8_t*)(vr + v_lane + d * 256);
   };
   if (active && t0 < t1) load_k(t0, 0);
 
@@ -153,8 +157,11 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
 #pragma unroll
         for (int c = 0; c < DC; ++c)
           {
-            s[i][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[SHARED ? 0 : i & 1][0][c], qf[Q_REG ? i : 0][c], s[i][0], 0, 0, 0);
-            s[i][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[SHARED ? 0 : i & 1][1][c], qf[Q_REG ? i : 0][c], s[i][1], 0, 0, 0);
+            bf16x8_t q;
+            if (Q_LDS && i == HW - 1) q = __builtin_bit_cast(bf16x8_t, QL[c * 64]);
+            else q = qf[Q_REG ? i : 0][c];
+            s[i][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[SHARED ? 0 : i & 1][0][c], q, s[i][0], 0, 0, 0);
+            s[i][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[SHARED ? 0 : i & 1][1][c], q, s[i][1], 0, 0, 0);
           }
         if (HW > 1) __builtin_amdgcn_sched_barrier(0);
       }
@@ -171,16 +178,22 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
     }
     lds_barrier();
 
-    // ---- mixing + softmax of queries 2w, 2w + 1, all heads
+    // ---- mixing + softmax of queries 2w, 2w + 1, all heads; a lane's two keys are neighbours (2 lc, 2 lc + 1)
+    const bool edge = t * 32 + 31 > past + q0 || t * 32 < first;         // some query of the tile does not see some key
 #pragma unroll QU
     for (int qi = 0; qi < 2; ++qi) {
-      const int q = 2 * wave + qi, qpos = past + q0 + q;
+      const int q = 2 * wave + qi;
       f32x4_t mx[C::HM][2];
+      float mo[C::HM][4];
+#pragma unroll
+      for (int m = 0; m < C::HM; ++m)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) mo[m][r] = MM[(m * 16 + lg * 4 + r) * 16 + q];
 #pragma unroll
       for (int kt = 0; kt < 2; ++kt) {
         float v[8];
-        const float* src = S + q * C::QS + (kt * 16 + lc) * C::HS + lg * 8;
-        if (lg * 8 < C::HP) {
+        const float* src = S + q * C::QS + (2 * lc + kt) * C::HS + lg * 8;
+        if (C::HP == 32 || lg * 8 < C::HP) {
           const float4 a = *(const float4*)src, c = *(const float4*)(src + 4);
           v[0] = a.x, v[1] = a.y, v[2] = a.z, v[3] = a.w, v[4] = c.x, v[5] = c.y, v[6] = c.z, v[7] = c.w;
         } else {
@@ -203,27 +216,34 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
 #pragma unroll
         for (int m = 0; m < C::HM; ++m) {
           f32x4_t a = {0.f, 0.f, 0.f, 0.f};
+          const bf16x8_t tf = __builtin_bit_cast(bf16x8_t, TF[m * 64 + lane]);
 #pragma unroll
-          for (int k = 2; k >= 0; --k) a = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tf[m], __builtin_bit_cast(bf16x8_t, part[k]), a, 0, 0, 0);
+          for (int k = 2; k >= 0; --k) a = __builtin_amdgcn_mfma_f32_16x16x32_bf16(tf, __builtin_bit_cast(bf16x8_t, part[k]), a, 0, 0, 0);
           mx[m][kt] = a;
         }
       }
-      const int key0 = t * 32 + lc, key1 = key0 + 16;
-      const bool live0 = key0 <= qpos && key0 >= first, live1 = key1 <= qpos && key1 >= first;
+      if (edge) {
+        const int qpos = past + q0 + q, key0 = t * 32 + 2 * lc;
+        const bool live0 = key0 <= qpos && key0 >= first, live1 = key0 < qpos && key0 + 1 >= first;
+#pragma unroll
+        for (int m = 0; m < C::HM; ++m)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) mx[m][0][r] = live0 ? mx[m][0][r] : -INFINITY, mx[m][1][r] = live1 ? mx[m][1][r] : -INFINITY;
+      }
+      float al_k = 0.f, mn_k = 0.f;                                      // of row (lc >> 2, lc & 3): what this lane writes
 #pragma unroll
       for (int m = 0; m < C::HM; ++m)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const int h = m * 16 + lg * 4 + r;
-          if (C::HP >= 16 || lg < 2) {
-            const float s0 = live0 ? mx[m][0][r] * sc : -INFINITY, s1 = live1 ? mx[m][1][r] * sc : -INFINITY;
-            const float mo = MM[h * 16 + q], mn = fmaxf(mo, row16_max(fmaxf(s0, s1)));
-            const float p0 = __builtin_amdgcn_exp2f(s0 - mn), p1 = __builtin_amdgcn_exp2f(s1 - mn);
-            bf16_t* dst = P + h * C::PH + q * C::PQ + lc;
-            dst[0] = f32_to_bf16(p0), dst[16] = f32_to_bf16(p1);
-            if (lc == 0) AL[h * 16 + q] = __builtin_amdgcn_exp2f(mo - mn), MM[h * 16 + q] = mn;
-          }
+          const float mn = fmaxf(mo[m][r], row16_max(fmaxf(mx[m][0][r], mx[m][1][r])) * sc), al = __builtin_amdgcn_exp2f(mo[m][r] - mn);
+          const float p0 = __builtin_amdgcn_exp2f(fmaf(mx[m][0][r], sc, -mn)), p1 = __builtin_amdgcn_exp2f(fmaf(mx[m][1][r], sc, -mn));
+          if (C::HP >= 16 || lg < 2) *(uint32_t*)(P + (m * 16 + lg * 4 + r) * C::PH + q * C::PQ + 2 * lc) = pack_bf16x2(p0, p1);
+          al_k = lc == m * 4 + r ? al : al_k, mn_k = lc == m * 4 + r ? mn : mn_k;
         }
+      if (lc < 4 * C::HM && (C::HP >= 16 || lg < 2)) {
+        const int h = (lc >> 2) * 16 + lg * 4 + (lc & 3);
+        AL[h * 16 + q] = al_k, MM[h * 16 + q] = mn_k;
+      }
     }
     lds_barrier();
 
@@ -237,11 +257,14 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
         const bf16x8_t pf = *(const bf16x8_t*)(P + h * C::PH + lc * C::PQ + lg * 8);
         const float al = AL[h * 16 + lc];
         if (__builtin_amdgcn_ballot_w64(al != 1.f)) {                    // (a maximum moved; rare behind a sequence's first tiles)
-          ol[i] *= al;
+          ol[i] *= lg == 0 ? al : 1.f;
 #pragma unroll
           for (int d = 0; d < NV; ++d) o[i][d] *= al;
         }
-        ol[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf, ol[i], 0, 0, 0);
+        uint32_t one = lc == i ? 0x3f803f80u : 0u;                       // A: a row of ones at row i
+        asm volatile("" : "+v"(one));                                    // (not kept in registers across the loop, one fragment per head)
+        const u32x4_t ones = {one, one, one, one};
+        ol = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, ones), pf, ol, 0, 0, 0);
 #pragma unroll
         for (int d = 0; d < NV; ++d)
           o[i][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[SHARED ? 0 : i & 1][d], pf, o[i][d], 0, 0, 0);
@@ -257,7 +280,7 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
   for (int i = 0; i < HW; ++i) {
     const int h = wave * HW + i;
     if (h >= p.H) continue;
-    const float m = MM[h * 16 + lc], l = ol[i][0];
+    const float m = MM[h * 16 + lc], l = __shfl(ol[i], lc, 64);           // (the sums sit in the first 16 lanes)
     float f = 1.f;
     if (p.n_split == 1) {
       const float sk = bf16_to_f32(p.sink[h]) * LOG2E, mm = fmaxf(m, sk), e = __builtin_amdgcn_exp2f(m - mm);
@@ -296,7 +319,7 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
 // A workgroup takes a run of 16-key tiles of one sequence, all heads: the query's whole-projection norm is recomputed in every
 // workgroup (a few KB), the workgroup whose run holds the new position also normalises and appends the new key and mixes and appends
 // the new value.  Partials of the runs are merged by k_attn_mix_combine.
-template <int GW, int DC, int NP>
+template <int GW, int DC, int NP, bool VEC>
 __global__ void __launch_bounds__(512) k_attn_mix_decode(QkvHeadsP hp, AttnMixP p) {
   constexpr int SS = 20;                                                 // S / P row stride (floats)
   __shared__ float S[MIX_MAX_H * SS], P[MIX_MAX_H * SS], talk[MIX_MAX_H * (MIX_MAX_H + 1)], AL[MIX_MAX_H], red[2][8];
@@ -347,46 +370,88 @@ __global__ void __launch_bounds__(512) k_attn_mix_decode(QkvHeadsP hp, AttnMixP 
       vv[j][0] = vr[0], vv[j][1] = vr[1];
     }
   };
-  const bool live = t_begin < t_end;
-  // ---- query (and key) norm
+  // ---- query (and key) norm.  VEC: 8 columns per thread, read once, together with the weights
+  constexpr u32x4_t zero4 = {0u, 0u, 0u, 0u};
+  u32x4_t qv = zero4, qw = zero4, kv = zero4, kw = zero4, nw = zero4, fw = zero4;
+  const int e8 = tid * 8;
   float sq = 0.f, sk = 0.f;
-#pragma unroll 1
-  for (int e = tid; e < nq; e += 512) { const float v = bf16_to_f32(row[e]); sq += v * v; }
-  if (owner)
-#pragma unroll 1
-    for (int e = tid; e < nk; e += 512) { const float v = bf16_to_f32(row[nq + e]); sk += v * v; }
-  if (!owner) load_k(t_begin), load_v(t_begin);
-#pragma unroll 1
+  if constexpr (VEC) {
+    if (e8 < nq) qv = *(const u32x4_t*)(row + e8), qw = *(const u32x4_t*)(hp.q_norm + e8);
+    if (owner) {
+      if (e8 < nk) kv = *(const u32x4_t*)(row + nq + e8), kw = *(const u32x4_t*)(hp.k_norm + e8);
+      if (e8 < nv) {
+        nw = *(const u32x4_t*)(row + nq + nk + e8);
+        if (hp.v_first) fw = *(const u32x4_t*)((const bf16_t*)hp.v_first + (size_t)b * hp.ld_first + e8);
+      }
+    }
+    if (!owner) load_k(t_begin), load_v(t_begin);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      sq += bf16lo(qv[j]) * bf16lo(qv[j]) + bf16hi(qv[j]) * bf16hi(qv[j]);
+      sk += bf16lo(kv[j]) * bf16lo(kv[j]) + bf16hi(kv[j]) * bf16hi(kv[j]);
+    }
+  } else {
+    for (int e = tid; e < nq; e += 512) { const float v = bf16_to_f32(row[e]); sq += v * v; }
+    if (owner)
+      for (int e = tid; e < nk; e += 512) { const float v = bf16_to_f32(row[nq + e]); sk += v * v; }
+    if (!owner) load_k(t_begin), load_v(t_begin);
+  }
   for (int e = tid; e < p.H * p.H; e += 512) { const int h = e / p.H; talk[h * (MIX_MAX_H + 1) + e - h * p.H] = bf16_to_f32(p.talk[e]); }
   sq = wave_sum(sq), sk = wave_sum(sk);
   if (lane == 0) red[0][wave] = sq, red[1][wave] = sk;
-  lds_barrier();                     // (not __syncthreads: the tile's loads stay in flight)
+  lds_barrier();                                                         // (the tile's loads stay in flight)
   sq = sk = 0.f;
 #pragma unroll
   for (int w = 0; w < 8; ++w) sq += red[0][w], sk += red[1][w];
   const float rq = 1.f / sqrtf(sq / (float)nq + hp.eps), rk = 1.f / sqrtf(sk / (float)nk + hp.eps);
-#pragma unroll 1
-  for (int e = tid; e < p.H * p.dimp; e += 512) {
-    const int h = e / p.dimp, d = e - h * p.dimp;
-    qs[e] = d < p.dim ? f32_to_bf16(bf16_to_f32(row[h * p.dim + d]) * rq * bf16_to_f32(hp.q_norm[h * p.dim + d])) : (bf16_t)0;
-  }
-  if (owner) {
-#pragma unroll 1
-    for (int e = tid; e < nk; e += 512) {
-      const int g = e / p.dim, d = e - g * p.dim;
-      ((bf16_t*)hp.k)[(((size_t)b * p.G + g) * p.Tp + past) * p.dimp + d] = f32_to_bf16(bf16_to_f32(row[nq + e]) * rk * bf16_to_f32(hp.k_norm[e]));
+  if constexpr (VEC) {
+    auto normed = [](u32x4_t x, u32x4_t w, float r) {
+      u32x4_t y;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) y[j] = pack_bf16x2(bf16lo(x[j]) * r * bf16lo(w[j]), bf16hi(x[j]) * r * bf16hi(w[j]));
+      return y;
+    };
+    if (e8 < nq) { const int h = e8 / p.dim; *(u32x4_t*)(qs + h * p.dimp + e8 - h * p.dim) = normed(qv, qw, rq); }
+    if (p.dimp != p.dim)
+      for (int e = tid; e < p.H * (p.dimp - p.dim); e += 512) { const int h = e / (p.dimp - p.dim); qs[h * p.dimp + p.dim + e - h * (p.dimp - p.dim)] = 0; }
+    if (owner) {
+      if (e8 < nk) {
+        const int g = e8 / p.dim;
+        *(u32x4_t*)((bf16_t*)hp.k + (((size_t)b * p.G + g) * p.Tp + past) * p.dimp + e8 - g * p.dim) = normed(kv, kw, rk);
+      }
+      if (e8 < nv) {
+        const int g = e8 / p.vdim;
+        bf16_t* dst = (bf16_t*)hp.v + ((((size_t)b * p.G + g) * (p.Tp >> 4) + own) * p.vdimp + e8 - g * p.vdim) * 16 + (past & 15);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          float lo = bf16lo(nw[j]), hi = bf16hi(nw[j]);
+          if (hp.v_first) lo = (1.f - hp.vmix) * lo + hp.vmix * bf16lo(fw[j]), hi = (1.f - hp.vmix) * hi + hp.vmix * bf16hi(fw[j]);
+          dst[32 * j] = f32_to_bf16(lo), dst[32 * j + 16] = f32_to_bf16(hi);
+        }
+      }
+      __syncthreads();                                                   // (the stores have to be visible to the whole workgroup)
     }
-#pragma unroll 1
-    for (int e = tid; e < nv; e += 512) {
-      const int g = e / p.vdim, d = e - g * p.vdim;
-      float v = bf16_to_f32(row[nq + nk + e]);
-      if (hp.v_first) v = (1.f - hp.vmix) * v + hp.vmix * bf16_to_f32(((const bf16_t*)hp.v_first)[(size_t)b * hp.ld_first + e]);
-      ((bf16_t*)hp.v)[((((size_t)b * p.G + g) * (p.Tp >> 4) + own) * p.vdimp + d) * 16 + (past & 15)] = f32_to_bf16(v);
+  } else {
+    for (int e = tid; e < p.H * p.dimp; e += 512) {
+      const int h = e / p.dimp, d = e - h * p.dimp;
+      qs[e] = d < p.dim ? f32_to_bf16(bf16_to_f32(row[h * p.dim + d]) * rq * bf16_to_f32(hp.q_norm[h * p.dim + d])) : (bf16_t)0;
     }
-    __syncthreads();                                                     // (the stores have to be visible to the whole workgroup)
+    if (owner) {
+      for (int e = tid; e < nk; e += 512) {
+        const int g = e / p.dim, d = e - g * p.dim;
+        ((bf16_t*)hp.k)[(((size_t)b * p.G + g) * p.Tp + past) * p.dimp + d] = f32_to_bf16(bf16_to_f32(row[nq + e]) * rk * bf16_to_f32(hp.k_norm[e]));
+      }
+      for (int e = tid; e < nv; e += 512) {
+        const int g = e / p.vdim, d = e - g * p.vdim;
+        float v = bf16_to_f32(row[nq + nk + e]);
+        if (hp.v_first) v = (1.f - hp.vmix) * v + hp.vmix * bf16_to_f32(((const bf16_t*)hp.v_first)[(size_t)b * hp.ld_first + e]);
+        ((bf16_t*)hp.v)[((((size_t)b * p.G + g) * (p.Tp >> 4) + own) * p.vdimp + d) * 16 + (past & 15)] = f32_to_bf16(v);
+      }
+      __syncthreads();                                                   // (as above)
+    }
   }
   lds_barrier();                     // the query (and the new key / value) is in LDS
-  if (!live) return;
+  if (t_begin >= t_end) return;
   if (owner) load_k(t_begin), load_v(t_begin);
 
   float acc[NP];
@@ -453,41 +518,32 @@ __device__ __forceinline__ int live_splits(const AttnMixP& p, size_t row, int sh
 }
 // one token per sequence: many splits, few rows -- a workgroup per (head, row), groups of threads share the splits
 #define MIX_MAX_SPLIT 1024
-__global__ void __launch_bounds__(512) k_attn_mix_combine(AttnMixP p) {
-  __shared__ float red[16], part[512], wt[MIX_MAX_SPLIT];
+__global__ void __launch_bounds__(1024) k_attn_mix_combine(AttnMixP p) {
+  constexpr int U = 16;                                                  // splits per thread group whose outputs are requested up front
+  __shared__ float red[16], part[1024], wt[MIX_MAX_SPLIT];
   const int h = blockIdx.x, tid = threadIdx.x;
   const size_t row = blockIdx.y, rows = (size_t)p.B * p.L;
   const int n = live_splits(p, row, 4);
-  const float sk = bf16_to_f32(p.sink[h]) * LOG2E;
-  float m = sk, lm[MIX_MAX_SPLIT / 512], ll[MIX_MAX_SPLIT / 512];
+  const int vw = p.vdim <= 32 ? 32 : p.vdim <= 64 ? 64 : 128, ng = 1024 / vw, grp = tid / vw, d = tid - grp * vw;
+  const float* o = ws_o(p.ws, p, rows, row, 0) + (size_t)h * p.vdim + min(d, p.vdim - 1);
+  const size_t step = (size_t)p.H * p.vdim;
+  f32x2_t q = {MIX_NEG, 0.f};
+  if (tid < n) q = *(const f32x2_t*)(ws_ml(p.ws, p, row, tid) + 2 * h);
+  float v[U];
 #pragma unroll
-  for (int i = 0; i < MIX_MAX_SPLIT / 512; ++i) {
-    const int s = tid + 512 * i;
-    lm[i] = MIX_NEG, ll[i] = 0.f;
-    if (s < n) { const f32x2_t q = *(const f32x2_t*)(ws_ml(p.ws, p, row, s) + 2 * h); lm[i] = q[0], ll[i] = q[1]; }
-    m = fmaxf(m, lm[i]);
-  }
-  m = block_max(m, red);
-  float l = 0.f;
-#pragma unroll
-  for (int i = 0; i < MIX_MAX_SPLIT / 512; ++i) {
-    const float w = __builtin_amdgcn_exp2f(lm[i] - m);
-    wt[tid + 512 * i] = lm[i] > 0.5f * MIX_NEG ? w : -1.f;               // (-1: a split of padding, whose outputs were not written)
-    l += ll[i] * w;
-  }
-  l = block_sum(l, red) + __builtin_amdgcn_exp2f(sk - m);
-  const float f = gate_of((const bf16_t*)p.gate + row * p.ld + h) / l;
-  const int vw = p.vdim <= 32 ? 32 : p.vdim <= 64 ? 64 : 128, ng = 512 / vw, grp = tid / vw, d = tid - grp * vw;
+  for (int u = 0; u < U; ++u) v[u] = o[min(grp + u * ng, n - 1) * step];
+  const float sk = bf16_to_f32(p.sink[h]) * LOG2E, gate = gate_of((const bf16_t*)p.gate + row * p.ld + h);
+  const float m = block_max(fmaxf(sk, q[0]), red), w = __builtin_amdgcn_exp2f(q[0] - m);
+  wt[tid] = q[0] > 0.5f * MIX_NEG ? w : -1.f;                            // (-1: no such split, or one of padding whose outputs were not written)
+  const float f = gate / (block_sum(q[1] * w, red) + __builtin_amdgcn_exp2f(sk - m));
   float a = 0.f;
-  if (d < p.vdim) {
-    const float* o = ws_o(p.ws, p, rows, row, 0) + (size_t)h * p.vdim + d;
-    const size_t step = (size_t)p.H * p.vdim;
-#pragma unroll 8
-    for (int s = grp; s < n; s += ng) {
-      const float w = wt[s], v = o[s * step];
-      a = w >= 0.f ? fmaf(w, v, a) : a;
-    }
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const int s = grp + u * ng;
+    const float x = wt[min(s, MIX_MAX_SPLIT - 1)];
+    a = s < n && x >= 0.f ? fmaf(x, v[u], a) : a;
   }
+  for (int s = grp + U * ng; s < n; s += ng) a = wt[s] >= 0.f ? fmaf(wt[s], o[s * step], a) : a;
   part[tid] = a;
   __syncthreads();
   if (grp == 0 && d < p.vdim) {
@@ -559,7 +615,7 @@ extern "C" int64_t p3v_attn_mix_ws_bytes(int B, int L, int H, int vdim, int n_sp
 }
 
 static int mix_combine(const AttnMixP& p, hipStream_t s) {
-  if (p.L == 1) hipLaunchKernelGGL(k_attn_mix_combine, dim3(p.H, p.B), dim3(512), 0, s, p);
+  if (p.L == 1) hipLaunchKernelGGL(k_attn_mix_combine, dim3(p.H, p.B), dim3(1024), 0, s, p);
   else hipLaunchKernelGGL(k_attn_mix_combine_rows, dim3(p.B * p.L), dim3(256), 0, s, p);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
@@ -614,7 +670,12 @@ extern "C" int p3v_attn_mix(const p3v_mix_args_t* a, void* stream) {
 
 template <int GW, int DC, int NP>
 static int launch_decode(const QkvHeadsP& hp, const AttnMixP& p, hipStream_t s) {
-  hipLaunchKernelGGL((k_attn_mix_decode<GW, DC, NP>), dim3(p.n_split, p.B), dim3(512), (size_t)p.H * p.dimp * 2, s, hp, p);
+  const bool vec = p.dim % 8 == 0 && p.vdim % 8 == 0 && hp.ld % 8 == 0 && (!hp.v_first || hp.ld_first % 8 == 0) && p.H * p.dim <= 4096 &&
+                   (((uintptr_t)hp.qkv | (uintptr_t)hp.q_norm | (uintptr_t)hp.k_norm | (uintptr_t)hp.v_first) & 15) == 0;
+  const dim3 grid(p.n_split, p.B);
+  const size_t lds = (size_t)p.H * p.dimp * 2;
+  if (vec) hipLaunchKernelGGL((k_attn_mix_decode<GW, DC, NP, true>), grid, dim3(512), lds, s, hp, p);
+  else hipLaunchKernelGGL((k_attn_mix_decode<GW, DC, NP, false>), grid, dim3(512), lds, s, hp, p);
   P3V_CHECK_LAUNCH();
   return mix_combine(p, s);
 }
