@@ -121,6 +121,8 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
     for (int d = 0; d < NV; ++d) o[i][d] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
   }
   for (int i = tid; i < C::HM * 256; i += 512) MM[i] = MIX_NEG;
+  if (p.H < C::HP)                                                       // heads that no wave writes: finite, talk's zero columns do the rest
+    for (int i = tid; i < C::S_BYTES / 4; i += 512) S[i] = 0.f;
   lds_barrier();
 
   const bf16_t* kb = (const bf16_t*)p.k + (size_t)b * p.G * p.Tp * p.dimp;
@@ -200,10 +202,6 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
 #pragma unroll
           for (int j = 0; j < 8; ++j) v[j] = 0.f;
         }
-        if (p.H < C::HP) {                                               // (heads that no wave wrote)
-#pragma unroll
-          for (int j = 0; j < 8; ++j) v[j] = lg * 8 + j < p.H ? v[j] : 0.f;
-        }
         u32x4_t part[3];
 #pragma unroll
         for (int k = 0; k < 3; ++k)
@@ -230,12 +228,20 @@ __global__ void __launch_bounds__(512, 1) k_attn_mix_prefill(AttnMixP p) {
 #pragma unroll
           for (int r = 0; r < 4; ++r) mx[m][0][r] = live0 ? mx[m][0][r] : -INFINITY, mx[m][1][r] = live1 ? mx[m][1][r] : -INFINITY;
       }
+      float rm[C::HM * 4];                                               // row maxima over the 16 lanes: stage by stage, so that no lane move waits
+#pragma unroll
+      for (int i = 0; i < C::HM * 4; ++i) rm[i] = fmaxf(mx[i >> 2][0][i & 3], mx[i >> 2][1][i & 3]);
+#define MIX_ROWS_STAGE(ctrl)                                                                              \
+  _Pragma("unroll") for (int i = 0; i < C::HM * 4; ++i) rm[i] = fmaxf(rm[i], P3V_DPP_F32(rm[i], ctrl));   \
+  __builtin_amdgcn_sched_barrier(0);
+      MIX_ROWS_STAGE(0xB1) MIX_ROWS_STAGE(0x4E) MIX_ROWS_STAGE(0x124) MIX_ROWS_STAGE(0x128)
+#undef MIX_ROWS_STAGE
       float al_k = 0.f, mn_k = 0.f;                                      // of row (lc >> 2, lc & 3): what this lane writes
 #pragma unroll
       for (int m = 0; m < C::HM; ++m)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float mn = fmaxf(mo[m][r], row16_max(fmaxf(mx[m][0][r], mx[m][1][r])) * sc), al = __builtin_amdgcn_exp2f(mo[m][r] - mn);
+          const float mn = fmaxf(mo[m][r], rm[m * 4 + r] * sc), al = __builtin_amdgcn_exp2f(mo[m][r] - mn);
           const float p0 = __builtin_amdgcn_exp2f(fmaf(mx[m][0][r], sc, -mn)), p1 = __builtin_amdgcn_exp2f(fmaf(mx[m][1][r], sc, -mn));
           if (C::HP >= 16 || lg < 2) *(uint32_t*)(P + (m * 16 + lg * 4 + r) * C::PH + q * C::PQ + 2 * lc) = pack_bf16x2(p0, p1);
           al_k = lc == m * 4 + r ? al : al_k, mn_k = lc == m * 4 + r ? mn : mn_k;

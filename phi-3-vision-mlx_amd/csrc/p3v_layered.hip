@@ -203,7 +203,41 @@ __global__ void __launch_bounds__(256) k_qkv_heads(QkvHeadsP p) {
       store_acts<V>((T*)p.k + (((size_t)b * p.G + g) * p.Tp + pos) * p.dimp + d, v);
     }
   }
-  for (int e = (part - 4) * 256 + threadIdx.x; part >= 4 && e < nv; e += 1024) {
+  if (part < 4) return;
+  if constexpr (V == 8) {
+    // a whole block of 16 tokens: 8 columns per thread, 16-byte loads, the 16 x 8 values turned around in registers
+    if (p.vdim % 8 == 0 && (!p.v_first || p.ld_first % 8 == 0) && pos_hi - pos_lo == 16) {
+      for (int e = ((part - 4) * 256 + threadIdx.x) * 8; e < nv; e += 8192) {
+        const int g = e / p.vdim, d = e - g * p.vdim;
+        T* dst = (T*)p.v + ((((size_t)b * p.G + g) * (p.Tp >> 4) + blk) * p.vdimp + d) * 16;
+        const T* src = base + ((size_t)b * p.L + pos_lo - past) * p.ld + nq + nk + e;
+        const T* first = p.v_first ? (const T*)p.v_first + ((size_t)b * p.L + pos_lo - past) * p.ld_first + e : nullptr;
+#pragma unroll
+        for (int half = 0; half < 2; ++half) {
+          float x[8][8];
+#pragma unroll
+          for (int j = 0; j < 8; ++j) {
+            load_acts<8>(src + (size_t)(half * 8 + j) * p.ld, x[j]);
+            if (first) {
+              float f[8];
+              load_acts<8>(first + (size_t)(half * 8 + j) * p.ld_first, f);
+#pragma unroll
+              for (int k = 0; k < 8; ++k) x[j][k] = (1.f - p.vmix) * x[j][k] + p.vmix * f[k];
+            }
+          }
+#pragma unroll
+          for (int k = 0; k < 8; ++k) {
+            float y[8];
+#pragma unroll
+            for (int j = 0; j < 8; ++j) y[j] = x[j][k];
+            store_acts<8>(dst + k * 16 + half * 8, y);
+          }
+        }
+      }
+      return;
+    }
+  }
+  for (int e = (part - 4) * 256 + threadIdx.x; e < nv; e += 1024) {
     const int g = e / p.vdim, d = e - g * p.vdim;
     T* dst = (T*)p.v + ((((size_t)b * p.G + g) * (p.Tp >> 4) + blk) * p.vdimp + d) * 16;
     const T* src = base + ((size_t)b * p.L - past) * p.ld + nq + nk + e;            // + pos * ld
