@@ -74,7 +74,8 @@ enum {
   P3V_EPI_SILU_MUL = 6,    /* W = [gate;up] (2N rows): out bf16[M,N] = silu(g)*u  phi.py:469-471 */
   P3V_EPI_PATCH = 7,       /* out f32 row (m/P)*(P+1)+1+m%P = acc + pos[1+m%P]   phi.py:199-205 */
   P3V_EPI_F32 = 8,         /* out f32 = acc (+ bias if given)                               */
-  P3V_EPI_SCALE_RESID_F32 = 9 /* out f32 = resid_f32 + col_scale[n] * acc (a residual branch with a per-channel scale) */
+  P3V_EPI_SCALE_RESID_F32 = 9, /* out f32 = resid_f32 + col_scale[n] * acc (a residual branch with a per-channel scale) */
+  P3V_EPI_GELU_MUL = 10    /* as SILU_MUL with the tanh form of GELU: out bf16[M,N] = gelu(g)*u, fp32 up to the one rounding */
 };
 typedef struct {
   const uint16_t* A;   /* [M, lda] bf16 */
@@ -479,6 +480,57 @@ int p3v_attn_mix(const p3v_mix_args_t* args /* host */, void* stream);
 int p3v_attn_mix_decode(const p3v_mix_args_t* args /* host */, void* stream);
 int p3v_attn_mix_plan(int B, int L, int H, int G, int dim, int vdim, int n_keys, int f32);
 int64_t p3v_attn_mix_ws_bytes(int B, int L, int H, int vdim, int n_split);
+
+/* RMS norm of fp32 rows: out = x / sqrt(mean x^2 + eps) * w * gain, one rounding (out bf16, or fp32 with out_f32) */
+int p3v_rms_rows(const float* x, const uint16_t* w, void* out, int out_f32, int rows, int H, float eps, float gain, void* stream);
+/* p3v_gemv whose input row is p3v_rms_rows of the fp32 row x with args->norm_w, args->norm_eps (args->x unused).  M = 1, K in {1024, 2048,
+ * 3072, 4096, 8192}, epilogue NONE, SILU_MUL or GELU_MUL: otherwise P3V_ERR_UNSUPPORTED and the caller runs the two calls. */
+int p3v_gemv_rms(const p3v_gemv_args_t* args /* host */, const float* x, float gain, void* stream);
+
+/* Gated linear attention of B x L new tokens.  y rows [B*L, ld]: H*dim query, H*dim key, H*vdim value, H*vdim gate, rank low-rank
+ * decay columns, then anything.  Per head, fp32:
+ *   a = sigmoid(a2 . low-rank + a2_b)^(1/tau) per key channel,  S_t = diag(a_t) S_{t-1} + k_t v_t^T,  o_t = q_scale S_t^T q_t,
+ *   out row = rms(o over vdim) norm silu(gate).
+ * s [B, R, H, dim, vdim] fp32: the state behind t columns in slot t % R; a call reads slot past (zero for a sequence that starts at or
+ * behind column past: pad_len) and writes slot past + keep, keep in 0 .. L being how many of the tokens stay.
+ * n_chunk from p3v_gla_plan (0: token by token), ws of p3v_gla_ws_bytes. */
+typedef struct {
+  const void* y; const uint16_t* a2; const uint16_t* a2_b; const uint16_t* norm; float* s; void* out; float* ws;
+  const int32_t* pad_len; const int32_t* d_past;
+  float eps, tau, q_scale;
+  int B, L, H, dim, vdim, rank, ld, past, R, keep, n_chunk, f32;
+} p3v_gla_args_t;
+int p3v_gla(const p3v_gla_args_t* args /* host */, void* stream);
+int p3v_gla_plan(int B, int L, int H, int dim, int vdim, int f32);
+int64_t p3v_gla_ws_bytes(int B, int L, int H, int dim, int vdim, int n_chunk);
+
+/* Latent attention of B x L new tokens.  y rows [B*L, ld]: H*(dim + rot) query (per head dim unrotated, rot rotated), rank latent, rot
+ * shared rotated key, H*vdim gate columns, then anything.  Cache c [B, Tp, rankp + rotp]: per token the normed latent (rank, zeros up to
+ * rankp, a multiple of 64) and the rotated key part (rot, zeros up to rotp, a multiple of 32).
+ *   score_h = scale (q_nope . (uk_h c) + q_rot . k_rot), softmax over the keys pad_len[b] .. own position with exp(sink_h) added to the
+ *   denominator,  out = (sum p (uv_h c)) sigmoid(gate).
+ * Rotation: cos_t, sin_t [tab_n, rot / 2] fp32 by position (column - pad_len[b]), dimension i paired with i + rot / 2.
+ * Weights: uk [H*dim, rankp], uv [H*vdim, rankp] (zeros behind rank), ukt [H, rankp, dimp] = uk per head transposed (dimp % 32 == 0).
+ *   p3v_latent_append   rotates the queries in y and appends the new tokens to the cache (any sizes and types)
+ *   p3v_latent_any      attention behind it, any sizes and types, fp32 arithmetic
+ *   p3v_latent_rows     append and attention in the latent space, a few tokens per sequence; q [B*L, H up to 16s, rankp + rotp] scratch
+ *   p3v_latent_prompt   attention behind p3v_latent_append over expanded keys kx [B, n_keys, H*dim] and values vx [B, H*vdim, n_keys]
+ *                       (n_keys % 64 == 0, past + L <= n_keys <= Tp)
+ * p3v_latent_plan: > 0 p3v_latent_rows with the keys split that many ways (ws of p3v_latent_ws_bytes), 0 p3v_latent_any,
+ * < 0 p3v_latent_prompt.  n_keys of the plan: the cache capacity for L = 1, past + L otherwise. */
+typedef struct {
+  void* y; const uint16_t* c_norm; const uint16_t* uk; const uint16_t* ukt; const uint16_t* uv; const uint16_t* sink;
+  const float* cos_t; const float* sin_t; void* c; void* q; const void* kx; const void* vx; void* out; float* ws;
+  const int32_t* pad_len; const int32_t* d_past;
+  float eps, scale;
+  int B, L, H, dim, rot, vdim, rank, rankp, rotp, dimp, ld, past, Tp, tab_n, n_keys, n_split, f32;
+} p3v_latent_args_t;
+int p3v_latent_append(const p3v_latent_args_t* args /* host */, void* stream);
+int p3v_latent_any(const p3v_latent_args_t* args /* host */, void* stream);
+int p3v_latent_rows(const p3v_latent_args_t* args /* host */, void* stream);
+int p3v_latent_prompt(const p3v_latent_args_t* args /* host */, void* stream);
+int p3v_latent_plan(int B, int L, int H, int dim, int rot, int vdim, int rank, int n_keys, int f32);
+int64_t p3v_latent_ws_bytes(int B, int L, int H, int rank, int n_split);
 
 /* p3v_argmax / p3v_log_softmax / p3v_topk / p3v_step_end on fp32 logits */
 int p3v_argmax_f32(const float* logits, int32_t* out, int rows, int n, int64_t row_stride, void* stream);

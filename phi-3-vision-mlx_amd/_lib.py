@@ -14,7 +14,7 @@ LIB_PATH = os.environ.get("P3V_LIB") or os.path.join(_HERE, "libp3v.so")     # P
 
 P3V_OK = 0
 (EPI_NONE, EPI_BIAS, EPI_BIAS_QGELU, EPI_BIAS_GELU, EPI_BIAS_RESID_F32, EPI_RESID_BF16, EPI_SILU_MUL, EPI_PATCH,
- EPI_F32, EPI_SCALE_RESID_F32) = range(10)
+ EPI_F32, EPI_SCALE_RESID_F32, EPI_GELU_MUL) = range(11)
 DECODE_MAX_L = 16
 
 vp, i32, i64, f32 = C.c_void_p, C.c_int, C.c_int64, C.c_float
@@ -104,6 +104,19 @@ class MixArgs(C.Structure):
                 ("ld", i32), ("ld_first", i32), ("past", i32), ("Tp", i32), ("n_split", i32), ("f32", i32)]
 
 
+class GlaArgs(C.Structure):
+    _fields_ = [("y", vp), ("a2", vp), ("a2_b", vp), ("norm", vp), ("s", vp), ("out", vp), ("ws", vp), ("pad_len", vp), ("d_past", vp),
+                ("eps", f32), ("tau", f32), ("q_scale", f32), ("B", i32), ("L", i32), ("H", i32), ("dim", i32), ("vdim", i32), ("rank", i32),
+                ("ld", i32), ("past", i32), ("R", i32), ("keep", i32), ("n_chunk", i32), ("f32", i32)]
+
+
+class LatentArgs(C.Structure):
+    _fields_ = [("y", vp), ("c_norm", vp), ("uk", vp), ("ukt", vp), ("uv", vp), ("sink", vp), ("cos_t", vp), ("sin_t", vp), ("c", vp), ("q", vp),
+                ("kx", vp), ("vx", vp), ("out", vp), ("ws", vp), ("pad_len", vp), ("d_past", vp), ("eps", f32), ("scale", f32),
+                ("B", i32), ("L", i32), ("H", i32), ("dim", i32), ("rot", i32), ("vdim", i32), ("rank", i32), ("rankp", i32), ("rotp", i32),
+                ("dimp", i32), ("ld", i32), ("past", i32), ("Tp", i32), ("tab_n", i32), ("n_keys", i32), ("n_split", i32), ("f32", i32)]
+
+
 # name -> (restype, argtypes); must list every symbol include/p3v.h declares
 SIGNATURES = {
     "p3v_version": (i32, []),
@@ -165,6 +178,17 @@ SIGNATURES = {
     "p3v_attn_mix_decode": (i32, [C.POINTER(MixArgs), vp]),
     "p3v_attn_mix_plan": (i32, [i32, i32, i32, i32, i32, i32, i32, i32]),
     "p3v_attn_mix_ws_bytes": (i64, [i32, i32, i32, i32, i32]),
+    "p3v_rms_rows": (i32, [vp, vp, vp, i32, i32, i32, f32, f32, vp]),
+    "p3v_gemv_rms": (i32, [C.POINTER(GemvArgs), vp, f32, vp]),
+    "p3v_gla": (i32, [C.POINTER(GlaArgs), vp]),
+    "p3v_gla_plan": (i32, [i32, i32, i32, i32, i32, i32]),
+    "p3v_gla_ws_bytes": (i64, [i32, i32, i32, i32, i32, i32]),
+    "p3v_latent_append": (i32, [C.POINTER(LatentArgs), vp]),
+    "p3v_latent_any": (i32, [C.POINTER(LatentArgs), vp]),
+    "p3v_latent_rows": (i32, [C.POINTER(LatentArgs), vp]),
+    "p3v_latent_prompt": (i32, [C.POINTER(LatentArgs), vp]),
+    "p3v_latent_plan": (i32, [i32, i32, i32, i32, i32, i32, i32, i32, i32]),
+    "p3v_latent_ws_bytes": (i64, [i32, i32, i32, i32, i32]),
     "p3v_argmax_f32": (i32, [vp, vp, i32, i32, i64, vp]),
     "p3v_log_softmax_f32": (i32, [vp, vp, i32, i32, vp]),
     "p3v_topk_f32": (i32, [vp, vp, i32, i32, i32, i64, vp]),

@@ -1,7 +1,7 @@
 """Cache states: what one prompt batch (or one slot group of the engine) keeps on the device between calls."""
 import torch
 
-from .config import head_dim
+from .config import GlaMixer, LatentMixer, Mixer, head_dim
 from .ops import BF16, F32, I32
 
 
@@ -75,8 +75,9 @@ class CacheState:
         captured-prefill entry built on these buffers must not be reused (model._prefill_captured drops it)."""
         self.shared["dirty"] = True
 
-    def note_written(self, lo, hi):
-        """A call is about to write columns [lo, hi): states that keep a bounded history beside the cache check and record it."""
+    def note_written(self, lo, hi, kept=None):
+        """A call is about to write columns [lo, hi), of which [lo, kept) stay (None: all): states that keep a bounded history beside the
+        cache check and record it."""
 
     def row_view(self, rows, S, offset, epoch):
         """Batch rows `rows` (a slice) as a state of their own over the same memory, at cache column `offset`, for the prefill of
@@ -130,65 +131,162 @@ def round_up(n, m):
     return (n + m - 1) // m * m
 
 
-class LayeredCacheState(CacheState):
-    """State of a layered decoder (config.LayerSpec): per layer its own key / value sizes, in the layout of the mixed-head attention
+class KVRows:
+    """Keys and values of one attention layer: k [B, G, Tp, dimp], v [B, G, Tp / 16, vdimp, 16], the widths rounded up to 32 with zeros."""
+    recurrent = False
 
-        k[i]     [B, G, Tp, dimp]             dimp = dim rounded up to 32, vdimp = vdim rounded up to 32, the padding zero
-        v[i]     [B, G, Tp / 16, vdimp, 16]
+    def __init__(self, m, B, Tp, R, dt, device):
+        self.k = torch.zeros((B, m.kv_heads, Tp, round_up(m.dim, 32)), dtype=dt, device=device)
+        self.v = torch.zeros((B, m.kv_heads, Tp // 16, round_up(m.vdim, 32), 16), dtype=dt, device=device)
+
+    @staticmethod
+    def token_bytes(m, e):
+        return e * m.kv_heads * (round_up(m.dim, 32) + round_up(m.vdim, 32))
+
+    def rows(self, sel):
+        return self._of(k=self.k[sel], v=self.v[sel])
+
+    def beams(self, n, Tp):
+        return self._of(k=_repeat(self.k, n, 2, Tp), v=_repeat(self.v, n, 2, Tp // 16))
+
+    def scrub(self, lo, hi):
+        self.k[:, :, lo:hi] = 0
+        for c in range(lo, hi):
+            self.v[:, :, c // 16, :, c % 16] = 0
+
+    def _of(self, **kw):
+        new = type(self).__new__(type(self))
+        new.__dict__.update(kw)
+        return new
+
+
+class LatentRows(KVRows):
+    """Latent attention's cache: c [B, Tp, rankp + rotp], a row = the normed latent (rank, zeros up to a multiple of 64), then the
+    rotated key part all heads share (zeros up to a multiple of 32)."""
+
+    def __init__(self, m, B, Tp, R, dt, device):
+        self.c = torch.zeros((B, Tp, latent_width(m)), dtype=dt, device=device)
+        self.cos = self.sin = None                               # rotation tables [>= Tp, rot / 2] fp32 by position (the model sets them)
+
+    @staticmethod
+    def token_bytes(m, e):
+        return e * latent_width(m)
+
+    def rows(self, sel):
+        return self._of(c=self.c[sel], cos=self.cos, sin=self.sin)
+
+    def beams(self, n, Tp):
+        return self._of(c=_repeat(self.c, n, 1, Tp), cos=self.cos, sin=self.sin)
+
+    def scrub(self, lo, hi):
+        self.c[:, lo:hi] = 0
+
+
+class RecurrentRows(KVRows):
+    """A recurrent layer's states: s [B, R, H, dim, vdim] fp32, the state behind t columns in slot t % R."""
+    recurrent = True
+
+    def __init__(self, m, B, Tp, R, dt, device):
+        self.s = torch.zeros((B, R, m.heads, m.dim, m.vdim), dtype=F32, device=device)
+
+    @staticmethod
+    def token_bytes(m, e):
+        return 0
+
+    def rows(self, sel):
+        return self._of(s=self.s[sel])
+
+    def beams(self, n, Tp):
+        return self._of(s=self.s.repeat_interleave(n, dim=0))
+
+    def scrub(self, lo, hi):
+        pass                                                     # (a step replaces the whole state, out of the slot before)
+
+
+MIXER_ROWS = {Mixer: KVRows, LatentMixer: LatentRows, GlaMixer: RecurrentRows}
+
+
+def latent_width(m):
+    return round_up(m.rank, 64) + round_up(m.rot.dims, 32)
+
+
+def _repeat(t, n, dim, cols):
+    out = torch.zeros((t.shape[0] * n,) + t.shape[1:dim] + (cols,) + t.shape[dim + 1:], dtype=t.dtype, device=t.device)
+    src = min(cols, t.shape[dim])
+    out.narrow(dim, 0, src).copy_(t.narrow(dim, 0, src).repeat_interleave(n, dim=0))
+    return out
+
+
+class LayeredCacheState(CacheState):
+    """State of a layered decoder (config.LayerSpec): per layer what its mixer keeps (mix[i], also of a layer that uses another one's
+    weights), and with a token shift
+
         shift[i] [B, R, width] fp32           the mixer's unshifted inputs of the last R columns (column c in row c % R)
 
-    A cache is rewound by lowering `offset`; the token shift then needs the input of the token before, so the state keeps a ring of R
-    of them: a rewind of up to R - 1 tokens is exact, a longer one raises."""
+    A cache is rewound by lowering `offset`.  The token shift then needs the input of the token before, so the state keeps a ring of
+    shift_rows of them: a rewind of up to that many less one is exact.  A recurrent layer needs the state itself; the ring of state_rows
+    of them holds those behind the last calls (`held`).  Any other rewind raises."""
 
     def __init__(self, cfg, B, S, max_tokens, device):
         self.B, self.S, self.max_tokens = B, S, max_tokens
         self.T = S + max(max_tokens, 0)
         self.quantized = False
         self.Tp = padded_columns(self.T)
-        self.R = cfg.shift_rows
-        self.hist_max = 0
+        self.R, self.state_rows = cfg.shift_rows, cfg.state_rows
+        self.hist_max, self.held = 0, frozenset()
         dt = F32 if cfg.dtype == "float32" else BF16
-        self.k, self.v, self.shift = [], [], []
-        for ly in cfg.layers:
-            m = ly.mixer
-            self.k.append(torch.zeros((B, m.kv_heads, self.Tp, round_up(m.dim, 32)), dtype=dt, device=device))
-            self.v.append(torch.zeros((B, m.kv_heads, self.Tp // 16, round_up(m.vdim, 32), 16), dtype=dt, device=device))
-            self.shift.append(torch.zeros((B, self.R, cfg.hidden_size), dtype=F32, device=device))
+        self.mix = [MIXER_ROWS[type(ly.mixer)](ly.mixer, B, self.Tp, self.state_rows, dt, device) for ly in cfg.layers]
+        self.shift = [torch.zeros((B, self.R, cfg.hidden_size), dtype=F32, device=device) if cfg.design.token_shift else None for _ in cfg.layers]
         self._loop_state()
 
-    def note_written(self, lo, hi):
+    @property
+    def k(self):
+        return [m.k for m in self.mix]
+
+    @property
+    def v(self):
+        return [m.v for m in self.mix]
+
+    @property
+    def recurrent(self):
+        return any(m.recurrent for m in self.mix)
+
+    def note_written(self, lo, hi, kept=None):
+        """Columns [lo, hi) are about to be written, [lo, kept) of them to stay (None: all)."""
+        kept = hi if kept is None else kept
         if getattr(self, "slots", False) or getattr(self, "fresh_rows", False):
             return                                              # (every row's history is rewritten by its own prefill)
+        if self.recurrent and not lo <= kept <= hi:
+            raise ValueError(f"columns [{lo}, {hi}) of which {kept - lo} stay: a recurrent state cannot follow")
         if lo == 0:
-            self.hist_max = 0
-        elif lo <= self.hist_max - self.R:
+            self.hist_max, self.held = 0, frozenset((0,))
+        elif self.recurrent and lo not in self.held:
+            raise ValueError(f"cache rewound to {lo}: the recurrent states held are those behind {sorted(self.held)} columns")
+        elif self.shift[0] is not None and lo <= self.hist_max - self.R:
             raise ValueError(f"cache rewound to {lo}: the token-shift history holds the last {self.R} of {self.hist_max} columns")
         self.hist_max = max(self.hist_max, hi)
+        if kept > lo:
+            self.held = frozenset(t for t in self.held if t <= lo and (t - kept) % self.state_rows) | {kept}
 
     def _view_rows(self, view, rows):
-        view.__dict__.update(k=[t[rows] for t in self.k], v=[t[rows] for t in self.v], shift=[t[rows] for t in self.shift], R=self.R, hist_max=0)
+        view.__dict__.update(mix=[m.rows(rows) for m in self.mix], shift=[None if t is None else t[rows] for t in self.shift], R=self.R,
+                             state_rows=self.state_rows, hist_max=0, held=frozenset())
 
     def beams(self, n, L):
         """A scratch copy with every row repeated n times and room for L more columns (beam calls read the cache, never write it)."""
         view = type(self).__new__(type(self))
-        Tp = round_up(self.offset + L, 32)
-
-        def rep(t, dim, cols):
-            out = torch.zeros((self.B * n,) + t.shape[1:dim] + (cols,) + t.shape[dim + 1:], dtype=t.dtype, device=t.device)
-            src = min(cols, t.shape[dim])
-            out.narrow(dim, 0, src).copy_(t.narrow(dim, 0, src).repeat_interleave(n, dim=0))
-            return out
+        Tp = round_up(self.offset + L, 64)
         view.__dict__.update(B=self.B * n, S=self.S, max_tokens=self.max_tokens, T=Tp, Tp=Tp, quantized=False, offset=self.offset, graphs={},
-                             epoch=self.epoch, R=self.R, hist_max=self.hist_max, fresh_rows=True,
+                             epoch=self.epoch, R=self.R, state_rows=self.state_rows, hist_max=self.hist_max, held=self.held, fresh_rows=True,
                              pad_len=None if self.pad_len is None else self.pad_len.repeat_interleave(n),
-                             k=[rep(t, 2, Tp) for t in self.k], v=[rep(t, 2, Tp // 16) for t in self.v],
-                             shift=[t.repeat_interleave(n, dim=0) for t in self.shift])
+                             mix=[m.beams(n, Tp) for m in self.mix],
+                             shift=[None if t is None else t.repeat_interleave(n, dim=0) for t in self.shift])
         return view
 
     def scrub(self, lo, hi):
         hi = min(hi, self.Tp)
-        for k, v, h in zip(self.k, self.v, self.shift):
-            k[:, :, lo:hi] = 0
-            for c in range(lo, hi):
-                v[:, :, c // 16, :, c % 16] = 0
-                h[:, c % self.R] = 0
+        for m, h in zip(self.mix, self.shift):
+            m.scrub(lo, hi)
+            if h is not None:
+                for c in range(lo, hi):
+                    h[:, c % self.R] = 0

@@ -8,9 +8,9 @@ reference's own notebook (assets/su_rope_explained.ipynb, cell 9); a real
 """
 import json
 import math
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 from types import SimpleNamespace
-from typing import Optional
+from typing import Optional, Tuple, Union
 
 SHORT_FACTOR = [
     1.05, 1.05, 1.05, 1.1, 1.1, 1.1, 1.2500000000000002, 1.2500000000000002,
@@ -110,46 +110,150 @@ class Mixer:
 
 
 @dataclass(frozen=True)
+class Rotary:
+    """Rotary positions on `dims` dimensions, dimension i paired with i + dims / 2.  yarn: None, or (factor, original, fast, slow)."""
+    dims: int
+    base: float
+    yarn: Optional[Tuple[float, float, float, float]] = None
+
+    def frequencies(self):
+        """(angle per position of every pair, factor on cos and sin), float64."""
+        pair = range(self.dims // 2)
+        f = [self.base ** (-2.0 * i / self.dims) for i in pair]
+        if self.yarn is None:
+            return f, 1.0
+        factor, original, fast, slow = self.yarn
+
+        def dim_of(turns):
+            return self.dims * math.log(original / (2 * math.pi * turns)) / (2 * math.log(self.base))
+        lo, hi = max(math.floor(dim_of(fast)), 0), min(math.ceil(dim_of(slow)), self.dims - 1)
+        ramp = [min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0) for i in pair]
+        return [x / factor * r + x * (1 - r) for x, r in zip(f, ramp)], 0.1 * math.log(factor) + 1.0
+
+
+@dataclass(frozen=True)
+class LatentMixer:
+    """Latent attention: one latent of `rank` values and one rotated key part of `rot.dims` values per token, shared by the heads."""
+    heads: int
+    dim: int
+    vdim: int
+    rank: int
+    rot: Rotary
+    scale: float
+
+
+@dataclass(frozen=True)
+class GlaMixer:
+    """Gated linear attention: a [dim, vdim] state per head, a decay per key channel out of a low-rank projection.  gate_rank: its rank
+    (None: what the checkpoint's tensors have)."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    gate_rank: Optional[int] = None
+
+
+@dataclass(frozen=True)
 class Mlp:
     ff: int
 
 
 @dataclass(frozen=True)
 class LayerSpec:
-    mixer: Mixer
+    mixer: Union[Mixer, LatentMixer, GlaMixer]
     mlp: Optional[Mlp]
+    owner: Optional[int] = None                      # the layer whose tensors this one uses (None: its own)
 
 
-def _layer_spec(i, d):
-    if d["type"] != "attention":
-        raise ValueError(f"layer {i}: unknown mixer type {d['type']!r}")
-    m = d["mixer"]
+def _attention(i, m):
     mixer = Mixer(int(m["heads"]), int(m["kv_heads"]), int(m["dim"]), int(m["vdim"]), float(m["scale"]), bool(m["v_mix"]))
     if mixer.heads % mixer.kv_heads:
         raise ValueError(f"layer {i}: {mixer.heads} query heads over {mixer.kv_heads} key / value heads")
+    return mixer
+
+
+def _latent_attention(i, m):
+    rot, s = m["rot"], m["rot"].get("scaling")
+    if int(rot.get("dims", m["rot_dim"])) != int(m["rot_dim"]) or int(m["rot_dim"]) % 2:
+        raise ValueError(f"layer {i}: rotary dimensions {rot.get('dims')} of a rotated part of {m['rot_dim']}")
+    yarn = None if s is None else tuple(float(s[k]) for k in ("factor", "original", "fast", "slow"))
+    return LatentMixer(int(m["heads"]), int(m["dim"]), int(m["vdim"]), int(m["kv_rank"]), Rotary(int(m["rot_dim"]), float(rot["base"]), yarn),
+                       float(m["scale"]))
+
+
+def _gla(i, m):
+    return GlaMixer(int(m["heads"]), int(m["dim"]), int(m["vdim"]), float(m["tau"]), None if m.get("gate_rank") is None else int(m["gate_rank"]))
+
+
+@dataclass(frozen=True)
+class Design:
+    """What is the same in every model of a layered design: its mixers ('type' of a layer -> reader of its sizes), the norm in front of
+    a branch ("dyt" | "rms"), the activation of its feed-forward, what the branches carry, whether the head is the embedding table."""
+    mixers: dict
+    norm: str
+    act: str
+    token_shift: bool = False
+    layer_scale: bool = False
+    tied_head: bool = False
+
+
+DESIGNS = {
+    "Pelalix": Design({"attention": _attention}, norm="dyt", act="silu", token_shift=True, layer_scale=True),
+    "Pudisun": Design({"latent_attention": _latent_attention, "gla": _gla}, norm="rms", act="gelu_tanh", tied_head=True),
+}
+
+
+def _layer_spec(design, i, d):
+    if d["type"] not in design.mixers:
+        raise ValueError(f"layer {i}: unknown mixer type {d['type']!r}")
+    mixer = design.mixers[d["type"]](i, d["mixer"])
     mlp = d.get("mlp")
     if mlp is not None and mlp["kind"] != "dense":
         raise ValueError(f"layer {i}: unknown feed-forward kind {mlp['kind']!r}")
-    return LayerSpec(mixer, None if mlp is None else Mlp(int(mlp["ff"])))
+    return LayerSpec(mixer, None if mlp is None else Mlp(int(mlp["ff"])), d.get("weights_of"))
 
 
-def layered_config(d, dtype=None, shift_rows=128, **kwargs):
-    """config.json of a layered decoder -> SimpleNamespace.  dtype: "bfloat16" (default) or "float32" activations; shift_rows: columns of
-    token-shift history a state keeps (how far a cache can be rewound)."""
+def _resolve_owners(layers):
+    """Layers that use another one's tensors name the layer that has them."""
+    out = []
+    for i, s in enumerate(layers):
+        j, seen = s.owner, {i}
+        while j is not None and 0 <= j < len(layers) and j not in seen and layers[j].owner is not None:
+            seen.add(j)
+            j = layers[j].owner
+        if j is not None:
+            if not 0 <= j < len(layers) or j in seen:
+                raise ValueError(f"layer {i}: no layer has the weights it names ({s.owner})")
+            if (layers[j].mixer, layers[j].mlp) != (s.mixer, s.mlp):
+                raise ValueError(f"layer {i}: other sizes than layer {j}, whose weights it uses")
+        out.append(replace(s, owner=j))
+    return tuple(out)
+
+
+def layered_config(d, dtype=None, shift_rows=128, state_rows=2, **kwargs):
+    """config.json of a layered decoder -> SimpleNamespace.  dtype: "bfloat16" (default) or "float32" activations; shift_rows /
+    state_rows: columns of token-shift history / recurrent states a cache keeps (how far it can be rewound)."""
     for k in ("use_quantized_cache", "quantized_fp8", "quantized_int4"):
         if kwargs.pop(k, False):
             raise ValueError(f"{k} is not available for {d['architecture']}")
     if dtype not in (None, "bfloat16", "float32"):
         raise ValueError(f"dtype must be 'bfloat16' or 'float32', got {dtype!r}")
-    layers = tuple(_layer_spec(i, x) for i, x in enumerate(d["layers"]))
-    mixing = {s.mixer.kv_heads * s.mixer.vdim for s in layers if s.mixer.v_mix}
+    if d["architecture"] not in DESIGNS:
+        raise ValueError(f"unknown architecture {d['architecture']!r}")
+    design = DESIGNS[d["architecture"]]
+    layers = _resolve_owners([_layer_spec(design, i, x) for i, x in enumerate(d["layers"])])
+    mixing = {s.mixer.kv_heads * s.mixer.vdim for s in layers if getattr(s.mixer, "v_mix", False)}
     if len(mixing) > 1:
         raise ValueError(f"value-mixing layers of different value widths {sorted(mixing)}")
     if not layers:
         raise ValueError("a model without layers")
-    return SimpleNamespace(architectures=[d["architecture"]], layers=layers, num_hidden_layers=len(layers), hidden_size=int(d["width"]),
-                           vocab_size=int(d["vocab"]), norm_eps=float(d["norm"]["eps"]), embed_scale=float(d["embedding"]["scale"]),
-                           dtype=dtype or "bfloat16", shift_rows=int(shift_rows), **kwargs)
+    if float(d.get("residual_mult", 1.0)) == 0.0:
+        raise ValueError("residual_mult 0: the layers would not reach the output")
+    return SimpleNamespace(architectures=[d["architecture"]], design=design, layers=layers, num_hidden_layers=len(layers),
+                           hidden_size=int(d["width"]), vocab_size=int(d["vocab"]), norm_eps=float(d["norm"]["eps"]),
+                           embed_scale=float(d.get("embedding", {}).get("scale", 1.0)), residual_mult=float(d.get("residual_mult", 1.0)),
+                           logit_scale=float(d.get("logit_scale", 1.0)), dtype=dtype or "bfloat16", shift_rows=int(shift_rows),
+                           state_rows=int(state_rows), **kwargs)
 
 
 def load_config(json_path, **kwargs):

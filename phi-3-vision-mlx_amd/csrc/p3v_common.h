@@ -59,6 +59,20 @@ __device__ __forceinline__ void p3v_rope_pair(float a, float b, float cs, float 
 // the gate_up epilogue gains nothing from it (205 vs 203 us).
 __device__ __forceinline__ float p3v_sigmoid(float x) { return __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 
+// Gated feed-forward epilogues (W = [gate; up]): act(gate) * up of fp32 sums, before the one rounding that follows.
+//  SiLU: every intermediate rounded to bf16, as the reference's array expression rounds it (phi.py:469-471)
+//  GELU (tanh form): 0.5 g (1 + tanh(sqrt(2/pi) (g + 0.044715 g^3))) in fp32 = g sigmoid(2 u): no cancellation for any g
+#define P3V_GATED(epi) ((epi) == P3V_EPI_SILU_MUL || (epi) == P3V_EPI_GELU_MUL)
+__device__ __forceinline__ float p3v_gelu_tanh(float g) {
+  const float u = 0.7978845608028654f * (g + 0.044715f * g * g * g);
+  return g / (1.f + __expf(-2.f * u));
+}
+__device__ __forceinline__ float p3v_gated(int epi, float gate, float up) {
+  if (epi == P3V_EPI_GELU_MUL) return p3v_gelu_tanh(gate) * up;
+  const float g = bf16_round(gate), u = bf16_round(up);
+  return bf16_round(g * bf16_round(1.f / (1.f + __expf(-g)))) * u;
+}
+
 // nn.RMSNorm = mx.fast.rms_norm (phi.py:478-479, 571): w * astype(x * rsqrt(mean x^2 + eps), bf16) -- the normalised value is
 // rounded to bf16 BEFORE the weight multiply, which rounds again (HF's Phi3RMSNorm does the same).  One bf16 pair at a time.
 __device__ __forceinline__ uint32_t rms_pair(uint32_t x2, float r, uint32_t g2) {

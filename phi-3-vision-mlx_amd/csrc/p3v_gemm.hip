@@ -59,7 +59,7 @@ __device__ __forceinline__ void store8_bf16(bf16_t* p, const float* v) {
 
 template <int EPI, int ORD = 0>
 __global__ void __launch_bounds__(256, 2) k_gemm(GemmP p) {
-  constexpr bool SILU = EPI == P3V_EPI_SILU_MUL, QKV = EPI == P3V_EPI_QKV;
+  constexpr bool SILU = P3V_GATED(EPI), QKV = EPI == P3V_EPI_QKV;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);   // uniform: LDS-DMA bases stay in SGPRs
   const int wr = wave >> 1, wc = wave & 1;
@@ -210,11 +210,7 @@ __global__ void __launch_bounds__(256, 2) k_gemm(GemmP p) {
       for (int j = 0; j < 2; ++j) {
         float o4[4];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          // reference rounds gate/up to bf16 (Linear output) and every elementwise op after it (phi.py:469-471)
-          const float g = bf16_round(acc[i][j][r]), u = bf16_round(acc[i][2 + j][r]);
-          o4[r] = bf16_round(g * bf16_round(1.f / (1.f + __expf(-g)))) * u;
-        }
+        for (int r = 0; r < 4; ++r) o4[r] = p3v_gated(EPI, acc[i][j][r], acc[i][2 + j][r]);
         pk[j][0] = pack_bf16x2(o4[0], o4[1]), pk[j][1] = pack_bf16x2(o4[2], o4[3]);
       }
       u32x4_t w;
@@ -312,7 +308,7 @@ static int launch_gemm_v(const GemmP& p, hipStream_t s) {
       return P3V_ERR_HIP;
     attr_set = true;
   }
-  const int n_tile = EPI == P3V_EPI_SILU_MUL ? BN / 2 : BN;
+  const int n_tile = P3V_GATED(EPI) ? BN / 2 : BN;
   dim3 grid(p3v_cdiv(p.N, n_tile), p3v_cdiv(p.M, BM), p.kslice ? p.K / p.kslice : 1);
   hipLaunchKernelGGL((k_gemm<EPI, ORD>), grid, dim3(256), GEMM_LDS, s, p);
   P3V_CHECK_LAUNCH();
@@ -331,7 +327,7 @@ static int gemm128(const p3v_gemm_args_t* a, hipStream_t s);
 // PFLOP/s), a last round that leaves every CU at most one small workgroup 0.42 -- pick the cheapest whole-round
 // packing, e.g. 2531 x 16384 (gate_up): 8 x 64 = 512 big tiles = 2 rounds + 4 x 128 small = 1 round.
 static int gemm_big_rows(const p3v_gemm_args_t* a) {
-  const int n_big = a->epilogue == P3V_EPI_SILU_MUL ? 128 : 256, n_small = n_big / 2;
+  const int n_big = P3V_GATED(a->epilogue) ? 128 : 256, n_small = n_big / 2;
   if (a->M < 1024 || a->N % n_big || a->epilogue == P3V_EPI_PATCH) return 0;
   if (const int force = p3v_tuning().gemm_big_rows; force >= 0) return min(force / 256 * 256, a->M);   // tests: pin the split
   const int mt = p3v_cdiv(a->M, 256), nt_big = a->N / n_big, nt_small = p3v_cdiv(a->N, n_small);
@@ -362,7 +358,7 @@ static int gemm_big_rows(const p3v_gemm_args_t* a) {
 template <int EPI>
 __global__ void __launch_bounds__(256) k_splitk_reduce(const float* __restrict__ part, void* __restrict__ out, const void* __restrict__ resid,
                                                        const bf16_t* __restrict__ col_scale, int M, int N, int ldp, int ldo, int S) {
-  constexpr bool SILU = EPI == P3V_EPI_SILU_MUL;             // part holds [gate | up] columns (2N), out N columns
+  constexpr bool SILU = P3V_GATED(EPI);             // part holds [gate | up] columns (2N), out N columns
   const int per_row = N / 8;
   const long i = (long)blockIdx.x * 256 + threadIdx.x;
   if (i >= (long)M * per_row) return;
@@ -380,10 +376,7 @@ __global__ void __launch_bounds__(256) k_splitk_reduce(const float* __restrict__
   const size_t o = (size_t)m * ldo + n;
   if (SILU) {
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const float g = bf16_round(v[e]), up = bf16_round(u[e]);
-      v[e] = bf16_round(g * bf16_round(1.f / (1.f + __expf(-g)))) * up;
-    }
+    for (int e = 0; e < 8; ++e) v[e] = p3v_gated(EPI, v[e], u[e]);
   } else if (EPI == P3V_EPI_RESID_BF16) {
     float r[8];
     load8_bf16((const bf16_t*)resid + o, r);
@@ -463,7 +456,7 @@ __global__ void __launch_bounds__(384) k_splitk_reduce_norm(const float* __restr
 // number of K slices for a shape (1 = not a split-K shape)
 static int splitk_slices(int M, int N, int K, int epilogue) {
   const P3vTuning& t = p3v_tuning();
-  const bool silu = epilogue == P3V_EPI_SILU_MUL;
+  const bool silu = P3V_GATED(epilogue);
   if (t.gemm_no_splitk || M <= 16 || M > t.gemm_splitk_max_m /* beyond, every projection has >= 256 tiles anyway */ ||
       N % 128 || K % 512)
     return 1;
@@ -483,7 +476,7 @@ extern "C" int64_t p3v_gemm_ws_bytes(int M, int N, int K, int epilogue) {
   const int sk = p3v_gemm_skinny_slices(M, N, K, epilogue);
   const int S = sk ? sk : splitk_slices(M, N, K, epilogue);
   if (S == 1) return 0;
-  return (int64_t)S * M * (epilogue == P3V_EPI_SILU_MUL ? 2 * N : N) * 4;
+  return (int64_t)S * M * (P3V_GATED(epilogue) ? 2 * N : N) * 4;
 }
 
 // ---- out = resid + bf16(A W^T) and normed = RMSNorm(out) (include/p3v.h): only where the projection runs as K slices anyway
@@ -507,11 +500,13 @@ extern "C" int p3v_gemm_resid_norm(const p3v_gemm_args_t* a, const uint16_t* nor
 
 // the second launch of a split: adds the S fp32 partials [S, M, W rows] in slice order and applies the epilogue
 int p3v_splitk_reduce(const float* part, const p3v_gemm_args_t* a, int S, hipStream_t s) {
-  const bool silu = a->epilogue == P3V_EPI_SILU_MUL;
+  const bool silu = P3V_GATED(a->epilogue);
   const int w_rows = silu ? 2 * a->N : a->N;
   const long items = (long)a->M * (a->N / 8);
   const dim3 grid((unsigned)p3v_cdiv(items, 256));
-  if (silu) hipLaunchKernelGGL(k_splitk_reduce<P3V_EPI_SILU_MUL>, grid, dim3(256), 0, s, part, a->out, a->resid, a->col_scale, a->M, a->N, w_rows, a->ldo, S);
+  if (a->epilogue == P3V_EPI_GELU_MUL)
+    hipLaunchKernelGGL(k_splitk_reduce<P3V_EPI_GELU_MUL>, grid, dim3(256), 0, s, part, a->out, a->resid, a->col_scale, a->M, a->N, w_rows, a->ldo, S);
+  else if (silu) hipLaunchKernelGGL(k_splitk_reduce<P3V_EPI_SILU_MUL>, grid, dim3(256), 0, s, part, a->out, a->resid, a->col_scale, a->M, a->N, w_rows, a->ldo, S);
   else if (a->epilogue == P3V_EPI_SCALE_RESID_F32)
     hipLaunchKernelGGL(k_splitk_reduce<P3V_EPI_SCALE_RESID_F32>, grid, dim3(256), 0, s, part, a->out, a->resid, a->col_scale, a->M, a->N, w_rows, a->ldo, S);
   else if (a->epilogue == P3V_EPI_RESID_BF16)
@@ -523,7 +518,7 @@ int p3v_splitk_reduce(const float* part, const p3v_gemm_args_t* a, int S, hipStr
 
 // returns P3V_ERR_UNSUPPORTED when the shape is not one for split-K (or the caller gave no workspace for it)
 static int gemm_splitk(const p3v_gemm_args_t* a, hipStream_t s) {
-  const bool silu = a->epilogue == P3V_EPI_SILU_MUL;
+  const bool silu = P3V_GATED(a->epilogue);
   const int S = splitk_slices(a->M, a->N, a->K, a->epilogue);
   if (S == 1) return P3V_ERR_UNSUPPORTED;
   const int w_rows = silu ? 2 * a->N : a->N;
@@ -544,11 +539,11 @@ extern "C" int p3v_gemm(const p3v_gemm_args_t* a, void* stream) {
     return P3V_ERR_ARG;
   if ((a->epilogue == P3V_EPI_BIAS_RESID_F32 || a->epilogue == P3V_EPI_RESID_BF16) && !a->resid) return P3V_ERR_ARG;
   if (a->epilogue == P3V_EPI_PATCH && (!a->pos || a->patches_per_img <= 0)) return P3V_ERR_ARG;
-  if (a->epilogue < 0 || a->epilogue > P3V_EPI_SCALE_RESID_F32) return P3V_ERR_ARG;
+  if (a->epilogue < 0 || a->epilogue > P3V_EPI_GELU_MUL) return P3V_ERR_ARG;
   if (a->epilogue == P3V_EPI_SCALE_RESID_F32 && (!a->resid || !a->col_scale || ((uintptr_t)a->col_scale & 15) || a->bias)) return P3V_ERR_ARG;
   if (a->M == 0) return P3V_OK;
   {                                                            // operands are addressed with 32-bit byte offsets (buffer loads)
-    const size_t w_rows = (size_t)a->N * (a->epilogue == P3V_EPI_SILU_MUL ? 2 : 1);
+    const size_t w_rows = (size_t)a->N * (P3V_GATED(a->epilogue) ? 2 : 1);
     if ((size_t)a->M * a->lda * 2 >= (1ull << 32) || w_rows * a->ldw * 2 >= (1ull << 32)) return P3V_ERR_UNSUPPORTED;
   }
   hipStream_t s = (hipStream_t)stream;
@@ -592,6 +587,7 @@ static int gemm128(const p3v_gemm_args_t* a, hipStream_t s) {
     case P3V_EPI_BIAS_RESID_F32: return launch_gemm<P3V_EPI_BIAS_RESID_F32>(p, s);
     case P3V_EPI_RESID_BF16: return launch_gemm<P3V_EPI_RESID_BF16>(p, s);
     case P3V_EPI_SILU_MUL: return launch_gemm<P3V_EPI_SILU_MUL>(p, s);
+    case P3V_EPI_GELU_MUL: return launch_gemm<P3V_EPI_GELU_MUL>(p, s);
     case P3V_EPI_PATCH: return launch_gemm<P3V_EPI_PATCH>(p, s);
     case P3V_EPI_F32: return launch_gemm<P3V_EPI_F32>(p, s);
     case P3V_EPI_SCALE_RESID_F32: return launch_gemm<P3V_EPI_SCALE_RESID_F32>(p, s);

@@ -38,7 +38,7 @@ extern "C" int p3v_g256dbg_read(unsigned long long* out) {
 #endif
 template <int EPI, int SCHED = 0x50, int ORDER = 0>
 __global__ void __launch_bounds__(512, 1) k_gemm256(Gemm256P p) {
-  constexpr bool SILU = EPI == P3V_EPI_SILU_MUL, QKV = EPI == P3V_EPI_QKV;
+  constexpr bool SILU = P3V_GATED(EPI), QKV = EPI == P3V_EPI_QKV;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);   // uniform: LDS-DMA bases stay in SGPRs
   const int wr = wave >> 2, wc = wave & 3;
@@ -278,7 +278,7 @@ static int launch_gemm256_v(const Gemm256P& p, hipStream_t s) {
       return P3V_ERR_HIP;
     attr_set = true;
   }
-  const int n_tile = EPI == P3V_EPI_SILU_MUL ? TN / 2 : TN;
+  const int n_tile = P3V_GATED(EPI) ? TN / 2 : TN;
   static int n_cu = 0;
   if (!n_cu) {
     int dev = 0;
@@ -307,9 +307,9 @@ int p3v_gemm256_qkv(const p3v_gemm_args_t* a, const QkvP& q, hipStream_t s) {
 
 // called by p3v_gemm (which decides how many rows get the big tile); returns P3V_ERR_UNSUPPORTED to fall back
 int p3v_gemm256_try(const p3v_gemm_args_t* a, hipStream_t s) {
-  const int n_tile = a->epilogue == P3V_EPI_SILU_MUL ? TN / 2 : TN;
+  const int n_tile = P3V_GATED(a->epilogue) ? TN / 2 : TN;
   if (a->N % n_tile || a->K % TK || a->epilogue == P3V_EPI_PATCH) return P3V_ERR_UNSUPPORTED;
-  const size_t w_rows = (size_t)a->N * (a->epilogue == P3V_EPI_SILU_MUL ? 2 : 1);
+  const size_t w_rows = (size_t)a->N * (P3V_GATED(a->epilogue) ? 2 : 1);
   if (w_rows * a->ldw * 2 >= ((size_t)1 << 32) || (size_t)256 * a->lda * 2 >= ((size_t)1 << 31)) return P3V_ERR_UNSUPPORTED;  // 32-bit buffer offsets
   const Gemm256P p = {a->A, a->W, a->out, a->epilogue == P3V_EPI_SCALE_RESID_F32 ? a->col_scale : a->bias, a->resid, a->M, a->N, a->K, a->lda, a->ldw, a->ldo, {}};
   switch (a->epilogue) {
@@ -320,6 +320,7 @@ int p3v_gemm256_try(const p3v_gemm_args_t* a, hipStream_t s) {
     case P3V_EPI_BIAS_RESID_F32: return launch_gemm256<P3V_EPI_BIAS_RESID_F32>(p, s);
     case P3V_EPI_RESID_BF16: return launch_gemm256<P3V_EPI_RESID_BF16>(p, s);
     case P3V_EPI_SILU_MUL: return launch_gemm256<P3V_EPI_SILU_MUL>(p, s);
+    case P3V_EPI_GELU_MUL: return launch_gemm256<P3V_EPI_GELU_MUL>(p, s);
     case P3V_EPI_F32: return launch_gemm256<P3V_EPI_F32>(p, s);
     case P3V_EPI_SCALE_RESID_F32: return launch_gemm256<P3V_EPI_SCALE_RESID_F32>(p, s);
     default: return P3V_ERR_UNSUPPORTED;

@@ -31,7 +31,7 @@ __device__ __forceinline__ float gelu_erf2(float x) { return 0.5f * x * (1.f + e
 // acc[i][j]: block row i (16 output rows), block column j (16 W rows) of the wave's 128 x 64 sub-tile at (wr, wc) of the tile at (m0, n0).
 template <int EPI>
 __device__ __forceinline__ void gemm256_epilogue(const Gemm256P& p, f32x4_t (&acc)[8][4], int m0, int n0, int wr, int wc, int lane) {
-  constexpr bool SILU = EPI == P3V_EPI_SILU_MUL;
+  constexpr bool SILU = P3V_GATED(EPI);
   const int fc = lane & 15, fq = lane >> 4;
   const int mrow0 = m0 + wr * 128 + fc;                                  // + i * 16
 #if defined(P3V_G256_ABL) && P3V_G256_ABL == 3                  // timing experiment: no epilogue at all
@@ -52,8 +52,7 @@ __device__ __forceinline__ void gemm256_epilogue(const Gemm256P& p, f32x4_t (&ac
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           // reference rounds gate/up to bf16 (Linear output) and every elementwise op after it (phi.py:469-471)
-          const float g = bf16_round(acc[i][j][r]), u = bf16_round(acc[i][2 + j][r]);
-          o4[r] = bf16_round(g * bf16_round(1.f / (1.f + __expf(-g)))) * u;
+          o4[r] = p3v_gated(EPI, acc[i][j][r], acc[i][2 + j][r]);
         }
         pk[j][0] = pack_bf16x2(o4[0], o4[1]), pk[j][1] = pack_bf16x2(o4[2], o4[3]);
       }

@@ -144,8 +144,7 @@ __global__ void __launch_bounds__(NW * 64, 1) k_gemm_rows(RowsP p) {
           dst[n] = v0;
           if (SILU) dst[p.N + n] = v1;
         } else if (SILU) {
-          const float gt = bf16_round(v0), up = bf16_round(v1);
-          ((bf16_t*)p.out)[(size_t)m * p.ldo + n] = f32_to_bf16(bf16_round(gt * bf16_round(1.f / (1.f + __expf(-gt)))) * up);
+          ((bf16_t*)p.out)[(size_t)m * p.ldo + n] = f32_to_bf16(p3v_gated(p.epi, v0, v1));
         } else if (p.epi == P3V_EPI_RESID_BF16) {
           ((bf16_t*)p.out)[(size_t)m * p.ldo + n] = f32_to_bf16(bf16_to_f32(p.resid[(size_t)m * p.ldo + n]) + bf16_round(v0));
         } else {
@@ -164,7 +163,7 @@ __global__ void __launch_bounds__(NW * 64, 1) k_gemm_rows(RowsP p) {
 struct RowsPlan { int S, NW, NST; };
 static RowsPlan rows_plan(int M, int N, int K, int epilogue) {
   const P3vTuning& t = p3v_tuning();
-  const bool silu = epilogue == P3V_EPI_SILU_MUL;
+  const bool silu = P3V_GATED(epilogue);
   RowsPlan none = {0, 0, 0};
   if (!t.gemm_rows || M <= 8 || M > 32 || N % (silu ? 8 : 16)) return none;
   const bool scaled = epilogue == P3V_EPI_SCALE_RESID_F32;                         // (its epilogue is the reduction launch's)
@@ -198,7 +197,7 @@ static int launch_rows_mt(const RowsP& p, int S, hipStream_t s) {
 int p3v_gemm_rows_launch(const p3v_gemm_args_t* a, float* part, hipStream_t s) {
   const RowsPlan pl = rows_plan(a->M, a->N, a->K, a->epilogue);
   if (pl.S == 0 || a->bias || (pl.S > 1) != (part != nullptr)) return P3V_ERR_UNSUPPORTED;
-  const bool silu = a->epilogue == P3V_EPI_SILU_MUL;
+  const bool silu = P3V_GATED(a->epilogue);
   const RowsP p = {a->A, a->W, a->out, (const bf16_t*)a->resid, part, a->M, a->N, a->K, a->lda, a->ldw, a->ldo, a->epilogue,
                    a->N / (silu ? 8 : 16), silu ? 2 * a->N : a->N};
   if (pl.S == 1) return silu ? launch_rows_mt<true, 4, 3, false>(p, 1, s) : launch_rows_mt<false, 4, 3, false>(p, 1, s);

@@ -78,7 +78,7 @@ template <int EPI, bool PART, int TN, int TM = SK_BM>
 __global__ void __launch_bounds__(512, 1) k_gemm_skinny(SkinnyP p) {
   typedef SkCfg<TN, TM> C;
   static_assert(TM == SK_BM || EPI != P3V_EPI_QKV, "the qkv epilogue's V tiles are 128 dimensions tall");
-  constexpr bool SILU = EPI == P3V_EPI_SILU_MUL;
+  constexpr bool SILU = P3V_GATED(EPI);
   constexpr int NS = C::NS, NI = C::NI;
   static_assert(NS - 2 <= 4 && (NS - 2) * C::PER < 64, "sk_wait_stages covers 4 stages in flight");
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
@@ -255,11 +255,7 @@ __global__ void __launch_bounds__(512, 1) k_gemm_skinny(SkinnyP p) {
       for (int j = 0; j < 2; ++j) {
         float o4[4];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          // reference rounds gate/up to bf16 (Linear output) and every elementwise op after it (phi.py:469-471)
-          const float g = bf16_round(acc[i][j][r]), u = bf16_round(acc[i][2 + j][r]);
-          o4[r] = bf16_round(g * bf16_round(1.f / (1.f + __expf(-g)))) * u;
-        }
+        for (int r = 0; r < 4; ++r) o4[r] = p3v_gated(EPI, acc[i][j][r], acc[i][2 + j][r]);
         pk[j][0] = pack_bf16x2(o4[0], o4[1]), pk[j][1] = pack_bf16x2(o4[2], o4[3]);
       }
       u32x4_t w;
@@ -333,7 +329,7 @@ int p3v_gemm_skinny_slices(int M, int N, int K, int epilogue) {
 }
 static int sk_slices(int M, int N, int K, int epilogue) {
   const P3vTuning& t = p3v_tuning();
-  const bool silu = epilogue == P3V_EPI_SILU_MUL;
+  const bool silu = P3V_GATED(epilogue);
   if (t.gemm_no_skinny || M <= 8 || M > t.gemm_skinny_max_m || K % SK_BK || N % (silu ? 32 : 64)) return 0;
   if (epilogue != P3V_EPI_NONE && epilogue != P3V_EPI_RESID_BF16 && epilogue != P3V_EPI_SCALE_RESID_F32 && !silu) return 0;
   const int tiles = p3v_cdiv(M, SK_BM) * ((silu ? 2 * N : N) / SK_TN);
@@ -354,7 +350,7 @@ static int launch_skinny_tm(const SkinnyP& p, int S, hipStream_t s) {
     if (hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, C::LDS) != hipSuccess) return P3V_ERR_HIP;
     attr_set[part] = true;
   }
-  const int n_tile = EPI == P3V_EPI_SILU_MUL ? SK_TN / 2 : SK_TN;
+  const int n_tile = P3V_GATED(EPI) ? SK_TN / 2 : SK_TN;
   const dim3 grid(p.N / n_tile, p3v_cdiv(p.M, TM), S);
   if (part) hipLaunchKernelGGL((k_gemm_skinny<EPI, true, SK_TN, TM>), grid, dim3(512), C::LDS, s, p);
   else hipLaunchKernelGGL((k_gemm_skinny<EPI, false, SK_TN, TM>), grid, dim3(512), C::LDS, s, p);
@@ -372,7 +368,7 @@ int p3v_splitk_reduce(const float* part, const p3v_gemm_args_t* a, int S, hipStr
 // the K-slice launch alone (fp32 partials into a->ws; *S_out slices): P3V_ERR_UNSUPPORTED, nothing launched, unless the shape is
 // one this kernel splits and the workspace holds the partials
 int p3v_gemm_skinny_partials(const p3v_gemm_args_t* a, int* S_out, hipStream_t s) {
-  const bool silu = a->epilogue == P3V_EPI_SILU_MUL;
+  const bool silu = P3V_GATED(a->epilogue);
   const int w_rows = silu ? 2 * a->N : a->N;
   const int RS = a->bias ? 0 : p3v_gemm_rows_slices(a->M, a->N, a->K, a->epilogue);
   if (RS > 1 && a->ws && a->ws_bytes >= (int64_t)RS * a->M * w_rows * 4) {        // 9 .. 32 rows: the register-streaming kernel's K slices
@@ -386,7 +382,7 @@ int p3v_gemm_skinny_partials(const p3v_gemm_args_t* a, int* S_out, hipStream_t s
   if ((uintptr_t)a->ws & 15) return P3V_ERR_ARG;
   *S_out = S;
   const SkinnyP p = {a->A, a->W, a->ws, a->resid, a->M, a->N, a->K, a->lda, a->ldw, a->ldo, a->col_scale, a->K / S, {}};
-  if (silu) return launch_skinny<P3V_EPI_SILU_MUL>(p, S, s);
+  if (silu) return launch_skinny<P3V_EPI_SILU_MUL>(p, S, s);                       // (partials: the activation is the reduction's)
   if (a->epilogue == P3V_EPI_RESID_BF16) return launch_skinny<P3V_EPI_RESID_BF16>(p, S, s);
   return launch_skinny<P3V_EPI_NONE>(p, S, s);
 }
@@ -407,6 +403,7 @@ int p3v_gemm_skinny_try(const p3v_gemm_args_t* a, hipStream_t s) {
   const SkinnyP p = {a->A, a->W, a->out, a->resid, a->M, a->N, a->K, a->lda, a->ldw, a->ldo, a->col_scale, 0, {}};
   if (a->epilogue == P3V_EPI_SCALE_RESID_F32) return launch_skinny<P3V_EPI_SCALE_RESID_F32>(p, 1, s);
   if (a->epilogue == P3V_EPI_SILU_MUL) return launch_skinny<P3V_EPI_SILU_MUL>(p, 1, s);
+  if (a->epilogue == P3V_EPI_GELU_MUL) return launch_skinny<P3V_EPI_GELU_MUL>(p, 1, s);
   if (a->epilogue == P3V_EPI_RESID_BF16) return launch_skinny<P3V_EPI_RESID_BF16>(p, 1, s);
   return launch_skinny<P3V_EPI_NONE>(p, 1, s);
 }

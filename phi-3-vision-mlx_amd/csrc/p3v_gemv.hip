@@ -53,7 +53,7 @@ __global__ void __launch_bounds__(256) k_gemv(GemvP p) {
   }
   __syncthreads();
 
-  const bool silu = p.epi == P3V_EPI_SILU_MUL;
+  const bool silu = P3V_GATED(p.epi);
   const int n_waves = gridDim.x * 4;
   for (int u = blockIdx.x * 4 + wave; u < p.units; u += n_waves) {
     const int r0 = silu ? u : 2 * u;
@@ -93,9 +93,7 @@ __global__ void __launch_bounds__(256) k_gemv(GemvP p) {
       for (int m = 0; m < MT; ++m) {
         if (m >= p.M) break;
         if (silu) {
-          const float g = bf16_round(a0[m]), up = bf16_round(a1[m]);
-          const float s = bf16_round(g * bf16_round(1.f / (1.f + __expf(-g))));
-          ((bf16_t*)p.out)[(size_t)m * p.N + u] = f32_to_bf16(s * up);
+          ((bf16_t*)p.out)[(size_t)m * p.N + u] = f32_to_bf16(p3v_gated(p.epi, a0[m], a1[m]));
         } else {
           for (int h = 0; h < (has1 ? 2 : 1); ++h) {
             const float v = h ? a1[m] : a0[m];
@@ -293,8 +291,7 @@ __global__ void __launch_bounds__(256) k_gemv_mfma(GemvP p) {
     const size_t o = (size_t)li * p.N + n;
     if (SILU) {
       const float v1 = ((cpart[0][1][e] + cpart[1][1][e]) + (cpart[2][1][e] + cpart[3][1][e])) * rs;
-      const float gt = bf16_round(v0), up = bf16_round(v1);
-      ((bf16_t*)p.out)[o] = f32_to_bf16(bf16_round(gt * bf16_round(1.f / (1.f + __expf(-gt)))) * up);
+      ((bf16_t*)p.out)[o] = f32_to_bf16(p3v_gated(p.epi, v0, v1));
     } else if (p.epi == P3V_EPI_F32) {
       ((float*)p.out)[o] = v0;
     } else if (p.epi == P3V_EPI_SCALE_RESID_F32) {
@@ -521,8 +518,7 @@ __global__ void __launch_bounds__(NW * 64) k_gemv_mfma8(GemvP p, int n_sets) {
         if constexpr (SCALED) {
           ((float*)p.out)[o] = e_rf + e_ls * v0;
         } else if (SILU) {
-          const float gt = bf16_round(v0), up = bf16_round(v1);
-          ((bf16_t*)p.out)[o] = f32_to_bf16(bf16_round(gt * bf16_round(1.f / (1.f + __expf(-gt)))) * up);
+          ((bf16_t*)p.out)[o] = f32_to_bf16(p3v_gated(p.epi, v0, v1));
         } else if (p.epi == P3V_EPI_F32) {
           ((float*)p.out)[o] = v0;
         } else if (p.epi == P3V_EPI_RESID_BF16) {
@@ -561,7 +557,7 @@ static int launch_gemv_mfma8(const GemvP& p, hipStream_t s) {
 
 static int launch_gemv_mfma(const GemvP& p, hipStream_t s) {
   dim3 grid(p3v_cdiv(p.N, 16));
-  if (p.epi == P3V_EPI_SILU_MUL) hipLaunchKernelGGL(k_gemv_mfma<true>, grid, dim3(256), 0, s, p);
+  if (P3V_GATED(p.epi)) hipLaunchKernelGGL(k_gemv_mfma<true>, grid, dim3(256), 0, s, p);
   else hipLaunchKernelGGL(k_gemv_mfma<false>, grid, dim3(256), 0, s, p);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
@@ -612,17 +608,27 @@ extern "C" int p3v_gemv_dyt(const p3v_gemv_args_t* a, const p3v_dyt_args_t* d, v
   if (!a || !d || !a->W || !a->out || a->M <= 0 || a->N <= 0 || a->K <= 0) return P3V_ERR_ARG;
   if (!d->x || !d->w || !d->b || d->B != a->M || d->L != 1 || d->H != a->K) return P3V_ERR_ARG;
   if (d->mu && (!d->hist || d->hist_rows < 2 || (!d->d_past && d->past < 0))) return P3V_ERR_ARG;
-  if (a->M != 1 || (a->epilogue != P3V_EPI_NONE && a->epilogue != P3V_EPI_SILU_MUL)) return P3V_ERR_UNSUPPORTED;
+  if (a->M != 1 || (a->epilogue != P3V_EPI_NONE && !P3V_GATED(a->epilogue))) return P3V_ERR_UNSUPPORTED;
   if (((uintptr_t)d->x | (uintptr_t)d->w | (uintptr_t)d->b | (uintptr_t)d->mu | (uintptr_t)d->hist | (uintptr_t)a->W) & 15) return P3V_ERR_UNSUPPORTED;
   const GemvP p = {nullptr, a->W, a->out, nullptr, nullptr, 0.f, a->M, a->N, a->K, a->epilogue,
-                   a->epilogue == P3V_EPI_SILU_MUL ? a->N : (a->N + 1) / 2, nullptr, dyt_params(d)};
+                   P3V_GATED(a->epilogue) ? a->N : (a->N + 1) / 2, nullptr, dyt_params(d)};
   return gemv3_layered<GEMV_DYT>(p, (hipStream_t)stream);
+}
+
+extern "C" int p3v_gemv_rms(const p3v_gemv_args_t* a, const float* x, float gain, void* stream) {
+  if (!a || !x || !a->norm_w || !a->W || !a->out || a->M <= 0 || a->N <= 0 || a->K <= 0) return P3V_ERR_ARG;
+  if (a->M != 1 || (a->epilogue != P3V_EPI_NONE && !P3V_GATED(a->epilogue))) return P3V_ERR_UNSUPPORTED;
+  if (((uintptr_t)x | (uintptr_t)a->norm_w | (uintptr_t)a->W) & 15) return P3V_ERR_UNSUPPORTED;
+  GemvP p = {nullptr, a->W, a->out, nullptr, nullptr, a->norm_eps, a->M, a->N, a->K, a->epilogue,
+             P3V_GATED(a->epilogue) ? a->N : (a->N + 1) / 2, nullptr, {}};
+  p.dyt.x = x, p.dyt.w = a->norm_w, p.dyt.alpha = gain;
+  return gemv3_layered<GEMV_RMS>(p, (hipStream_t)stream);
 }
 
 extern "C" int p3v_gemv(const p3v_gemv_args_t* a, void* stream) {
   if (!a || !a->x || !a->W || !a->out) return P3V_ERR_ARG;
   if (a->M <= 0 || a->M > 16 || a->N <= 0 || a->K <= 0 || a->K % 8) return P3V_ERR_ARG;
-  if (a->epilogue != P3V_EPI_NONE && a->epilogue != P3V_EPI_RESID_BF16 && a->epilogue != P3V_EPI_SILU_MUL &&
+  if (a->epilogue != P3V_EPI_NONE && a->epilogue != P3V_EPI_RESID_BF16 && !P3V_GATED(a->epilogue) &&
       a->epilogue != P3V_EPI_F32 && a->epilogue != P3V_EPI_SCALE_RESID_F32)
     return P3V_ERR_UNSUPPORTED;
   if (a->epilogue == P3V_EPI_RESID_BF16 && !a->resid) return P3V_ERR_ARG;
@@ -630,7 +636,7 @@ extern "C" int p3v_gemv(const p3v_gemv_args_t* a, void* stream) {
   if (scaled && (!a->resid || !a->col_scale)) return P3V_ERR_ARG;
   const int mt = a->M <= 1 ? 1 : a->M <= 2 ? 2 : a->M <= 4 ? 4 : 8;
   GemvP p = {a->x, a->W, a->out, a->resid, a->norm_w, a->norm_eps, a->M, a->N, a->K, a->epilogue,
-             a->epilogue == P3V_EPI_SILU_MUL ? a->N : (a->N + 1) / 2, a->col_scale, {}};
+             P3V_GATED(a->epilogue) ? a->N : (a->N + 1) / 2, a->col_scale, {}};
   hipStream_t s = (hipStream_t)stream;
   if (scaled) {
     const int rc = gemv3_layered<GEMV_SCALED>(p, s);
@@ -666,7 +672,7 @@ extern "C" int p3v_gemv(const p3v_gemv_args_t* a, void* stream) {
   }
   const int rows8 = p3v_tuning().gemv_mfma8;
   if (rows8 && !scaled && a->M >= rows8_min && a->M <= 8) {
-    const bool silu = a->epilogue == P3V_EPI_SILU_MUL;
+    const bool silu = P3V_GATED(a->epilogue);
     switch (a->K) {                                      // K = NW waves x NST stages x 256
       case 1024: return silu ? launch_gemv_mfma8<true, 4, 1>(p, s) : launch_gemv_mfma8<false, 4, 1>(p, s);
       case 2048: return silu ? launch_gemv_mfma8<true, 4, 2>(p, s) : launch_gemv_mfma8<false, 4, 2>(p, s);

@@ -14,8 +14,9 @@ struct GemvP {
   DytP dyt;                              // GEMV_DYT: dyt.x (fp32) in place of x
 };
 // Variants of the one-row body for the layered decoders (fp32 residual stream): GEMV_DYT = the input row is a dynamic tanh (+ token
-// shift) of the residual row, computed while the first weights are on their way; GEMV_SCALED = out = resid + col_scale * acc in fp32.
-enum { GEMV_DYT = 1, GEMV_SCALED = 2 };
+// shift) of the residual row, computed while the first weights are on their way; GEMV_RMS = it is the RMS norm of that row (dyt.x, dyt.w,
+// dyt.alpha = the gain, eps); GEMV_SCALED = out = resid + col_scale * acc in fp32.
+enum { GEMV_DYT = 1, GEMV_SCALED = 2, GEMV_RMS = 4 };
 
 // 8 bf16 x 8 bf16 -> fp32 accumulate on v_dot2c_f32_bf16 (two products per instruction straight from the packed
 // operands): 4 VALU instructions per 16-byte weight chunk instead of 8 unpacks + 8 FMAs -- the GEMV's VALU pipe was
@@ -159,14 +160,14 @@ __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, i
   constexpr int XC = (CHUNKS + 255) / 256;              // x chunks per thread
   u32x4_t* xs = (u32x4_t*)smem;                         // [MT][CHUNKS] bf16 x (normalised)
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const bool silu = p.epi == P3V_EPI_SILU_MUL;
+  const bool silu = P3V_GATED(p.epi);
   const bool has_res = p.epi == P3V_EPI_RESID_BF16;
   const int u_begin = wave < wpw ? min(p.units, (bx * wpw + wave) * units_per_wave) : p.units;
   const int u_end = min(p.units, u_begin + units_per_wave);
   const int n_st = (u_end - u_begin) * NST;
 
   // ---- 1. x / norm-weight loads (oldest in the queue)
-  constexpr bool DYT = (VAR & GEMV_DYT) != 0, SCALED = (VAR & GEMV_SCALED) != 0;
+  constexpr bool DYT = (VAR & GEMV_DYT) != 0, SCALED = (VAR & GEMV_SCALED) != 0, RMS = (VAR & GEMV_RMS) != 0;
   static_assert(VAR == 0 || (MT == 1 && STEP == STEP_NONE), "one-row variants");
   float4 dx[XC][2], dh[XC][2];                           // GEMV_DYT: residual chunk, the token before's unshifted input
   u32x4_t db[XC], dm[XC];
@@ -187,6 +188,13 @@ __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, i
       dm[k] = ((const u32x4_t*)(p.dyt.mu ? p.dyt.mu : p.dyt.b))[c];
     }
   }
+  if constexpr (RMS) {
+#pragma unroll
+    for (int k = 0; k < XC; ++k) {
+      const int c = min(tid + k * 256, CHUNKS - 1);
+      dx[k][0] = ((const float4*)p.dyt.x)[2 * c], dx[k][1] = ((const float4*)p.dyt.x)[2 * c + 1];
+    }
+  }
   u32x4_t xv[MT][XC], gv[XC];
   const bf16_t* xrow[MT];
 #pragma unroll
@@ -204,8 +212,8 @@ __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, i
     const int c = min(tid + k * 256, CHUNKS - 1);
 #pragma unroll
     for (int m = 0; m < MT; ++m)
-      if constexpr (!DYT) xv[m][k] = ((const u32x4_t*)xrow[m])[c];
-    if constexpr (DYT) gv[k] = ((const u32x4_t*)p.dyt.w)[c];
+      if constexpr (!DYT && !RMS) xv[m][k] = ((const u32x4_t*)xrow[m])[c];
+    if constexpr (DYT || RMS) gv[k] = ((const u32x4_t*)p.dyt.w)[c];
     else gv[k] = p.norm_w ? ((const u32x4_t*)p.norm_w)[c] : (u32x4_t){0, 0, 0, 0};
   }
 
@@ -262,8 +270,31 @@ __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, i
       }
     }
   }
+  if constexpr (RMS) {
+    float ss = 0.f;
 #pragma unroll
-  for (int m = 0; m < (DYT ? 0 : MT); ++m) {
+    for (int k = 0; k < XC; ++k)
+      if (tid + k * 256 < CHUNKS) {
+        ss += dx[k][0].x * dx[k][0].x + dx[k][0].y * dx[k][0].y + dx[k][0].z * dx[k][0].z + dx[k][0].w * dx[k][0].w;
+        ss += dx[k][1].x * dx[k][1].x + dx[k][1].y * dx[k][1].y + dx[k][1].z * dx[k][1].z + dx[k][1].w * dx[k][1].w;
+      }
+    ss = wave_sum(ss);
+    if (lane == 0) red[wave] = ss;
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    const float r = p.dyt.alpha / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)(CHUNKS * 8) + p.eps);
+#pragma unroll
+    for (int k = 0; k < XC; ++k) {
+      const int c = tid + k * 256;
+      if (c < CHUNKS)
+        xs[c] = (u32x4_t){pack_bf16x2(dx[k][0].x * (r * bf16lo(gv[k][0])), dx[k][0].y * (r * bf16hi(gv[k][0]))),
+                          pack_bf16x2(dx[k][0].z * (r * bf16lo(gv[k][1])), dx[k][0].w * (r * bf16hi(gv[k][1]))),
+                          pack_bf16x2(dx[k][1].x * (r * bf16lo(gv[k][2])), dx[k][1].y * (r * bf16hi(gv[k][2]))),
+                          pack_bf16x2(dx[k][1].z * (r * bf16lo(gv[k][3])), dx[k][1].w * (r * bf16hi(gv[k][3])))};
+    }
+  }
+#pragma unroll
+  for (int m = 0; m < (DYT || RMS ? 0 : MT); ++m) {
     float r = 1.f;
     if (p.norm_w) {
       float ss = 0.f;
@@ -328,10 +359,7 @@ __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, i
             if constexpr (SCALED) {
               *(float2*)((float*)p.out + 2 * u) = make_float2(fbuf[buf].x + bf16lo(rbuf[buf][0]) * a0[0], fbuf[buf].y + bf16hi(rbuf[buf][0]) * a1[0]);
             } else if (silu) {
-              const float g = bf16_round(a0[m]), up = bf16_round(a1[m]);
-              const float sg = bf16_round(g * bf16_round(1.f / (1.f + __expf(-g))));
-              bf16_t* dst = (bf16_t*)p.out + (size_t)m * p.N + u;
-              *dst = f32_to_bf16(sg * up);
+              ((bf16_t*)p.out)[(size_t)m * p.N + u] = f32_to_bf16(p3v_gated(p.epi, a0[m], a1[m]));
             } else if (p.epi == P3V_EPI_F32) {
               ((float*)p.out)[(size_t)m * p.N + 2 * u] = a0[m];
               ((float*)p.out)[(size_t)m * p.N + 2 * u + 1] = a1[m];

@@ -1,5 +1,6 @@
-// Row kernels and plain projections of the layered text decoders (config.py: LayerSpec): a residual stream in fp32, dynamic-tanh
-// "norms", token shift, whole-projection query / key norms, value mixing, and a projection for every size and for fp32 activations.
+// Row kernels and plain projections of the layered text decoders (config.py: LayerSpec): a residual stream in fp32, RMS norms and
+// dynamic-tanh "norms" of it, token shift, whole-projection query / key norms, value mixing, and a projection for every size and for
+// fp32 activations.
 // Activations are bf16 or fp32 (the element type T of a model); weights are bf16 in either case, which fp32 arithmetic reads exactly.
 #include "p3v_layered.h"
 
@@ -17,6 +18,64 @@ extern "C" int p3v_embed_scale(const int32_t* ids, const uint16_t* table, float*
   if (!ids || !table || !out || n_tok < 0 || hidden <= 0 || vocab <= 0) return P3V_ERR_ARG;
   if (n_tok == 0) return P3V_OK;
   hipLaunchKernelGGL(k_embed_scale, dim3(n_tok), dim3(256), 0, (hipStream_t)stream, ids, table, out, hidden, vocab, scale);
+  P3V_CHECK_LAUNCH();
+  return P3V_OK;
+}
+
+// ---------------------------------------------------------------- RMS norm of fp32 rows
+// out = x / sqrt(mean x^2 + eps) * w * gain, fp32 up to the one rounding of out; a wave per row, CH 16-byte chunks per lane in registers
+// (CH = 0: any width, the row read twice)
+template <typename T, int CH>
+__global__ void __launch_bounds__(256) k_rms_rows(const float* __restrict__ x, const bf16_t* __restrict__ w, T* __restrict__ out, int rows, int H,
+                                                  float eps, float gain) {
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (row >= rows) return;
+  const float* xr = x + (size_t)row * H;
+  T* o = out + (size_t)row * H;
+  float ss = 0.f;
+  if constexpr (CH > 0) {
+    const int chunks = H / 8;
+    float v[CH][8];
+    u32x4_t g[CH];
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+      const int c = min(i * 64 + lane, chunks - 1);
+      load_acts<8>(xr + 8 * c, v[i]);
+      g[i] = *(const u32x4_t*)(w + 8 * c);
+    }
+#pragma unroll
+    for (int i = 0; i < CH; ++i)
+      if (i * 64 + lane < chunks) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) ss += v[i][j] * v[i][j];
+      }
+    const float r = gain / sqrtf(wave_sum(ss) / (float)H + eps);
+#pragma unroll
+    for (int i = 0; i < CH; ++i)
+      if (i * 64 + lane < chunks) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[i][j] *= r * (j & 1 ? bf16hi(g[i][j >> 1]) : bf16lo(g[i][j >> 1]));
+        store_acts<8>(o + 8 * (i * 64 + lane), v[i]);
+      }
+  } else {
+    for (int c = lane; c < H; c += 64) ss += xr[c] * xr[c];
+    const float r = gain / sqrtf(wave_sum(ss) / (float)H + eps);
+    for (int c = lane; c < H; c += 64) store_act(o + c, xr[c] * (r * bf16_to_f32(w[c])));
+  }
+}
+template <typename T>
+static void launch_rms_rows(const float* x, const bf16_t* w, T* out, int rows, int H, float eps, float gain, hipStream_t s) {
+  const dim3 grid(p3v_cdiv(rows, 4));
+  if (H % 8 || (((uintptr_t)x | (uintptr_t)w | (uintptr_t)out) & 15) || H > 4096) hipLaunchKernelGGL((k_rms_rows<T, 0>), grid, dim3(256), 0, s, x, w, out, rows, H, eps, gain);
+  else if (H <= 1024) hipLaunchKernelGGL((k_rms_rows<T, 2>), grid, dim3(256), 0, s, x, w, out, rows, H, eps, gain);
+  else if (H <= 2048) hipLaunchKernelGGL((k_rms_rows<T, 4>), grid, dim3(256), 0, s, x, w, out, rows, H, eps, gain);
+  else hipLaunchKernelGGL((k_rms_rows<T, 8>), grid, dim3(256), 0, s, x, w, out, rows, H, eps, gain);
+}
+extern "C" int p3v_rms_rows(const float* x, const uint16_t* w, void* out, int out_f32, int rows, int H, float eps, float gain, void* stream) {
+  if (!x || !w || !out || rows < 0 || H <= 0) return P3V_ERR_ARG;
+  if (rows == 0) return P3V_OK;
+  if (out_f32) launch_rms_rows(x, w, (float*)out, rows, H, eps, gain, (hipStream_t)stream);
+  else launch_rms_rows(x, w, (bf16_t*)out, rows, H, eps, gain, (hipStream_t)stream);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
 }
@@ -86,7 +145,7 @@ struct GemmAnyP {
 };
 template <typename T, int EPI>
 __global__ void __launch_bounds__(256) k_gemm_any(GemmAnyP p) {
-  constexpr bool SILU = EPI == P3V_EPI_SILU_MUL;
+  constexpr bool SILU = P3V_GATED(EPI);
   __shared__ float sa[16][68], sw[SILU ? 2 : 1][16][68];
   const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4, n0 = blockIdx.x * 64, m0 = blockIdx.y * 64;
   const int lr = tid >> 2, lk = (tid & 3) * 4;
@@ -126,7 +185,10 @@ __global__ void __launch_bounds__(256) k_gemm_any(GemmAnyP p) {
       if (m >= p.M || n >= p.N) continue;
       const size_t o = (size_t)m * p.ldo + n;
       const float v = acc[0][i][j];
-      if (SILU) {
+      if (EPI == P3V_EPI_GELU_MUL) {
+        const float t = 1.5957691216057308f * (v + 0.044715f * v * v * v);
+        store_act((T*)p.out + o, v / (1.f + expf(-t)) * acc[SILU ? 1 : 0][i][j]);
+      } else if (SILU) {
         const float g = round_act<T>(v), u = round_act<T>(acc[SILU ? 1 : 0][i][j]);
         store_act((T*)p.out + o, round_act<T>(g * round_act<T>(1.f / (1.f + expf(-g)))) * u);
       } else if (EPI == P3V_EPI_SCALE_RESID_F32) {
@@ -155,6 +217,7 @@ extern "C" int p3v_gemm_any(const p3v_gemm_args_t* a, int a_f32, void* stream) {
     P3V_ANY(P3V_EPI_NONE)
     P3V_ANY(P3V_EPI_F32)
     P3V_ANY(P3V_EPI_SILU_MUL)
+    P3V_ANY(P3V_EPI_GELU_MUL)
     P3V_ANY(P3V_EPI_SCALE_RESID_F32)
     default: return P3V_ERR_UNSUPPORTED;
   }

@@ -5,7 +5,7 @@ captured short-prompt prefill.  A model class (model.Phi3VModel, layered.Layered
     _new_state(B, S, max_tokens, pids, mask) a CacheState
     _slot_rows(st, row, lens)                per-row tables of a slot prefill (none by default)
     _alloc_bufs(B, L), _step_bufs(st)        activations of one call / of the captured step
-    _embed(ids, out=None), _layers(...), _head(x, out=None, bufs=None)
+    _embed(ids, out=None), _layers(...), _head(x, out=None, bufs=None)    (_layers' keep: how many of the L columns stay)
     _step(g, st)                             the launches of one captured greedy step
     _prefill_key(S, max_tokens), _cache_token_bytes()   what a captured prefill depends on (None: not capturable), its cache size
 """
@@ -227,9 +227,10 @@ class DecoderModel:
             raise ValueError(f"KV cache overflow: {past}+{L} > {st.T} (prompt + max_tokens)")
         if full_logits is None:
             full_logits = not prefill
+        keep = L if advance_offset is None else advance_offset
         if n_beam == 1:
-            st.note_written(past, past + L)
-        x = self._layers(x, st, B, L, past, n_beam, last_only=not full_logits)
+            st.note_written(past, past + L, past + keep)
+        x = self._layers(x, st, B, L, past, n_beam, last_only=not full_logits, keep=keep)
         if n_beam == 1:
             st.offset = past + L                                 # KVCache.__call__ auto-advance (phi.py:544-547)
         if advance_offset is not None:

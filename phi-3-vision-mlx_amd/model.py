@@ -462,7 +462,7 @@ class Phi3VModel(DecoderModel):
                 fused = False
             bufs["attn_merge"] = bool(fused)
 
-    def _layers(self, x, st, B, L, past, n_beam, bufs=None, d_past=None, last_only=False, step_begin=None):
+    def _layers(self, x, st, B, L, past, n_beam, bufs=None, d_past=None, last_only=False, step_begin=None, keep=None):
         """Phi3DecoderLayer stack (phi.py:473-485).  `d_past` (device int32) makes every
         position-dependent kernel read the cache length from HBM -> graph-replayable.
         last_only: the caller reads the LAST position only (prefill of generate / choose, Q8): the final layer still builds

@@ -10,7 +10,7 @@ import ctypes as C
 import torch
 
 from . import _lib as L
-from ._lib import (EPI_BIAS, EPI_BIAS_GELU, EPI_BIAS_QGELU, EPI_BIAS_RESID_F32, EPI_F32, EPI_NONE,  # noqa: F401
+from ._lib import (EPI_BIAS, EPI_BIAS_GELU, EPI_BIAS_QGELU, EPI_BIAS_RESID_F32, EPI_F32, EPI_GELU_MUL, EPI_NONE,  # noqa: F401
                    EPI_PATCH, EPI_RESID_BF16, EPI_SCALE_RESID_F32, EPI_SILU_MUL)
 
 BF16, F32, I32 = torch.bfloat16, torch.float32, torch.int32
@@ -32,6 +32,9 @@ def _chk(t, dtype, name):
     if not t.is_contiguous():
         raise ValueError(f"{name}: expected a contiguous tensor")
     return t
+
+
+GATED = (EPI_SILU_MUL, EPI_GELU_MUL)                             # W = [gate; up]: out has half of its rows as columns
 
 
 def embed_gather(ids, table, out=None):
@@ -118,7 +121,7 @@ def gemm(a, w, epilogue=EPI_NONE, bias=None, resid=None, out=None, n_out=None, p
     """nn.Linear / patch conv: out[M,N] = a[M,K] @ w[N,K]^T (+ epilogue), bf16 MFMA."""
     _chk(a, BF16, "a"), _chk(w, BF16, "w")
     M, K = a.shape
-    N = n_out if n_out is not None else (w.shape[0] // 2 if epilogue == EPI_SILU_MUL else w.shape[0])
+    N = n_out if n_out is not None else (w.shape[0] // 2 if epilogue in GATED else w.shape[0])
     if w.shape[1] != K:
         raise ValueError(f"gemm: K mismatch {a.shape} x {w.shape}")
     f32_out = epilogue in (EPI_BIAS_RESID_F32, EPI_PATCH, EPI_F32, EPI_SCALE_RESID_F32)
@@ -163,7 +166,7 @@ def gemv(x, w, epilogue=EPI_NONE, resid=None, norm_w=None, norm_eps=0.0, out=Non
     """Skinny nn.Linear for decode (M<=16) with optional fused RMSNorm / epilogue."""
     _chk(x, BF16, "x"), _chk(w, BF16, "w")
     M, K = x.shape
-    N = w.shape[0] // 2 if epilogue == EPI_SILU_MUL else w.shape[0]
+    N = w.shape[0] // 2 if epilogue in GATED else w.shape[0]
     if out is None:
         out = torch.empty((M, N), dtype=F32 if epilogue in (EPI_F32, EPI_SCALE_RESID_F32) else BF16, device=x.device)
     args = L.GemvArgs(_p(x), _p(w), _p(out), _p(resid), _p(norm_w), float(norm_eps), M, N, K, epilogue, _p(col_scale))
@@ -641,7 +644,7 @@ def project_dyt(x, norm, w, h, epilogue=EPI_NONE, out=None, B=1, Lq=1, **shift):
     M, H = B * Lq, x.shape[-1]
     if M == 1 and h.dtype == BF16 and out is not None:
         _chk(w, BF16, "w"), _chk(out, BF16, "out")
-        N = w.shape[0] // 2 if epilogue == EPI_SILU_MUL else w.shape[0]
+        N = w.shape[0] // 2 if epilogue in GATED else w.shape[0]
         if w.shape[1] != H or out.numel() != N:
             raise ValueError(f"project_dyt: {tuple(w.shape)} on rows of {H} -> {tuple(out.shape)}")
         d = _dyt_args(x, norm, 1, 1, **{**dict(shift=None, hist=None, past=0, d_past=None, pad_len=None), **shift})
@@ -654,13 +657,41 @@ def project_dyt(x, norm, w, h, epilogue=EPI_NONE, out=None, B=1, Lq=1, **shift):
     return project(h[:M], w, epilogue, out=out)
 
 
+def rms_rows(x, norm, out):
+    """RMS norm of the fp32 rows x: norm = (w, eps, gain) -> out (bf16 or fp32 rows), rounded once."""
+    w, eps, gain = norm
+    _chk(x, F32, "x"), _chk(w, BF16, "w"), _chk(out, F32 if out.dtype == F32 else BF16, "out")
+    H = x.shape[-1]
+    if w.numel() != H or out.numel() < x.numel():
+        raise ValueError(f"rms_rows: rows {tuple(x.shape)}, weight {tuple(w.shape)}, output {tuple(out.shape)}")
+    L.check(L.lib().p3v_rms_rows(_p(x), _p(w), _p(out), int(out.dtype == F32), x.numel() // H, H, float(eps), float(gain), _stream()), "rms_rows")
+    return out
+
+
+def project_rms(x, norm, w, h, epilogue=EPI_NONE, out=None):
+    """project(rms_rows(x)): one launch for a single bf16 row of a width the streaming kernel takes, else the two (h: their scratch rows)."""
+    M, H = x.shape
+    if M == 1 and h.dtype == BF16 and out is not None:
+        _chk(x, F32, "x"), _chk(w, BF16, "w"), _chk(out, BF16, "out"), _chk(norm[0], BF16, "norm")
+        N = w.shape[0] // 2 if epilogue in GATED else w.shape[0]
+        if w.shape[1] != H or out.numel() != N or norm[0].numel() != H:
+            raise ValueError(f"project_rms: {tuple(w.shape)} on rows of {H} -> {tuple(out.shape)}")
+        args = L.GemvArgs(0, _p(w), _p(out), 0, _p(norm[0]), float(norm[1]), 1, N, H, epilogue, 0)
+        rc = L.lib().p3v_gemv_rms(C.byref(args), _p(x), float(norm[2]), _stream())
+        if rc != L.ERR_UNSUPPORTED:
+            L.check(rc, "gemv_rms")
+            return out
+    rms_rows(x, norm, h)
+    return project(h[:M], w, epilogue, out=out)
+
+
 def project(x, w, epilogue=EPI_NONE, resid=None, col_scale=None, out=None):
     """One projection of a layered decoder, x [M, K] bf16 or fp32: the weight-streaming GEMV, the MFMA GEMM, or -- fp32 rows, and sizes
     those do not take -- the fp32-arithmetic kernel of every size."""
     f32 = x.dtype == F32
     _chk(x, F32 if f32 else BF16, "x"), _chk(w, BF16, "w")
     M, K = x.shape
-    N = w.shape[0] // 2 if epilogue == EPI_SILU_MUL else w.shape[0]
+    N = w.shape[0] // 2 if epilogue in GATED else w.shape[0]
     if w.shape[1] != K:
         raise ValueError(f"project: K mismatch {tuple(x.shape)} x {tuple(w.shape)}")
     if out is None:
@@ -723,6 +754,103 @@ def attention_mixed(qkv, q, k, v, out, norms, talk, sink, B, Lq, H, G, dim, vdim
         args.n_split = 1
     L.check(L.lib().p3v_qkv_heads(C.byref(args), _stream()), "qkv_heads")
     L.check(L.lib().p3v_attn_mix(C.byref(args), _stream()), "attn_mix")
+    return out
+
+
+def latent_plan(m, B, Lq, n_keys, dtype):
+    """How a latent-attention call runs: > 0 in the latent space with that many key splits, 0 the any-size kernel, < 0 over expanded keys."""
+    return int(L.lib().p3v_latent_plan(B, Lq, m.heads, m.dim, m.rot.dims, m.vdim, m.rank, int(n_keys), int(dtype == F32)))
+
+
+def latent_ws_bytes(m, B, Lq, n_split):
+    return int(L.lib().p3v_latent_ws_bytes(B, Lq, m.heads, m.rank, n_split))
+
+
+def _gemm_rows(a, w, out, M, N, K, lda, ldw):
+    """out[M, N] = a w^T of raw row pointers (bf16), rows of a and w lda / ldw elements apart."""
+    ws_bytes = L.lib().p3v_gemm_ws_bytes(M, N, K, EPI_NONE)
+    ws = _gemm_workspace(out.device, ws_bytes) if ws_bytes else None
+    args = L.GemmArgs(a, w, _p(out), 0, 0, 0, M, N, K, lda, ldw, N, EPI_NONE, 0, _p(ws), ws.numel() if ws is not None else 0, 0)
+    L.check(L.lib().p3v_gemm(C.byref(args), _stream()), "gemm")
+
+
+def attention_latent(mx, y, out, c, cos, sin, bufs, call, plan):
+    """Latent attention of a call's new tokens (include/p3v.h: p3v_latent_args_t).  mx: the layer's weights (mixers.LatentHeads), y its packed
+    projection rows [B*L, ld] (the queries in it are rotated in place), c its cache rows [B, Tp, ..], out [B*L, H vdim]."""
+    m, B, Lq = mx.m, call.B, call.L
+    f32 = y.dtype == F32
+    for t, n in ((y, "y"), (c, "c"), (out, "out")):
+        _chk(t, F32 if f32 else BF16, n)
+    for t, n in ((cos, "cos"), (sin, "sin")):
+        _chk(t, F32, n)
+    H, R, rot = m.heads, m.rank, m.rot.dims
+    Tp, cw, rankp, dimp = c.shape[1], c.shape[2], mx.uk.shape[1], mx.ukt.shape[2]
+    if (c.shape[0] != B or cw < rankp + rot or y.shape[0] != B * Lq or y.shape[1] < H * (m.dim + rot + m.vdim) + R + rot or out.numel() < B * Lq * H * m.vdim
+            or tuple(mx.uk.shape) != (H * m.dim, rankp) or tuple(mx.uv.shape) != (H * m.vdim, rankp) or tuple(mx.ukt.shape) != (H, rankp, dimp)
+            or mx.c_norm.numel() != R or mx.sink.numel() != H or cos.shape != sin.shape or cos.shape[1] != rot // 2 or cos.shape[0] < Tp
+            or (call.pad_len is not None and call.pad_len.numel() != B)):
+        raise ValueError(f"attention_latent: shapes y {tuple(y.shape)}, c {tuple(c.shape)}, out {tuple(out.shape)}, tables {tuple(cos.shape)}")
+    if call.d_past is None and call.past + Lq > Tp:
+        raise ValueError(f"attention_latent: columns {call.past} + {Lq} > {Tp}")
+    args = L.LatentArgs(y=_p(y), c_norm=_p(mx.c_norm), uk=_p(mx.uk), ukt=_p(mx.ukt), uv=_p(mx.uv), sink=_p(mx.sink), cos_t=_p(cos), sin_t=_p(sin), c=_p(c),
+                        out=_p(out), pad_len=_p(call.pad_len), d_past=_p(call.d_past), eps=float(mx.eps), scale=float(m.scale), B=B, L=Lq, H=H,
+                        dim=m.dim, rot=rot, vdim=m.vdim, rank=R, rankp=rankp, rotp=cw - rankp, dimp=dimp, ld=y.shape[1], past=int(call.past), Tp=Tp,
+                        tab_n=cos.shape[0], f32=int(f32))
+    lib = L.lib()
+    if plan > 0:
+        q, ws = bufs["q"], bufs["attn_ws"]
+        if q.dtype != BF16 or q.numel() < B * Lq * ((H + 15) // 16 * 16) * cw or ws.numel() * 4 < latent_ws_bytes(m, B, Lq, plan):
+            raise ValueError("attention_latent: scratch smaller than the call needs")
+        args.q, args.ws, args.n_split = _p(q), _p(ws), plan
+        L.check(lib.p3v_latent_rows(C.byref(args), _stream()), "latent_rows")
+        return out
+    L.check(lib.p3v_latent_append(C.byref(args), _stream()), "latent_append")
+    if plan == 0:
+        L.check(lib.p3v_latent_any(C.byref(args), _stream()), "latent_any")
+        return out
+    if call.d_past is not None:
+        raise ValueError("attention_latent: a prompt's position is a host value")
+    n = (call.past + Lq + 63) // 64 * 64
+    kx, vx = bufs["kx"], bufs["vx"]
+    if kx.numel() < B * n * H * m.dim or vx.numel() < B * n * H * m.vdim:
+        raise ValueError("attention_latent: scratch smaller than the call needs")
+    row = c.element_size() * Tp * cw
+    for b in range(B):                                           # keys as rows, values as columns: the value product reads consecutive keys
+        lat, k, v = _p(c) + b * row, kx[b * n * H * m.dim:], vx[b * n * H * m.vdim:]
+        _gemm_rows(lat, _p(mx.uk), k, n, H * m.dim, rankp, cw, rankp)
+        _gemm_rows(_p(mx.uv), lat, v, H * m.vdim, n, rankp, rankp, cw)
+    args.kx, args.vx, args.n_keys = _p(kx), _p(vx), n
+    L.check(lib.p3v_latent_prompt(C.byref(args), _stream()), "latent_prompt")
+    return out
+
+
+def gla_plan(m, B, Lq, dtype):
+    """Chunks of a gated-linear-attention call (0: token by token)."""
+    return int(L.lib().p3v_gla_plan(B, Lq, m.heads, m.dim, m.vdim, int(dtype == F32)))
+
+
+def gla_ws_bytes(m, B, Lq, n_chunk):
+    return int(L.lib().p3v_gla_ws_bytes(B, Lq, m.heads, m.dim, m.vdim, n_chunk))
+
+
+def gated_linear_attention(mx, y, out, s, ws, call, plan):
+    """Gated linear attention of a call's new tokens (include/p3v.h: p3v_gla_args_t).  mx: the layer's weights (mixers.LinearState), y its
+    packed projection rows [B*L, ld], s its ring of states [B, R, H, dim, vdim] fp32, out [B*L, H vdim]."""
+    m, B, Lq = mx.m, call.B, call.L
+    f32 = y.dtype == F32
+    _chk(y, F32 if f32 else BF16, "y"), _chk(out, F32 if f32 else BF16, "out"), _chk(s, F32, "s")
+    H, r = m.heads, mx.rank
+    if (s.shape[0] != B or tuple(s.shape[2:]) != (H, m.dim, m.vdim) or y.shape[0] != B * Lq or y.shape[1] < 2 * H * (m.dim + m.vdim) + r
+            or out.numel() < B * Lq * H * m.vdim or tuple(mx.a2.shape) != (H * m.dim, r) or mx.a2_b.numel() != H * m.dim or mx.norm.numel() != m.vdim
+            or not 0 <= call.keep <= Lq or (call.pad_len is not None and call.pad_len.numel() != B)):
+        raise ValueError(f"gated_linear_attention: shapes y {tuple(y.shape)}, s {tuple(s.shape)}, out {tuple(out.shape)}; {call.keep} of {Lq} stay")
+    need = gla_ws_bytes(m, B, Lq, plan)
+    if need and (ws is None or ws.numel() * 4 < need):
+        raise ValueError("gated_linear_attention: workspace smaller than gla_ws_bytes")
+    args = L.GlaArgs(y=_p(y), a2=_p(mx.a2), a2_b=_p(mx.a2_b), norm=_p(mx.norm), s=_p(s), out=_p(out), ws=_p(ws) if need else 0,
+                     pad_len=_p(call.pad_len), d_past=_p(call.d_past), eps=float(mx.eps), tau=float(m.tau), q_scale=float(m.dim) ** -0.5, B=B, L=Lq, H=H,
+                     dim=m.dim, vdim=m.vdim, rank=r, ld=y.shape[1], past=int(call.past), R=s.shape[1], keep=int(call.keep), n_chunk=int(plan), f32=int(f32))
+    L.check(L.lib().p3v_gla(C.byref(args), _stream()), "gla")
     return out
 
 

@@ -31,6 +31,8 @@ FAMILIES = [
     Family("Phi3F", "model:Phi3VModel", "processor:Phi3FProcessor", "weights:phi3_weight_specs"),
     Family("Pelalix", "layered:LayeredModel", "processor:TextProcessor", "weights:layered_weight_specs", layered=True,
            units=("elementwise", "gemm", "gemm256", "gemm_skinny", "gemm_rows", "gemv", "layered", "attn_mix", "runtime")),
+    Family("Pudisun", "layered:LayeredModel", "processor:TextProcessor", "weights:layered_weight_specs", layered=True,
+           units=("elementwise", "gemm", "gemm256", "gemm_skinny", "gemm_rows", "gemv", "layered", "latent", "latent_prompt", "gla", "runtime")),
 ]
 
 

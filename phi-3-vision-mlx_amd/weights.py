@@ -14,7 +14,7 @@ import zlib
 
 import torch
 
-from .config import is_vision
+from .config import GlaMixer, LatentMixer, is_vision
 from .registry import family
 
 _M32 = 0xFFFFFFFF
@@ -65,29 +65,53 @@ def weight_specs(cfg):
     return family(cfg).weight_specs(cfg)
 
 
+FREE_RANK = 16                                                   # of a low-rank projection whose rank no configuration gives (synthetic weights)
+
+
+class FreeDim(int):
+    """A size that the checkpoint decides (synthetic weights: the value)."""
+
+
+def _mixer_specs(p, m, D, first_v, i):
+    if isinstance(m, LatentMixer):
+        H, rot = m.heads, m.rot.dims
+        return [(p + "q", (H * (m.dim + rot), D), "matrix"), (p + "dkv", (m.rank + rot, D), "matrix"), (p + "dkv.norm", (m.rank,), "norm"),
+                (p + "uk", (H * m.dim, m.rank), "matrix"), (p + "uv", (H * m.vdim, m.rank), "matrix"), (p + "sink", (H,), "sink"),
+                (p + "g", (H * m.vdim, D), "matrix"), (p + "o", (D, H * m.vdim), "matrix")]
+    if isinstance(m, GlaMixer):
+        H, r = m.heads, FreeDim(FREE_RANK) if m.gate_rank is None else m.gate_rank
+        return [(p + "q", (H * m.dim, D), "matrix"), (p + "k", (H * m.dim, D), "matrix"), (p + "v", (H * m.vdim, D), "matrix"),
+                (p + "g", (H * m.vdim, D), "matrix"), (p + "o", (D, H * m.vdim), "matrix"), (p + "norm", (m.vdim,), "norm"),
+                (p + "a1", (r, D), "matrix"), (p + "a2", (H * m.dim, r), "matrix"), (p + "a2.b", (H * m.dim,), "decay")]
+    H, G = m.heads, m.kv_heads
+    specs = [(p + "q", (H * m.dim, D), "matrix"), (p + "k", (G * m.dim, D), "matrix"), (p + "v", (G * m.vdim, D), "matrix"),
+             (p + "q.norm", (H * m.dim,), "norm"), (p + "k.norm", (G * m.dim,), "norm"),
+             (p + "talk", (H, H), "talk"), (p + "sink", (H,), "sink"), (p + "g", (H, D), "matrix"), (p + "o", (D, H * m.vdim), "matrix")]
+    if m.v_mix and i != first_v:                                 # (the first such layer blends nothing in: a tensor of it is not read)
+        specs.append((p + "vmix", (), "alpha"))
+    return specs
+
+
 def layered_weight_specs(cfg):
-    """The tensors of a layered decoder (config.LayerSpec)."""
-    D, V = cfg.hidden_size, cfg.vocab_size
-    first_v = next((i for i, s in enumerate(cfg.layers) if s.mixer.v_mix), None)
+    """The tensors of a layered decoder (config.LayerSpec, config.Design)."""
+    D, V, ds = cfg.hidden_size, cfg.vocab_size, cfg.design
+    first_v = next((i for i, s in enumerate(cfg.layers) if getattr(s.mixer, "v_mix", False)), None)
 
     def norm(name):
-        return [(name, (D,), "norm"), (name + ".b", (D,), "bias"), (name + ".alpha", (), "alpha")]
+        return [(name, (D,), "norm")] + ([(name + ".b", (D,), "bias"), (name + ".alpha", (), "alpha")] if ds.norm == "dyt" else [])
     specs = [("embed", (V, D), "embed")]
     for i, s in enumerate(cfg.layers):
-        p, m = f"l{i}.", s.mixer
-        H, G = m.heads, m.kv_heads
-        specs += norm(p + "norm1")
-        specs += [(p + "mix.q", (H * m.dim, D), "matrix"), (p + "mix.k", (G * m.dim, D), "matrix"), (p + "mix.v", (G * m.vdim, D), "matrix"),
-                  (p + "mix.q.norm", (H * m.dim,), "norm"), (p + "mix.k.norm", (G * m.dim,), "norm"),
-                  (p + "mix.talk", (H, H), "talk"), (p + "mix.sink", (H,), "sink"), (p + "mix.g", (H, D), "matrix"),
-                  (p + "mix.o", (D, H * m.vdim), "matrix"), (p + "ls1", (D,), "norm"), (p + "shift", (D,), "shift")]
-        if m.v_mix and i != first_v:                             # (the first such layer blends nothing in: a tensor of it is not read)
-            specs.append((p + "mix.vmix", (), "alpha"))
+        if s.owner is not None:
+            continue
+        p = f"l{i}."
+        specs += norm(p + "norm1") + _mixer_specs(p + "mix.", s.mixer, D, first_v, i)
+        specs += [(p + "ls1", (D,), "norm")] if ds.layer_scale else []
+        specs += [(p + "shift", (D,), "shift")] if ds.token_shift else []
         if s.mlp is not None:
             specs += norm(p + "norm2")
-            specs += [(p + "mlp.gate", (s.mlp.ff, D), "matrix"), (p + "mlp.up", (s.mlp.ff, D), "matrix"), (p + "mlp.down", (D, s.mlp.ff), "matrix"),
-                      (p + "ls2", (D,), "norm")]
-    return specs + norm("final.norm") + [("head", (V, D), "matrix")]
+            specs += [(p + "mlp.gate", (s.mlp.ff, D), "matrix"), (p + "mlp.up", (s.mlp.ff, D), "matrix"), (p + "mlp.down", (D, s.mlp.ff), "matrix")]
+            specs += [(p + "ls2", (D,), "norm")] if ds.layer_scale else []
+    return specs + norm("final.norm") + ([] if ds.tied_head else [("head", (V, D), "matrix")])
 
 
 def phi3_weight_specs(cfg):
@@ -145,6 +169,7 @@ _KIND = {  # kind -> (std, mean)
     "matrix": (0.02, 0.0), "embed": (0.02, 0.0), "bias": (0.02, 0.0),
     "gn": (0.02, 0.0), "norm": (0.05, 1.0),
     "alpha": (0.1, 0.6), "sink": (0.5, 1.0), "shift": (0.2, 0.4), "talk": (0.1, 0.0),     # ("talk": around the identity)
+    "decay": (1.0, 3.0),
 }
 
 
@@ -279,7 +304,8 @@ def load_safetensors_dir(model_path, cfg, device="cpu"):
     if missing:
         raise KeyError(f"weights missing from {model_path}: {missing[:4]}{'...' if len(missing) > 4 else ''}")
     if family(cfg).layered:
-        wrong = [(n, tuple(out[n].shape), s) for n, s, _ in specs if tuple(out[n].shape) != tuple(s)]
+        wrong = [(n, tuple(out[n].shape), s) for n, s, _ in specs
+                 if len(out[n].shape) != len(s) or any(a != b for a, b in zip(out[n].shape, s) if not isinstance(b, FreeDim))]
         if wrong:
             raise ValueError(f"weights of other shapes than the config's in {model_path}: {wrong[:4]}")
     return out
