@@ -49,8 +49,9 @@ def parse():
     ap.add_argument("--config4", action="store_true", help="BASELINE configs[3]: 8 mixed image+text requests per GPU, batched (B = 8)")
     ap.add_argument("--config5", action="store_true", help="BASELINE configs[4]: fp8 (e4m3) weights, W8A8 prefill on the fp8 MFMA, int8 KV cache")
     ap.add_argument("--fp8-weight-only", action="store_true", help="with --config5: fp8_activations=False (dequantise + bf16 MFMA prefill)")
-    ap.add_argument("--layered", action="store_true", help="the layered text decoders (Pelalix layers of realistic sizes, random weights) beside "
-                    "Phi-3 layers of equal size: prefill and decode throughput; its own JSON line instead of the headline one")
+    ap.add_argument("--layered", nargs="?", const="Pelalix", default=None, choices=("Pelalix", "Pudisun"),
+                    help="a layered text decoder (layers of realistic sizes, random weights) beside Phi-3 layers (Pudisun: and Pelalix layers) of equal "
+                    "size: prefill and decode throughput; its own JSON line instead of the headline one")
     ap.add_argument("--tiny", action="store_true", help="tiny config (debug only; the result is NOT the headline metric)")
     return ap.parse_args()
 
@@ -279,6 +280,21 @@ def layered_config_dict(width, heads, kv, dim, ff, layers=LAYERED_LAYERS):
     return {"architecture": "Pelalix", "width": width, "vocab": LAYERED_VOCAB, "norm": {"eps": 1e-5}, "embedding": {"scale": 1.0}, "layers": [layer] * layers}
 
 
+# Pudisun: width, ff, latent attention (heads, dim, rotated dim, vdim, rank), gated linear attention (heads, dim, vdim); the layers alternate.
+# Beside them Phi-3 and Pelalix layers of the same width and feed-forward whose attention has as many 96-wide heads as the width holds.
+PUDISUN_SIZES = [(3072, 8192, (32, 64, 32, 96, 512), (32, 64, 96)), (3072, 8192, (24, 128, 64, 128, 512), (16, 96, 192)),
+                 (1536, 4096, (16, 64, 32, 96, 256), (16, 48, 96))]
+
+
+def pudisun_config_dict(width, ff, latent, gla, layers=LAYERED_LAYERS):
+    H, dim, rot, vdim, rank = latent
+    rotary = {"base": 10000.0, "dims": rot, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}
+    mixers = [("latent_attention", {"heads": H, "dim": dim, "rot_dim": rot, "vdim": vdim, "kv_rank": rank, "rot": rotary, "scale": (dim + rot) ** -0.5}),
+              ("gla", {"heads": gla[0], "dim": gla[1], "vdim": gla[2], "tau": 16.0})]
+    return {"architecture": "Pudisun", "width": width, "vocab": LAYERED_VOCAB, "norm": {"eps": 1e-5}, "residual_mult": 0.7, "logit_scale": 0.25,
+            "layers": [{"type": t, "mixer": m, "mlp": {"kind": "dense", "ff": ff}} for t, m in (mixers * layers)[:layers]]}
+
+
 def layered_run(model, prompts, decodes, steps, reps=5):
     """{prompt length: (ms, tokens/s)} of the whole prompt call and {(batch, context): (ms per step, tokens/s)} of the captured greedy step."""
     import numpy as np
@@ -322,22 +338,35 @@ def bench_layered(args):
     from phi_3_vision_mlx_amd.config import phi3v_config_dict
     torch.cuda.set_device(0)
     prompts, decodes = (512, 2048, 8192), ((1, 512), (1, 2048), (1, 8192), (8, 2048))
+    own = args.layered.lower()
+
+    def phi3(width, heads, kv, ff):
+        return dict(phi3v_config_dict(vision=False), hidden_size=width, num_attention_heads=heads, num_key_value_heads=kv, intermediate_size=ff,
+                    num_hidden_layers=LAYERED_LAYERS)
+    if own == "pelalix":
+        sizes = [({"width": width, "heads": heads, "kv_heads": kv, "head_size": dim, "ff": ff},
+                  {"pelalix": layered_config_dict(width, heads, kv, dim, ff), "phi3": phi3(width, heads, kv, ff)})
+                 for width, heads, kv, dim, ff in LAYERED_SIZES]
+    else:
+        sizes = [({"width": width, "ff": ff, "latent_heads_dim_rot_vdim_rank": latent, "gla_heads_dim_vdim": gla},
+                  {"pudisun": pudisun_config_dict(width, ff, latent, gla), "pelalix": layered_config_dict(width, width // 96, width // 96, 96, ff),
+                   "phi3": phi3(width, width // 96, width // 96, ff)}) for width, ff, latent, gla in PUDISUN_SIZES]
     rows = []
-    for width, heads, kv, dim, ff in LAYERED_SIZES:
-        row = {"width": width, "heads": heads, "kv_heads": kv, "head_size": dim, "ff": ff, "layers": LAYERED_LAYERS, "vocab": LAYERED_VOCAB}
-        phi = dict(phi3v_config_dict(vision=False), hidden_size=width, num_attention_heads=heads, num_key_value_heads=kv, intermediate_size=ff,
-                   num_hidden_layers=LAYERED_LAYERS)
-        for name, cfg in (("pelalix", layered_config_dict(width, heads, kv, dim, ff)), ("phi3", phi)):
+    for size, configs in sizes:
+        row = dict(size, layers=LAYERED_LAYERS, vocab=LAYERED_VOCAB)
+        for name, cfg in configs.items():
             model, _ = load_synthetic(config=cfg, device="cuda:0")
-            print("layered:", name, width, heads, kv, file=sys.stderr, flush=True)
+            print("layered:", name, size, file=sys.stderr, flush=True)
             row[name] = layered_run(model, prompts, decodes, args.steps if args.steps != 128 else 48)
             del model
             torch.cuda.empty_cache()
-        row["pelalix_over_phi3_time"] = {
-            k: {s: round(row["pelalix"][k][s][f] / row["phi3"][k][s][f], 3) for s in row["phi3"][k]} for k, f in (("prefill", "ms"), ("decode", "ms_per_step"))}
+        for other in configs:
+            if other != own:
+                row[f"{own}_over_{other}_time"] = {k: {s: round(row[own][k][s][f] / row[other][k][s][f], 3) for s in row[other][k]}
+                                                   for k, f in (("prefill", "ms"), ("decode", "ms_per_step"))}
         rows.append(row)
-    print(json.dumps({"metric": "layered decoders: prefill ms and decode ms per step beside Phi-3 layers of equal size", "dtype": "bf16",
-                      "data": "synthetic", "higher_is_better": False, "sizes": rows}), flush=True)
+    print(json.dumps({"metric": f"layered decoders ({args.layered}): prefill ms and decode ms per step beside layers of equal size of the other models",
+                      "dtype": "bf16", "data": "synthetic", "higher_is_better": False, "sizes": rows}), flush=True)
 
 
 def main():

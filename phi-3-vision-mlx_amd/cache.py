@@ -241,11 +241,11 @@ class LayeredCacheState(CacheState):
 
     @property
     def k(self):
-        return [m.k for m in self.mix]
+        return [getattr(m, "k", None) for m in self.mix]
 
     @property
     def v(self):
-        return [m.v for m in self.mix]
+        return [getattr(m, "v", None) for m in self.mix]
 
     @property
     def recurrent(self):

@@ -7,12 +7,13 @@
 //
 // One new token: a workgroup per (head, sequence) reads the state out of the ring's slot past % R and writes the next slot.
 // A prompt: chunks of 64 tokens in three launches --
-//   k_gla_chunk   per chunk: what its tokens leave in the state, sum_s (k_s a_{s+1} .. a_end) v_s^T, and the whole chunk's decay
+//   k_gla_chunk   per chunk: the decays c_t (running sums of log2 a), what the chunk's tokens leave in the state,
+//                 sum_s (k_s 2^(c_end - c_s)) v_s^T, and the whole chunk's decay 2^c_end
 //   k_gla_scan    per state element: the states at the chunks' starts, in order
-//   k_gla_out     per chunk: (q_t a_1 .. a_t) S_start + sum_{s <= t} (q_t a_{s+1} .. a_t . k_s) v_s, norm, gate
-// Decays are kept as running sums of log2 a (c_t); every exponential taken is of c_t - c_s with s <= t, never positive, so that no decay
-// is too strong for it: across the 16-token blocks of a chunk both factors refer to the later block's start, inside a block the
-// difference is taken pair by pair.
+//   k_gla_out     per chunk: (q_t 2^c_t) S_start + sum_{s <= t} (q_t . k_s 2^(c_t - c_s)) v_s, norm, gate
+// No decay is too strong for it: an exponential is taken of c_t - c_s with s <= t only, never positive.  Across the 16-token blocks of a
+// chunk both factors refer to the later block's start; inside a block the keys' factor would be positive, so a block over which some
+// channel decays by more than 2^GLA_SAFE takes its exponentials pair by pair.
 #include "p3v_layered.h"
 
 #define GLA_C 64                     // tokens of a chunk
@@ -25,15 +26,19 @@ struct GlaP {
   int B, L, H, dim, vdim, rank, ld, past, R, keep, n_tok, store;
 };
 
-// log2 of the decay, from z = W_a2 a1 + b
+// log2 of the decay, from z = W_a2 a1 + b: log sigmoid(z) = min(z, 0) - log(1 + x) with x = e^-|z|, the rounding of 1 + x given back
 __device__ __forceinline__ float log2_decay(float z, float inv_tau) {
-  return (fminf(z, 0.f) - log1pf(expf(-fabsf(z)))) * inv_tau * GLA_LOG2E;
+  const float x = __builtin_amdgcn_exp2f(-fabsf(z) * GLA_LOG2E), u = 1.f + x;
+  const float l = __builtin_amdgcn_logf(u) + (x - (u - 1.f)) * GLA_LOG2E * __builtin_amdgcn_rcpf(u);
+  return (fminf(z, 0.f) * GLA_LOG2E - l) * inv_tau;
 }
-__device__ __forceinline__ float row16_sum(float v) {
-  v += P3V_DPP_F32(v, 0xB1);
-  v += P3V_DPP_F32(v, 0x4E);
-  v += P3V_DPP_F32(v, 0x124);
-  return v + P3V_DPP_F32(v, 0x128);
+// 2^x - 1 for -1 < x <= 0, 2^x below: what a step multiplies a state with, next to the state itself or next to nothing.  (A slow decay is
+// 1 - tiny: rounded to fp32 before it meets the state, it would be off by up to 2^-25 in every step, the same way each time.)
+__device__ __forceinline__ float decay_less_one(float x) {
+  if (x <= -1.f) return __builtin_amdgcn_exp2f(x);
+  const float t = x * 0.6931471805599453f;
+  const float series = t * fmaf(t, fmaf(t, fmaf(t, fmaf(t, 1.f / 120.f, 1.f / 24.f), 1.f / 6.f), 0.5f), 1.f);
+  return t > -0.03f ? series : __builtin_amdgcn_exp2f(x) - 1.f;
 }
 __device__ __forceinline__ float silu32(float g) { return g / (1.f + expf(-g)); }
 
@@ -46,7 +51,7 @@ __global__ void __launch_bounds__(512) k_gla_steps(GlaP p) {
   extern __shared__ float sm[];
   const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x, dim = p.dim, vdim = p.vdim;
   const int nc = (vdim + V - 1) / V, ng = max(1, 512 / nc);
-  float *q = sm, *k = q + dim, *al = k + dim, *v = al + dim, *po = v + vdim;      // po [ng][vdim]
+  float *q = sm, *k = q + dim, *al = k + dim, *rest = al + dim, *v = rest + dim, *po = v + vdim;      // po [ng][vdim]
   __shared__ float red[8];
   const int past = p.d_past ? *p.d_past : p.past, first = p.pad_len ? p.pad_len[b] : 0;
   const size_t head = (size_t)dim * vdim, at = (size_t)b * p.R * p.H + h;
@@ -81,8 +86,17 @@ __global__ void __launch_bounds__(512) k_gla_steps(GlaP p) {
       k[d] = load_act(row + (p.H + h) * dim + d);
       float z = bf16_to_f32(p.a2b[h * dim + d]);
       const bf16_t* w = p.a2 + (size_t)(h * dim + d) * p.rank;
-      for (int r = 0; r < p.rank; ++r) z = fmaf(bf16_to_f32(w[r]), load_act(a1 + r), z);
-      al[d] = __builtin_amdgcn_exp2f(log2_decay(z, p.inv_tau));
+      int r = 0;
+      for (; r + 16 <= p.rank; r += 16) {                        // (sixteen at a time: all loads in flight)
+        float wr[16], ar[16];
+#pragma unroll
+        for (int j = 0; j < 16; ++j) wr[j] = bf16_to_f32(w[r + j]), ar[j] = load_act(a1 + r + j);
+#pragma unroll
+        for (int j = 0; j < 16; ++j) z = fmaf(wr[j], ar[j], z);
+      }
+      for (; r < p.rank; ++r) z = fmaf(bf16_to_f32(w[r]), load_act(a1 + r), z);
+      const float x = log2_decay(z, p.inv_tau);
+      al[d] = decay_less_one(x), rest[d] = x > -1.f ? 1.f : 0.f;
     }
     for (int i = tid; i < vdim; i += 512) v[i] = load_act(row + 2 * p.H * dim + h * vdim + i);
     __syncthreads();
@@ -91,10 +105,10 @@ __global__ void __launch_bounds__(512) k_gla_steps(GlaP p) {
 #pragma unroll
       for (int j = 0; j < V; ++j) o[j] = 0.f, vv[j] = v[c + j];
       auto update = [&](int d, float (&x)[V]) {
-        const float a = al[d], kd = k[d], qd = q[d];
+        const float a = al[d], kd = k[d], qd = q[d], one = rest[d];
 #pragma unroll
         for (int j = 0; j < V; ++j) {
-          x[j] = live ? fmaf(a, x[j], kd * vv[j]) : 0.f;
+          x[j] = live ? fmaf(a, x[j], fmaf(one, x[j], kd * vv[j])) : 0.f;
           o[j] = fmaf(qd, x[j], o[j]);
         }
         if (dst) {
@@ -132,7 +146,22 @@ __global__ void __launch_bounds__(512) k_gla_steps(GlaP p) {
 }
 
 // ================================================================ prompts: chunks
-// c[t][d] (row stride S) = sum of log2 a over the chunk's tokens up to t, 256 threads.  a1: LDS scratch of 64 x 17 floats.  Tokens that
+// the live tokens [lo, hi) of a chunk
+__device__ __forceinline__ void gla_span(const GlaP& p, int b, int l0, int& lo, int& hi) {
+  const int past = p.d_past ? *p.d_past : p.past, first = p.pad_len ? p.pad_len[b] : 0;
+  lo = min(max(first - past - l0, 0), GLA_C);
+  hi = max(min(p.n_tok - l0, GLA_C), lo);
+}
+// LDS row strides (elements): token rows of channels (16 rows of 4 floats in distinct banks), channel rows of tokens
+__host__ __device__ __forceinline__ int gla_dim16(int n) { return (n + 15) / 16 * 16; }
+__host__ __device__ __forceinline__ int gla_stride(int n) { return gla_dim16(n) + 4; }
+#define GLA_TS (GLA_C + 4)
+__host__ __device__ __forceinline__ int gla_key_rows(int dim) { return max(gla_dim16(dim), 32); }     // (also the scratch of gla_decays)
+// workspace: states [chunk, B, H, dim, vdim], decays of whole chunks [chunk, B, H, dim], running sums [B L, H, dim]
+__host__ __device__ __forceinline__ size_t gla_decay_at(const GlaP& p, int nc) { return (size_t)nc * p.B * p.H * p.dim * p.vdim; }
+__host__ __device__ __forceinline__ size_t gla_sums_at(const GlaP& p, int nc) { return gla_decay_at(p, nc) + (size_t)nc * p.B * p.H * p.dim; }
+
+// c[t][d] (row stride S) = sum of log2 a over the chunk's tokens up to t, 256 threads.  a1: LDS scratch of 64 x 20 floats.  Tokens that
 // are none (padding, behind the end) decay nothing.
 template <typename T>
 __device__ __forceinline__ void gla_decays(const GlaP& p, int b, int h, int l0, int lo, int hi, float* c, int S, float* a1) {
@@ -144,30 +173,35 @@ __device__ __forceinline__ void gla_decays(const GlaP& p, int b, int h, int l0, 
   const T* base = (const T*)p.y + ((size_t)b * p.L + l0) * p.ld + 2 * p.H * (dim + p.vdim);
   for (int r0 = 0; r0 < p.rank; r0 += 16) {
     const int nr = min(16, p.rank - r0);
-    __syncthreads();
-    for (int i = tid; i < GLA_C * 16; i += 256) {
-      const int t = i >> 4, r = i & 15;
-      a1[t * 17 + r] = t >= lo && t < hi && r < nr ? load_act(base + (size_t)t * p.ld + r0 + r) : 0.f;
+    if (r0) __syncthreads();
+#pragma unroll
+    for (int i = 0; i < GLA_C * 16 / 256; ++i) {
+      const int t = (tid >> 4) + i * 16, r = tid & 15;
+      a1[t * 20 + r] = t >= lo && t < hi && r < nr ? load_act(base + (size_t)t * p.ld + r0 + r) : 0.f;
+    }
+    float w[16];
+    if (mine) {
+#pragma unroll
+      for (int r = 0; r < 16; ++r) w[r] = r < nr ? bf16_to_f32(p.a2[(size_t)(h * dim + d) * p.rank + r0 + r]) : 0.f;
     }
     __syncthreads();
     if (mine) {
-      float w[16];
-#pragma unroll
-      for (int r = 0; r < 16; ++r) w[r] = r < nr ? bf16_to_f32(p.a2[(size_t)(h * dim + d) * p.rank + r0 + r]) : 0.f;
       const float bias = bf16_to_f32(p.a2b[h * dim + d]);
+      const bool last = r0 + 16 >= p.rank;
+      float run = 0.f;
       for (int t = g * per; t < (g + 1) * per; ++t) {
         float z = r0 == 0 ? bias : c[t * S + d];
 #pragma unroll
-        for (int r = 0; r < 16; ++r) z = fmaf(w[r], a1[t * 17 + r], z);
+        for (int r = 0; r < 16; r += 4) {
+          const float4 x = *(const float4*)(a1 + t * 20 + r);
+          z = fmaf(w[r], x.x, z), z = fmaf(w[r + 1], x.y, z), z = fmaf(w[r + 2], x.z, z), z = fmaf(w[r + 3], x.w, z);
+        }
+        if (last) {
+          run += t >= lo && t < hi ? log2_decay(z, p.inv_tau) : 0.f;
+          z = run;
+        }
         c[t * S + d] = z;
       }
-    }
-  }
-  if (mine) {
-    float run = 0.f;
-    for (int t = g * per; t < (g + 1) * per; ++t) {
-      if (t >= lo && t < hi) run += log2_decay(c[t * S + d], p.inv_tau);
-      c[t * S + d] = run;
     }
   }
   __syncthreads();
@@ -179,76 +213,100 @@ __device__ __forceinline__ void gla_decays(const GlaP& p, int b, int h, int l0, 
     for (int t = g * per; t < (g + 1) * per; ++t) c[t * S + d] += off;
   __syncthreads();
 }
-// the live tokens [lo, hi) of a chunk
-__device__ __forceinline__ void gla_span(const GlaP& p, int b, int l0, int& lo, int& hi) {
-  const int past = p.d_past ? *p.d_past : p.past, first = p.pad_len ? p.pad_len[b] : 0;
-  lo = min(max(first - past - l0, 0), GLA_C);
-  hi = max(min(p.n_tok - l0, GLA_C), lo);
+
+// rows of 64 tokens -> LDS, channel rows of tokens (row stride GLA_TS); dead tokens and channels behind n are zero.  A wave takes 32
+// tokens x 16 channels, 8 channels a lane: its LDS writes fall into distinct banks.
+template <typename T>
+__device__ __forceinline__ void gla_transpose(const T* src, int ld, int n, int lo, int hi, T* dst, int tid) {
+  const int t8 = tid & 31, c8 = (tid >> 5) * 8;
+  for (int c0 = c8; c0 < gla_dim16(n); c0 += 64)
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int t = t8 + 32 * i;
+      __attribute__((aligned(16))) T x[8] = {};
+      if (t >= lo && t < hi && c0 < n) {
+#pragma unroll
+        for (int j = 0; j < 8; j += 16 / (int)sizeof(T)) *(u32x4_t*)(x + j) = *(const u32x4_t*)(src + (size_t)t * ld + c0 + j);
+      }
+#pragma unroll
+      for (int j = 0; j < 8; ++j) dst[(c0 + j) * GLA_TS + t] = x[j];
+    }
 }
-__host__ __device__ __forceinline__ int gla_stride1(int n) { return (n + 63) / 64 * 64 + 16; }   // four rows of 16 floats in distinct banks
-__host__ __device__ __forceinline__ int gla_stride(int n) { return (n + 7) / 8 * 8 + 4; }        // sixteen rows of 4 floats in distinct banks
+__device__ __forceinline__ void load4(const bf16_t* p, float (&v)[4]) {
+  const u32x2_t w = *(const u32x2_t*)p;
+  v[0] = bf16lo(w[0]), v[1] = bf16hi(w[0]), v[2] = bf16lo(w[1]), v[3] = bf16hi(w[1]);
+}
+__device__ __forceinline__ void load4(const float* p, float (&v)[4]) {
+  const float4 w = *(const float4*)p;
+  v[0] = w.x, v[1] = w.y, v[2] = w.z, v[3] = w.w;
+}
+__device__ __forceinline__ void store4(bf16_t* p, const float (&v)[4]) { *(u32x2_t*)p = (u32x2_t){pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])}; }
+__device__ __forceinline__ void store4(float* p, const float (&v)[4]) { *(float4*)p = make_float4(v[0], v[1], v[2], v[3]); }
 
-__host__ __device__ __forceinline__ size_t gla_decay_at(const GlaP& p, int nc) { return (size_t)nc * p.B * p.H * p.dim * p.vdim; }
-
+// The fp32 MFMA takes one k per lane group; four of them in a row are given k = 4 group + 0 .. 3 of a run of 16, so that an operand's four
+// values are one LDS read.
 template <typename T>
 __global__ void __launch_bounds__(256) k_gla_chunk(GlaP p) {
-  extern __shared__ float sm[];
+  extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   const int ch = blockIdx.x, h = blockIdx.y, b = blockIdx.z, tid = threadIdx.x, lane = tid & 63, lc = lane & 15, lg = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int dim = p.dim, vdim = p.vdim, KS = gla_stride1(dim), VS = gla_stride1(vdim), l0 = ch * GLA_C;
-  float *kd = sm, *v = kd + GLA_C * KS, *a1 = v;                 // (the values come when the decays are done)
+  const int dim = p.dim, vdim = p.vdim, DS = gla_stride(dim), l0 = ch * GLA_C;
+  float *cum = (float*)smem, *kd = cum + GLA_C * DS;                     // [64][DS], [dim16][TS]
+  T* vt = (T*)(kd + gla_key_rows(dim) * GLA_TS);                           // [vdim16][TS]
   int lo, hi;
   gla_span(p, b, l0, lo, hi);
-  gla_decays<T>(p, b, h, l0, lo, hi, kd, KS, a1);
   const T* base = (const T*)p.y + ((size_t)b * p.L + l0) * p.ld;
-  for (int i = tid; i < GLA_C * (vdim / 8); i += 256) {
-    const int t = i / (vdim / 8), c = (i - t * (vdim / 8)) * 8;
-    float x[8] = {0, 0, 0, 0, 0, 0, 0, 0};
-    if (t >= lo && t < hi) load_acts<8>(base + (size_t)t * p.ld + 2 * p.H * dim + h * vdim + c, x);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) v[t * VS + c + j] = x[j];
-  }
+  gla_transpose<T>(base + 2 * p.H * dim + h * vdim, p.ld, vdim, lo, hi, vt, tid);
+  gla_decays<T>(p, b, h, l0, lo, hi, cum, DS, kd);
   const size_t row = (size_t)ch * p.B * p.H + (size_t)b * p.H + h;
   float* decay = p.ws + gla_decay_at(p, gridDim.x) + row * dim;
-  float end[8];                                                  // this thread's 8 channels at the chunk's end
-  const int per = dim / 8, c8 = (tid % per) * 8, t8 = tid / per, nt = 256 / per;
+  float* sums = p.ws + gla_sums_at(p, gridDim.x) + ((size_t)b * p.L + l0) * p.H * dim + h * dim;
+  const int t8 = tid & 31, c8 = (tid >> 5) * 8;
+  for (int c0 = c8; c0 < gla_dim16(dim); c0 += 64) {
+    float end[8] = {};
+    if (c0 < dim) load_acts<8>(cum + (GLA_C - 1) * DS + c0, end);
+    if (t8 == 0 && c0 < dim)
 #pragma unroll
-  for (int j = 0; j < 8; ++j) end[j] = kd[(GLA_C - 1) * KS + c8 + j];
-  if (t8 == 0)
+      for (int j = 0; j < 8; ++j) decay[c0 + j] = __builtin_amdgcn_exp2f(end[j]);
 #pragma unroll
-    for (int j = 0; j < 8; ++j) decay[c8 + j] = __builtin_amdgcn_exp2f(end[j]);
-  __syncthreads();
-  if (t8 < nt)
-    for (int t = t8; t < GLA_C; t += nt) {
-      float x[8] = {0, 0, 0, 0, 0, 0, 0, 0};
-      if (t >= lo && t < hi) load_acts<8>(base + (size_t)t * p.ld + (p.H + h) * dim + c8, x);
+    for (int i = 0; i < 2; ++i) {
+      const int t = t8 + 32 * i;
+      float x[8] = {}, c[8] = {};
+      if (c0 < dim) load_acts<8>(cum + t * DS + c0, c);
+      if (t >= lo && t < hi && c0 < dim) load_acts<8>(base + (size_t)t * p.ld + (p.H + h) * dim + c0, x);
+      if (l0 + t < p.L && c0 < dim) store_acts<8>(sums + (size_t)t * p.H * dim + c0, c);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) kd[t * KS + c8 + j] = x[j] * __builtin_amdgcn_exp2f(fminf(end[j] - kd[t * KS + c8 + j], 0.f));
+      for (int j = 0; j < 8; ++j) kd[(c0 + j) * GLA_TS + t] = x[j] * __builtin_amdgcn_exp2f(fminf(end[j] - c[j], 0.f));
     }
+  }
   __syncthreads();
-  // A operand: row = key channel, k = token; B operand: column = value channel
-  const int dt = (dim + 15) / 16, vg = (vdim + 63) / 64;
+  // A operand: row = key channel; B operand: column = value channel; a wave takes consecutive tiles, the keys of a row of them stay
+  const int VT = (vdim + 15) / 16, tiles = (dim + 15) / 16 * VT, per = (tiles + 3) / 4;
   float* dst = p.ws + row * dim * vdim;
-  for (int u = wave; u < dt * vg; u += 4) {
-    const int d0 = (u / vg) * 16, v0 = (u % vg) * 64;
-    f32x4_t acc[4];
+  float ka[4][4];
+  int have = -1;
+  for (int u = wave * per; u < min((wave + 1) * per, tiles); ++u) {
+    const int dt = u / VT, v0 = (u - dt * VT) * 16;
+    if (dt != have) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j) acc[j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-    const float* ka = kd + lg * KS + d0 + lc;
-    const float* va = v + lg * VS + v0 + lc;
-#pragma unroll 4
-    for (int s = 0; s < GLA_C; s += 4) {
-      const float a = ka[s * KS];
-#pragma unroll
-      for (int j = 0; j < 4; ++j) acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, va[s * VS + j * 16], acc[j], 0, 0, 0);
+      for (int q = 0; q < 4; ++q) load4(kd + (dt * 16 + lc) * GLA_TS + q * 16 + lg * 4, ka[q]);
+      have = dt;
     }
+    f32x4_t acc = {0.f, 0.f, 0.f, 0.f}, acc2 = {0.f, 0.f, 0.f, 0.f};     // (two chains: the products do not wait for each other)
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
+    for (int q = 0; q < 4; ++q) {
+      float vb[4];
+      load4(vt + (v0 + lc) * GLA_TS + q * 16 + lg * 4, vb);
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = d0 + lg * 4 + r, c = v0 + j * 16 + lc;
-        if (d < dim && c < vdim) dst[(size_t)d * vdim + c] = acc[j][r];
+      for (int i = 0; i < 4; ++i) {
+        if (q & 1) acc2 = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[q][i], vb[i], acc2, 0, 0, 0);
+        else acc = __builtin_amdgcn_mfma_f32_16x16x4f32(ka[q][i], vb[i], acc, 0, 0, 0);
       }
+    }
+    if (v0 + lc < vdim)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (dt * 16 + lg * 4 + r < dim) dst[(size_t)(dt * 16 + lg * 4 + r) * vdim + v0 + lc] = acc[r] + acc2[r];
   }
 }
 
@@ -282,169 +340,153 @@ __global__ void __launch_bounds__(256) k_gla_scan(GlaP p, int nc) {
   if (p.store) *(float4*)(p.s + (((size_t)b * p.R + (past + p.n_tok) % p.R) * p.H + h) * head + 4 * i) = s;
 }
 
-// Wave w owns the chunk's tokens 16 w .. 16 w + 15; VG: groups of 64 value channels.
-template <typename T> struct GlaOutLds {
-  int DS, VS, PS, cum, k, qt, v, p, total;                       // strides (elements) and byte offsets
-  __host__ __device__ GlaOutLds(int dim, int vdim) {
-    DS = gla_stride(dim), VS = (vdim + 15) / 16 * 16 + 8, PS = GLA_C + 4;
-    cum = 0, qt = cum + GLA_C * DS * 4, p = qt + GLA_C * DS * 4, k = p + GLA_C * PS * 4, v = k + GLA_C * DS * (int)sizeof(T);
-    total = v + GLA_C * VS * (int)sizeof(T);
-  }
-};
-template <typename T, int VG>
+// Wave w owns the chunk's tokens 16 w .. 16 w + 15, one per lane column; everything is transposed: pairs [s, t] and outputs [v, t], so that a
+// lane's pairs are the operand of the product with the values as they lie.  VT: 16-channel tiles of a value.
+#define GLA_SAFE 60.f
+template <typename T, int VT>
 __global__ void __launch_bounds__(256) k_gla_out(GlaP p) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   const int ch = blockIdx.x, h = blockIdx.y, b = blockIdx.z, tid = threadIdx.x, lane = tid & 63, lc = lane & 15, lg = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int dim = p.dim, vdim = p.vdim, l0 = ch * GLA_C;
-  const GlaOutLds<T> o_(dim, vdim);
-  const int DS = o_.DS, VS = o_.VS, PS = o_.PS;
-  float *cum = (float*)(smem + o_.cum), *qt = (float*)(smem + o_.qt), *P = (float*)(smem + o_.p);
-  T *k = (T*)(smem + o_.k), *v = (T*)(smem + o_.v);
+  const int dim = p.dim, vdim = p.vdim, DS = gla_stride(dim), l0 = ch * GLA_C, t0 = wave * 16;
+  float* cum = (float*)smem;                                             // [64][DS]
+  T *k = (T*)(cum + GLA_C * DS), *vt = k + GLA_C * DS;                   // [64][DS], [vdim16][TS]
   int lo, hi;
   gla_span(p, b, l0, lo, hi);
-  gla_decays<T>(p, b, h, l0, lo, hi, cum, DS, P);
   const T* base = (const T*)p.y + ((size_t)b * p.L + l0) * p.ld;
-  for (int i = tid; i < GLA_C * (dim / 4); i += 256) {           // (4 at a time: the strides are multiples of 4)
-    const int t = i / (dim / 4), c = (i - t * (dim / 4)) * 4;
-    const bool live = t >= lo && t < hi;
+  const float* sums = p.ws + gla_sums_at(p, gridDim.x) + ((size_t)b * p.L + l0) * p.H * dim + h * dim;
+  gla_transpose<T>(base + 2 * p.H * dim + h * vdim, p.ld, vdim, lo, hi, vt, tid);
+  const int n4 = gla_dim16(dim) / 4, t4 = tid >> 4;
+  for (int c = tid & 15; c < n4; c += 16)
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      k[t * DS + c + j] = live ? base[(size_t)t * p.ld + (p.H + h) * dim + c + j] : (T)0;
-      qt[t * DS + c + j] = live ? load_act(base + (size_t)t * p.ld + h * dim + c + j) * p.q_scale : 0.f;
+    for (int i = 0; i < 4; ++i) {
+      const int t = t4 + 16 * i;
+      float x[4] = {0.f, 0.f, 0.f, 0.f}, y[4] = {0.f, 0.f, 0.f, 0.f};
+      if (l0 + t < p.L && 4 * c < dim) load4(sums + (size_t)t * p.H * dim + 4 * c, x);
+      if (t >= lo && t < hi && 4 * c < dim) load4(base + (size_t)t * p.ld + (p.H + h) * dim + 4 * c, y);
+      store4(cum + t * DS + 4 * c, x), store4(k + t * DS + 4 * c, y);
     }
-  }
-  for (int i = tid; i < GLA_C * (vdim / 4); i += 256) {
-    const int t = i / (vdim / 4), c = (i - t * (vdim / 4)) * 4;
-    const bool live = t >= lo && t < hi;
-#pragma unroll
-    for (int j = 0; j < 4; ++j) v[t * VS + c + j] = live ? base[(size_t)t * p.ld + 2 * p.H * dim + h * vdim + c + j] : (T)0;
-  }
   __syncthreads();
-  const int t0 = wave * 16;
+  const float* ref = cum + max(t0 - 1, 0) * DS;                          // decays before this block (wave 0: none)
+  bool strong = false;                                                   // does some channel decay too much over the block?
+  const int tl = min(t0 + 15, p.L - 1 - l0);                             // its last row in memory
+  if (tl >= t0)
+    for (int d = lane; d < dim; d += 64) strong |= (wave ? ref[d] : 0.f) - cum[tl * DS + d] > GLA_SAFE;
+  strong = __builtin_amdgcn_ballot_w64(strong) != 0;
 
-  // ---- the block's own pairs: lane = (token s, quarter of the channels), all 16 tokens t
-  {
-    float sc[16];
-#pragma unroll
-    for (int t = 0; t < 16; ++t) sc[t] = 0.f;
-    for (int d = lg; d < dim; d += 4) {
-      const float ks = load_act(k + (t0 + lc) * DS + d), cs = cum[(t0 + lc) * DS + d];
-#pragma unroll
-      for (int t = 0; t < 16; ++t)
-        sc[t] = fmaf(qt[(t0 + t) * DS + d] * ks, __builtin_amdgcn_exp2f(fminf(cum[(t0 + t) * DS + d] - cs, 0.f)), sc[t]);
-    }
-#pragma unroll
-    for (int t = 0; t < 16; ++t) {
-      const float x = rows_sum(sc[t]);
-      if (lg == (t >> 2)) P[(t0 + t) * PS + t0 + lc] = t >= lc ? x : 0.f;
-    }
-  }
-  // ---- earlier blocks of the chunk: both factors refer to the block's start
-  const float* ref = cum + max(t0 - 1, 0) * DS;                  // (wave 0: the chunk's start, zero)
-  for (int i = lane; i < 16 * dim; i += 64) {
-    const int t = t0 + i / dim, d = i % dim;
-    qt[t * DS + d] *= __builtin_amdgcn_exp2f(fminf(cum[t * DS + d] - (wave ? ref[d] : 0.f), 0.f));
-  }
-  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");             // (the wave's own rows: no barrier)
-  const float* qa = qt + (t0 + lc) * DS + lg;
-  if (wave) {
-    f32x4_t sc[3];
-#pragma unroll
-    for (int j = 0; j < 3; ++j) sc[j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-    for (int d0 = 0; d0 < dim; d0 += 4) {
-      const float a = qa[d0], rd = ref[d0 + lg];
-#pragma unroll
-      for (int j = 0; j < 3; ++j)
-        if (j < wave) {
-          const int s = j * 16 + lc;
-          const float kb = load_act(k + s * DS + d0 + lg) * __builtin_amdgcn_exp2f(fminf(rd - cum[s * DS + d0 + lg], 0.f));
-          sc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, kb, sc[j], 0, 0, 0);
-        }
-    }
-#pragma unroll
-    for (int j = 0; j < 3; ++j)
-      if (j < wave) {
-#pragma unroll
-        for (int r = 0; r < 4; ++r) P[(t0 + lg * 4 + r) * PS + j * 16 + lc] = sc[j][r];
-      }
-  }
-  // ---- the state at the chunk's start, then the pairs
-  f32x4_t o[VG][4];
-#pragma unroll
-  for (int g = 0; g < VG; ++g)
-#pragma unroll
-    for (int j = 0; j < 4; ++j) o[g][j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+  const int l = min(l0 + t0 + lc, p.L - 1);                              // this lane's token
+  const T* q = (const T*)p.y + ((size_t)b * p.L + l) * p.ld + h * dim;
   const float* S = p.ws + ((size_t)ch * p.B * p.H + (size_t)b * p.H + h) * dim * vdim;
-  int vc[VG][4];
+  f32x4_t sc[4], o[VT];
 #pragma unroll
-  for (int g = 0; g < VG; ++g)
+  for (int j = 0; j < 4; ++j) sc[j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int j = 0; j < 4; ++j) vc[g][j] = min(g * 64 + j * 16 + lc, vdim - 1);
-#pragma unroll 2
-  for (int d0 = 0; d0 < dim; d0 += 4) {
-    const float a = wave ? qa[d0] * __builtin_amdgcn_exp2f(ref[d0 + lg]) : qa[d0];
-    const float* sr = S + (size_t)(d0 + lg) * vdim;
+  for (int j = 0; j < VT; ++j) o[j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+  for (int d0 = 0; d0 < dim; d0 += 16) {
+    const int d = d0 + 4 * lg;
+    float qv[4] = {0.f, 0.f, 0.f, 0.f}, ct[4], rf[4] = {0.f, 0.f, 0.f, 0.f}, qd[4];
+    if (d < dim) load4(q + d, qv);
+    float sv[VT][4];
 #pragma unroll
-    for (int g = 0; g < VG; ++g)
+    for (int j = 0; j < VT; ++j)
 #pragma unroll
-      for (int j = 0; j < 4; ++j) o[g][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, sr[vc[g][j]], o[g][j], 0, 0, 0);
-  }
-  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-  const float* pa = P + (t0 + lc) * PS + lg;
-#pragma unroll 2
-  for (int s = 0; s < t0 + 16; s += 4) {
-    const float a = pa[s];
-    const T* vr = v + (s + lg) * VS;
+      for (int i = 0; i < 4; ++i) sv[j][i] = S[(size_t)min(d + i, dim - 1) * vdim + min(j * 16 + lc, vdim - 1)];
+    load4(cum + (t0 + lc) * DS + d, ct);
+    if (wave) load4(ref + d, rf);
 #pragma unroll
-    for (int g = 0; g < VG; ++g)
+    for (int i = 0; i < 4; ++i) {
+      qv[i] *= p.q_scale * __builtin_amdgcn_exp2f(fminf(ct[i] - rf[i], 0.f));
+      qd[i] = qv[i] * __builtin_amdgcn_exp2f(rf[i]);
+    }
 #pragma unroll
-      for (int j = 0; j < 4; ++j) o[g][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(a, load_act(vr + vc[g][j]), o[g][j], 0, 0, 0);
-  }
-  // ---- norm over the value channels (a token: 4 registers rows x 16 lanes), gate
+    for (int j = 0; j < 4; ++j)
+      if (j < wave || (j == wave && !strong)) {
+        float kb[4], cs[4];
+        load4(k + (j * 16 + lc) * DS + d, kb), load4(cum + (j * 16 + lc) * DS + d, cs);
 #pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    float ss = 0.f;
+        for (int i = 0; i < 4; ++i) kb[i] *= __builtin_amdgcn_exp2f(rf[i] - cs[i]);
 #pragma unroll
-    for (int g = 0; g < VG; ++g)
-#pragma unroll
-      for (int j = 0; j < 4; ++j) ss += g * 64 + j * 16 + lc < vdim ? o[g][j][r] * o[g][j][r] : 0.f;
-    const float rs = 1.f / sqrtf(row16_sum(ss) / (float)vdim + p.eps);
-    const int t = t0 + lg * 4 + r, l = l0 + t;
-    if (l >= p.L) continue;
-    const T* gate = base + (size_t)t * p.ld + 2 * p.H * dim + (p.H + h) * vdim;
-    T* out = (T*)p.out + ((size_t)b * p.L + l) * p.H * vdim + (size_t)h * vdim;
-#pragma unroll
-    for (int g = 0; g < VG; ++g)
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int c = g * 64 + j * 16 + lc;
-        if (c < vdim) store_act(out + c, o[g][j][r] * rs * bf16_to_f32(p.norm[c]) * silu32(load_act(gate + c)));
+        for (int i = 0; i < 4; ++i) sc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(kb[i], qv[i], sc[j], 0, 0, 0);
       }
+#pragma unroll
+    for (int j = 0; j < VT; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) o[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(sv[j][i], qd[i], o[j], 0, 0, 0);
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j)
+    if (j == wave) {                                                     // the block's own pairs: s <= t
+      if (strong) {
+        for (int d = 0; d < dim; ++d) {
+          const float qs = load_act(q + d) * p.q_scale, ct = cum[(t0 + lc) * DS + d];
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int s = (t0 + lg * 4 + r) * DS + d;
+            sc[j][r] = fmaf(qs * load_act(k + s), __builtin_amdgcn_exp2f(fminf(ct - cum[s], 0.f)), sc[j][r]);
+          }
+        }
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) sc[j][r] = lg * 4 + r <= lc ? sc[j][r] : 0.f;
+    }
+#pragma unroll
+  for (int j = 0; j < 4; ++j)
+    if (j <= wave) {
+#pragma unroll
+      for (int v = 0; v < VT; ++v) {
+        float va[4];
+        load4(vt + min(v * 16 + lc, gla_dim16(vdim) - 1) * GLA_TS + j * 16 + lg * 4, va);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) o[v] = __builtin_amdgcn_mfma_f32_16x16x4f32(va[i], sc[j][i], o[v], 0, 0, 0);
+      }
+    }
+  // ---- norm over the value channels, gate
+  float ss = 0.f;
+#pragma unroll
+  for (int v = 0; v < VT; ++v)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) ss += v * 16 + lg * 4 + r < vdim ? o[v][r] * o[v][r] : 0.f;
+  const float rs = 1.f / sqrtf(rows_sum(ss) / (float)vdim + p.eps);
+  if (l0 + t0 + lc >= p.L) return;
+  const T* gate = base + (size_t)(t0 + lc) * p.ld + 2 * p.H * dim + (p.H + h) * vdim;
+  T* out = (T*)p.out + ((size_t)b * p.L + l) * p.H * vdim + (size_t)h * vdim;
+#pragma unroll
+  for (int v = 0; v < VT; ++v) {
+    const int c = v * 16 + lg * 4;
+    if (c < vdim) {
+      float g[4], w[4];
+      load4(gate + c, g), load4(p.norm + c, w);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) g[r] = o[v][r] * rs * w[r] * (g[r] / (1.f + __expf(-g[r])));
+      store4(out + c, g);
+    }
   }
 }
 
 // ---------------------------------------------------------------- host side
 #define GLA_MAX_LDS (160 * 1024)
-static int gla_lds_out(int dim, int vdim, int f32) { return f32 ? GlaOutLds<float>(dim, vdim).total : GlaOutLds<bf16_t>(dim, vdim).total; }
-static int gla_lds_chunk(int dim, int vdim) { return GLA_C * (gla_stride1(dim) + max(gla_stride1(vdim), 17)) * 4; }
+static int gla_lds_out(int dim, int vdim, int e) { return GLA_C * gla_stride(dim) * (4 + e) + gla_dim16(vdim) * GLA_TS * e; }
+static int gla_lds_chunk(int dim, int vdim, int e) {
+  return GLA_C * gla_stride(dim) * 4 + gla_key_rows(dim) * GLA_TS * 4 + gla_dim16(vdim) * GLA_TS * e;
+}
 
 // chunks of a call (0: token by token)
 extern "C" int p3v_gla_plan(int B, int L, int H, int dim, int vdim, int f32) {
   if (B <= 0 || L <= 8 || H <= 0 || dim <= 0 || vdim <= 0 || dim % 8 || vdim % 8 || dim > 128 || vdim > 256 || H > 65535 || B > 65535) return 0;
-  if (gla_lds_out(dim, vdim, f32) > GLA_MAX_LDS || gla_lds_chunk(dim, vdim) > GLA_MAX_LDS) return 0;
+  const int e = f32 ? 4 : 2;
+  if (gla_lds_out(dim, vdim, e) > GLA_MAX_LDS || gla_lds_chunk(dim, vdim, e) > GLA_MAX_LDS) return 0;
   return p3v_cdiv(L, GLA_C);
 }
 extern "C" int64_t p3v_gla_ws_bytes(int B, int L, int H, int dim, int vdim, int n_chunk) {
   if (B <= 0 || L <= 0 || H <= 0 || dim <= 0 || vdim <= 0 || n_chunk < 0) return 0;
   if (n_chunk == 0) return L == 1 ? 0 : (int64_t)B * H * dim * vdim * 4;        // the state behind tokens that do not stay
-  return (int64_t)n_chunk * B * H * ((int64_t)dim * vdim + dim) * 4;
+  return ((int64_t)n_chunk * B * H * ((int64_t)dim * vdim + dim) + (int64_t)B * L * H * dim) * 4;
 }
 
 template <typename T> static int gla_steps(const GlaP& p, hipStream_t s) {
   const bool vec = p.vdim % 4 == 0;
   const int nc = vec ? p.vdim / 4 : p.vdim, ng = max(1, 512 / nc);
-  const size_t lds = (size_t)(3 * p.dim + p.vdim + ng * p.vdim) * 4;
+  const size_t lds = (size_t)(4 * p.dim + p.vdim + ng * p.vdim) * 4;
   if (nc > 512 || lds > 64 * 1024) return P3V_ERR_UNSUPPORTED;
   if (vec) hipLaunchKernelGGL((k_gla_steps<T, 4>), dim3(p.H, p.B), dim3(512), lds, s, p);
   else hipLaunchKernelGGL((k_gla_steps<T, 1>), dim3(p.H, p.B), dim3(512), lds, s, p);
@@ -461,15 +503,15 @@ template <typename T> static int gla_states(GlaP p, int n_tok, int store, hipStr
   if (gla_set_lds((const void*)k_gla_chunk<T>, set) != P3V_OK) return P3V_ERR_HIP;
   const int nc = p3v_cdiv(n_tok, GLA_C);
   p.n_tok = n_tok, p.store = store;
-  hipLaunchKernelGGL(k_gla_chunk<T>, dim3(nc, p.H, p.B), dim3(256), gla_lds_chunk(p.dim, p.vdim), s, p);
+  hipLaunchKernelGGL(k_gla_chunk<T>, dim3(nc, p.H, p.B), dim3(256), gla_lds_chunk(p.dim, p.vdim, (int)sizeof(T)), s, p);
   hipLaunchKernelGGL(k_gla_scan, dim3(p3v_cdiv((long)p.dim * p.vdim / 4, 256), p.B * p.H), dim3(256), 0, s, p, nc);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
 }
-template <typename T, int VG> static int gla_out(const GlaP& p, int nc, hipStream_t s) {
+template <typename T, int VT> static int gla_out(const GlaP& p, int nc, hipStream_t s) {
   static bool set = false;
-  if (gla_set_lds((const void*)k_gla_out<T, VG>, set) != P3V_OK) return P3V_ERR_HIP;
-  hipLaunchKernelGGL((k_gla_out<T, VG>), dim3(nc, p.H, p.B), dim3(256), GlaOutLds<T>(p.dim, p.vdim).total, s, p);
+  if (gla_set_lds((const void*)k_gla_out<T, VT>, set) != P3V_OK) return P3V_ERR_HIP;
+  hipLaunchKernelGGL((k_gla_out<T, VT>), dim3(nc, p.H, p.B), dim3(256), gla_lds_out(p.dim, p.vdim, (int)sizeof(T)), s, p);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
 }
@@ -477,7 +519,8 @@ template <typename T> static int gla_chunks(GlaP p, int nc, hipStream_t s) {
   int rc = gla_states<T>(p, p.L, p.keep == p.L, s);
   if (rc != P3V_OK) return rc;
   p.n_tok = p.L;
-  rc = p.vdim <= 64 ? gla_out<T, 1>(p, nc, s) : p.vdim <= 128 ? gla_out<T, 2>(p, nc, s) : gla_out<T, 4>(p, nc, s);
+  rc = p.vdim <= 32 ? gla_out<T, 2>(p, nc, s) : p.vdim <= 64 ? gla_out<T, 4>(p, nc, s) : p.vdim <= 96 ? gla_out<T, 6>(p, nc, s)
+     : p.vdim <= 128 ? gla_out<T, 8>(p, nc, s) : p.vdim <= 192 ? gla_out<T, 12>(p, nc, s) : gla_out<T, 16>(p, nc, s);
   if (rc == P3V_OK && p.keep > 0 && p.keep < p.L) rc = gla_states<T>(p, p.keep, 1, s);      // (the workspace is free again)
   return rc;
 }

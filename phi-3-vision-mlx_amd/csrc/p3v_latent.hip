@@ -112,16 +112,7 @@ __global__ void __launch_bounds__(256) k_latent_attn(LatP p) {
   float* red = (float*)(smem + C::TILE + C::Q + C::P);                   // [4][16]
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lc = lane & 15, lg = lane >> 4;
   const int split = blockIdx.x, h0 = blockIdx.y * 16, row = blockIdx.z, b = row / p.L;
-  const int past = p.d_past ? *p.d_past : p.past, pos = past + row - b * p.L, first = p.pad_len ? p.pad_len[b] : 0;
-  const int t_first = split * p.tiles_per_split, last = pos >> 6;
-  if (t_first > last) return;                                            // beyond the live keys: the merge does not look here
-  const int t0 = max(t_first, first >> 6), t1 = min(t_first + p.tiles_per_split, last + 1), h = h0 + lc;
-  float* ml = lat_ml(p.ws, p, row, split);
-  if (t0 >= t1) {                                                        // only padding here
-    if (tid < 16 && h < p.H) ml[2 * h] = LAT_NEG, ml[2 * h + 1] = 0.f;
-    return;
-  }
-  const int QW = p.rankp + p.rotp, HP = (p.H + 15) / 16 * 16;
+  const int QW = p.rankp + p.rotp, HP = (p.H + 15) / 16 * 16, t_first = split * p.tiles_per_split;
   const bf16_t* kb = (const bf16_t*)p.c + ((size_t)b * p.Tp + wave * 16 + lc) * QW + lg * 8;
   bf16x8_t kf[C::NC];
   auto load = [&](int t) {
@@ -129,7 +120,16 @@ __global__ void __launch_bounds__(256) k_latent_attn(LatP p) {
 #pragma unroll
     for (int c = 0; c < C::NC; ++c) kf[c] = *(const bf16x8_t*)(kr + c * 32);
   };
-  load(t0);
+  load(min(t_first, (p.Tp >> 6) - 1));                                   // (ahead of the position: the run's first tile, in most calls)
+  const int past = p.d_past ? *p.d_past : p.past, pos = past + row - b * p.L, first = p.pad_len ? p.pad_len[b] : 0, last = pos >> 6;
+  if (t_first > last) return;                                            // beyond the live keys: the merge does not look here
+  const int t0 = max(t_first, first >> 6), t1 = min(t_first + p.tiles_per_split, last + 1), h = h0 + lc;
+  float* ml = lat_ml(p.ws, p, row, split);
+  if (t0 >= t1) {                                                        // only padding here
+    if (tid < 16 && h < p.H) ml[2 * h] = LAT_NEG, ml[2 * h + 1] = 0.f;
+    return;
+  }
+  if (t0 != t_first) load(t0);
   const bf16_t* qg = (const bf16_t*)p.q + ((size_t)row * HP + h0) * QW;
   for (int e = tid; e < 16 * (C::NC * 4); e += 256) {
     const int i = e / (C::NC * 4), c = (e - i * (C::NC * 4)) * 8;
@@ -188,24 +188,37 @@ __global__ void __launch_bounds__(256) k_latent_attn(LatP p) {
 }
 
 // ---------------------------------------------------------------- merge, value up-projection, gate
-// A workgroup per (head, 64 value dimensions, 16 rows); its weights are requested before the merge.
+// A workgroup per (head, 128 value dimensions, 16 rows); its weights are requested before the merge.
 #define LAT_MAX_SPLIT 128
 template <int RC>
-__global__ void __launch_bounds__(256) k_latent_out(LatP p) {
+__global__ void __launch_bounds__(512) k_latent_out(LatP p) {
   constexpr int OS = RC * 64 + 8;
   __shared__ float wt[16][LAT_MAX_SPLIT];
   __shared__ __attribute__((aligned(16))) bf16_t ol[16 * OS];
-  __shared__ float4 part[256];
+  __shared__ float4 part[512];
   const int h = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lc = lane & 15, lg = lane >> 4;
-  const int row0 = blockIdx.z * 16, M = p.B * p.L, n_row = min(16, M - row0), past = p.d_past ? *p.d_past : p.past;
-  const int v0 = blockIdx.y * 64 + wave * 16;
+  const int row0 = blockIdx.z * 16, M = p.B * p.L, n_row = min(16, M - row0), v0 = blockIdx.y * 128 + wave * 16;
+  constexpr int R4 = RC * 16, U = 8;                                     // float4 columns of a latent; splits requested at once
+  const int items = n_row * R4, G = items >= 512 ? 1 : 512 / items, g = G > 1 ? tid / items : 0;
+  const size_t step = (size_t)p.H * p.rankp;
+  auto part_of = [&](int e) { return lat_o(p.ws, p, M, row0 + e / R4, 0) + (size_t)h * p.rankp + 4 * (e % R4); };
+  // few rows: the partials are requested before anything else -- which of them were written is known later
+  float4 x0[U];
+  if (G > 1) {
+    const float* o = part_of(tid - g * items);
+#pragma unroll
+    for (int u = 0; u < U; ++u) x0[u] = *(const float4*)(o + min(min(g, G - 1) + u * G, p.n_split - 1) * step);
+  }
+  const int past = p.d_past ? *p.d_past : p.past;
   bf16x8_t w[2 * RC];
   const bf16_t* wr = p.uv + ((size_t)h * p.vdim + min(v0 + lc, p.vdim - 1)) * p.rankp + lg * 8;
 #pragma unroll
   for (int c = 0; c < 2 * RC; ++c) w[c] = *(const bf16x8_t*)(wr + c * 32);
   auto live = [&](int row) { return min(p.n_split, ((past + row % p.L) >> 6) / p.tiles_per_split + 1); };
   const float sk = bf16_to_f32(p.sink[h]) * LAT_LOG2E;
-  for (int i = wave; i < n_row; i += 4) {
+  const int v = v0 + lg * 4;
+  const u32x2_t z = *(const u32x2_t*)((const bf16_t*)p.y + (size_t)(row0 + min(lc, n_row - 1)) * p.ld + lat_gate_col(p) + h * p.vdim + min(v, p.vdim - 4));
+  for (int i = wave; i < n_row; i += 8) {
     const int row = row0 + i, n = live(row);
     float m[2], l[2];
 #pragma unroll
@@ -219,26 +232,27 @@ __global__ void __launch_bounds__(256) k_latent_out(LatP p) {
     wt[i][lane] = m[0] > 0.5f * LAT_NEG ? w0 * f : -1.f;                 // (-1: no such split, or one of padding whose outputs were not written)
     wt[i][lane + 64] = m[1] > 0.5f * LAT_NEG ? w1 * f : -1.f;
   }
-  for (int e = tid; e < (16 - n_row) * OS; e += 256) ol[n_row * OS + e] = 0;
+  for (int e = tid; e < (16 - n_row) * OS; e += 512) ol[n_row * OS + e] = 0;
   __syncthreads();
-  constexpr int R4 = RC * 16;                                            // float4 columns of a latent
-  const int items = n_row * R4, G = items >= 256 ? 1 : 256 / items, g = G > 1 ? tid / items : 0;
-  const size_t step = (size_t)p.H * p.rankp;
-  for (int e = G > 1 ? tid - g * items : tid; e < items; e += 256) {
-    const int i = e / R4, c = e - i * R4, row = row0 + i, n = live(row);
-    const float* o = lat_o(p.ws, p, M, row, 0) + (size_t)h * p.rankp + 4 * c;
+  for (int e = G > 1 ? tid - g * items : tid; e < items; e += 512) {
+    const int i = e / R4, c = e - i * R4, n = live(row0 + i);
+    const float* o = part_of(e);
     float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
+    auto add = [&](const float4 (&x)[U], int s0) {
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int s = s0 + u * G;
+        const float f = s < n ? wt[i][s] : -1.f;
+        if (f >= 0.f) a.x = fmaf(f, x[u].x, a.x), a.y = fmaf(f, x[u].y, a.y), a.z = fmaf(f, x[u].z, a.z), a.w = fmaf(f, x[u].w, a.w);
+      }
+    };
     if (g < G) {
-      for (int s0 = g; s0 < n; s0 += 8 * G) {
-        float4 x[8];
+      if (G > 1) add(x0, g);
+      for (int s0 = G > 1 ? g + U * G : g; s0 < n; s0 += U * G) {
+        float4 x[U];
 #pragma unroll
-        for (int u = 0; u < 8; ++u) x[u] = *(const float4*)(o + min(s0 + u * G, n - 1) * step);
-#pragma unroll
-        for (int u = 0; u < 8; ++u) {
-          const int s = s0 + u * G;
-          const float f = s < n ? wt[i][s] : -1.f;
-          if (f >= 0.f) a.x = fmaf(f, x[u].x, a.x), a.y = fmaf(f, x[u].y, a.y), a.z = fmaf(f, x[u].z, a.z), a.w = fmaf(f, x[u].w, a.w);
-        }
+        for (int u = 0; u < U; ++u) x[u] = *(const float4*)(o + min(s0 + u * G, n - 1) * step);
+        add(x, s0);
       }
     }
     if (G == 1) *(u32x2_t*)(ol + i * OS + 4 * c) = (u32x2_t){pack_bf16x2(a.x, a.y), pack_bf16x2(a.z, a.w)};
@@ -257,10 +271,8 @@ __global__ void __launch_bounds__(256) k_latent_out(LatP p) {
   f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int c = 0; c < 2 * RC; ++c) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[c], *(const bf16x8_t*)(ol + lc * OS + c * 32 + lg * 8), acc, 0, 0, 0);
-  const int v = v0 + lg * 4;
   if (lc < n_row && v < p.vdim) {
     const size_t row = row0 + lc;
-    const u32x2_t z = *(const u32x2_t*)((const bf16_t*)p.y + row * p.ld + lat_gate_col(p) + h * p.vdim + v);
     *(u32x2_t*)((bf16_t*)p.out + row * p.H * p.vdim + h * p.vdim + v) =
         (u32x2_t){pack_bf16x2(acc[0] * lat_gate(bf16lo(z[0])), acc[1] * lat_gate(bf16hi(z[0]))),
                   pack_bf16x2(acc[2] * lat_gate(bf16lo(z[1])), acc[3] * lat_gate(bf16hi(z[1])))};
@@ -379,7 +391,7 @@ template <int RC, int RT> static int launch_attn(const LatP& p, hipStream_t s) {
     set = true;
   }
   hipLaunchKernelGGL((k_latent_attn<RC, RT>), dim3(p.n_split, p3v_cdiv(p.H, 16), p.B * p.L), dim3(256), (LatCfg<RC, RT>::LDS), s, p);
-  hipLaunchKernelGGL(k_latent_out<RC>, dim3(p.H, p3v_cdiv(p.vdim, 64), p3v_cdiv(p.B * p.L, 16)), dim3(256), 0, s, p);
+  hipLaunchKernelGGL(k_latent_out<RC>, dim3(p.H, p3v_cdiv(p.vdim, 128), p3v_cdiv(p.B * p.L, 16)), dim3(512), 0, s, p);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
 }

@@ -13,7 +13,7 @@ template <int KC, int VT> struct PromptCfg {                              // KC:
 };
 
 template <int KC, int VT>
-__global__ void __launch_bounds__(256) k_latent_prompt(LatP p) {
+__global__ void __launch_bounds__(256, KC * 4 + VT * 16 <= 112 && (KC <= 12 || VT <= 2) ? 2 : 1) k_latent_prompt(LatP p) {
   typedef PromptCfg<KC, VT> C;
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   bf16_t *Ks = (bf16_t*)smem, *Vs = (bf16_t*)(smem + C::K);
