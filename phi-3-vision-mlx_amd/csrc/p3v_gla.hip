@@ -26,6 +26,12 @@ struct GlaP {
   int B, L, H, dim, vdim, rank, ld, past, R, keep, n_tok, store;
 };
 
+// workgroup barrier for LDS data only: global loads stay in flight across it
+__device__ __forceinline__ void lds_barrier() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
 // log2 of the decay, from z = W_a2 a1 + b: log sigmoid(z) = min(z, 0) - log(1 + x) with x = e^-|z|, the rounding of 1 + x given back
 __device__ __forceinline__ float log2_decay(float z, float inv_tau) {
   const float x = __builtin_amdgcn_exp2f(-fabsf(z) * GLA_LOG2E), u = 1.f + x;
@@ -173,7 +179,7 @@ __device__ __forceinline__ void gla_decays(const GlaP& p, int b, int h, int l0, 
   const T* base = (const T*)p.y + ((size_t)b * p.L + l0) * p.ld + 2 * p.H * (dim + p.vdim);
   for (int r0 = 0; r0 < p.rank; r0 += 16) {
     const int nr = min(16, p.rank - r0);
-    if (r0) __syncthreads();
+    if (r0) lds_barrier();
 #pragma unroll
     for (int i = 0; i < GLA_C * 16 / 256; ++i) {
       const int t = (tid >> 4) + i * 16, r = tid & 15;
@@ -184,7 +190,7 @@ __device__ __forceinline__ void gla_decays(const GlaP& p, int b, int h, int l0, 
 #pragma unroll
       for (int r = 0; r < 16; ++r) w[r] = r < nr ? bf16_to_f32(p.a2[(size_t)(h * dim + d) * p.rank + r0 + r]) : 0.f;
     }
-    __syncthreads();
+    lds_barrier();
     if (mine) {
       const float bias = bf16_to_f32(p.a2b[h * dim + d]);
       const bool last = r0 + 16 >= p.rank;
@@ -204,48 +210,61 @@ __device__ __forceinline__ void gla_decays(const GlaP& p, int b, int h, int l0, 
       }
     }
   }
-  __syncthreads();
+  lds_barrier();
   float off = 0.f;
   if (mine)
     for (int i = 0; i < g; ++i) off += c[((i + 1) * per - 1) * S + d];
-  __syncthreads();
+  lds_barrier();
   if (mine && g > 0)
     for (int t = g * per; t < (g + 1) * per; ++t) c[t * S + d] += off;
-  __syncthreads();
+  lds_barrier();
 }
 
-// rows of 64 tokens -> LDS, channel rows of tokens (row stride GLA_TS); dead tokens and channels behind n are zero.  A wave takes 32
-// tokens x 16 channels, 8 channels a lane: its LDS writes fall into distinct banks.
-template <typename T>
-__device__ __forceinline__ void gla_transpose(const T* src, int ld, int n, int lo, int hi, T* dst, int tid) {
-  const int t8 = tid & 31, c8 = (tid >> 5) * 8;
-  for (int c0 = c8; c0 < gla_dim16(n); c0 += 64)
+// Rows of 64 tokens, NC x 64 channels at most, through registers (requested early, written to LDS late).  A wave takes 32 tokens x 16 channels,
+// 8 channels a lane: transposed LDS writes then fall into distinct banks.  Dead tokens and channels behind n are zero.
+template <typename T, int NC> struct GlaRows {
+  static constexpr int W = (int)sizeof(T) / 2;                           // 16-byte pieces of 8 values
+  u32x4_t x[NC][2][W];
+  __device__ __forceinline__ void load(const T* src, int ld, int n, int lo, int hi, int tid) {
+    const int t8 = tid & 31, c8 = (tid >> 5) * 8;
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const int t = t8 + 32 * i;
-      __attribute__((aligned(16))) T x[8] = {};
-      if (t >= lo && t < hi && c0 < n) {
+    for (int c = 0; c < NC; ++c)
 #pragma unroll
-        for (int j = 0; j < 8; j += 16 / (int)sizeof(T)) *(u32x4_t*)(x + j) = *(const u32x4_t*)(src + (size_t)t * ld + c0 + j);
+      for (int i = 0; i < 2; ++i) {
+        const int t = t8 + 32 * i, c0 = c * 64 + c8;
+        const bool live = t >= lo && t < hi && c0 < n;
+#pragma unroll
+        for (int j = 0; j < W; ++j) {
+          x[c][i][j] = (u32x4_t){0u, 0u, 0u, 0u};
+          if (live) x[c][i][j] = *(const u32x4_t*)(src + (size_t)t * ld + c0 + j * (8 / W));
+        }
       }
+  }
+  __device__ __forceinline__ float get(int c, int i, int j) const {
+    if constexpr (W == 1) return j & 1 ? bf16hi(x[c][i][0][j >> 1]) : bf16lo(x[c][i][0][j >> 1]);
+    else return __uint_as_float(x[c][i][j >> 2][j & 3]);
+  }
+  __device__ __forceinline__ T raw(int c, int i, int j) const {
+    if constexpr (W == 1) return (T)(x[c][i][0][j >> 1] >> (16 * (j & 1)));
+    else return __uint_as_float(x[c][i][j >> 2][j & 3]);
+  }
+  // channel rows of tokens, row stride GLA_TS
+  __device__ __forceinline__ void put_transposed(T* dst, int n, int tid) const {
+    const int t8 = tid & 31, c8 = (tid >> 5) * 8;
 #pragma unroll
-      for (int j = 0; j < 8; ++j) dst[(c0 + j) * GLA_TS + t] = x[j];
-    }
-}
-__device__ __forceinline__ void load4(const bf16_t* p, float (&v)[4]) {
-  const u32x2_t w = *(const u32x2_t*)p;
-  v[0] = bf16lo(w[0]), v[1] = bf16hi(w[0]), v[2] = bf16lo(w[1]), v[3] = bf16hi(w[1]);
-}
-__device__ __forceinline__ void load4(const float* p, float (&v)[4]) {
-  const float4 w = *(const float4*)p;
-  v[0] = w.x, v[1] = w.y, v[2] = w.z, v[3] = w.w;
-}
-__device__ __forceinline__ void store4(bf16_t* p, const float (&v)[4]) { *(u32x2_t*)p = (u32x2_t){pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])}; }
-__device__ __forceinline__ void store4(float* p, const float (&v)[4]) { *(float4*)p = make_float4(v[0], v[1], v[2], v[3]); }
+    for (int c = 0; c < NC; ++c)
+      if (c * 64 + c8 < gla_dim16(n))
+#pragma unroll
+        for (int i = 0; i < 2; ++i)
+#pragma unroll
+          for (int j = 0; j < 8; ++j) dst[(c * 64 + c8 + j) * GLA_TS + t8 + 32 * i] = raw(c, i, j);
+  }
+};
 
 // The fp32 MFMA takes one k per lane group; four of them in a row are given k = 4 group + 0 .. 3 of a run of 16, so that an operand's four
 // values are one LDS read.
-template <typename T>
+// NK, NV: 64-channel groups of a key, of a value
+template <typename T, int NK, int NV>
 __global__ void __launch_bounds__(256) k_gla_chunk(GlaP p) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   const int ch = blockIdx.x, h = blockIdx.y, b = blockIdx.z, tid = threadIdx.x, lane = tid & 63, lc = lane & 15, lg = lane >> 4;
@@ -256,13 +275,20 @@ __global__ void __launch_bounds__(256) k_gla_chunk(GlaP p) {
   int lo, hi;
   gla_span(p, b, l0, lo, hi);
   const T* base = (const T*)p.y + ((size_t)b * p.L + l0) * p.ld;
-  gla_transpose<T>(base + 2 * p.H * dim + h * vdim, p.ld, vdim, lo, hi, vt, tid);
+  GlaRows<T, NK> kx;
+  GlaRows<T, NV> vx;
+  vx.load(base + 2 * p.H * dim + h * vdim, p.ld, vdim, lo, hi, tid);
+  kx.load(base + (p.H + h) * dim, p.ld, dim, lo, hi, tid);
   gla_decays<T>(p, b, h, l0, lo, hi, cum, DS, kd);
+  vx.put_transposed(vt, vdim, tid);
   const size_t row = (size_t)ch * p.B * p.H + (size_t)b * p.H + h;
   float* decay = p.ws + gla_decay_at(p, gridDim.x) + row * dim;
   float* sums = p.ws + gla_sums_at(p, gridDim.x) + ((size_t)b * p.L + l0) * p.H * dim + h * dim;
   const int t8 = tid & 31, c8 = (tid >> 5) * 8;
-  for (int c0 = c8; c0 < gla_dim16(dim); c0 += 64) {
+#pragma unroll
+  for (int n = 0; n < NK; ++n) {
+    const int c0 = n * 64 + c8;
+    if (c0 >= gla_dim16(dim)) continue;
     float end[8] = {};
     if (c0 < dim) load_acts<8>(cum + (GLA_C - 1) * DS + c0, end);
     if (t8 == 0 && c0 < dim)
@@ -271,12 +297,11 @@ __global__ void __launch_bounds__(256) k_gla_chunk(GlaP p) {
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
       const int t = t8 + 32 * i;
-      float x[8] = {}, c[8] = {};
+      float c[8] = {};
       if (c0 < dim) load_acts<8>(cum + t * DS + c0, c);
-      if (t >= lo && t < hi && c0 < dim) load_acts<8>(base + (size_t)t * p.ld + (p.H + h) * dim + c0, x);
       if (l0 + t < p.L && c0 < dim) store_acts<8>(sums + (size_t)t * p.H * dim + c0, c);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) kd[(c0 + j) * GLA_TS + t] = x[j] * __builtin_amdgcn_exp2f(fminf(end[j] - c[j], 0.f));
+      for (int j = 0; j < 8; ++j) kd[(c0 + j) * GLA_TS + t] = kx.get(n, i, j) * __builtin_amdgcn_exp2f(fminf(end[j] - c[j], 0.f));
     }
   }
   __syncthreads();
@@ -344,7 +369,7 @@ __global__ void __launch_bounds__(256) k_gla_scan(GlaP p, int nc) {
 // lane's pairs are the operand of the product with the values as they lie.  VT: 16-channel tiles of a value.
 #define GLA_SAFE 60.f
 template <typename T, int VT>
-__global__ void __launch_bounds__(256) k_gla_out(GlaP p) {
+__global__ void __launch_bounds__(256, VT <= 8 ? 3 : 2) k_gla_out(GlaP p) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   const int ch = blockIdx.x, h = blockIdx.y, b = blockIdx.z, tid = threadIdx.x, lane = tid & 63, lc = lane & 15, lg = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -355,7 +380,8 @@ __global__ void __launch_bounds__(256) k_gla_out(GlaP p) {
   gla_span(p, b, l0, lo, hi);
   const T* base = (const T*)p.y + ((size_t)b * p.L + l0) * p.ld;
   const float* sums = p.ws + gla_sums_at(p, gridDim.x) + ((size_t)b * p.L + l0) * p.H * dim + h * dim;
-  gla_transpose<T>(base + 2 * p.H * dim + h * vdim, p.ld, vdim, lo, hi, vt, tid);
+  GlaRows<T, (VT + 3) / 4> vx;
+  vx.load(base + 2 * p.H * dim + h * vdim, p.ld, vdim, lo, hi, tid);
   const int n4 = gla_dim16(dim) / 4, t4 = tid >> 4;
   for (int c = tid & 15; c < n4; c += 16)
 #pragma unroll
@@ -366,7 +392,22 @@ __global__ void __launch_bounds__(256) k_gla_out(GlaP p) {
       if (t >= lo && t < hi && 4 * c < dim) load4(base + (size_t)t * p.ld + (p.H + h) * dim + 4 * c, y);
       store4(cum + t * DS + 4 * c, x), store4(k + t * DS + 4 * c, y);
     }
-  __syncthreads();
+  vx.put_transposed(vt, vdim, tid);
+  const int l = min(l0 + t0 + lc, p.L - 1);                              // this lane's token
+  const T* q = (const T*)p.y + ((size_t)b * p.L + l) * p.ld + h * dim;
+  const float* S = p.ws + ((size_t)ch * p.B * p.H + (size_t)b * p.H + h) * dim * vdim;
+  struct { float q[4], s[VT][4]; } x;                                    // query and starting state of 16 key channels
+  auto request = [&](int d0) {
+    const int d = d0 + 4 * lg;
+    x.q[0] = x.q[1] = x.q[2] = x.q[3] = 0.f;
+    if (d < dim) load4(q + d, x.q);
+#pragma unroll
+    for (int j = 0; j < VT; ++j)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) x.s[j][i] = S[(size_t)min(d + i, dim - 1) * vdim + min(j * 16 + lc, vdim - 1)];
+  };
+  request(0);
+  lds_barrier();
   const float* ref = cum + max(t0 - 1, 0) * DS;                          // decays before this block (wave 0: none)
   bool strong = false;                                                   // does some channel decay too much over the block?
   const int tl = min(t0 + 15, p.L - 1 - l0);                             // its last row in memory
@@ -374,28 +415,20 @@ __global__ void __launch_bounds__(256) k_gla_out(GlaP p) {
     for (int d = lane; d < dim; d += 64) strong |= (wave ? ref[d] : 0.f) - cum[tl * DS + d] > GLA_SAFE;
   strong = __builtin_amdgcn_ballot_w64(strong) != 0;
 
-  const int l = min(l0 + t0 + lc, p.L - 1);                              // this lane's token
-  const T* q = (const T*)p.y + ((size_t)b * p.L + l) * p.ld + h * dim;
-  const float* S = p.ws + ((size_t)ch * p.B * p.H + (size_t)b * p.H + h) * dim * vdim;
   f32x4_t sc[4], o[VT];
 #pragma unroll
   for (int j = 0; j < 4; ++j) sc[j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int j = 0; j < VT; ++j) o[j] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
   for (int d0 = 0; d0 < dim; d0 += 16) {
+    if (d0) request(d0);                                                 // (not a step ahead: the registers are worth more as occupancy)
     const int d = d0 + 4 * lg;
-    float qv[4] = {0.f, 0.f, 0.f, 0.f}, ct[4], rf[4] = {0.f, 0.f, 0.f, 0.f}, qd[4];
-    if (d < dim) load4(q + d, qv);
-    float sv[VT][4];
-#pragma unroll
-    for (int j = 0; j < VT; ++j)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) sv[j][i] = S[(size_t)min(d + i, dim - 1) * vdim + min(j * 16 + lc, vdim - 1)];
+    float qv[4], ct[4], rf[4] = {0.f, 0.f, 0.f, 0.f}, qd[4];
     load4(cum + (t0 + lc) * DS + d, ct);
     if (wave) load4(ref + d, rf);
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      qv[i] *= p.q_scale * __builtin_amdgcn_exp2f(fminf(ct[i] - rf[i], 0.f));
+      qv[i] = x.q[i] * p.q_scale * __builtin_amdgcn_exp2f(fminf(ct[i] - rf[i], 0.f));
       qd[i] = qv[i] * __builtin_amdgcn_exp2f(rf[i]);
     }
 #pragma unroll
@@ -411,7 +444,7 @@ __global__ void __launch_bounds__(256) k_gla_out(GlaP p) {
 #pragma unroll
     for (int j = 0; j < VT; ++j)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) o[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(sv[j][i], qd[i], o[j], 0, 0, 0);
+      for (int i = 0; i < 4; ++i) o[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(x.s[j][i], qd[i], o[j], 0, 0, 0);
   }
 #pragma unroll
   for (int j = 0; j < 4; ++j)
@@ -498,12 +531,21 @@ static int gla_set_lds(const void* fn, bool& done) {
   done = true;
   return P3V_OK;
 }
-template <typename T> static int gla_states(GlaP p, int n_tok, int store, hipStream_t s) {
+template <typename T, int NK, int NV> static int gla_chunk(const GlaP& p, int nc, hipStream_t s) {
   static bool set = false;
-  if (gla_set_lds((const void*)k_gla_chunk<T>, set) != P3V_OK) return P3V_ERR_HIP;
+  if (gla_set_lds((const void*)k_gla_chunk<T, NK, NV>, set) != P3V_OK) return P3V_ERR_HIP;
+  hipLaunchKernelGGL((k_gla_chunk<T, NK, NV>), dim3(nc, p.H, p.B), dim3(256), gla_lds_chunk(p.dim, p.vdim, (int)sizeof(T)), s, p);
+  P3V_CHECK_LAUNCH();
+  return P3V_OK;
+}
+template <typename T, int NK> static int gla_chunk_v(const GlaP& p, int nc, hipStream_t s) {
+  return p.vdim <= 64 ? gla_chunk<T, NK, 1>(p, nc, s) : p.vdim <= 128 ? gla_chunk<T, NK, 2>(p, nc, s) : gla_chunk<T, NK, 4>(p, nc, s);
+}
+template <typename T> static int gla_states(GlaP p, int n_tok, int store, hipStream_t s) {
   const int nc = p3v_cdiv(n_tok, GLA_C);
   p.n_tok = n_tok, p.store = store;
-  hipLaunchKernelGGL(k_gla_chunk<T>, dim3(nc, p.H, p.B), dim3(256), gla_lds_chunk(p.dim, p.vdim, (int)sizeof(T)), s, p);
+  const int rc = p.dim <= 64 ? gla_chunk_v<T, 1>(p, nc, s) : gla_chunk_v<T, 2>(p, nc, s);
+  if (rc != P3V_OK) return rc;
   hipLaunchKernelGGL(k_gla_scan, dim3(p3v_cdiv((long)p.dim * p.vdim / 4, 256), p.B * p.H), dim3(256), 0, s, p, nc);
   P3V_CHECK_LAUNCH();
   return P3V_OK;

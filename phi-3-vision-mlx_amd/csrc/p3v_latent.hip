@@ -11,8 +11,9 @@
 #include "p3v_latent.h"
 
 // ---------------------------------------------------------------- append: one wave per new token
-// latent = rms(c) c_norm, key part rotated -> cache row.  ROT_Q: the queries of the row are rotated in place.
-template <typename T>
+#define LAT_VEC_RANK 1024            // widest latent of the vector form
+// latent = rms(c) c_norm, key part rotated -> cache row.  rot_q: the queries of the row are rotated in place, four pairs at a time where V = 4.
+template <typename T, int V = 1>
 __device__ __forceinline__ void latent_append_row(const LatP& p, int row, int lane, bool rot_q) {
   const int b = row / p.L, past = p.d_past ? *p.d_past : p.past, col = past + row - b * p.L, first = p.pad_len ? p.pad_len[b] : 0;
   const int pos = min(max(col - first, 0), p.tab_n - 1), half = p.rot / 2, W = p.dim + p.rot;
@@ -21,13 +22,52 @@ __device__ __forceinline__ void latent_append_row(const LatP& p, int row, int la
   T* dst = (T*)p.c + ((size_t)b * p.Tp + col) * (p.rankp + p.rotp);
   const float *cs = p.cos_t + (size_t)pos * half, *sn = p.sin_t + (size_t)pos * half;
   float ss = 0.f;
-  for (int i = lane; i < p.rank; i += 64) { const float v = load_act(d + i); ss += v * v; }
-  const float r = 1.f / sqrtf(wave_sum(ss) / (float)p.rank + p.eps);
-  for (int i = lane; i < p.rank; i += 64) store_act(dst + i, load_act(d + i) * r * bf16_to_f32(p.c_norm[i]));
+  if constexpr (V == 4) {                                                // the latent in registers, read once
+    float x[LAT_VEC_RANK / 512][8], w[LAT_VEC_RANK / 512][8];
+#pragma unroll
+    for (int k = 0; k < LAT_VEC_RANK / 512; ++k) {
+      const int i = (k * 64 + lane) * 8;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[k][j] = 0.f;
+      if (i < p.rank) load_acts<8>(d + i, x[k]), load_acts<8>(p.c_norm + i, w[k]);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss += x[k][j] * x[k][j];
+    }
+    const float r = 1.f / sqrtf(wave_sum(ss) / (float)p.rank + p.eps);
+#pragma unroll
+    for (int k = 0; k < LAT_VEC_RANK / 512; ++k) {
+      const int i = (k * 64 + lane) * 8;
+      if (i < p.rank) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[k][j] *= r * w[k][j];
+        store_acts<8>(dst + i, x[k]);
+      }
+    }
+  } else {
+    for (int i = lane; i < p.rank; i += 64) { const float v = load_act(d + i); ss += v * v; }
+    const float r = 1.f / sqrtf(wave_sum(ss) / (float)p.rank + p.eps);
+    for (int i = lane; i < p.rank; i += 64) store_act(dst + i, load_act(d + i) * r * bf16_to_f32(p.c_norm[i]));
+  }
   for (int i = lane; i < half; i += 64) {
     const float u = load_act(d + p.rank + i), v = load_act(d + p.rank + half + i);
     store_act(dst + p.rankp + i, u * cs[i] - v * sn[i]);
     store_act(dst + p.rankp + half + i, v * cs[i] + u * sn[i]);
+  }
+  if constexpr (V == 4) {
+    if (rot_q) {
+      const int per = half / 4;
+#pragma unroll 2
+      for (int e = lane; e < p.H * per; e += 64) {
+        const int h = e / per, i = (e - h * per) * 4;
+        T* q = y + h * W + p.dim + i;
+        float u[4], v[4], c[4], s[4], a[4], b4[4];
+        load4(q, u), load4(q + half, v), load4(cs + i, c), load4(sn + i, s);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) a[j] = u[j] * c[j] - v[j] * s[j], b4[j] = v[j] * c[j] + u[j] * s[j];
+        store4(q, a), store4(q + half, b4);
+      }
+    }
+    return;
   }
   if (rot_q)
     for (int e = lane; e < p.H * half; e += 64) {
@@ -38,10 +78,10 @@ __device__ __forceinline__ void latent_append_row(const LatP& p, int row, int la
       store_act(q + half, v * cs[i] + u * sn[i]);
     }
 }
-template <typename T>
+template <typename T, int V>
 __global__ void __launch_bounds__(256) k_latent_append(LatP p) {
   const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (row < p.B * p.L) latent_append_row<T>(p, row, threadIdx.x & 63, true);
+  if (row < p.B * p.L) latent_append_row<T, V>(p, row, threadIdx.x & 63, true);
 }
 
 // ---------------------------------------------------------------- queries into the latent space
@@ -51,7 +91,7 @@ __global__ void __launch_bounds__(256) k_latent_q(LatP p) {
   if (h == p.H) {
     if (blockIdx.y == 0)
       for (int i = wave; i < 16; i += 4)
-        if (row0 + i < M) latent_append_row<bf16_t>(p, row0 + i, lane, false);
+        if (row0 + i < M) latent_append_row<bf16_t, 4>(p, row0 + i, lane, false);
     return;
   }
   const int r0 = blockIdx.y * 64 + wave * 16, row = min(row0 + lc, M - 1);
@@ -188,7 +228,8 @@ __global__ void __launch_bounds__(256) k_latent_attn(LatP p) {
 }
 
 // ---------------------------------------------------------------- merge, value up-projection, gate
-// A workgroup per (head, 128 value dimensions, 16 rows); its weights are requested before the merge.
+// A workgroup per (head, 32 value dimensions, 16 rows): two 16-dimension tiles x four quarters of the rank; weights and, for few rows, the
+// partials are requested before anything else.
 #define LAT_MAX_SPLIT 128
 template <int RC>
 __global__ void __launch_bounds__(512) k_latent_out(LatP p) {
@@ -197,7 +238,7 @@ __global__ void __launch_bounds__(512) k_latent_out(LatP p) {
   __shared__ __attribute__((aligned(16))) bf16_t ol[16 * OS];
   __shared__ float4 part[512];
   const int h = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, lc = lane & 15, lg = lane >> 4;
-  const int row0 = blockIdx.z * 16, M = p.B * p.L, n_row = min(16, M - row0), v0 = blockIdx.y * 128 + wave * 16;
+  const int row0 = blockIdx.z * 16, M = p.B * p.L, n_row = min(16, M - row0), kq = wave >> 1, v0 = blockIdx.y * 32 + (wave & 1) * 16;
   constexpr int R4 = RC * 16, U = 8;                                     // float4 columns of a latent; splits requested at once
   const int items = n_row * R4, G = items >= 512 ? 1 : 512 / items, g = G > 1 ? tid / items : 0;
   const size_t step = (size_t)p.H * p.rankp;
@@ -210,10 +251,11 @@ __global__ void __launch_bounds__(512) k_latent_out(LatP p) {
     for (int u = 0; u < U; ++u) x0[u] = *(const float4*)(o + min(min(g, G - 1) + u * G, p.n_split - 1) * step);
   }
   const int past = p.d_past ? *p.d_past : p.past;
-  bf16x8_t w[2 * RC];
+  constexpr int NW = (RC + 1) / 2;                                       // 32-rank chunks kq, kq + 4, .. of this wave
+  bf16x8_t w[NW];
   const bf16_t* wr = p.uv + ((size_t)h * p.vdim + min(v0 + lc, p.vdim - 1)) * p.rankp + lg * 8;
 #pragma unroll
-  for (int c = 0; c < 2 * RC; ++c) w[c] = *(const bf16x8_t*)(wr + c * 32);
+  for (int c = 0; c < NW; ++c) w[c] = *(const bf16x8_t*)(wr + min(kq + 4 * c, 2 * RC - 1) * 32);
   auto live = [&](int row) { return min(p.n_split, ((past + row % p.L) >> 6) / p.tiles_per_split + 1); };
   const float sk = bf16_to_f32(p.sink[h]) * LAT_LOG2E;
   const int v = v0 + lg * 4;
@@ -270,8 +312,14 @@ __global__ void __launch_bounds__(512) k_latent_out(LatP p) {
   __syncthreads();
   f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-  for (int c = 0; c < 2 * RC; ++c) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[c], *(const bf16x8_t*)(ol + lc * OS + c * 32 + lg * 8), acc, 0, 0, 0);
-  if (lc < n_row && v < p.vdim) {
+  for (int c = 0; c < NW; ++c)
+    if (kq + 4 * c < 2 * RC) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[c], *(const bf16x8_t*)(ol + lc * OS + (kq + 4 * c) * 32 + lg * 8), acc, 0, 0, 0);
+  f32x4_t* sum = (f32x4_t*)part;
+  if (kq) sum[tid] = acc;                                                // (nobody reads the merge's use of it any more)
+  __syncthreads();
+  if (kq == 0 && lc < n_row && v < p.vdim) {
+#pragma unroll
+    for (int k = 1; k < 4; ++k) acc += sum[tid + 128 * k];
     const size_t row = row0 + lc;
     *(u32x2_t*)((bf16_t*)p.out + row * p.H * p.vdim + h * p.vdim + v) =
         (u32x2_t){pack_bf16x2(acc[0] * lat_gate(bf16lo(z[0])), acc[1] * lat_gate(bf16hi(z[0]))),
@@ -364,8 +412,16 @@ extern "C" int p3v_latent_append(const p3v_latent_args_t* a, void* stream) {
   if (rc != P3V_OK) return rc;
   const LatP p = lat_params(a);
   const dim3 grid(p3v_cdiv((long)p.B * p.L, 4));
-  if (a->f32) hipLaunchKernelGGL(k_latent_append<float>, grid, dim3(256), 0, (hipStream_t)stream, p);
-  else hipLaunchKernelGGL(k_latent_append<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, p);
+  hipStream_t s = (hipStream_t)stream;
+  const bool vec = lat_aligned(p.dim, p.rot, p.vdim, p.rank) && p.ld % 8 == 0 && p.rank <= LAT_VEC_RANK &&
+                   (((uintptr_t)p.y | (uintptr_t)p.c | (uintptr_t)p.c_norm | (uintptr_t)p.cos_t | (uintptr_t)p.sin_t) & 15) == 0;
+  if (a->f32) {
+    if (vec) hipLaunchKernelGGL((k_latent_append<float, 4>), grid, dim3(256), 0, s, p);
+    else hipLaunchKernelGGL((k_latent_append<float, 1>), grid, dim3(256), 0, s, p);
+  } else {
+    if (vec) hipLaunchKernelGGL((k_latent_append<bf16_t, 4>), grid, dim3(256), 0, s, p);
+    else hipLaunchKernelGGL((k_latent_append<bf16_t, 1>), grid, dim3(256), 0, s, p);
+  }
   P3V_CHECK_LAUNCH();
   return P3V_OK;
 }
@@ -391,7 +447,7 @@ template <int RC, int RT> static int launch_attn(const LatP& p, hipStream_t s) {
     set = true;
   }
   hipLaunchKernelGGL((k_latent_attn<RC, RT>), dim3(p.n_split, p3v_cdiv(p.H, 16), p.B * p.L), dim3(256), (LatCfg<RC, RT>::LDS), s, p);
-  hipLaunchKernelGGL(k_latent_out<RC>, dim3(p.H, p3v_cdiv(p.vdim, 128), p3v_cdiv(p.B * p.L, 16)), dim3(512), 0, s, p);
+  hipLaunchKernelGGL(k_latent_out<RC>, dim3(p.H, p3v_cdiv(p.vdim, 32), p3v_cdiv(p.B * p.L, 16)), dim3(512), 0, s, p);
   P3V_CHECK_LAUNCH();
   return P3V_OK;
 }
@@ -403,7 +459,7 @@ extern "C" int p3v_latent_rows(const p3v_latent_args_t* a, void* stream) {
   if (!a->ukt || !a->uv || !a->q || !a->out || !a->ws || a->n_split <= 0 || a->n_split > LAT_MAX_SPLIT) return P3V_ERR_ARG;
   if (a->f32 || !lat_aligned(a->dim, a->rot, a->vdim, a->rank) || !lat_rows_fit(a->rank, a->rot) || a->ld % 8) return P3V_ERR_UNSUPPORTED;
   if (a->rankp != (a->rank + 63) / 64 * 64 || a->rotp != (a->rot + 31) / 32 * 32 || a->dimp < a->dim || a->dimp % 32) return P3V_ERR_ARG;
-  if ((long)a->B * a->L > 65535 || (((uintptr_t)a->y | (uintptr_t)a->ukt | (uintptr_t)a->uv | (uintptr_t)a->c | (uintptr_t)a->q | (uintptr_t)a->ws | (uintptr_t)a->out) & 15)) return P3V_ERR_ARG;
+  if ((long)a->B * a->L > 65535 || (((uintptr_t)a->y | (uintptr_t)a->ukt | (uintptr_t)a->uv | (uintptr_t)a->c | (uintptr_t)a->c_norm | (uintptr_t)a->q | (uintptr_t)a->ws | (uintptr_t)a->out) & 15)) return P3V_ERR_ARG;
   LatP p = lat_params(a);
   // (the position may be a device value: the splits then cover the capacity)
   p.tiles_per_split = p3v_cdiv(p3v_cdiv(a->L == 1 || a->d_past ? a->Tp : a->past + a->L, 64), a->n_split);

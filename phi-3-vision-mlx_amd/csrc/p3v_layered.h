@@ -47,6 +47,18 @@ template <int V> __device__ __forceinline__ void store_acts(float* p, const floa
   }
 }
 
+// four consecutive ones, 8-byte (bf16) or 16-byte (fp32) aligned
+__device__ __forceinline__ void load4(const bf16_t* p, float (&v)[4]) {
+  const u32x2_t w = *(const u32x2_t*)p;
+  v[0] = bf16lo(w[0]), v[1] = bf16hi(w[0]), v[2] = bf16lo(w[1]), v[3] = bf16hi(w[1]);
+}
+__device__ __forceinline__ void load4(const float* p, float (&v)[4]) {
+  const float4 w = *(const float4*)p;
+  v[0] = w.x, v[1] = w.y, v[2] = w.z, v[3] = w.w;
+}
+__device__ __forceinline__ void store4(bf16_t* p, const float (&v)[4]) { *(u32x2_t*)p = (u32x2_t){pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3])}; }
+__device__ __forceinline__ void store4(float* p, const float (&v)[4]) { *(float4*)p = make_float4(v[0], v[1], v[2], v[3]); }
+
 // ---- kernel parameters
 struct DytP {
   const float* x; const bf16_t* w; const bf16_t* b; const bf16_t* mu; float* hist; const int32_t* pad_len; const int32_t* d_past;
