@@ -111,7 +111,7 @@ int p3v_gemm_rows_slices(int M, int N, int K, int epilogue);
  * (M == 1: VALU dot products; 2 <= M <= 16: the weight rows go straight from HBM into MFMA fragments).
  * Same call sites as p3v_gemm when L*B is small.  Optional fused RMSNorm of x
  * (norm_w != null: x is normalised with norm_w/eps before use, phi.py:482,484).
- * Epilogues: NONE, RESID_BF16, SILU_MUL (W = [gate;up]), F32, SCALE_RESID_F32. */
+ * Epilogues: NONE, RESID_BF16, SILU_MUL / GELU_MUL (W = [gate;up]), F32, SCALE_RESID_F32. */
 typedef struct {
   const uint16_t* x;      /* [M, K] bf16 */
   const uint16_t* W;      /* [N or 2N, K] bf16 */
@@ -449,11 +449,11 @@ typedef struct {
 int p3v_dyt(const p3v_dyt_args_t* args /* host */, void* out, int out_f32, void* stream);
 
 /* p3v_gemv whose input row is p3v_dyt of the fp32 residual row (a->x unused; d: B = 1, L = 1): the dynamic tanh and the token shift
- * in the projection's prologue.  M = 1, K in {1024, 2048, 3072, 4096, 8192}, epilogue NONE or SILU_MUL: otherwise P3V_ERR_UNSUPPORTED and
+ * in the projection's prologue.  M = 1, K in {1024, 2048, 3072, 4096, 8192}, epilogue NONE, SILU_MUL or GELU_MUL: otherwise P3V_ERR_UNSUPPORTED and
  * the caller runs the two calls. */
 int p3v_gemv_dyt(const p3v_gemv_args_t* args /* host */, const p3v_dyt_args_t* d /* host */, void* stream);
 
-/* p3v_gemm for every size and for fp32 A (a_f32: A is float*), plain fp32 arithmetic.  Epilogues NONE (out in A's type), F32, SILU_MUL,
+/* p3v_gemm for every size and for fp32 A (a_f32: A is float*), plain fp32 arithmetic.  Epilogues NONE (out in A's type), F32, SILU_MUL, GELU_MUL,
  * SCALE_RESID_F32. */
 int p3v_gemm_any(const p3v_gemm_args_t* args /* host */, int a_f32, void* stream);
 
