@@ -291,7 +291,7 @@ def pudisun_config_dict(width, ff, latent, gla, layers=LAYERED_LAYERS):
     rotary = {"base": 10000.0, "dims": rot, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}
     mixers = [("latent_attention", {"heads": H, "dim": dim, "rot_dim": rot, "vdim": vdim, "kv_rank": rank, "rot": rotary, "scale": (dim + rot) ** -0.5}),
               ("gla", {"heads": gla[0], "dim": gla[1], "vdim": gla[2], "tau": 16.0})]
-    return {"architecture": "Pudisun", "width": width, "vocab": LAYERED_VOCAB, "norm": {"eps": 1e-5}, "residual_mult": 0.7, "logit_scale": 0.25,
+    return {"architecture": "Pudisun", "width": width, "vocab": LAYERED_VOCAB, "norm": {"eps": 1e-5}, "residual_mult": 0.5, "logit_scale": 1.0,
             "layers": [{"type": t, "mixer": m, "mlp": {"kind": "dense", "ff": ff}} for t, m in (mixers * layers)[:layers]]}
 
 

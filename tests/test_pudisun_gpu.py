@@ -219,7 +219,7 @@ def test_rotation_reaches_far_positions():
 
 # ---------------------------------------------------------------- gated linear attention
 class Gla:
-    def __init__(self, H, dim, vdim, rank, B, dt, seed=0, tau=16.0, bias=(2.0, 1.5), R=2):
+    def __init__(self, H, dim, vdim, rank, B, dt, seed=0, tau=12.0, bias=(2.0, 1.5), R=2):
         from phi_3_vision_mlx_amd import config, mixers
         self.r, self.B, self.dt, self.R, self.tau = np.random.default_rng(seed), B, dt, R, tau
         self.m = config.GlaMixer(H, dim, vdim, tau)
@@ -262,7 +262,7 @@ class Gla:
         return np.concatenate([np.zeros((pad, o.shape[1])), o]), s
 
 
-GLA_SIZES = [(4, 48, 64, 16), (2, 96, 192, 16), (3, 128, 256, 40), (5, 8, 8, 4), (2, 64, 24, 33), (3, 24, 96, 8), (2, 20, 36, 16), (1, 7, 10, 3), (2, 160, 64, 16)]
+GLA_SIZES = [(6, 56, 72, 12), (2, 96, 192, 16), (3, 128, 256, 40), (5, 8, 8, 4), (2, 64, 24, 33), (3, 24, 96, 8), (2, 20, 36, 16), (1, 7, 10, 3), (2, 160, 64, 16)]
 
 
 @pytest.mark.parametrize("dt", [F32, BF16])
@@ -345,7 +345,7 @@ CONFIGS = {
     "shared": dict(width=192, vocab=512, eps=1e-5, mult=1.0, lscale=0.5, layers=[
         latent(8, 32, 16, 32, 64, ff=320), gla(4, 24, 32, ff=192), gla(4, 24, 32, ff=192, weights_of=1), latent(8, 32, 16, 32, 64, ff=320, weights_of=0),
         latent(6, 48, 32, 40, 96, ff=64), gla(4, 24, 32, ff=192, weights_of=2)]),
-    "streamed": dict(width=1024, vocab=330, eps=1e-5, mult=0.8, lscale=0.25, layers=[latent(16, 64, 32, 64, 256, ff=1024), gla(8, 64, 128, tau=16.0, ff=2048)]),
+    "streamed": dict(width=1024, vocab=330, eps=1e-5, mult=0.8, lscale=0.4, layers=[latent(16, 64, 32, 64, 256, ff=1024), gla(8, 64, 128, tau=16.0, ff=2048)]),
     "many": dict(width=256, vocab=384, eps=1e-6, mult=-0.5, lscale=3.0, layers=[latent(32, 128, 64, 128, 512, ff=256), latent(20, 16, 32, 96, 136, ff=64), gla(16, 96, 160, ff=128)]),
 }
 
