@@ -651,8 +651,12 @@ extern "C" int p3v_gemv(const p3v_gemv_args_t* a, void* stream) {
         default: break;
       }
   }
+  if (mt == 1 && a->epilogue == P3V_EPI_GELU_MUL && (a->K == 3072 || a->K == 8192)) {
+    const int rc = gemv3_layered<GEMV_GATED>(p, s);
+    if (rc != P3V_ERR_UNSUPPORTED) return rc;
+  }
   const int variant = p3v_tuning().gemv_variant;       // 1: generic kernel only; 3: streaming kernel where it applies
-  if (variant == 3 && mt == 1 && !scaled && a->N % 2 == 0 && (a->K == 3072 || a->K == 8192)) {
+  if (variant == 3 && mt == 1 && !scaled && a->epilogue != P3V_EPI_GELU_MUL && a->N % 2 == 0 && (a->K == 3072 || a->K == 8192)) {
     if (a->K == 3072) return launch_gemv3<1, 1, 6>(p, s);
     return launch_gemv3<1, 4, 4>(p, s);                  // 8192 = 4 stages x 4 chunks: keeps 2 waves/SIMD resident
   }
@@ -665,7 +669,7 @@ extern "C" int p3v_gemv(const p3v_gemv_args_t* a, void* stream) {
   // at ctx 2531, B = 2 / 3 / 4: 2.08 / 2.43 / 2.66 ms with the MT-row streaming kernel, 1.99 / 2.16 / 2.35 with this one);
   // P3V_GEMV8_MIN=5 restores the round-1 split
   const int rows8_min = p3v_tuning().gemv8_min;
-  if (rows_variant && variant == 3 && a->M >= 2 && a->M <= 4 && a->M < rows8_min && a->N % 2 == 0 && a->epilogue != P3V_EPI_F32 && !scaled &&
+  if (rows_variant && variant == 3 && a->M >= 2 && a->M <= 4 && a->M < rows8_min && a->N % 2 == 0 && a->epilogue != P3V_EPI_F32 && a->epilogue != P3V_EPI_GELU_MUL && !scaled &&
       (a->K == 3072 || a->K == 8192)) {
     if (a->K == 3072) return mt == 2 ? launch_gemv3<2, 1, 6>(p, s) : launch_gemv3<4, 1, 6>(p, s);
     return mt == 2 ? launch_gemv3<2, 4, 4>(p, s) : launch_gemv3<4, 4, 4>(p, s);

@@ -15,8 +15,9 @@ struct GemvP {
 };
 // Variants of the one-row body for the layered decoders (fp32 residual stream): GEMV_DYT = the input row is a dynamic tanh (+ token
 // shift) of the residual row, computed while the first weights are on their way; GEMV_RMS = it is the RMS norm of that row (dyt.x, dyt.w,
-// dyt.alpha = the gain, eps); GEMV_SCALED = out = resid + col_scale * acc in fp32.
-enum { GEMV_DYT = 1, GEMV_SCALED = 2, GEMV_RMS = 4 };
+// dyt.alpha = the gain, eps); GEMV_SCALED = out = resid + col_scale * acc in fp32; GEMV_GATED = nothing but any gated epilogue, which the plain body
+// does not carry (SiLU alone: the choice at run time costs its launches 0.7 %).
+enum { GEMV_DYT = 1, GEMV_SCALED = 2, GEMV_RMS = 4, GEMV_GATED = 8 };
 
 // 8 bf16 x 8 bf16 -> fp32 accumulate on v_dot2c_f32_bf16 (two products per instruction straight from the packed
 // operands): 4 VALU instructions per 16-byte weight chunk instead of 8 unpacks + 8 FMAs -- the GEMV's VALU pipe was
@@ -160,7 +161,7 @@ __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, i
   constexpr int XC = (CHUNKS + 255) / 256;              // x chunks per thread
   u32x4_t* xs = (u32x4_t*)smem;                         // [MT][CHUNKS] bf16 x (normalised)
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const bool silu = P3V_GATED(p.epi);
+  const bool silu = VAR ? P3V_GATED(p.epi) : p.epi == P3V_EPI_SILU_MUL;
   const bool has_res = p.epi == P3V_EPI_RESID_BF16;
   const int u_begin = wave < wpw ? min(p.units, (bx * wpw + wave) * units_per_wave) : p.units;
   const int u_end = min(p.units, u_begin + units_per_wave);
@@ -359,7 +360,7 @@ __device__ __forceinline__ void gemv3_body(const GemvP& p, int units_per_wave, i
             if constexpr (SCALED) {
               *(float2*)((float*)p.out + 2 * u) = make_float2(fbuf[buf].x + bf16lo(rbuf[buf][0]) * a0[0], fbuf[buf].y + bf16hi(rbuf[buf][0]) * a1[0]);
             } else if (silu) {
-              ((bf16_t*)p.out)[(size_t)m * p.N + u] = f32_to_bf16(p3v_gated(p.epi, a0[m], a1[m]));
+              ((bf16_t*)p.out)[(size_t)m * p.N + u] = f32_to_bf16(p3v_gated(VAR ? p.epi : P3V_EPI_SILU_MUL, a0[m], a1[m]));
             } else if (p.epi == P3V_EPI_F32) {
               ((float*)p.out)[(size_t)m * p.N + 2 * u] = a0[m];
               ((float*)p.out)[(size_t)m * p.N + 2 * u + 1] = a1[m];
